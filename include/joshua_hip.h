@@ -52,6 +52,12 @@ extern "C" {
 #define JQ_TYPE_Q5_1 7u
 #define JQ_TYPE_Q3_K 11u
 #define JQ_TYPE_Q5_K 13u
+/* Plain rows: jq_upload takes n x k elements in row-major order and keeps them in rows padded to 64 elements.
+ * A product with F32 weights runs in f32 throughout.  One with BF16 weights takes up to 8 activation rows in f32;
+ * more are rounded to bf16 for the matrix cores (f32 accumulation either way).  jq_block_geometry, which describes
+ * block formats, knows neither. */
+#define JQ_TYPE_F32 0u
+#define JQ_TYPE_BF16 30u
 
 typedef struct jq_weight jq_weight;
 
@@ -196,7 +202,8 @@ typedef struct {
     uint32_t n_expert_used;  /* k */
     uint32_t hidden;         /* h */
     uint32_t inter;          /* expert feed-forward length */
-    uint32_t gating;         /* 0 softmax, 1 sigmoid (src/quantized_deepseek2.rs:529-532) */
+    uint32_t gating;         /* 0 softmax, 1 sigmoid (src/quantized_deepseek2.rs:529-532), 2 softmax with the
+                              * router's bias part of the logits (it then counts in the weights, too) */
     uint32_t norm_topk;      /* divide the k weights by max(sum, 6.103515625e-5) */
     float weights_scale;     /* 0 or 1: none (src/quantized_deepseek2.rs:549-551) */
     uint32_t n_group;        /* <= 1: no group limit (src/quantized_deepseek2.rs:563-566) */
@@ -205,6 +212,10 @@ typedef struct {
      * expert has a limit of its own (src/quantized_deepseek4.rs:445-462, :2419-2448). */
     float swiglu_clamp;
     float swiglu_clamp_shared;
+    /* The gated unit of BF16 / F32 experts: g sigmoid(alpha g) (u + up_shift) over the clamped g and u; alpha 0
+     * stands for 1 (SwiGLU).  Experts in block formats take 0 or 1, and 0, only. */
+    float act_alpha;
+    float act_up_shift;
 } jq_moe_config;
 
 /* router_w is [E, h] row-major f32 on the host (ffn_gate_inp), router_bias [E]
@@ -394,11 +405,34 @@ int jq_gguf_upload(const jq_gguf *g, const char *name, jq_weight **out);
  * context_length. */
 int jq_qwen3_load_gguf(const char *path, uint32_t n_ctx, jq_model **out);
 
+/* ---- Models of any architecture ------------------------------------------------------
+ * jq_model_load picks the loader by what the path holds: a GGUF file by its general.architecture (qwen3, qwen3moe),
+ * a folder with config.json and model.safetensors by the configuration's "architecture" (Bozosun).  The jq_qwen3_*
+ * calls above and these work on the same objects.  No counterpart in the reference, whose model object is one Rust
+ * type per architecture. */
+#define JQ_COMPUTE_DEFAULT 0u  /* the precision the architecture is served with */
+#define JQ_COMPUTE_F32 1u      /* every product and activation in 32-bit; fails where the architecture has no such form */
+int jq_model_load(const char *path, uint32_t n_ctx, uint32_t compute, jq_model **out);
+void jq_model_free(jq_model *model);
+uint32_t jq_model_vocab(const jq_model *model);
+uint32_t jq_model_context(const jq_model *model);        /* tokens the caches hold */
+uint32_t jq_model_cached_tokens(const jq_model *model);  /* tokens fed so far */
+
+/* Appends n_tokens tokens at absolute position pos (the number of tokens fed so far) and writes the logits of the
+ * n_want places among them that `want` lists, [n_want, vocab], in that order.  n_want 0: none.  tokens and want are
+ * host pointers; logits goes to host or device memory, or may be NULL (jq_model_greedy then reads the last row). */
+int jq_model_forward(jq_model *model, const uint32_t *tokens, uint32_t n_tokens, uint32_t pos, const uint32_t *want,
+                     uint32_t n_want, float *logits, int logits_on_device, void *stream);
+/* Greedy pick over the last row of logits of the last forward (jq_qwen3_greedy's rule). */
+int jq_model_greedy(jq_model *model, uint32_t *token, void *stream);
+/* Forgets the fed tokens: keys, values and recurrent states. */
+int jq_model_reset(jq_model *model);
+
 /* ---- Model-level plugin boundary ----------------------------------------------------
  * The four symbols the reference engine looks up when it is started with a backend
  * library (reference: src/npu/mod.rs:32-50 contract; src/npu/vendor.rs:17-20
  * signatures, :49-56 symbol check, :95-121 init; src/main.rs:166-172 the switch).
- * init loads the GGUF at model_path as a dense Qwen3 decoder with a KV cache of
+ * init loads the model at model_path (jq_model_load) with caches of
  * n_ctx tokens and reports the vocabulary size; forward appends n_tokens tokens at
  * absolute position pos, which must equal the number of tokens fed so far, and
  * writes vocab logits for the last one; reset forgets the fed tokens.  0 is success;

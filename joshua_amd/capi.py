@@ -19,9 +19,12 @@ ALL_TYPES = (Q8_0, Q2_K, Q4_K, Q6_K, IQ2_XXS, MXFP4)
 # formats the reference serves through the canonical decode plus its 8-lane dot
 # (reference: src/quant_matmul.rs:228-248; sizes src/gguf_ext.rs:487-500)
 Q4_0, Q4_1, Q5_0, Q5_1, Q3_K, Q5_K = 2, 3, 6, 7, 11, 13
+# plain rows
+F32, BF16 = 0, 30
 GENERIC_TYPES = (Q4_0, Q4_1, Q5_0, Q5_1, Q3_K, Q5_K)
 TYPE_NAMES = {Q8_0: "Q8_0", Q2_K: "Q2_K", Q4_K: "Q4_K", Q6_K: "Q6_K", IQ2_XXS: "IQ2_XXS", MXFP4: "MXFP4", Q4_0: "Q4_0",
-              Q4_1: "Q4_1", Q5_0: "Q5_0", Q5_1: "Q5_1", Q3_K: "Q3_K", Q5_K: "Q5_K"}
+              Q4_1: "Q4_1", Q5_0: "Q5_0", Q5_1: "Q5_1", Q3_K: "Q3_K", Q5_K: "Q5_K",
+              F32: "F32", BF16: "BF16"}
 
 # Every symbol include/joshua_hip.h declares.
 EXPORTS = (
@@ -34,7 +37,8 @@ EXPORTS = (
     "jq_gguf_version", "jq_gguf_tensor_data_offset", "jq_gguf_tensor_count", "jq_gguf_metadata_count",
     "jq_gguf_tensor_at", "jq_gguf_find_tensor", "jq_gguf_tensor_bytes", "jq_gguf_meta_u32", "jq_gguf_meta_f32",
     "jq_gguf_meta_bool", "jq_gguf_meta_str", "jq_gguf_meta_array_len", "jq_gguf_upload",
-    "joshua_npu_init", "joshua_npu_forward", "joshua_npu_reset", "joshua_npu_free",
+    "jq_model_load", "jq_model_free", "jq_model_vocab", "jq_model_context", "jq_model_cached_tokens", "jq_model_forward",
+    "jq_model_greedy", "jq_model_reset", "joshua_npu_init", "joshua_npu_forward", "joshua_npu_reset", "joshua_npu_free",
 )
 
 
@@ -47,7 +51,8 @@ class MoeConfig(ctypes.Structure):
     _fields_ = [("n_expert", ctypes.c_uint32), ("n_expert_used", ctypes.c_uint32), ("hidden", ctypes.c_uint32),
                 ("inter", ctypes.c_uint32), ("gating", ctypes.c_uint32), ("norm_topk", ctypes.c_uint32),
                 ("weights_scale", ctypes.c_float), ("n_group", ctypes.c_uint32), ("topk_group", ctypes.c_uint32),
-                ("swiglu_clamp", ctypes.c_float), ("swiglu_clamp_shared", ctypes.c_float)]
+                ("swiglu_clamp", ctypes.c_float), ("swiglu_clamp_shared", ctypes.c_float),
+                ("act_alpha", ctypes.c_float), ("act_up_shift", ctypes.c_float)]
 
 
 class MlaConfig(ctypes.Structure):
@@ -71,21 +76,40 @@ class Qwen3Config(ctypes.Structure):
 _lib = None
 
 
-def lib() -> ctypes.CDLL:
+class _Library(ctypes.CDLL):
+    """The loaded library.  One that holds a subset of the symbols raises at the call of another."""
+
+    def __getattr__(self, name):
+        try:
+            return super().__getattr__(name)
+        except AttributeError:
+            if name not in EXPORTS:
+                raise
+
+            def missing(*_):
+                raise JoshuaHipError(f"{name} is not part of {self._name}")
+            setattr(self, name, missing)
+            return missing
+
+
+def lib(path: str = LIB_PATH, beside_torch: bool = True) -> ctypes.CDLL:
+    """The library, loaded by the first call: from `path`, and (`beside_torch`) into a process that also holds
+    PyTorch's HIP runtime."""
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
+        if not os.path.exists(path):
             raise JoshuaHipError(
-                f"{LIB_PATH} is missing: build it with `python -m joshua_amd.build` (there is no CPU fallback)")
+                f"{path} is missing: build it with `python -m joshua_amd.build` (there is no CPU fallback)")
         # One process must hold one HIP runtime.  PyTorch ships its own copy of
         # libamdhip64 under the same soname the library links against, so when
         # torch is installed it is loaded first and the loader binds this
         # library to that copy; without torch the system runtime is used.
-        try:
-            import torch  # noqa: F401
-        except ImportError:
-            pass
-        L = ctypes.CDLL(LIB_PATH)
+        if beside_torch:
+            try:
+                import torch  # noqa: F401
+            except ImportError:
+                pass
+        L = _Library(path)
         sz, u32, vp, i32 = ctypes.c_size_t, ctypes.c_uint32, ctypes.c_void_p, ctypes.c_int
         L.jq_last_error.restype = ctypes.c_char_p
         L.jq_last_kernel.restype = ctypes.c_char_p
@@ -155,6 +179,15 @@ def lib() -> ctypes.CDLL:
         L.jq_gguf_meta_str.argtypes = [vp, ctypes.c_char_p, ctypes.POINTER(vp), ctypes.POINTER(sz)]
         L.jq_gguf_meta_array_len.argtypes = [vp, ctypes.c_char_p, ctypes.POINTER(sz)]
         L.jq_gguf_upload.argtypes = [vp, ctypes.c_char_p, ctypes.POINTER(vp)]
+        L.jq_model_load.argtypes = [ctypes.c_char_p, u32, u32, ctypes.POINTER(vp)]
+        L.jq_model_free.argtypes = [vp]
+        L.jq_model_free.restype = None
+        for f in (L.jq_model_vocab, L.jq_model_context, L.jq_model_cached_tokens):
+            f.argtypes = [vp]
+            f.restype = u32
+        L.jq_model_forward.argtypes = [vp, vp, u32, u32, vp, u32, vp, i32, vp]
+        L.jq_model_greedy.argtypes = [vp, ctypes.POINTER(u32), vp]
+        L.jq_model_reset.argtypes = [vp]
         L.joshua_npu_init.argtypes = [ctypes.c_char_p, u32, ctypes.POINTER(u32), ctypes.POINTER(vp)]
         L.joshua_npu_init.restype = ctypes.c_int32
         L.joshua_npu_forward.argtypes = [vp, vp, u32, u32, vp]
@@ -424,7 +457,79 @@ class Mla:
         return int(lib().jq_mla_cached_tokens(self._h))
 
 
-class Qwen3:
+COMPUTE_DEFAULT, COMPUTE_F32 = 0, 1
+
+
+class Model:
+    """A model of any architecture the library knows, picked by what `path` holds: a GGUF file, or a folder with
+    config.json and model.safetensors.  compute=COMPUTE_F32 runs every product in 32-bit where the architecture has
+    that form."""
+
+    def __init__(self, path: str, n_ctx: int = 0, compute: int = COMPUTE_DEFAULT):
+        out = ctypes.c_void_p()
+        _check(lib().jq_model_load(os.fsencode(path), n_ctx, compute, ctypes.byref(out)))
+        self._h = out
+
+    def close(self) -> None:
+        if self._h:
+            lib().jq_model_free(self._h)
+            self._h = ctypes.c_void_p()
+
+    def __del__(self):
+        try:
+            self.close()
+        except Exception:
+            pass
+
+    @property
+    def vocab(self) -> int:
+        return int(lib().jq_model_vocab(self._h))
+
+    @property
+    def context(self) -> int:
+        return int(lib().jq_model_context(self._h))
+
+    @property
+    def cached_tokens(self) -> int:
+        return int(lib().jq_model_cached_tokens(self._h))
+
+    def logits_at(self, tokens, pos: int, want) -> np.ndarray:
+        """Appends the tokens at position `pos`; the logits of the places among them that `want` lists, [len(want), vocab]."""
+        t, w = np.ascontiguousarray(tokens, dtype=np.uint32), np.ascontiguousarray(want, dtype=np.uint32)
+        logits = np.empty((w.size, self.vocab), np.float32)
+        _check(lib().jq_model_forward(self._h, t.ctypes.data, t.size, pos, w.ctypes.data, w.size, logits.ctypes.data, 0, None))
+        return logits
+
+    def forward(self, tokens, pos: int) -> np.ndarray:
+        """The last token's logits."""
+        return self.logits_at(tokens, pos, [max(len(tokens), 1) - 1])[0]
+
+    def forward_only(self, tokens, pos: int, stream: int = 0) -> None:
+        """Enqueues the step and leaves the last token's logits on the device (for greedy())."""
+        t, w = np.ascontiguousarray(tokens, dtype=np.uint32), np.array([max(len(tokens), 1) - 1], np.uint32)
+        _check(lib().jq_model_forward(self._h, t.ctypes.data, t.size, pos, w.ctypes.data, 1, None, 1, stream or None))
+
+    def greedy(self, stream: int = 0) -> int:
+        tok = ctypes.c_uint32()
+        _check(lib().jq_model_greedy(self._h, ctypes.byref(tok), stream or None))
+        return tok.value
+
+    def reset(self) -> None:
+        _check(lib().jq_model_reset(self._h))
+
+    def generate(self, prompt, n_new: int) -> list:
+        """A new sequence: the prompt in one step, then n_new greedy tokens, one step each."""
+        self.reset()
+        out, step, pos = [], list(prompt), 0
+        for _ in range(n_new):
+            self.forward_only(step, pos)
+            pos += len(step)
+            step = [self.greedy()]
+            out += step
+        return out
+
+
+class Qwen3(Model):
     """The dense Qwen3 decoder graph on the device, fed and stepped like the reference's
     model object (reference: src/quantized_qwen3_moe.rs:792-826 forward / clear_kv_cache;
     driver loop src/engine.rs:1149-1294)."""
@@ -447,40 +552,10 @@ class Qwen3:
         _check(lib().jq_qwen3_get_config(out, ctypes.byref(self.cfg)))
         return self
 
-    def close(self) -> None:
-        if self._h:
-            lib().jq_qwen3_free(self._h)
-            self._h = ctypes.c_void_p()
-
-    def __del__(self):
-        try:
-            self.close()
-        except Exception:
-            pass
-
     def set_tensor(self, name: str, qtype: int, data) -> None:
         """qtype 0: f32 vector; else packed blocks of that GGUF type."""
         a = np.ascontiguousarray(data, dtype=np.float32) if qtype == 0 else _host_bytes(data)
         _check(lib().jq_qwen3_set_tensor(self._h, name.encode(), qtype, a.ctypes.data, a.nbytes))
-
-    def forward(self, tokens, pos: int) -> np.ndarray:
-        t = np.ascontiguousarray(tokens, dtype=np.uint32)
-        logits = np.empty(self.cfg.vocab, np.float32)
-        _check(lib().jq_qwen3_forward(self._h, t.ctypes.data, t.size, pos, logits.ctypes.data, 0, None))
-        return logits
-
-    def forward_only(self, tokens, pos: int, stream: int = 0) -> None:
-        """Enqueues the step and leaves the logits on the device (for greedy())."""
-        t = np.ascontiguousarray(tokens, dtype=np.uint32)
-        _check(lib().jq_qwen3_forward(self._h, t.ctypes.data, t.size, pos, None, 1, stream or None))
-
-    def greedy(self, stream: int = 0) -> int:
-        tok = ctypes.c_uint32()
-        _check(lib().jq_qwen3_greedy(self._h, ctypes.byref(tok), stream or None))
-        return tok.value
-
-    def reset(self) -> None:
-        _check(lib().jq_qwen3_reset(self._h))
 
 
 def type_size_bytes(qtype: int, elems: int) -> "int | None":

@@ -1,23 +1,9 @@
 // C ABI of libjoshua_hip.so (declared in include/joshua_hip.h): weight objects
 // resident in HBM in native GGUF block layout, shape validation with the
 // reference's error behaviour, and kernel dispatch.
-#include <hip/hip_runtime.h>
-
-#include <cstdarg>
-#include <cmath>
-#include <cstdio>
-#include <cstdlib>
-#include <algorithm>
-#include <cstring>
-#include <map>
-#include <tuple>
-#include <memory>
-#include <set>
-#include <mutex>
-#include <string>
-#include <vector>
-
-#include "../../include/joshua_hip.h"
+#include "dense.hpp"
+#include "moe.hpp"
+#include "model.hpp"
 #include "kernels_mfma_q4k.hpp"
 #include "kernels_graph.hpp"
 #include "kernels_mla.hpp"
@@ -39,60 +25,7 @@
 
 namespace {
 
-thread_local char g_err[512] = "";
-// Name of the kernel the calling thread's last matmul dispatch chose (jq_last_kernel).
-thread_local const char *g_last_kernel = "";
-void note_kernel(const char *name) { g_last_kernel = name; }
 
-int fail(const char *fmt, ...) {
-    va_list ap;
-    va_start(ap, fmt);
-    vsnprintf(g_err, sizeof g_err, fmt, ap);
-    va_end(ap);
-    return 1;
-}
-
-#define HIP_TRY(expr)                                                                      \
-    do {                                                                                   \
-        hipError_t e_ = (expr);                                                            \
-        if (e_ != hipSuccess) return fail("%s: %s", #expr, hipGetErrorString(e_));         \
-    } while (0)
-
-struct Geometry {
-    size_t elems, bytes;
-};
-
-bool geometry(uint32_t t, Geometry *g) {
-    switch (t) {  // reference: src/gguf_ext.rs:483-512
-    case JQ_TYPE_Q8_0: *g = {32, 34}; return true;
-    case JQ_TYPE_Q2_K: *g = {256, 84}; return true;
-    case JQ_TYPE_Q4_K: *g = {256, 144}; return true;
-    case JQ_TYPE_Q6_K: *g = {256, 210}; return true;
-    case JQ_TYPE_IQ2_XXS: *g = {256, 66}; return true;
-    case JQ_TYPE_MXFP4: *g = {32, 17}; return true;
-    case JQ_TYPE_Q4_0: *g = {32, 18}; return true;
-    case JQ_TYPE_Q4_1: *g = {32, 20}; return true;
-    case JQ_TYPE_Q5_0: *g = {32, 22}; return true;
-    case JQ_TYPE_Q5_1: *g = {32, 24}; return true;
-    case JQ_TYPE_Q3_K: *g = {256, 110}; return true;
-    case JQ_TYPE_Q5_K: *g = {256, 176}; return true;
-    default: return false;
-    }
-}
-
-const char *type_name(uint32_t t) {
-    switch (t) {
-    case JQ_TYPE_Q8_0: return "quantized";
-    case JQ_TYPE_Q2_K: return "quantized";
-    case JQ_TYPE_Q4_K: return "quantized";
-    case JQ_TYPE_Q6_K: return "quantized";
-    case JQ_TYPE_Q4_0: case JQ_TYPE_Q4_1: case JQ_TYPE_Q5_0: case JQ_TYPE_Q5_1: case JQ_TYPE_Q3_K: case JQ_TYPE_Q5_K:
-        return "quantized";
-    case JQ_TYPE_IQ2_XXS: return "iq2_xxs";
-    case JQ_TYPE_MXFP4: return "mxfp4";
-    default: return "unknown";
-    }
-}
 
 // Every block format the library decodes: X(type id, trait).
 #define JQ_FOR_EACH_FORMAT(X) \
@@ -100,62 +33,9 @@ const char *type_name(uint32_t t) {
     X(JQ_TYPE_MXFP4, MXFP4) X(JQ_TYPE_Q4_0, Q4_0) X(JQ_TYPE_Q4_1, Q4_1) X(JQ_TYPE_Q5_0, Q5_0) X(JQ_TYPE_Q5_1, Q5_1)  \
     X(JQ_TYPE_Q3_K, Q3_K) X(JQ_TYPE_Q5_K, Q5_K)
 
-std::once_flag g_init_once;
-int g_init_rc = 0;
-int g_device = 0;
-
 }  // namespace
 
-// Scratch memory of jq_matmul_t_noalloc: a fixed array in every device's memory, held from the moment the
-// library is loaded on that device until the process ends.  Host code never uses the array's name as an
-// address (on the host it is a stand-in, not device memory): noalloc_scratch_on() asks the runtime for the
-// array's address on a device, once, with that device current, and every launch gets that pointer.
-static __device__ __align__(256) uint8_t scratch[JQ_NOALLOC_SCRATCH_BYTES];
 
-namespace {
-
-constexpr int MAX_DEVICES = 64;
-uint8_t *g_scratch_ptr[MAX_DEVICES] = {};
-std::mutex g_scratch_mu[MAX_DEVICES];  // one call at a time enqueues launches that use a device's array
-std::mutex g_scratch_table_mu;
-
-// The address of `scratch` on `device`, which must be the current device.
-int noalloc_scratch_on(int device, uint8_t **out) {
-    if (device < 0 || device >= MAX_DEVICES) return fail("device %d is beyond the %d this library keeps scratch for", device, MAX_DEVICES);
-    std::lock_guard<std::mutex> g(g_scratch_table_mu);
-    if (!g_scratch_ptr[device]) {
-        void *p = nullptr;
-        HIP_TRY(hipGetSymbolAddress(&p, HIP_SYMBOL(scratch)));
-        if (!p) return fail("hipGetSymbolAddress returned no address for the scratch array on device %d", device);
-        g_scratch_ptr[device] = (uint8_t *)p;
-    }
-    *out = g_scratch_ptr[device];
-    return 0;
-}
-
-int do_init(int device) {
-    int count = 0;
-    HIP_TRY(hipGetDeviceCount(&count));
-    if (device < 0 || device >= count) return fail("jq_init: device %d out of range (%d visible)", device, count);
-    HIP_TRY(hipSetDevice(device));
-    g_device = device;
-    uint8_t *p = nullptr;
-    return noalloc_scratch_on(device, &p);
-}
-
-int ensure_init() {
-    std::call_once(g_init_once, [] { g_init_rc = do_init(0); });
-    return g_init_rc;
-}
-
-}  // namespace
-
-struct jq_weight {
-    uint32_t type;
-    size_t n, k, nbytes, row_bytes;
-    uint8_t *dev;
-    bool owns;
-};
 
 namespace {
 
@@ -164,7 +44,8 @@ namespace {
 // src/mxfp4.rs:142-172).
 int validate(uint32_t type, size_t m, size_t k, size_t n, size_t lhs_len, size_t nbytes, size_t dst_len) {
     Geometry g;
-    if (!geometry(type, &g)) return fail("unsupported tensor type id %u", type);
+    if (const size_t eb = dense_elem_bytes(type)) g = {1, eb};
+    else if (!geometry(type, &g)) return fail("unsupported tensor type id %u", type);
     if (k % g.elems != 0)
         return fail("%s matmul: k=%zu is not a multiple of the block size %zu", type_name(type), k, g.elems);
     size_t bpr = k / g.elems;
@@ -639,125 +520,6 @@ void launch_q4k_acts_prep(const float *X, size_t rows, size_t k, uint8_t *out, h
     hipLaunchKernelGGL(jq::q4k_acts_prep, dim3((unsigned)((units + 7) / 8)), dim3(256), 0, s, X, (int)rows, (int)k, out);
 }
 
-// Device memory for what one call's launches hand to each other (prepared activation operands, partial
-// sums of a product split over k), on stream s.  Requests up to SCRATCH_KEEP bytes are served from one
-// allocation per (device, stream), made at first use and kept until the process ends: the launches of a
-// stream run in order, so consecutive calls can share it, and a call pays no allocator round trip
-// (hipMallocAsync with hipFreeAsync takes some 18 us of host time a call, more than the kernels of a
-// small matmul take on the device).  A call that needs more than the stream's buffer holds gets a new,
-// larger one; the old one is retired, not freed, because a HIP graph captured earlier on the stream
-// still names it (sizes at least double, so a stream retires at most a handful of buffers).  The holder
-// keeps that allocation's lock until it goes out of scope, after the call's last launch is enqueued, so
-// host threads that share a stream enqueue their calls one after the other.  Larger requests are
-// stream-ordered allocations, freed behind the call's launches.  First use and growth allocate: neither
-// is possible while the stream is being captured, so a caller warms a stream up with its largest call
-// before capturing it.
-//
-// jq_matmul_t_noalloc serves the same requests from a fixed array in device memory instead (below): it
-// installs the array for the calling thread with FixedScratchScope, and get() then hands out that
-// array, or fails when the request exceeds it, and never reaches an allocator.
-constexpr size_t SCRATCH_KEEP = 64u << 20;
-
-struct StreamBuffer {
-    std::mutex mu;
-    uint8_t *ptr = nullptr;
-    size_t bytes = 0;
-    std::vector<uint8_t *> retired;
-};
-
-std::mutex g_stream_table_mu;
-// keyed by (device, stream, kind): kind 0 is what a product's launches hand to each other, kind 1 the f32 copies of
-// jq_matmul_t_f16's operands around such a product (which takes buffer 0 itself)
-std::map<std::tuple<int, hipStream_t, int>, std::unique_ptr<StreamBuffer>> g_stream_table;
-
-// jq_stream_release: waits for the stream, then frees its buffer and the retired ones.
-int release_stream_scratch(hipStream_t s) {
-    int dev = 0;
-    HIP_TRY(hipGetDevice(&dev));
-    std::vector<std::unique_ptr<StreamBuffer>> bufs;
-    {
-        std::lock_guard<std::mutex> g(g_stream_table_mu);
-        for (int kind = 0; kind < 2; kind++) {
-            auto it = g_stream_table.find({dev, s, kind});
-            if (it == g_stream_table.end()) continue;
-            bufs.push_back(std::move(it->second));
-            g_stream_table.erase(it);
-        }
-    }
-    if (bufs.empty()) return 0;
-    for (auto &b : bufs) { std::lock_guard<std::mutex> wait_for_the_last_holder(b->mu); }
-    HIP_TRY(hipStreamSynchronize(s));
-    for (auto &b : bufs) {
-        if (b->ptr) (void)hipFree(b->ptr);
-        for (uint8_t *p : b->retired) (void)hipFree(p);
-    }
-    return 0;
-}
-
-struct FixedScratch {
-    uint8_t *ptr = nullptr;
-    size_t bytes = 0;
-    std::mutex *mu = nullptr;
-};
-thread_local const FixedScratch *tl_fixed_scratch = nullptr;
-
-struct FixedScratchScope {
-    explicit FixedScratchScope(const FixedScratch *f) { tl_fixed_scratch = f; }
-    ~FixedScratchScope() { tl_fixed_scratch = nullptr; }
-};
-
-class CallScratch {
-    std::unique_lock<std::mutex> lock_;
-    hipStream_t stream_ = nullptr;
-    uint8_t *transient_ = nullptr;
-    int kind_ = 0;
-
-public:
-    CallScratch() = default;
-    explicit CallScratch(int kind) : kind_(kind) {}
-    CallScratch(const CallScratch &) = delete;
-    CallScratch &operator=(const CallScratch &) = delete;
-    ~CallScratch() {
-        if (transient_) (void)hipFreeAsync(transient_, stream_);
-    }
-    // 0 on success; on failure the message is set
-    int get(size_t bytes, hipStream_t s, uint8_t **out) {
-        stream_ = s;
-        if (const FixedScratch *f = kind_ == 0 ? tl_fixed_scratch : nullptr) {
-            if (bytes > f->bytes)
-                return fail("this product needs %zu bytes of scratch memory; the entry point that allocates nothing "
-                            "holds %zu", bytes, f->bytes);
-            lock_ = std::unique_lock<std::mutex>(*f->mu);
-            *out = f->ptr;
-            return 0;
-        }
-        if (bytes > SCRATCH_KEEP) {
-            HIP_TRY(hipMallocAsync((void **)&transient_, bytes, s));
-            *out = transient_;
-            return 0;
-        }
-        int dev = 0;
-        HIP_TRY(hipGetDevice(&dev));
-        StreamBuffer *b;
-        {
-            std::lock_guard<std::mutex> g(g_stream_table_mu);
-            auto &slot = g_stream_table[{dev, s, kind_}];
-            if (!slot) slot.reset(new StreamBuffer);
-            b = slot.get();
-        }
-        lock_ = std::unique_lock<std::mutex>(b->mu);
-        if (b->bytes < bytes) {
-            const size_t want = std::min(SCRATCH_KEEP, std::max<size_t>({(bytes + 0xFFFFF) & ~(size_t)0xFFFFF, 2 * b->bytes,
-                                                                          (size_t)1 << 20}));
-            uint8_t *fresh = nullptr;
-            HIP_TRY(hipMalloc((void **)&fresh, want));
-            if (b->ptr) b->retired.push_back(b->ptr);
-            b->ptr = fresh, b->bytes = want;
-        }
-        *out = b->ptr;
-        return 0;
-    }
-};
 
 // Workgroups of the LDS-ring MFMA kernel that fit a compute unit (LDS and the 16 waves of a SIMD group).
 constexpr int ring_wgs_per_cu(int maxnb) { return maxnb == 16 ? 1 : maxnb == 8 ? 2 : 4; }
@@ -1102,6 +864,7 @@ int dispatch_gemm_decoded(uint32_t type, const uint8_t *W, size_t row_bytes, con
 int dispatch_matmul(uint32_t type, const uint8_t *W, size_t row_bytes, const float *X, float *Y, size_t m,
                     size_t k, size_t n, hipStream_t s) {
     if (m > 0x7FFFFFFF || k > 0x7FFFFFFF || n > 0x7FFFFFFF) return fail("matmul: dimension exceeds 2^31-1");
+    if (dense_elem_bytes(type)) return dense_matmul(type, W, row_bytes, X, Y, m, k, n, s);
     if (type == JQ_TYPE_Q4_K && m == 1) {
         const int rc = dispatch_q4k_dot4(W, row_bytes, X, Y, k, n, s);
         if (rc >= 0) return rc;
@@ -1264,6 +1027,7 @@ void launch_decode(const jq_weight *w, const uint32_t *ids, float *out, size_t r
 }
 
 int dispatch_decode(const jq_weight *w, const uint32_t *ids, float *out, size_t rows, hipStream_t s) {
+    if (dense_elem_bytes(w->type)) return dense_decode(w, ids, out, rows, 1.0f, s);
     switch (w->type) {
 #define JQ_CASE(ID, Q) \
     case ID: launch_decode<jq::Q>(w, ids, out, rows, s); break;
@@ -1275,97 +1039,10 @@ int dispatch_decode(const jq_weight *w, const uint32_t *ids, float *out, size_t 
     return 0;
 }
 
-// Frees a device allocation when it goes out of scope.
-struct DevBuf {
-    void *p = nullptr;
-    ~DevBuf() {
-        if (p) (void)hipFree(p);
-    }
-    hipError_t alloc(size_t bytes) { return hipMalloc(&p, bytes ? bytes : 1); }
-};
-
 }  // namespace
 
 extern "C" {
 
-const char *jq_last_error(void) { return g_err; }
-const char *jq_last_kernel(void) { return g_last_kernel; }
-
-int jq_block_geometry(uint32_t ggml_type, size_t *elems, size_t *bytes) {
-    Geometry g;
-    if (!geometry(ggml_type, &g)) return fail("unsupported tensor type id %u", ggml_type);
-    if (elems) *elems = g.elems;
-    if (bytes) *bytes = g.bytes;
-    return 0;
-}
-
-int jq_init(int device) {
-    bool first = false;
-    std::call_once(g_init_once, [&] {
-        first = true;
-        g_init_rc = do_init(device);
-    });
-    if (!first && g_init_rc == 0 && device != g_device)
-        return fail("jq_init: already initialised on device %d", g_device);
-    return g_init_rc;
-}
-
-int jq_upload(uint32_t ggml_type, const void *blocks, size_t nbytes, size_t n, size_t k, int src_is_device,
-              jq_weight **out) {
-    if (!out) return fail("jq_upload: out is null");
-    *out = nullptr;
-    Geometry g;
-    if (!geometry(ggml_type, &g)) return fail("unsupported tensor type id %u", ggml_type);
-    if (k % g.elems != 0)
-        return fail("%s tensor: k=%zu is not a multiple of the block size %zu", type_name(ggml_type), k, g.elems);
-    size_t want = n * (k / g.elems) * g.bytes;
-    if (nbytes != want)
-        return fail("%s tensor: %zu bytes for %zu x %zu elements (expected %zu)", type_name(ggml_type), nbytes, n, k,
-                    want);
-    if (nbytes && !blocks) return fail("jq_upload: blocks is null");
-    if (ensure_init()) return 1;
-    uint8_t *dev = nullptr;
-    // Kernels read a row in 16-byte pieces that may start before the unit they
-    // need; 64 spare bytes keep every such read inside the allocation.
-    HIP_TRY(hipMalloc((void **)&dev, nbytes + 64));
-    hipError_t e = hipMemcpy(dev, blocks, nbytes, src_is_device ? hipMemcpyDeviceToDevice : hipMemcpyHostToDevice);
-    if (e == hipSuccess) e = hipMemset(dev + nbytes, 0, 64);
-    if (e != hipSuccess) {
-        (void)hipFree(dev);
-        return fail("jq_upload: copy to device failed: %s", hipGetErrorString(e));
-    }
-    *out = new jq_weight{ggml_type, n, k, nbytes, (k / g.elems) * g.bytes, dev, true};
-    return 0;
-}
-
-int jq_view(const jq_weight *parent, size_t byte_offset, size_t n, size_t k, jq_weight **out) {
-    if (!out) return fail("jq_view: out is null");
-    *out = nullptr;
-    if (!parent) return fail("jq_view: parent is null");
-    Geometry g;
-    geometry(parent->type, &g);
-    if (k % g.elems != 0)
-        return fail("%s tensor: k=%zu is not a multiple of the block size %zu", type_name(parent->type), k, g.elems);
-    size_t need = n * (k / g.elems) * g.bytes;
-    // reference: src/mmap_tensor.rs:105-110 (range must lie inside the mapping)
-    if (byte_offset > parent->nbytes || need > parent->nbytes - byte_offset)
-        return fail("jq_view: range %zu+%zu exceeds the parent's %zu bytes", byte_offset, need, parent->nbytes);
-    if (byte_offset % g.bytes != 0) return fail("jq_view: offset %zu is not a whole number of blocks", byte_offset);
-    *out = new jq_weight{parent->type, n, k, need, (k / g.elems) * g.bytes, parent->dev + byte_offset, false};
-    return 0;
-}
-
-void jq_free(jq_weight *w) {
-    if (!w) return;
-    if (w->owns && w->dev) (void)hipFree(w->dev);
-    delete w;
-}
-
-uint32_t jq_dtype(const jq_weight *w) { return w ? w->type : 0; }
-size_t jq_rows(const jq_weight *w) { return w ? w->n : 0; }
-size_t jq_cols(const jq_weight *w) { return w ? w->k : 0; }
-size_t jq_storage_size_in_bytes(const jq_weight *w) { return w ? w->nbytes : 0; }
-const void *jq_device_ptr(const jq_weight *w) { return w ? w->dev : nullptr; }
 
 int jq_matmul_t(const jq_weight *w, size_t m, const float *lhs, size_t lhs_len, float *dst, size_t dst_len,
                 int ptrs_are_device, void *stream) {
@@ -1428,7 +1105,7 @@ int jq_matmul_t_noalloc(const jq_weight *w, size_t m, const float *lhs_dev, size
     FixedScratch f;
     if (noalloc_scratch_on(dev, &f.ptr)) return 1;  // resolved by jq_init; the first call on another device resolves it there
     f.bytes = JQ_NOALLOC_SCRATCH_BYTES;
-    f.mu = &g_scratch_mu[dev];
+    f.mu = &noalloc_scratch_mutex(dev);
     FixedScratchScope scope(&f);
     return dispatch_matmul(w->type, w->dev, w->row_bytes, lhs_dev, dst_dev, m, w->k, w->n, (hipStream_t)stream);
 }
@@ -1448,11 +1125,6 @@ int jq_try_matmul_fused(uint32_t ggml_type, size_t m, size_t k, size_t n, const 
     if (ensure_init()) return 1;
     return dispatch_matmul(ggml_type, (const uint8_t *)blocks_dev, (k / g.elems) * g.bytes, lhs_dev, dst_dev, m, k, n,
                            (hipStream_t)stream);
-}
-
-int jq_stream_release(void *stream) {
-    if (ensure_init()) return 1;
-    return release_stream_scratch((hipStream_t)stream);
 }
 
 int jq_dequantize(const jq_weight *w, float *out, size_t out_len, int out_is_device, void *stream) {
@@ -1568,53 +1240,12 @@ int jq_embedding(const jq_weight *w, const uint32_t *ids, size_t n_ids, float *o
     return 0;
 }
 
-int jq_stream_synchronize(void *stream) {
-    HIP_TRY(hipStreamSynchronize((hipStream_t)stream));
-    return 0;
-}
-
-
-// ---- mixture of experts -----------------------------------------------------------
 
 }  // extern "C"
 
-struct jq_moe {
-    jq_moe_config cfg;
-    const jq_weight *gate, *up, *down, *sgate, *sup, *sdown;
-    float *router_w = nullptr, *router_bias = nullptr;
-    const uint8_t **pgate = nullptr, **pup = nullptr, **pdown = nullptr;  // device tables of expert bases
-    bool fold_shared = false;  // the shared expert rides along as table entry n_expert of the grouped kernels
-    // scratch, grown to the largest token count seen
-    size_t cap_tokens = 0;
-    float *logits = nullptr, *wts = nullptr, *G = nullptr, *U = nullptr, *out = nullptr;
-    float *sG = nullptr, *sU = nullptr, *sH = nullptr, *sOut = nullptr;
-    uint32_t *ids = nullptr;
-    int *gexp = nullptr, *offsets = nullptr, *xrow = nullptr, *yrow = nullptr;
-    uint8_t *qacts = nullptr;  // activations as MFMA operand records (Q4_K experts, grouped path)
-    uint8_t *gacts = nullptr;  // activations of the grouped int8 GEMM, and its tables
-    int *gtab = nullptr;
-    size_t gtab_rows = 0;      // row groups (and tiles) the tables hold
-    int gtile_rgs = 8;         // row groups a tile of the current plan: 8 (waves share the rows), 2 (the weight rows), 0 (both: two launches)
-    jq::ActsI8 qi8{nullptr, nullptr, nullptr, nullptr};  // activations as int8 planes (decode path, long rows)
-    std::mutex mu;
-};
+// ---- mixture of experts -----------------------------------------------------------
 
 namespace {
-
-void moe_free_scratch(jq_moe *m) {
-    for (void *p : {(void *)m->logits, (void *)m->wts, (void *)m->G, (void *)m->U, (void *)m->out, (void *)m->sG,
-                    (void *)m->sU, (void *)m->sH, (void *)m->sOut, (void *)m->ids, (void *)m->gexp,
-                    (void *)m->offsets, (void *)m->xrow, (void *)m->yrow, (void *)m->qacts, (void *)m->qi8.xl,
-                    (void *)m->qi8.xh, (void *)m->qi8.sx, (void *)m->qi8.sxs, (void *)m->gacts, (void *)m->gtab})
-        if (p) (void)hipFree(p);
-    m->qacts = nullptr;
-    m->gacts = nullptr, m->gtab = nullptr, m->gtab_rows = 0;
-    m->qi8 = jq::ActsI8{nullptr, nullptr, nullptr, nullptr};
-    m->logits = m->wts = m->G = m->U = m->out = m->sG = m->sU = m->sH = m->sOut = nullptr;
-    m->ids = nullptr;
-    m->gexp = m->offsets = m->xrow = m->yrow = nullptr;
-    m->cap_tokens = 0;
-}
 
 // Formats whose decode-shaped expert matmuls run on integer dot products (Q::dot8).
 bool moe_has_dot8(uint32_t type) {
@@ -1640,22 +1271,9 @@ bool moe_has_gemm_i8(uint32_t type) {
            type == JQ_TYPE_Q5_1;
 }
 
-int moe_reserve(jq_moe *m, size_t T) {
-    if (T <= m->cap_tokens) return 0;
-    moe_free_scratch(m);
+int moe_reserve_quantized(jq_moe *m, size_t T) {
     const jq_moe_config &c = m->cfg;
-    // rows of the pair buffers: the routed pairs, then one per token for a folded shared expert
-    size_t P = T * c.n_expert_used, PR = P + T, groups = std::max<size_t>(PR, c.n_expert + 1) + 1;
-    HIP_TRY(hipMalloc((void **)&m->logits, T * c.n_expert * sizeof(float)));
-    HIP_TRY(hipMalloc((void **)&m->wts, P * sizeof(float)));
-    HIP_TRY(hipMalloc((void **)&m->ids, P * sizeof(uint32_t)));
-    HIP_TRY(hipMalloc((void **)&m->G, PR * c.inter * sizeof(float)));
-    HIP_TRY(hipMalloc((void **)&m->U, PR * c.inter * sizeof(float)));
-    HIP_TRY(hipMalloc((void **)&m->out, PR * c.hidden * sizeof(float)));
-    HIP_TRY(hipMalloc((void **)&m->gexp, groups * sizeof(int)));
-    HIP_TRY(hipMalloc((void **)&m->offsets, (groups + 1) * sizeof(int)));
-    HIP_TRY(hipMalloc((void **)&m->xrow, PR * sizeof(int)));
-    HIP_TRY(hipMalloc((void **)&m->yrow, PR * sizeof(int)));
+    const size_t P = T * c.n_expert_used, PR = P + T;
     if (moe_has_dot8(m->gate->type) || moe_has_dot8(m->down->type)) {
         const size_t words = PR * (std::max<size_t>(c.hidden, c.inter) / 4);
         HIP_TRY(hipMalloc((void **)&m->qi8.xl, words * sizeof(uint32_t) + 16));
@@ -1671,14 +1289,6 @@ int moe_reserve(jq_moe *m, size_t T) {
         HIP_TRY(hipMalloc((void **)&m->gacts, m->gtab_rows * (std::max<size_t>(c.hidden, c.inter) / 256 + 1) * jq::QI_REC));
         HIP_TRY(hipMalloc((void **)&m->gtab, (8 * m->gtab_rows + 4) * sizeof(int)));
     }
-    if (m->sgate) {
-        size_t si = m->sgate->n;
-        HIP_TRY(hipMalloc((void **)&m->sG, T * si * sizeof(float)));
-        HIP_TRY(hipMalloc((void **)&m->sU, T * si * sizeof(float)));
-        HIP_TRY(hipMalloc((void **)&m->sH, T * si * sizeof(float)));
-        HIP_TRY(hipMalloc((void **)&m->sOut, T * c.hidden * sizeof(float)));
-    }
-    m->cap_tokens = T;
     return 0;
 }
 
@@ -2303,70 +1913,6 @@ int dispatch_moe_gemm_i8(jq_moe *m, uint32_t type, const uint8_t *const *wptr, s
     }
 }
 
-// `planes`: also leave x as fixed-point planes there (the one-expert-a-workgroup router kernel does; *planes_made
-// says whether it ran)
-// `gate_later`: when the gating can run by one wave a token, it is left to the caller's next kernel (the logits are
-// in m->logits) and *gate_later holds its operands; else it is cleared.
-// `pre`: the decoder layer's residual add and RMSNorm run inside the router launch (one token; x is then pre->hn_out,
-// which that launch writes).
-int moe_route_dev(jq_moe *m, size_t T, const float *x, hipStream_t s, jq::MoePairGroups pg,
-                  jq::ActsI8 planes = jq::ActsI8{nullptr, nullptr, nullptr, nullptr}, bool *planes_made = nullptr,
-                  jq::MoeGateIn *gate_later = nullptr, const jq::MoePreNormArgs *pre = nullptr) {
-    const jq_moe_config &c = m->cfg;
-    const unsigned token_runs = (unsigned)((T + jq::ROUTER_TOKENS_PER_WG - 1) / jq::ROUTER_TOKENS_PER_WG);
-    static const char *no_tile = getenv("JQ_MOE_NO_ROUTER_TILE");
-    // (a router of a million weights or more, 256 experts of 7168: from 8 tokens, 16 us against 27)
-    const size_t tile_from = (size_t)c.hidden * c.n_expert >= (1u << 20) ? 8 : 32;
-    jq::MoeGateParams gp{(int)c.n_expert, (int)c.n_expert_used, (int)c.gating, (int)c.norm_topk, c.weights_scale,
-                         (int)c.n_group, (int)c.topk_group};
-    static const char *no_wave = getenv("JQ_MOE_NO_WAVE_GATE");
-    const bool wave_gate = !no_wave && c.n_group <= 1 && c.n_expert <= 256 && c.n_expert_used <= 64;
-    if (pre)
-        hipLaunchKernelGGL(jq::moe_router_logits_norm, dim3(c.n_expert), dim3(256), 0, s, m->router_w, *pre, m->logits,
-                           (int)c.hidden, (int)c.n_expert);
-    else if (T >= tile_from && !no_tile)  // many tokens: a token's activations read once per eight experts (the same bits)
-        hipLaunchKernelGGL(jq::moe_router_logits_tile, dim3((c.n_expert + 7) / 8, (unsigned)((T + 7) / 8)), dim3(256), 0, s,
-                           m->router_w, x, m->logits, (int)T, (int)c.hidden, (int)c.n_expert,
-                           c.hidden % 32 == 0 ? planes : jq::ActsI8{nullptr, nullptr, nullptr, nullptr});
-    else
-        hipLaunchKernelGGL(jq::moe_router_logits, dim3(c.n_expert, token_runs), dim3(256), 0, s, m->router_w, x, m->logits,
-                           (int)T, (int)c.hidden, (int)c.n_expert, planes);
-    if (planes_made) *planes_made = !pre && planes.xl && (c.hidden % 32 == 0 || !(T >= tile_from && !no_tile));
-    size_t sm = (2 * c.n_expert + std::max<uint32_t>(c.n_group, 1) + c.n_expert_used + 4) * sizeof(float);
-    if (gate_later) {
-        if (wave_gate) {
-            *gate_later = jq::MoeGateIn{m->logits, m->router_bias, gp, m->ids, m->wts, pg, (int)T};
-            HIP_TRY(hipGetLastError());
-            return 0;
-        }
-        gate_later->logits = nullptr;
-    }
-    // no expert groups and at most 256 experts: one wave a token, reductions in registers
-    if (wave_gate) {
-        const int ne = (int)(c.n_expert + 63) / 64;
-#define JQ_GATE(NE) hipLaunchKernelGGL(jq::moe_gate_topk_wave<NE>, dim3((unsigned)T), dim3(64), 0, s, m->logits, m->router_bias, gp, m->ids, m->wts, pg)
-        if (ne == 1) JQ_GATE(1);
-        else if (ne == 2) JQ_GATE(2);
-        else if (ne == 3) JQ_GATE(3);
-        else JQ_GATE(4);
-#undef JQ_GATE
-        HIP_TRY(hipGetLastError());
-        return 0;
-    }
-    hipLaunchKernelGGL(jq::moe_gate_topk, dim3((unsigned)T), dim3(256), sm, s, m->logits, m->router_bias, gp, m->ids,
-                       m->wts, pg);
-    HIP_TRY(hipGetLastError());
-    return 0;
-}
-
-// The decoder's residual add and RMSNorm in front of a layer's mixture of experts: x_out = x + res,
-// hn_out = rmsnorm(x_out) w, and the experts run over hn_out.  `fused` says whether the router launch did it
-// (then the caller's residual row is x_out) or a launch of its own in place (then it is still x).
-struct MoePreNorm {
-    jq::MoePreNormArgs a;
-    bool fused;
-};
-
 int moe_forward_dev(jq_moe *m, size_t T, const float *x, float *y, hipStream_t s, MoePreNorm *pre = nullptr) {
     const jq_moe_config &c = m->cfg;
     const int P = (int)(T * c.n_expert_used), extra = m->fold_shared ? 1 : 0;
@@ -2463,26 +2009,7 @@ int moe_forward_dev(jq_moe *m, size_t T, const float *x, float *y, hipStream_t s
         if (moe_route_dev(m, T, x, s, jq::MoePairGroups{nullptr, nullptr, nullptr, nullptr, 0}, planes, &planes_ready)) return 1;
         groups = (int)c.n_expert + extra;
         max_group = (int)T;
-        const int in_lds = (size_t)P <= 12288;
-        const size_t chunks = ((size_t)P + 63) / 64, rank_ints = chunks * c.n_expert + c.n_expert + 1;
-        static const char *no_ranked = getenv("JQ_MOE_NO_RANKED_GROUPING");
-        // (its rank table: chunks x experts ints of LDS, up to 144 KB)
-        if (!no_ranked && chunks <= (size_t)jq::GROUP_RANK_CHUNKS && rank_ints <= 36864) {
-            static std::once_flag big_lds;
-            static hipError_t attr_rc = hipSuccess;
-            std::call_once(big_lds, [&] {
-                attr_rc = hipFuncSetAttribute((const void *)jq::moe_group_pairs_ranked, hipFuncAttributeMaxDynamicSharedMemorySize,
-                                              36864 * (int)sizeof(int));
-            });
-            HIP_TRY(attr_rc);
-            hipLaunchKernelGGL(jq::moe_group_pairs_ranked, dim3(1), dim3(jq::GROUP_PAIRS_THREADS), rank_ints * sizeof(int), s,
-                               m->ids, (int)T, (int)c.n_expert_used, (int)c.n_expert, m->gexp, m->offsets, m->xrow, m->yrow,
-                               extra);
-        }
-        else
-            hipLaunchKernelGGL(jq::moe_group_pairs, dim3(1), dim3(jq::GROUP_PAIRS_THREADS), (c.n_expert + 1 + (in_lds ? P : 0)) * sizeof(int), s,
-                               m->ids, (int)T, (int)c.n_expert_used, (int)c.n_expert, m->gexp, m->offsets, m->xrow, m->yrow,
-                               extra, in_lds);
+        if (moe_group_dev(m, T, extra, s)) return 1;
     }
     HIP_TRY(hipGetLastError());
     // silu(gate x) * (up x) of every pair into G, then down over it
@@ -2655,134 +2182,19 @@ int moe_forward_dev(jq_moe *m, size_t T, const float *x, float *y, hipStream_t s
     return 0;
 }
 
-// Device table of expert base pointers; `extra` (the shared expert's weight, or null) becomes entry
-// n_expert.
-int moe_ptr_table(const jq_weight *w, size_t n_expert, size_t rows_per_expert, const jq_weight *extra,
-                  const uint8_t ***out) {
-    std::vector<const uint8_t *> host(n_expert + 1);
-    for (size_t e = 0; e < n_expert; e++) host[e] = w->dev + e * rows_per_expert * w->row_bytes;
-    host[n_expert] = extra ? extra->dev : w->dev;
-    HIP_TRY(hipMalloc((void **)out, host.size() * sizeof(uint8_t *)));
-    HIP_TRY(hipMemcpy((void *)*out, host.data(), host.size() * sizeof(uint8_t *), hipMemcpyHostToDevice));
-    return 0;
+bool moe_takes_quantized(const jq_weight *gate, const jq_weight *up, const jq_weight *down) {
+    return !dense_elem_bytes(gate->type) && !dense_elem_bytes(up->type) && !dense_elem_bytes(down->type);
 }
+
+const MoeBackend g_quantized_moe{moe_takes_quantized, moe_reserve_quantized, nullptr,
+                                 [](jq_moe *m, size_t T, const float *x, float *y, hipStream_t s, MoePreNorm *pre) {
+                                     return moe_forward_dev(m, T, x, y, s, pre);
+                                 }};
+const RegisterMoeBackend g_register_quantized_moe(&g_quantized_moe);
 
 }  // namespace
 
 extern "C" {
-
-int jq_moe_create(const jq_moe_config *cfg, const float *router_w, const float *router_bias,
-                  const jq_weight *gate_exps, const jq_weight *up_exps, const jq_weight *down_exps,
-                  const jq_weight *shared_gate, const jq_weight *shared_up, const jq_weight *shared_down,
-                  jq_moe **out) {
-    if (!out) return fail("jq_moe_create: out is null");
-    *out = nullptr;
-    if (!cfg || !router_w || !gate_exps || !up_exps || !down_exps) return fail("jq_moe_create: null argument");
-    const jq_moe_config &c = *cfg;
-    if (c.n_expert == 0 || c.n_expert_used == 0 || c.n_expert_used > c.n_expert)
-        return fail("moe: %u experts used of %u", c.n_expert_used, c.n_expert);
-    if (c.hidden % 4 != 0) return fail("moe: hidden size %u is not a multiple of 4", c.hidden);
-    if (c.n_group > 1 && (c.n_expert % c.n_group != 0 || c.topk_group == 0 || c.topk_group > c.n_group))
-        return fail("moe: %u experts in %u groups, %u groups kept", c.n_expert, c.n_group, c.topk_group);
-    // reference: src/quantized_qwen3_moe.rs:567-571 (expert tensor shaped [n_expert, out, in])
-    if (gate_exps->n != (size_t)c.n_expert * c.inter || gate_exps->k != c.hidden || up_exps->n != gate_exps->n ||
-        up_exps->k != c.hidden || down_exps->n != (size_t)c.n_expert * c.hidden || down_exps->k != c.inter)
-        return fail("moe: expected expert tensors shaped [%u*%u, %u], [%u*%u, %u], [%u*%u, %u]", c.n_expert, c.inter,
-                    c.hidden, c.n_expert, c.inter, c.hidden, c.n_expert, c.hidden, c.inter);
-    bool any_shared = shared_gate || shared_up || shared_down;
-    if (any_shared) {
-        if (!(shared_gate && shared_up && shared_down)) return fail("moe: shared expert needs gate, up and down");
-        if (shared_gate->k != c.hidden || shared_up->k != c.hidden || shared_up->n != shared_gate->n ||
-            shared_down->k != shared_gate->n || shared_down->n != c.hidden)
-            return fail("moe: shared expert shapes do not chain");
-    }
-    if (ensure_init()) return 1;
-    jq_moe *m = new jq_moe;
-    m->cfg = c;
-    m->gate = gate_exps;
-    m->up = up_exps;
-    m->down = down_exps;
-    m->sgate = shared_gate;
-    m->sup = shared_up;
-    m->sdown = shared_down;
-    auto cleanup = [&] {
-        jq_moe_free(m);
-        return 1;
-    };
-    size_t rbytes = (size_t)c.n_expert * c.hidden * sizeof(float);
-    if (hipMalloc((void **)&m->router_w, rbytes) != hipSuccess ||
-        hipMemcpy(m->router_w, router_w, rbytes, hipMemcpyHostToDevice) != hipSuccess) {
-        fail("moe: router upload failed");
-        return cleanup();
-    }
-    if (router_bias) {
-        if (hipMalloc((void **)&m->router_bias, c.n_expert * sizeof(float)) != hipSuccess ||
-            hipMemcpy(m->router_bias, router_bias, c.n_expert * sizeof(float), hipMemcpyHostToDevice) != hipSuccess) {
-            fail("moe: router bias upload failed");
-            return cleanup();
-        }
-    }
-    // A shared expert of the routed experts' own type and shape rides along in the grouped kernels.
-    m->fold_shared = any_shared && shared_gate->type == gate_exps->type && shared_up->type == up_exps->type &&
-                     shared_down->type == down_exps->type && shared_gate->n == c.inter;
-    if (moe_ptr_table(gate_exps, c.n_expert, c.inter, m->fold_shared ? shared_gate : nullptr, &m->pgate) ||
-        moe_ptr_table(up_exps, c.n_expert, c.inter, m->fold_shared ? shared_up : nullptr, &m->pup) ||
-        moe_ptr_table(down_exps, c.n_expert, c.hidden, m->fold_shared ? shared_down : nullptr, &m->pdown))
-        return cleanup();
-    *out = m;
-    return 0;
-}
-
-void jq_moe_free(jq_moe *m) {
-    if (!m) return;
-    moe_free_scratch(m);
-    for (void *p : {(void *)m->router_w, (void *)m->router_bias, (void *)m->pgate, (void *)m->pup, (void *)m->pdown})
-        if (p) (void)hipFree(p);
-    delete m;
-}
-
-int jq_moe_route(jq_moe *m, size_t n_tokens, const float *x, uint32_t *ids, float *weights, int ptrs_are_device,
-                 void *stream) {
-    if (!m) return fail("jq_moe_route: layer is null");
-    if (n_tokens == 0) return 0;
-    if (!x || !ids || !weights) return fail("jq_moe_route: null pointer");
-    hipStream_t s = (hipStream_t)stream;
-    std::lock_guard<std::mutex> lock(m->mu);
-    if (moe_reserve(m, n_tokens)) return 1;
-    size_t P = n_tokens * m->cfg.n_expert_used;
-    DevBuf xd;
-    const float *xdev = x;
-    if (!ptrs_are_device) {
-        HIP_TRY(xd.alloc(n_tokens * m->cfg.hidden * sizeof(float)));
-        HIP_TRY(hipMemcpyAsync(xd.p, x, n_tokens * m->cfg.hidden * sizeof(float), hipMemcpyHostToDevice, s));
-        xdev = (const float *)xd.p;
-    }
-    if (moe_route_dev(m, n_tokens, xdev, s, jq::MoePairGroups{nullptr, nullptr, nullptr, nullptr, 0})) return 1;
-    hipMemcpyKind kind = ptrs_are_device ? hipMemcpyDeviceToDevice : hipMemcpyDeviceToHost;
-    HIP_TRY(hipMemcpyAsync(ids, m->ids, P * sizeof(uint32_t), kind, s));
-    HIP_TRY(hipMemcpyAsync(weights, m->wts, P * sizeof(float), kind, s));
-    if (!ptrs_are_device) HIP_TRY(hipStreamSynchronize(s));
-    return 0;
-}
-
-int jq_moe_forward(jq_moe *m, size_t n_tokens, const float *x, float *y, int ptrs_are_device, void *stream) {
-    if (!m) return fail("jq_moe_forward: layer is null");
-    if (n_tokens == 0) return 0;
-    if (!x || !y) return fail("jq_moe_forward: null pointer");
-    hipStream_t s = (hipStream_t)stream;
-    std::lock_guard<std::mutex> lock(m->mu);
-    if (moe_reserve(m, n_tokens)) return 1;
-    if (ptrs_are_device) return moe_forward_dev(m, n_tokens, x, y, s);
-    size_t bytes = n_tokens * m->cfg.hidden * sizeof(float);
-    DevBuf xd, yd;
-    HIP_TRY(xd.alloc(bytes));
-    HIP_TRY(yd.alloc(bytes));
-    HIP_TRY(hipMemcpyAsync(xd.p, x, bytes, hipMemcpyHostToDevice, s));
-    if (moe_forward_dev(m, n_tokens, (const float *)xd.p, (float *)yd.p, s)) return 1;
-    HIP_TRY(hipMemcpyAsync(y, yd.p, bytes, hipMemcpyDeviceToHost, s));
-    HIP_TRY(hipStreamSynchronize(s));
-    return 0;
-}
 
 }  // extern "C"
 
@@ -3123,7 +2535,7 @@ size_t jq_mla_cached_tokens(const jq_mla *m) { return m ? m->n_past : 0; }
 
 // ---- dense Qwen3 decoder ------------------------------------------------------------
 
-struct jq_model {
+struct Qwen3Model : jq_model {
     jq_qwen3_config cfg;
     std::map<std::string, jq_weight *> q;   // quantized matrices by GGUF name
     std::map<std::string, float *> f;       // f32 vectors by GGUF name
@@ -3135,42 +2547,35 @@ struct jq_model {
     bool fused_ready = false;
     float *cat = nullptr;     // the fused result of a single-token step (q|k|v, gate|up)
     std::vector<float *> kc, vc;            // per layer [n_kv, n_ctx, d]
-    uint32_t n_past = 0;
     size_t cap_tokens = 0;
-    uint32_t *ids = nullptr, *pick = nullptr;
-    float *pick_v = nullptr;  // the greedy pick's candidates, one per slice of the logits
-    int *pick_i = nullptr;
+    uint32_t *ids = nullptr;
     int *pos = nullptr;       // device copy of the position of the step being run
     float *part = nullptr;    // split-attention partials
     float2 *rope_cs = nullptr;  // (cos, sin) of the rotary angles of a step's tokens, [8][head_dim / 2]
     float *x2 = nullptr;      // second residual row of a single-token step (the fused norm + matmul launches alternate)
     float *x = nullptr, *hn = nullptr, *qb = nullptr, *kb = nullptr, *vb = nullptr, *att = nullptr, *proj = nullptr,
-          *g = nullptr, *u = nullptr, *mid = nullptr, *logits = nullptr;
+          *g = nullptr, *u = nullptr, *mid = nullptr;
     // Mixture-of-experts feed-forward blocks (cfg.n_expert > 0): the routers as they arrived from the host,
     // one layer object each (built at the first step, rebuilt when a tensor of the layer is replaced), and
     // the index of the one that currently holds the scratch buffers all of them take turns with.
     std::map<std::string, std::vector<float>> router_host;
     std::vector<jq_moe *> moe;
     int moe_scratch_at = -1;
-    std::mutex mu;
+
+    ~Qwen3Model() override;
+    int step(const uint32_t *tokens, uint32_t n, const uint32_t *want, uint32_t n_want, hipStream_t s) override;
 };
 
 namespace {
 
-// Hands the scratch buffers of one layer object to another of the same configuration.  Work on a stream
-// runs in launch order and every kernel got its pointers when it was launched, so the layers of a model
-// can take turns with one set.
-void moe_swap_scratch(jq_moe *a, jq_moe *b) {
-    std::swap(a->cap_tokens, b->cap_tokens);
-    std::swap(a->logits, b->logits), std::swap(a->wts, b->wts), std::swap(a->G, b->G), std::swap(a->U, b->U);
-    std::swap(a->out, b->out), std::swap(a->sG, b->sG), std::swap(a->sU, b->sU), std::swap(a->sH, b->sH);
-    std::swap(a->sOut, b->sOut), std::swap(a->ids, b->ids), std::swap(a->gexp, b->gexp);
-    std::swap(a->offsets, b->offsets), std::swap(a->xrow, b->xrow), std::swap(a->yrow, b->yrow);
-    std::swap(a->qacts, b->qacts), std::swap(a->gacts, b->gacts), std::swap(a->gtab, b->gtab);
-    std::swap(a->gtab_rows, b->gtab_rows), std::swap(a->gtile_rgs, b->gtile_rgs), std::swap(a->qi8, b->qi8);
+// A handle of the C ABI as this architecture's model; null, with the message set, for another one's.
+Qwen3Model *qwen3_of(jq_model *m, const char *call) {
+    Qwen3Model *q = dynamic_cast<Qwen3Model *>(m);
+    if (!q) fail("%s: not a qwen3 model", call);
+    return q;
 }
 
-void model_free_scratch(jq_model *m) {
+void model_free_scratch(Qwen3Model *m) {
     for (void *p : {(void *)m->ids, (void *)m->x, (void *)m->x2, (void *)m->hn, (void *)m->qb, (void *)m->kb, (void *)m->vb,
                     (void *)m->att, (void *)m->proj, (void *)m->g, (void *)m->mid})  // u is the second half of g
         if (p) (void)hipFree(p);
@@ -3180,7 +2585,7 @@ void model_free_scratch(jq_model *m) {
     m->cap_tokens = 0;
 }
 
-int model_reserve(jq_model *m, size_t T) {
+int model_reserve(Qwen3Model *m, size_t T) {
     if (T <= m->cap_tokens) return 0;
     model_free_scratch(m);
     const jq_qwen3_config &c = m->cfg;
@@ -3228,14 +2633,14 @@ bool qwen3_shape(const jq_qwen3_config &c, const std::string &name, size_t *n, s
     return false;
 }
 
-int model_mm(jq_model *m, const std::string &name, const float *x, float *y, size_t T, hipStream_t s) {
+int model_mm(Qwen3Model *m, const std::string &name, const float *x, float *y, size_t T, hipStream_t s) {
     auto it = m->q.find(name);
     if (it == m->q.end()) return fail("qwen3: missing tensor `%s`", name.c_str());
     const jq_weight *w = it->second;
     return dispatch_matmul(w->type, w->dev, w->row_bytes, x, y, T, w->k, w->n, s);
 }
 
-int model_vec(jq_model *m, const std::string &name, const float **out) {
+int model_vec(Qwen3Model *m, const std::string &name, const float **out) {
     auto it = m->f.find(name);
     if (it == m->f.end()) return fail("qwen3: missing tensor `%s`", name.c_str());
     *out = it->second;
@@ -3246,7 +2651,7 @@ int model_vec(jq_model *m, const std::string &name, const float **out) {
 // replaces their entries in m->q by views of it.  Skipped when any is missing or the types differ.
 // With `pair_rows` (two parts of equal shape) the rows alternate instead: row 2j of the fused matrix is
 // row j of the first part, row 2j + 1 row j of the second, and the views stride over every other row.
-int model_fuse(jq_model *m, const std::string &key, const std::vector<std::string> &names, bool pair_rows = false) {
+int model_fuse(Qwen3Model *m, const std::string &key, const std::vector<std::string> &names, bool pair_rows = false) {
     std::vector<jq_weight *> parts;
     for (const auto &nm : names) {
         auto it = m->q.find(nm);
@@ -3292,7 +2697,7 @@ int model_fuse(jq_model *m, const std::string &key, const std::vector<std::strin
 }
 
 // The layer objects of a mixture-of-experts model that are not built yet (all of them at the first step).
-int model_prepare_moe(jq_model *m) {
+int model_prepare_moe(Qwen3Model *m) {
     const jq_qwen3_config &c = m->cfg;
     if (!c.n_expert) return 0;
     m->moe.resize(c.n_layer, nullptr);
@@ -3316,7 +2721,7 @@ int model_prepare_moe(jq_model *m) {
     return 0;
 }
 
-int model_prepare_fused(jq_model *m) {
+int model_prepare_fused(Qwen3Model *m) {
     if (model_prepare_moe(m)) return 1;
     if (m->fused_ready) return 0;
     const jq_qwen3_config &c = m->cfg;
@@ -3347,8 +2752,6 @@ int model_prepare_fused(jq_model *m) {
     return 0;
 }
 
-unsigned grid_for(size_t total) { return (unsigned)std::min<size_t>((total + 255) / 256, 8192); }
-
 // x_out = x + res; y = W rmsnorm(x_out) as one launch (hn_out also gets the normalised row when
 // given).  False when no kernel has that form for this weight: the caller then runs the two steps.
 // With `swiglu`, w pairs gate and up rows and y gets the w->n / 2 activations.
@@ -3360,7 +2763,7 @@ bool model_norm_mm(const jq_weight *w, const float *x, const float *res, const f
     return dispatch_q4k_dot4(w->dev, w->row_bytes, x, y, w->k, w->n, s, &nm, swiglu) == 0;
 }
 
-int model_forward_dev(jq_model *m, uint32_t T, uint32_t pos, hipStream_t s) {
+int model_forward_dev(Qwen3Model *m, uint32_t T, uint32_t pos, const uint32_t *want, uint32_t n_want, hipStream_t s) {
     const jq_qwen3_config &c = m->cfg;
     const int d = (int)c.head_dim, nh = (int)c.n_head, nkv = (int)c.n_kv_head, h = (int)c.hidden;
     auto emb = m->q.find("token_embd.weight");
@@ -3537,20 +2940,49 @@ int model_forward_dev(jq_model *m, uint32_t T, uint32_t pos, hipStream_t s) {
         if (!down_done && model_mm(m, p + ".ffn_down.weight", m->mid, m->proj, T, s)) return 1;
         pending = m->proj;
     }
+    if (!n_want) return 0;
     const float *w_on;
     if (model_vec(m, "output_norm.weight", &w_on)) return 1;
-    // logits only for the last position (reference: src/quantized_qwen3_moe.rs:816-818)
-    const size_t last = (size_t)(T - 1) * h;
-    hipLaunchKernelGGL(jq::rmsnorm_rows, dim3(1), dim3(1024), 0, s, xc + last, pending ? pending + last : nullptr, w_on,
-                       c.rms_eps, m->hn, h);
+    // logits only for the wanted positions (the last one of a plugin step; reference: src/quantized_qwen3_moe.rs:816-818)
+    for (uint32_t i = 0; i < n_want; i++) {
+        const size_t at = (size_t)want[i] * h;
+        // (a position wanted twice: its residual is added once)
+        bool again = false;
+        for (uint32_t j = 0; j < i; j++) again |= want[j] == want[i];
+        hipLaunchKernelGGL(jq::rmsnorm_rows, dim3(1), dim3(1024), 0, s, xc + at, pending && !again ? pending + at : nullptr, w_on,
+                           c.rms_eps, m->hn + (size_t)i * h, h);
+    }
     // tie_word_embeddings conversions ship no output head (src/quantized_qwen3_moe.rs:739-743)
     const char *head = m->q.count("output.weight") ? "output.weight" : "token_embd.weight";
-    if (model_mm(m, head, m->hn, m->logits, 1, s)) return 1;
+    if (model_mm(m, head, m->hn, m->logits, n_want, s)) return 1;
     HIP_TRY(hipGetLastError());
     return 0;
 }
 
 }  // namespace
+
+Qwen3Model::~Qwen3Model() {
+    Qwen3Model *m = this;
+    model_free_scratch(m);
+    for (jq_moe *e : m->moe) jq_moe_free(e);
+    for (auto &kv : m->q) jq_free(kv.second);
+    for (auto &kv : m->fused) jq_free(kv.second);
+    for (auto *w : m->retired) jq_free(w);
+    if (m->cat) (void)hipFree(m->cat);
+    for (auto &kv : m->f) (void)hipFree(kv.second);
+    for (float *p : m->kc) (void)hipFree(p);
+    for (float *p : m->vc) (void)hipFree(p);
+    if (m->pos) (void)hipFree(m->pos);
+    if (m->part) (void)hipFree(m->part);
+    if (m->rope_cs) (void)hipFree(m->rope_cs);
+}
+
+int Qwen3Model::step(const uint32_t *tokens, uint32_t n, const uint32_t *want, uint32_t n_want, hipStream_t s) {
+    if (model_reserve(this, std::max(n, n_want))) return 1;
+    if (model_prepare_fused(this)) return 1;  // first step only: q|k(|v) and gate|up as single matrices
+    HIP_TRY(hipMemcpyAsync(ids, tokens, n * sizeof(uint32_t), hipMemcpyHostToDevice, s));
+    return model_forward_dev(this, n, n_past, want, n_want, s);
+}
 
 extern "C" {
 
@@ -3570,8 +3002,9 @@ int jq_qwen3_create(const jq_qwen3_config *cfg, jq_model **out) {
     if (c.head_dim % 8 != 0 || c.hidden % 4 != 0 || c.ffn % 4 != 0) return fail("qwen3: dimensions must be multiples of 4/8");
     if (c.head_dim > (uint32_t)jq::AR_MAX_D) return fail("qwen3: head_dim %u exceeds %d", c.head_dim, jq::AR_MAX_D);
     if (ensure_init()) return 1;
-    jq_model *m = new jq_model;
+    Qwen3Model *m = new Qwen3Model;
     m->cfg = c;
+    m->arch = c.n_expert ? "qwen3moe" : "qwen3", m->vocab = c.vocab, m->n_ctx = c.n_ctx;
     size_t per = (size_t)c.n_kv_head * c.n_ctx * c.head_dim * sizeof(float);
     for (uint32_t l = 0; l < c.n_layer; l++) {
         float *k = nullptr, *v = nullptr;
@@ -3584,11 +3017,11 @@ int jq_qwen3_create(const jq_qwen3_config *cfg, jq_model **out) {
         m->vc.push_back(v);
     }
     const size_t part_floats = (size_t)8 * c.n_head * ((c.n_ctx + jq::ATT_CHUNK - 1) / jq::ATT_CHUNK) * (c.head_dim + 2);
-    if (hipMalloc((void **)&m->logits, c.vocab * sizeof(float)) != hipSuccess ||
-        hipMalloc((void **)&m->pick, sizeof(uint32_t)) != hipSuccess ||
-        hipMalloc((void **)&m->pick_v, jq::ARGMAX_PARTS * sizeof(float)) != hipSuccess ||
-        hipMalloc((void **)&m->pick_i, jq::ARGMAX_PARTS * sizeof(int)) != hipSuccess ||
-        hipMalloc((void **)&m->pos, sizeof(int)) != hipSuccess ||
+    if (m->init_outputs()) {
+        jq_qwen3_free(m);
+        return 1;
+    }
+    if (hipMalloc((void **)&m->pos, sizeof(int)) != hipSuccess ||
         hipMalloc((void **)&m->part, part_floats * sizeof(float)) != hipSuccess ||
         hipMalloc((void **)&m->rope_cs, (size_t)8 * (c.head_dim / 2) * sizeof(float2)) != hipSuccess) {
         jq_qwen3_free(m);
@@ -3598,29 +3031,12 @@ int jq_qwen3_create(const jq_qwen3_config *cfg, jq_model **out) {
     return 0;
 }
 
-void jq_qwen3_free(jq_model *m) {
-    if (!m) return;
-    model_free_scratch(m);
-    for (jq_moe *e : m->moe) jq_moe_free(e);
-    for (auto &kv : m->q) jq_free(kv.second);
-    for (auto &kv : m->fused) jq_free(kv.second);
-    for (auto *w : m->retired) jq_free(w);
-    if (m->cat) (void)hipFree(m->cat);
-    for (auto &kv : m->f) (void)hipFree(kv.second);
-    for (float *p : m->kc) (void)hipFree(p);
-    for (float *p : m->vc) (void)hipFree(p);
-    if (m->logits) (void)hipFree(m->logits);
-    if (m->pick) (void)hipFree(m->pick);
-    if (m->pick_v) (void)hipFree(m->pick_v);
-    if (m->pick_i) (void)hipFree(m->pick_i);
-    if (m->pos) (void)hipFree(m->pos);
-    if (m->part) (void)hipFree(m->part);
-    if (m->rope_cs) (void)hipFree(m->rope_cs);
-    delete m;
-}
+void jq_qwen3_free(jq_model *m) { jq_model_free(m); }
 
-int jq_qwen3_set_tensor(jq_model *m, const char *name, uint32_t ggml_type, const void *data, size_t nbytes) {
-    if (!m || !name || !data) return fail("jq_qwen3_set_tensor: null argument");
+int jq_qwen3_set_tensor(jq_model *model, const char *name, uint32_t ggml_type, const void *data, size_t nbytes) {
+    if (!model || !name || !data) return fail("jq_qwen3_set_tensor: null argument");
+    Qwen3Model *m = qwen3_of(model, "jq_qwen3_set_tensor");
+    if (!m) return 1;
     size_t n, k;
     if (!qwen3_shape(m->cfg, name, &n, &k)) return fail("qwen3: unknown tensor `%s`", name);
     std::lock_guard<std::mutex> lock(m->mu);
@@ -3697,53 +3113,21 @@ int jq_qwen3_set_tensor(jq_model *m, const char *name, uint32_t ggml_type, const
 
 int jq_qwen3_forward(jq_model *m, const uint32_t *tokens, uint32_t n_tokens, uint32_t pos, float *logits,
                      int logits_on_device, void *stream) {
-    if (!m || !tokens) return fail("jq_qwen3_forward: null argument");
-    if (n_tokens == 0) return fail("qwen3: forward needs at least one token");
-    std::lock_guard<std::mutex> lock(m->mu);
-    // the KV-cache contract of the plugin boundary (reference: crates/joshua-mock-npu/src/lib.rs:89-95)
-    if (pos != m->n_past) return fail("qwen3: pos %u does not match the %u tokens fed so far", pos, m->n_past);
-    if ((uint64_t)pos + n_tokens > m->cfg.n_ctx)
-        return fail("qwen3: %u + %u tokens exceed the context of %u", pos, n_tokens, m->cfg.n_ctx);
-    for (uint32_t i = 0; i < n_tokens; i++)
-        if (tokens[i] >= m->cfg.vocab) return fail("embedding id %u is out of range for %u rows", tokens[i], m->cfg.vocab);
-    hipStream_t s = (hipStream_t)stream;
-    if (model_reserve(m, n_tokens)) return 1;
-    if (model_prepare_fused(m)) return 1;  // first step only: q|k(|v) and gate|up as single matrices
-    HIP_TRY(hipMemcpyAsync(m->ids, tokens, n_tokens * sizeof(uint32_t), hipMemcpyHostToDevice, s));
-    if (model_forward_dev(m, n_tokens, pos, s)) return 1;
-    m->n_past = pos + n_tokens;
-    if (logits) {
-        HIP_TRY(hipMemcpyAsync(logits, m->logits, m->cfg.vocab * sizeof(float),
-                               logits_on_device ? hipMemcpyDeviceToDevice : hipMemcpyDeviceToHost, s));
-        if (!logits_on_device) HIP_TRY(hipStreamSynchronize(s));
-    }
-    return 0;
+    const uint32_t last = n_tokens - 1;
+    return jq_model_forward(m, tokens, n_tokens, pos, &last, n_tokens ? 1 : 0, logits, logits_on_device, stream);
 }
 
-int jq_qwen3_greedy(jq_model *m, uint32_t *token, void *stream) {
-    if (!m || !token) return fail("jq_qwen3_greedy: null argument");
-    hipStream_t s = (hipStream_t)stream;
-    std::lock_guard<std::mutex> lock(m->mu);
-    hipLaunchKernelGGL(jq::argmax_last_parts, dim3(jq::ARGMAX_PARTS), dim3(256), 0, s, m->logits, (int)m->cfg.vocab,
-                       m->pick_v, m->pick_i);
-    hipLaunchKernelGGL(jq::argmax_last_merge, dim3(1), dim3(jq::ARGMAX_PARTS), 0, s, m->pick_v, m->pick_i, m->pick);
-    HIP_TRY(hipMemcpyAsync(token, m->pick, sizeof(uint32_t), hipMemcpyDeviceToHost, s));
-    HIP_TRY(hipStreamSynchronize(s));
-    return 0;
-}
+int jq_qwen3_greedy(jq_model *m, uint32_t *token, void *stream) { return jq_model_greedy(m, token, stream); }
 
-int jq_qwen3_get_config(const jq_model *m, jq_qwen3_config *out) {
-    if (!m || !out) return fail("jq_qwen3_get_config: null argument");
+int jq_qwen3_get_config(const jq_model *model, jq_qwen3_config *out) {
+    if (!model || !out) return fail("jq_qwen3_get_config: null argument");
+    const Qwen3Model *m = qwen3_of(const_cast<jq_model *>(model), "jq_qwen3_get_config");
+    if (!m) return 1;
     *out = m->cfg;
     return 0;
 }
 
-int jq_qwen3_reset(jq_model *m) {
-    if (!m) return fail("jq_qwen3_reset: model is null");
-    std::lock_guard<std::mutex> lock(m->mu);
-    m->n_past = 0;
-    return 0;
-}
+int jq_qwen3_reset(jq_model *m) { return jq_model_reset(m); }
 
 }  // extern "C"
 
@@ -3764,7 +3148,7 @@ int gguf_wrap(std::unique_ptr<jq::Gguf> g, const std::string &err, jq_gguf **out
 }
 
 // Every tensor the graph reads is installed, or the name of the first one that is not.
-int model_check_complete(jq_model *m) {
+int model_check_complete(Qwen3Model *m) {
     std::vector<std::string> names = {"token_embd.weight", "output_norm.weight", "output.weight"};
     const bool moe = m->cfg.n_expert != 0;
     for (uint32_t l = 0; l < m->cfg.n_layer; l++) {
@@ -3966,8 +3350,9 @@ int jq_qwen3_load_gguf(const char *path, uint32_t n_ctx, jq_model **out) {
     if (!g) return fail("%s", err.c_str());
     jq_qwen3_config cfg{};
     if (qwen3_config_from_gguf(*g, n_ctx, &cfg)) return 1;
-    jq_model *m = nullptr;
-    if (jq_qwen3_create(&cfg, &m)) return 1;
+    jq_model *model = nullptr;
+    if (jq_qwen3_create(&cfg, &model)) return 1;
+    Qwen3Model *m = static_cast<Qwen3Model *>(model);
     bool have_output = false;
     for (const jq::GgufTensor &t : g->tensors) {
         size_t n, k;
@@ -4020,41 +3405,16 @@ int jq_qwen3_load_gguf(const char *path, uint32_t n_ctx, jq_model **out) {
     return 0;
 }
 
-// The four symbols the reference engine binds when it loads a backend as a shared library
-// (reference: src/npu/mod.rs:32-50 contract, src/npu/vendor.rs:17-20 signatures, :49-56 symbol
-// check, :95-121 init; crates/joshua-mock-npu/src/lib.rs:41-131 return codes of the model plugin).
-int32_t joshua_npu_init(const char *model_path, uint32_t n_ctx, uint32_t *out_vocab, void **out_handle) {
-    if (!model_path || !out_vocab || !out_handle) return -1;
-    *out_handle = nullptr;
-    jq_model *m = nullptr;
-    if (jq_qwen3_load_gguf(model_path, n_ctx, &m)) return -2;
-    *out_vocab = m->cfg.vocab;
-    *out_handle = m;
-    return 0;
-}
-
-int32_t joshua_npu_forward(void *handle, const uint32_t *tokens, uint32_t n_tokens, uint32_t pos, float *out_logits) {
-    if (!handle || !tokens || !out_logits || n_tokens == 0) return -1;
-    jq_model *m = (jq_model *)handle;
-    // the handle may arrive on another thread than the one that made it; the device is per thread
-    if (hipSetDevice(g_device) != hipSuccess) return -5;
-    {
-        std::lock_guard<std::mutex> lock(m->mu);
-        if (pos != m->n_past) return -3;
-        if ((uint64_t)pos + n_tokens > m->cfg.n_ctx) return -4;
-    }
-    return jq_qwen3_forward(m, tokens, n_tokens, pos, out_logits, 0, nullptr) ? -5 : 0;
-}
-
-int32_t joshua_npu_reset(void *handle) {
-    if (!handle) return -1;
-    return jq_qwen3_reset((jq_model *)handle) ? -5 : 0;
-}
-
-void joshua_npu_free(void *handle) {
-    if (!handle) return;
-    (void)hipSetDevice(g_device);
-    jq_qwen3_free((jq_model *)handle);
-}
-
 }  // extern "C"
+
+namespace {
+
+int load_qwen3(const char *path, const ModelLoadOptions &opt, jq_model **out) {
+    if (opt.compute == JQ_COMPUTE_F32)
+        return fail("qwen3: products of quantized blocks run on fixed-point activations; there is no 32-bit form");
+    return jq_qwen3_load_gguf(path, opt.n_ctx, out);
+}
+const RegisterModelArch g_register_qwen3({"qwen3", false, load_qwen3});
+const RegisterModelArch g_register_qwen3moe({"qwen3moe", false, load_qwen3});
+
+}  // namespace

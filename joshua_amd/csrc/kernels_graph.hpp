@@ -22,7 +22,7 @@ __device__ __forceinline__ float block_sum(float v, float *red) {  // blockDim.x
 // out[r, :] = x[r, :] / sqrt(mean(x[r, :]^2) + eps) * w.  One workgroup of 1024 per row,
 // float4 per thread, the row kept in registers between the two passes (h <= 8192),
 // so a 4096-wide row costs one memory round trip instead of sixteen.
-__global__ __launch_bounds__(1024) void rmsnorm_rows(float *__restrict__ x, const float *__restrict__ res,
+static __global__ __launch_bounds__(1024) void rmsnorm_rows(float *__restrict__ x, const float *__restrict__ res,
                                                       const float *__restrict__ w, float eps,
                                                       float *__restrict__ out, int h) {
     __shared__ float red[16];
@@ -59,7 +59,7 @@ __global__ __launch_bounds__(1024) void rmsnorm_rows(float *__restrict__ x, cons
 // (reference: src/quantized_qwen3_moe.rs:237-262,345-364; closed form in its test :867-895).
 // cache layout [kv_head, n_ctx, d]; *pos_ptr is the number of tokens already cached.  A token's q, k and v
 // heads start qs, ks and vs floats after the previous token's (the three may be parts of one product's rows).
-__global__ __launch_bounds__(64) void qkv_norm_rope_cache(float *__restrict__ q, const float *__restrict__ k,
+static __global__ __launch_bounds__(64) void qkv_norm_rope_cache(float *__restrict__ q, const float *__restrict__ k,
                                                            const float *__restrict__ v, const float *__restrict__ wq,
                                                            const float *__restrict__ wk, float eps, int n_head, int n_kv,
                                                            int d, const int *__restrict__ pos_ptr, float theta,
@@ -101,7 +101,7 @@ __global__ __launch_bounds__(64) void qkv_norm_rope_cache(float *__restrict__ q,
 // when the maximum moves), so the LDS a launch needs does not grow with the context.  d <= 4 * 256.
 constexpr int AR_CHUNK = 1024, AR_MAX_D = 1024;
 
-__global__ __launch_bounds__(256) void attention_rows(const float *__restrict__ q, const float *__restrict__ kc,
+static __global__ __launch_bounds__(256) void attention_rows(const float *__restrict__ q, const float *__restrict__ kc,
                                                        const float *__restrict__ vc, float *__restrict__ out,
                                                        int n_head, int n_kv, int d, const int *__restrict__ pos_ptr,
                                                        int n_ctx, float sqrt_d, int q_stride) {
@@ -320,7 +320,7 @@ __global__ __launch_bounds__(64 * G * KS) void attention_tiles(const float *__re
 // *pos = p, and the rotary angles of the T positions p .. p + T - 1 of a step: cs[t][i] = (cos, sin) of
 // (p + t) * theta^(-2i/d), i < d/2 — the arithmetic of qkv_norm_rope_cache, done once a step for the
 // attention kernel that applies head norm and rotation itself.
-__global__ __launch_bounds__(256) void rope_table(int *pos, int p, int T, int d, float theta, float2 *__restrict__ cs) {
+static __global__ __launch_bounds__(256) void rope_table(int *pos, int p, int T, int d, float theta, float2 *__restrict__ cs) {
     if (threadIdx.x == 0) *pos = p;
     const int half = d / 2;
     for (int e = threadIdx.x; e < T * half; e += blockDim.x) {
@@ -507,7 +507,7 @@ __global__ __launch_bounds__(256) void attention_split(int n_head, int n_kv, int
 // out[(t, head), :] = sum_ch exp(m_ch - m) acc_ch / sum_ch exp(m_ch - m) l_ch over the chunks with keys.
 // Every read of the partials is issued side by side (a thread per chunk for m and l, 16 chunks at a
 // time for the sums): the kernel is a few round trips to memory long, whatever the chunk count.
-__global__ __launch_bounds__(128) void attention_merge(const float *__restrict__ part, float *__restrict__ out, int d,
+static __global__ __launch_bounds__(128) void attention_merge(const float *__restrict__ part, float *__restrict__ out, int d,
                                                         int n_chunks) {
     extern __shared__ float wch[];  // [n_chunks] maxima, then rescaling weights; [n_chunks] l
     float *lch = wch + n_chunks;
@@ -543,16 +543,16 @@ __global__ __launch_bounds__(128) void attention_merge(const float *__restrict__
 }
 
 // out[i] = silu(gu[2i]) * gu[2i + 1]: the activation over a product with a row-paired gate|up matrix
-__global__ __launch_bounds__(256) void swiglu_pairs(const float *__restrict__ gu, float *__restrict__ out, size_t total) {
+static __global__ __launch_bounds__(256) void swiglu_pairs(const float *__restrict__ gu, float *__restrict__ out, size_t total) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
         const float2 v = ((const float2 *)gu)[i];
         out[i] = silu(v.x) * v.y;
     }
 }
 
-__global__ void set_int(int *p, int v) { *p = v; }
+static __global__ void set_int(int *p, int v) { *p = v; }
 
-__global__ __launch_bounds__(256) void add_rows(const float *__restrict__ a, const float *__restrict__ b,
+static __global__ __launch_bounds__(256) void add_rows(const float *__restrict__ a, const float *__restrict__ b,
                                                  float *__restrict__ out, size_t total) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x)
         out[i] = a[i] + b[i];
@@ -588,7 +588,7 @@ __device__ __forceinline__ void argmax_last_block(float &best, int &idx, float *
     }
 }
 
-__global__ __launch_bounds__(256) void argmax_last_parts(const float *__restrict__ v, int n, float *__restrict__ pv,
+static __global__ __launch_bounds__(256) void argmax_last_parts(const float *__restrict__ v, int n, float *__restrict__ pv,
                                                          int *__restrict__ pi) {
     __shared__ float bv[4];
     __shared__ int bi[4];
@@ -605,7 +605,7 @@ __global__ __launch_bounds__(256) void argmax_last_parts(const float *__restrict
     if (threadIdx.x == 0) pv[blockIdx.x] = best, pi[blockIdx.x] = idx;
 }
 
-__global__ __launch_bounds__(ARGMAX_PARTS) void argmax_last_merge(const float *__restrict__ pv, const int *__restrict__ pi,
+static __global__ __launch_bounds__(ARGMAX_PARTS) void argmax_last_merge(const float *__restrict__ pv, const int *__restrict__ pi,
                                                                   uint32_t *__restrict__ out) {
     __shared__ float bv[ARGMAX_PARTS / 64];
     __shared__ int bi[ARGMAX_PARTS / 64];

@@ -89,7 +89,7 @@ __device__ __forceinline__ void moe_router_logits_body(const float *__restrict__
     }
 }
 
-__global__ __launch_bounds__(256) void moe_router_logits(const float *__restrict__ Wr, const float *__restrict__ X,
+static __global__ __launch_bounds__(256) void moe_router_logits(const float *__restrict__ Wr, const float *__restrict__ X,
                                                           float *__restrict__ logits, int T, int h, int E, ActsI8 planes) {
     moe_router_logits_body(Wr, X, logits, T, h, E, planes);
 }
@@ -106,7 +106,7 @@ struct MoePreNormArgs {
     float *x_out, *hn_out;
 };
 
-__global__ __launch_bounds__(256) void moe_router_logits_norm(const float *__restrict__ Wr, MoePreNormArgs nm,
+static __global__ __launch_bounds__(256) void moe_router_logits_norm(const float *__restrict__ Wr, MoePreNormArgs nm,
                                                                float *__restrict__ logits, int h, int E) {
     __shared__ float red[2][4];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, e = blockIdx.x;
@@ -151,7 +151,7 @@ __global__ __launch_bounds__(256) void moe_router_logits_norm(const float *__res
 // reduced the same way, so the two kernels give the same bits.
 // With `planes` (h a multiple of 32) the launch also leaves the tokens' activations as fixed-point planes for the expert
 // kernels behind it: the workgroups of a token tile share its 8 h / 32 blocks, eight lanes a block.
-__global__ __launch_bounds__(256) void moe_router_logits_tile(const float *__restrict__ Wr, const float *__restrict__ X,
+static __global__ __launch_bounds__(256) void moe_router_logits_tile(const float *__restrict__ Wr, const float *__restrict__ X,
                                                                float *__restrict__ logits, int T, int h, int E,
                                                                ActsI8 planes = ActsI8{nullptr, nullptr, nullptr, nullptr}) {
     __shared__ float red[4][64];
@@ -204,10 +204,13 @@ __global__ __launch_bounds__(256) void moe_router_logits_tile(const float *__res
 
 struct MoeGateParams {
     int E, k_used;
-    int sigmoid;      // 0: softmax over experts, 1: sigmoid per expert
+    int sigmoid;      // 0: softmax over experts, 1: sigmoid per expert, 2: softmax over the biased logits
     int norm_topk;    // divide the k weights by their sum (clamped below at 2^-14)
     float scale;      // multiply the weights (0 or 1: leave alone)
     int n_group, topk_group;
+    // softmax only: the bias is part of the logits (and so of the weights) instead of the selection alone
+    __host__ __device__ bool logit_bias() const { return sigmoid == 2; }
+    __host__ __device__ bool is_sigmoid() const { return sigmoid == 1; }
 };
 
 // One wave per token: probabilities, selection scores (bias, group limit),
@@ -222,7 +225,7 @@ struct MoePairGroups {
     int n_extra;
 };
 
-__global__ __launch_bounds__(256) void moe_gate_topk(const float *__restrict__ logits, const float *__restrict__ bias,
+static __global__ __launch_bounds__(256) void moe_gate_topk(const float *__restrict__ logits, const float *__restrict__ bias,
                                                       MoeGateParams p, uint32_t *__restrict__ ids,
                                                       float *__restrict__ wts, MoePairGroups pg) {
     extern __shared__ __attribute__((aligned(16))) float sm[];  // probs[E], sel[E], gscore[n_group], selw[k_used], red[4]
@@ -231,11 +234,12 @@ __global__ __launch_bounds__(256) void moe_gate_topk(const float *__restrict__ l
     const int t = blockIdx.x, lane = threadIdx.x, wv = threadIdx.x >> 6;  // `lane` strides the experts by 256
     constexpr int NT = 256;
     const float *lg = logits + (size_t)t * p.E;
-    if (p.sigmoid) {
+    if (p.is_sigmoid()) {
         for (int e = lane; e < p.E; e += NT) probs[e] = 1.0f / (1.0f + expf(-lg[e]));
     } else {
         float mx = -INFINITY;
-        for (int e = lane; e < p.E; e += NT) mx = fmaxf(mx, lg[e]);
+        const float *lb = p.logit_bias() ? bias : nullptr;
+        for (int e = lane; e < p.E; e += NT) mx = fmaxf(mx, lb ? lg[e] + lb[e] : lg[e]);
 #pragma unroll
         for (int off = 32; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
         if ((lane & 63) == 0) red[wv] = mx;
@@ -244,7 +248,7 @@ __global__ __launch_bounds__(256) void moe_gate_topk(const float *__restrict__ l
         __syncthreads();
         float sum = 0.0f;
         for (int e = lane; e < p.E; e += NT) {
-            const float v = expf(lg[e] - mx);
+            const float v = expf((lb ? lg[e] + lb[e] : lg[e]) - mx);
             probs[e] = v;
             sum += v;
         }
@@ -254,7 +258,7 @@ __global__ __launch_bounds__(256) void moe_gate_topk(const float *__restrict__ l
         sum = (red[0] + red[1]) + (red[2] + red[3]);
         for (int e = lane; e < p.E; e += NT) probs[e] = probs[e] / sum;
     }
-    for (int e = lane; e < p.E; e += NT) sel[e] = probs[e] + (bias ? bias[e] : 0.0f);
+    for (int e = lane; e < p.E; e += NT) sel[e] = probs[e] + (bias && !p.logit_bias() ? bias[e] : 0.0f);
     __syncthreads();
     if (p.n_group > 1) {
         const int per = p.E / p.n_group;
@@ -269,7 +273,7 @@ __global__ __launch_bounds__(256) void moe_gate_topk(const float *__restrict__ l
                     b2 = v;
                 }
             }
-            gscore[g] = p.sigmoid ? b1 + b2 : b1;
+            gscore[g] = p.is_sigmoid() ? b1 + b2 : b1;
         }
         __syncthreads();
         for (int e = lane; e < p.E; e += NT) {
@@ -345,7 +349,12 @@ __device__ __forceinline__ void moe_gate_topk_wave_body(int t, int T, int lane, 
         float v[NE];
 #pragma unroll
         for (int i = 0; i < NE; i++) v[i] = lane + 64 * i < p.E ? lg[lane + 64 * i] : -INFINITY;
-        if (p.sigmoid) {
+        if (p.logit_bias() && bias) {
+#pragma unroll
+            for (int i = 0; i < NE; i++)
+                if (lane + 64 * i < p.E) v[i] += bias[lane + 64 * i];
+        }
+        if (p.is_sigmoid()) {
 #pragma unroll
             for (int i = 0; i < NE; i++) prob[i] = 1.0f / (1.0f + expf(-v[i]));
         } else {
@@ -365,7 +374,7 @@ __device__ __forceinline__ void moe_gate_topk_wave_body(int t, int T, int lane, 
         }
 #pragma unroll
         for (int i = 0; i < NE; i++)
-            sel[i] = lane + 64 * i < p.E ? prob[i] + (bias ? bias[lane + 64 * i] : 0.0f) : -INFINITY;
+            sel[i] = lane + 64 * i < p.E ? prob[i] + (bias && !p.logit_bias() ? bias[lane + 64 * i] : 0.0f) : -INFINITY;
     }
     int my_e = 0;
     float my_p = 0.0f;  // lane r keeps slot r
@@ -428,6 +437,16 @@ __global__ __launch_bounds__(64) void moe_gate_topk_wave(const float *__restrict
     moe_gate_topk_wave_body<NE>((int)blockIdx.x, (int)gridDim.x, (int)threadIdx.x, logits, bias, p, ids, wts, pg, true, &slot_e);
 }
 
+// The operands of a gating that a kernel behind the router runs itself.
+struct MoeGateIn {
+    const float *logits, *bias;
+    MoeGateParams p;
+    uint32_t *ids;
+    float *wts;
+    MoePairGroups pg;
+    int T;
+};
+
 // Groups the T*k routed (token, slot) pairs by expert, keeping pair order inside
 // a group (the reference buckets the same way on the host,
 // src/quantized_qwen3_moe.rs:459-480).  Group e is expert e:
@@ -435,7 +454,7 @@ __global__ __launch_bounds__(64) void moe_gate_topk_wave(const float *__restrict
 //   xrow[pos]  activation row (token) of the pair,  yrow[pos]  the pair index
 constexpr int GROUP_PAIRS_THREADS = 1024;
 
-__global__ __launch_bounds__(GROUP_PAIRS_THREADS) void moe_group_pairs(const uint32_t *__restrict__ ids, int T,
+static __global__ __launch_bounds__(GROUP_PAIRS_THREADS) void moe_group_pairs(const uint32_t *__restrict__ ids, int T,
                                                                        int k_used, int E, int *__restrict__ gexp,
                                                                        int *__restrict__ offsets,
                                                                        int *__restrict__ xrow, int *__restrict__ yrow,
@@ -507,7 +526,7 @@ __global__ __launch_bounds__(GROUP_PAIRS_THREADS) void moe_group_pairs(const uin
 // LDS: chunks * E + E + 1 ints.
 constexpr int GROUP_RANK_CHUNKS = 64, GROUP_RANK_PER_WAVE = GROUP_RANK_CHUNKS * 64 / GROUP_PAIRS_THREADS;
 
-__global__ __launch_bounds__(GROUP_PAIRS_THREADS) void moe_group_pairs_ranked(const uint32_t *__restrict__ ids, int T,
+static __global__ __launch_bounds__(GROUP_PAIRS_THREADS) void moe_group_pairs_ranked(const uint32_t *__restrict__ ids, int T,
                                                                               int k_used, int E, int *__restrict__ gexp,
                                                                               int *__restrict__ offsets,
                                                                               int *__restrict__ xrow, int *__restrict__ yrow,
@@ -760,7 +779,7 @@ __global__ __launch_bounds__(64 * ROWS_PER_WG) void moe_rows_staged(const uint8_
     }
 }
 
-__global__ __launch_bounds__(256) void acts_i8_prep(const float *__restrict__ X, size_t rows, int k, ActsI8 out) {
+static __global__ __launch_bounds__(256) void acts_i8_prep(const float *__restrict__ X, size_t rows, int k, ActsI8 out) {
     const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;  // four elements a thread, eight threads a block
     if (i >= rows * (size_t)(k / 4)) return;  // whole groups of 8 lanes leave together (k % 32 == 0)
     acts_i8_quantize(X, i, out);
@@ -1176,7 +1195,7 @@ __global__ __launch_bounds__(64 * ROWS_PER_WG) void moe_down_combine_dot8(const 
 // y[t, :] = sum_s w[t, s] * out[t*k + s, :]  (+ shared_out[t, :] of the shared expert),
 // slots added in order s = 0..k-1 (reference: src/quantized_qwen3_moe.rs:516-518,
 // src/quantized_deepseek2.rs:553-557).
-__global__ __launch_bounds__(256) void moe_combine(const float *__restrict__ out, const float *__restrict__ wts, int T,
+static __global__ __launch_bounds__(256) void moe_combine(const float *__restrict__ out, const float *__restrict__ wts, int T,
                                                     int k_used, int h, const float *__restrict__ shared_out,
                                                     float *__restrict__ y) {
     const size_t total = (size_t)T * h;
@@ -1194,14 +1213,14 @@ __global__ __launch_bounds__(256) void moe_combine(const float *__restrict__ out
 namespace jq {
 
 // h[i] = silu(g[i]) * u[i], both clamped first when limit > 0  (the shared expert's activation; the decoder's)
-__global__ __launch_bounds__(256) void swiglu_rows(const float *__restrict__ g, const float *__restrict__ u,
+static __global__ __launch_bounds__(256) void swiglu_rows(const float *__restrict__ g, const float *__restrict__ u,
                                                     float *__restrict__ h, size_t total, float limit) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x)
         h[i] = swiglu(g[i], u[i], limit);
 }
 
 // g[i] = silu(g[i]) * u[i] in place (gate and up results of the grouped GEMM, in front of the down projection)
-__global__ __launch_bounds__(256) void swiglu_in_place(float *__restrict__ g, const float *__restrict__ u, size_t total,
+static __global__ __launch_bounds__(256) void swiglu_in_place(float *__restrict__ g, const float *__restrict__ u, size_t total,
                                                         float limit) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x)
         g[i] = swiglu(g[i], u[i], limit);

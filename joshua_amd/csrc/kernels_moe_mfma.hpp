@@ -200,15 +200,6 @@ constexpr int moe_gate_up_mfma_lds() {
 // expert from there; the first workgroup of a token's first pair writes ids, weights and pair groups for the down
 // projection.  A launch less than gating on its own, which costs 4 us of which 3 are the launch and its wait for
 // the router.
-struct MoeGateIn {
-    const float *logits, *bias;
-    MoeGateParams p;
-    uint32_t *ids;
-    float *wts;
-    MoePairGroups pg;
-    int T;
-};
-
 template <class F, int NB, bool GATE>
 __global__ __launch_bounds__(64 * NB) void moe_gate_up_mfma(MoeStack Wa, MoeStack Wb, const float *__restrict__ X,
                                                             const int *__restrict__ gexp, const int *__restrict__ xrow,

@@ -1,0 +1,163 @@
+// A selective state-space mixer: short causal convolutions a channel, and the recurrence
+//   S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,   y_c = sum_n S[c, n] C_n + D_c x_c
+// with its output gate.  States, step sizes and decays are f32; the carried state of a sequence is S [channels][N] and
+// the convolution's last taps - 1 inputs [taps - 1][channels].
+#pragma once
+#include "kernels_dense.hpp"
+
+namespace jq {
+
+// out[t, c] = silu(b[c] + sum_j w[c, j] x[t - (taps - 1) + j, c]); inputs in front of the step come from tail_in,
+// the step's last taps - 1 go to tail_out (another buffer: a step may be shorter than the tail).
+template <class O>
+__global__ __launch_bounds__(256) void causal_conv_silu(const float *__restrict__ x, size_t ldx, const float *__restrict__ w,
+                                                        const float *__restrict__ b, const float *__restrict__ tail_in,
+                                                        float *__restrict__ tail_out, O *__restrict__ out, size_t ldo, int T, int C,
+                                                        int taps) {
+    const size_t total = (size_t)(T + taps - 1) * C;
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
+        const int t = (int)(i / C), c = (int)(i % C);
+        if (t >= T) {
+            const int at = t - (taps - 1);  // place t - T of the new tail
+            tail_out[(size_t)(t - T) * C + c] = at >= 0 ? x[(size_t)at * ldx + c] : tail_in[(size_t)(at + taps - 1) * C + c];
+            continue;
+        }
+        float acc = b[c];
+        for (int j = 0; j < taps; j++) {
+            const int at = t - (taps - 1) + j;
+            const float v = at >= 0 ? x[(size_t)at * ldx + c] : tail_in[(size_t)(at + taps - 1) * C + c];
+            acc = fmaf(w[(size_t)c * taps + j], v, acc);
+        }
+        out[(size_t)t * ldo + c] = (O)silu(acc);
+    }
+}
+
+__device__ __forceinline__ float softplus(float v) { return v > 20.0f ? v : log1pf(expf(v)); }
+
+template <int LPC>
+__device__ __forceinline__ float sum_lanes(float v) {
+    if constexpr (LPC == 64) return wave_sum(v);
+    else if constexpr (LPC == 32) return sum_row16(sum_xor16(v));
+    else if constexpr (LPC == 16) return sum_row16(v);
+    else if constexpr (LPC == 8) return sum_row8(v);
+    else {
+        v += dpp_f<0xB1>(v);
+        v += dpp_f<0x4E>(v);
+        return v;
+    }
+}
+
+struct SsmScan {
+    const float *dt_raw;      // [T][C]: step sizes before bias and softplus
+    const float *dt_bias;     // [C]
+    const float *bc;          // [T][ld_bc]: B (N) then C (N) of a token
+    size_t ld_bc;
+    const float *z;           // [T][ld_z]: output gate
+    size_t ld_z;
+    const float *A_log2;      // [C][N]: A log2(e)
+    const float *D;           // [C]
+    float *S;                 // [C][N]
+    int T, C, N;
+    size_t ldx, ldo;
+};
+
+// The recurrence over a step's tokens, LPC lanes a channel with NS states each (N <= LPC NS), tokens in runs of
+// SCAN_RUN: a run's step sizes (softplus once a channel), inputs, B and C are put into LDS, the states advance in
+// registers, and the run's outputs leave together, gated.
+constexpr int SCAN_MAX_STATES = 512;
+
+template <int LPC, int NS, class IO>
+__global__ __launch_bounds__(256) void selective_scan(SsmScan a, const IO *__restrict__ x, IO *__restrict__ out) {
+    constexpr int CPW = 256 / LPC, NP = LPC * NS, SCAN_RUN = NP <= 128 ? 32 : 4096 / NP;
+    __shared__ float2 sd[SCAN_RUN][CPW];                                           // dt, dt x
+    __shared__ float sy[SCAN_RUN][CPW];                                            // D x, then the output
+    __shared__ __attribute__((aligned(16))) float sb[SCAN_RUN][NP], scc[SCAN_RUN][NP];
+    const int tid = threadIdx.x, ln = tid % LPC, ch = tid / LPC, c0 = (int)blockIdx.x * CPW, c = c0 + ch;
+    float S[NS], A[NS];
+#pragma unroll
+    for (int j = 0; j < NS; j++) {
+        const int n = ln * NS + j;
+        const bool in = c < a.C && n < a.N;
+        A[j] = in ? a.A_log2[(size_t)c * a.N + n] : 0.0f;
+        S[j] = in ? a.S[(size_t)c * a.N + n] : 0.0f;
+    }
+    for (int t0 = 0; t0 < a.T; t0 += SCAN_RUN) {
+        const int nt = min(SCAN_RUN, a.T - t0), padded = (nt + 3) & ~3;  // (tokens past the end: dt = 0 leaves the states alone)
+        for (int i = tid; i < padded * CPW; i += 256) {
+            const int t = i / CPW, k = i % CPW, cc = c0 + k;
+            float dt = 0.0f, xv = 0.0f, d = 0.0f;
+            if (cc < a.C && t < nt) {
+                dt = softplus(a.dt_raw[(size_t)(t0 + t) * a.C + cc] + a.dt_bias[cc]);
+                xv = (float)x[(size_t)(t0 + t) * a.ldx + cc], d = a.D[cc];
+            }
+            sd[t][k] = float2{dt, dt * xv};
+            sy[t][k] = d * xv;
+        }
+        for (int i = tid; i < padded * NP; i += 256) {
+            const int t = i / NP, n = i % NP;
+            const float *p = a.bc + (size_t)(t0 + t) * a.ld_bc;
+            sb[t][n] = n < a.N && t < nt ? p[n] : 0.0f;
+            scc[t][n] = n < a.N && t < nt ? p[a.N + n] : 0.0f;
+        }
+        __syncthreads();
+        for (int t = 0; t < nt; t += 4) {
+            float y[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int u = 0; u < 4; u++) {
+                const float2 d = sd[t + u][ch];
+#pragma unroll
+                for (int j = 0; j < NS; j++) {
+                    const int n = ln * NS + j;
+                    S[j] = fmaf(__builtin_amdgcn_exp2f(d.x * A[j]), S[j], d.y * sb[t + u][n]);
+                    y[u] = fmaf(S[j], scc[t + u][n], y[u]);
+                }
+            }
+#pragma unroll
+            for (int u = 0; u < 4; u++) y[u] = sum_lanes<LPC>(y[u]);
+            if (ln == 0) {
+#pragma unroll
+                for (int u = 0; u < 4; u++) sy[t + u][ch] += y[u];
+            }
+        }
+        __syncthreads();
+        for (int i = tid; i < nt * CPW; i += 256) {
+            const int t = i / CPW, k = i % CPW, cc = c0 + k;
+            if (cc < a.C) out[(size_t)(t0 + t) * a.ldo + cc] = (IO)(sy[t][k] * silu(a.z[(size_t)(t0 + t) * a.ld_z + cc]));
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int j = 0; j < NS; j++) {
+        const int n = ln * NS + j;
+        if (c < a.C && n < a.N) a.S[(size_t)c * a.N + n] = S[j];
+    }
+}
+
+// One token, with the projection of its step sizes in front: 16 lanes a channel take the channel's row of W_dt
+// (dt = softplus(W_dt p + bias)) and then its N states.
+template <class E>
+__global__ __launch_bounds__(256) void selective_step(SsmScan a, const uint8_t *__restrict__ Wdt, size_t pitch, const float *__restrict__ p,
+                                                      int rank, const float *__restrict__ x, float *__restrict__ out) {
+    const int sub = threadIdx.x & 15, c = 16 * (int)blockIdx.x + ((int)threadIdx.x >> 4), cc = min(c, a.C - 1);
+    const uint8_t *row = Wdt + (size_t)cc * pitch;
+    float dot = 0.0f;
+    for (int k = sub * E::CH; k < rank; k += 16 * E::CH) {
+        float w[E::CH], v[E::CH];
+        E::widen(chunk_of<E>(row, k), w);
+        load_acts<E::CH>(p, k, rank, v);
+#pragma unroll
+        for (int i = 0; i < E::CH; i++) dot = fmaf(w[i], v[i], dot);
+    }
+    const float dt = softplus(sum_row16(dot) + a.dt_bias[cc]), xv = x[cc], dx = dt * xv;
+    float y = 0.0f;
+    for (int n = sub; n < a.N; n += 16) {
+        const size_t at = (size_t)cc * a.N + n;
+        const float S = fmaf(__builtin_amdgcn_exp2f(dt * a.A_log2[at]), a.S[at], dx * a.bc[n]);
+        y = fmaf(S, a.bc[a.N + n], y);
+        if (c < a.C) a.S[at] = S;
+    }
+    y = sum_row16(y);
+    if (sub == 0 && c < a.C) out[c] = fmaf(a.D[c], xv, y) * silu(a.z[c]);
+}
+
+}  // namespace jq

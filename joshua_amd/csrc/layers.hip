@@ -1,0 +1,746 @@
+// Layered decoders with plain BF16 / F32 weights: a stack whose layers each name a mixer (attention, selective scan)
+// and a feed-forward block (none, dense, mixture of experts), normalised in front and behind.  A design is a reader of
+// its configuration into StackConfig plus its tensor names; the step below runs any of them.
+#include "dense.hpp"
+#include "kernels_attention.hpp"
+#include "kernels_ssm.hpp"
+#include "model.hpp"
+#include "safetensors.hpp"
+
+namespace {
+
+// ---- what a design's configuration comes down to ------------------------------------------------------
+
+struct RotaryConfig {
+    int dims = 0;
+    double base = 10000.0;
+    double factor = 1.0, original = 0.0, fast = 0.0, slow = 0.0;  // YaRN; factor 1 with `yarn` false: none
+    bool yarn = false;
+    bool operator==(const RotaryConfig &o) const {
+        return dims == o.dims && base == o.base && yarn == o.yarn && factor == o.factor && original == o.original && fast == o.fast && slow == o.slow;
+    }
+};
+
+struct LayerConfig {
+    enum Mixer { ATTENTION, MAMBA1 } mixer = ATTENTION;
+    // attention
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+    float scale = 1.0f;
+    bool v_mix = false;
+    RotaryConfig rot;
+    // selective scan
+    int inner = 0, state = 0, dt_rank = 0, taps = 0;
+    // feed-forward
+    enum Mlp { NONE, DENSE, MOE } mlp = NONE;
+    int ff = 0, experts = 0, top = 0;
+    float limit = INFINITY;
+};
+
+struct StackConfig {
+    const char *arch = "";
+    uint32_t vocab = 0, width = 0;
+    float embedding_scale = 1.0f, norm_eps = 1e-6f, residual_mult = 1.0f;
+    bool rms = false;                         // norms: root mean square instead of mean and variance with bias
+    float act_alpha = 1.0f, act_shift = 0.0f;  // the gated unit: g sigmoid(alpha g) (u + shift)
+    std::vector<LayerConfig> layers;
+};
+
+// The frequencies of the rotated pairs, and the factor on cos and sin.
+double rotary_frequencies(const RotaryConfig &r, std::vector<double> *freq) {
+    const int half = r.dims / 2;
+    freq->resize(half);
+    for (int i = 0; i < half; i++) (*freq)[i] = std::pow(r.base, -2.0 * i / r.dims);
+    if (!r.yarn) return 1.0;
+    // a pair keeps its frequency where it turns `fast` times or more over the original context, is slowed by
+    // `factor` where it turns `slow` times or less, and goes over linearly between
+    auto index_of = [&](double turns) { return r.dims * std::log(r.original / (2.0 * M_PI * turns)) / (2.0 * std::log(r.base)); };
+    const double lo = std::max(std::floor(index_of(r.fast)), 0.0), hi = std::min(std::ceil(index_of(r.slow)), r.dims - 1.0);
+    for (int i = 0; i < half; i++) {
+        const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+        (*freq)[i] = (*freq)[i] / r.factor * ramp + (*freq)[i] * (1.0 - ramp);
+    }
+    return 0.1 * std::log(r.factor) + 1.0;
+}
+
+// ---- the model -----------------------------------------------------------------------------------------
+
+struct NormWeights {
+    float *w = nullptr, *b = nullptr;
+};
+
+struct Layer {
+    LayerConfig c;
+    NormWeights norm1, norm1b, norm2, norm2b;
+    jq_weight *in = nullptr;   // q | k | v rows, or the scan's x | z
+    jq_weight *o = nullptr;
+    float lambda = 0.0f;
+    bool v_first = false;      // the first layer that mixes values: the others mix in its own
+    int rot = -1;              // which of the model's rotary tables
+    void *kc = nullptr, *vc = nullptr;
+    // selective scan
+    jq_weight *wx = nullptr, *wdt = nullptr;
+    float *conv = nullptr, *conv_b = nullptr, *dt_b = nullptr, *A_log2 = nullptr, *D = nullptr;
+    float *S = nullptr, *tail[2] = {nullptr, nullptr};
+    int tail_at = 0;
+    // feed-forward
+    jq_weight *gate = nullptr, *up = nullptr, *down = nullptr;
+    jq_moe *moe = nullptr;
+    int moe_shares = -1;       // the first layer with experts of the same sizes: their scratch buffers take turns
+    // this layer's activation buffers (shared between layers of equal size)
+    void *mix_e = nullptr, *conv_e = nullptr, *dt_e = nullptr, *ff_e = nullptr;
+
+    int DP() const { return (c.dim + 31) / 32 * 32; }
+    int DVP() const { return (c.vdim + 31) / 32 * 32; }
+    int mix_width() const { return c.mixer == LayerConfig::ATTENTION ? c.heads * c.vdim : c.inner; }
+};
+
+struct RotaryTable {
+    RotaryConfig c;
+    double *freq = nullptr;
+    float mag = 1.0f;
+    float2 *cs = nullptr;  // [tokens of the step][dims / 2]
+};
+
+struct LayeredModel : jq_model {
+    StackConfig cfg;
+    uint32_t type = JQ_TYPE_BF16;  // of the matrices, the caches and a many-token step's activations
+    std::vector<Layer> layers;
+    std::vector<RotaryTable> rots;
+    jq_weight *embed = nullptr, *head = nullptr;
+    NormWeights final_norm;
+    std::vector<void *> owned;     // weights and states in device memory
+    std::vector<jq_weight *> matrices;
+    // scratch for cap_tokens tokens and cap_want wanted rows
+    size_t cap_tokens = 0, cap_want = 0;
+    std::vector<void *> scratch;
+    uint32_t *ids = nullptr, *want_ids = nullptr;
+    float *x = nullptr, *x2 = nullptr, *h = nullptr, *y = nullptr, *proj = nullptr, *mid = nullptr, *conv_f = nullptr, *bc = nullptr,
+          *dt = nullptr, *first_v = nullptr, *part = nullptr;
+    void *h_e = nullptr, *q_e = nullptr;
+    std::vector<int> moe_holder;   // per layer index of the first of its size: which layer holds the scratch now
+    bool broken = false;           // a step failed half way: the states are those of no sequence
+
+    ~LayeredModel() override;
+    int step(const uint32_t *tokens, uint32_t n, const uint32_t *want, uint32_t n_want, hipStream_t s) override;
+    void forget() override { broken = false; }
+    int reserve(size_t T, size_t W);
+    int run_layers(int T, const uint32_t *want, int n_want, hipStream_t s);
+    size_t esz() const { return dense_elem_bytes(type); }
+
+    template <class T>
+    int device_alloc(T **out, size_t n) {
+        void *p = nullptr;
+        HIP_TRY(hipMalloc(&p, std::max<size_t>(n * sizeof(T), 16)));
+        owned.push_back(p);
+        *out = (T *)p;
+        return 0;
+    }
+};
+
+void free_all(std::vector<void *> *v) {
+    for (void *p : *v) (void)hipFree(p);
+    v->clear();
+}
+
+LayeredModel::~LayeredModel() {
+    for (Layer &l : layers) jq_moe_free(l.moe);
+    for (jq_weight *w : matrices) jq_free(w);
+    free_all(&scratch);
+    free_all(&owned);
+}
+
+int LayeredModel::reserve(size_t T, size_t W) {
+    if (T <= cap_tokens && W <= cap_want) return 0;
+    T = std::max(T, cap_tokens), W = std::max(W, cap_want);
+    free_all(&scratch);
+    cap_tokens = cap_want = 0;
+    size_t proj_w = 0, mid_w = 0, inner_w = 0, bc_w = 0, v_w = 0, part_w = 0, q_w = 0;
+    for (const Layer &l : layers) {
+        const LayerConfig &c = l.c;
+        proj_w = std::max(proj_w, l.in->n);
+        mid_w = std::max<size_t>({mid_w, (size_t)l.mix_width(), (size_t)c.ff});
+        if (c.mixer == LayerConfig::ATTENTION) {
+            q_w = std::max(q_w, (size_t)c.heads * l.DP());
+            if (c.v_mix) v_w = std::max(v_w, (size_t)c.kv_heads * c.vdim);
+            part_w = std::max(part_w, (size_t)c.heads * ((n_ctx + jq::ATT_CHUNK - 1) / jq::ATT_CHUNK) * (c.vdim + 2));
+        } else {
+            inner_w = std::max(inner_w, (size_t)c.inner);
+            bc_w = std::max(bc_w, l.wx->n);
+        }
+    }
+    auto get = [&](auto **out, size_t n) {  // zeroed: the padding of activation rows is never written
+        using P = std::remove_reference_t<decltype(**out)>;
+        const size_t bytes = std::max<size_t>(n * sizeof(P), 256);
+        void *p = nullptr;
+        HIP_TRY(hipMalloc(&p, bytes));
+        scratch.push_back(p);
+        HIP_TRY(hipMemset(p, 0, bytes));
+        *out = (P *)p;
+        return 0;
+    };
+    const size_t w = cfg.width, R = std::max(T, W);
+    if (get(&ids, T) || get(&want_ids, W) || get(&x, T * w) || get(&x2, w) || get(&h, R * w) || get(&y, T * w) || get(&proj, T * proj_w) ||
+        get(&mid, (size_t)GEMV_MAX_ROWS * mid_w) || get(&conv_f, (size_t)GEMV_MAX_ROWS * inner_w) || get(&bc, T * bc_w) ||
+        get(&dt, T * inner_w) || get(&first_v, T * v_w) || get(&part, (size_t)GEMV_MAX_ROWS * part_w))
+        return 1;
+    uint8_t *p = nullptr;
+    if (get(&p, R * dense_stride(w) * esz())) return 1;
+    h_e = p;
+    if (get(&p, T * q_w * esz())) return 1;
+    q_e = p;
+    for (RotaryTable &r : rots)
+        if (get(&r.cs, T * (r.c.dims / 2))) return 1;
+    std::map<std::pair<int, size_t>, void *> by_size;  // (role, row length)
+    auto rows = [&](int role, size_t k, void **out) {
+        void *&slot = by_size[{role, k}];
+        if (!slot) {
+            uint8_t *b = nullptr;
+            if (get(&b, T * dense_stride(k) * esz())) return 1;
+            slot = b;
+        }
+        *out = slot;
+        return 0;
+    };
+    for (Layer &l : layers) {
+        if (rows(0, l.mix_width(), &l.mix_e)) return 1;
+        if (l.c.mixer == LayerConfig::MAMBA1 && (rows(1, l.c.inner, &l.conv_e) || rows(2, l.c.dt_rank, &l.dt_e))) return 1;
+        if (l.c.mlp == LayerConfig::DENSE && rows(3, l.c.ff, &l.ff_e)) return 1;
+    }
+    cap_tokens = T, cap_want = W;
+    return 0;
+}
+
+int LayeredModel::step(const uint32_t *tokens, uint32_t n, const uint32_t *want, uint32_t n_want, hipStream_t s) {
+    if (broken) return fail("%s: an earlier step failed half way; reset the model", arch);
+    if (reserve(n, std::max<uint32_t>(n_want, 1))) return 1;
+    HIP_TRY(hipMemcpyAsync(ids, tokens, n * sizeof(uint32_t), hipMemcpyHostToDevice, s));
+    if (n_want) HIP_TRY(hipMemcpyAsync(want_ids, want, n_want * sizeof(uint32_t), hipMemcpyHostToDevice, s));
+    broken = true;
+    if (run_layers((int)n, want, (int)n_want, s)) return 1;
+    HIP_TRY(hipGetLastError());
+    broken = false;
+    return 0;
+}
+
+#define JQ_ELEM_OF(TYPE, CALL)                                 \
+    do {                                                       \
+        if ((TYPE) == JQ_TYPE_BF16) {                          \
+            using E = jq::ElemBf16;                            \
+            CALL;                                              \
+        } else {                                               \
+            using E = jq::ElemF32;                             \
+            CALL;                                              \
+        }                                                      \
+    } while (0)
+
+// The attention of one layer over its projections a.qkv.  Steps of up to 8 tokens leave f32 rows in out_f, longer
+// ones rows of the element type in out_e.
+int run_attention(LayeredModel *m, Layer &l, const jq::AttnLayer &a, bool small, float *out_f, void *out_e, hipStream_t s) {
+    const uint32_t type = m->type;
+    const int dc = std::max(a.DP, a.DVP), gq = a.H / a.G, T = a.T;
+    const size_t ldo = dense_stride((size_t)a.H * a.dv);
+    if (small && dc <= 256) {
+        const int n_chunks = (a.pos0 + T + jq::ATT_CHUNK - 1) / jq::ATT_CHUNK, runs = (gq + jq::DEC_HEADS - 1) / jq::DEC_HEADS;
+        const dim3 grid((unsigned)(n_chunks * a.G * runs), (unsigned)T);
+#define JQ_DEC(DC) JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attention_decode<E, DC>), grid, dim3(256), 0, s, a, n_chunks, m->part))
+        if (dc <= 64) JQ_DEC(64);
+        else if (dc <= 128) JQ_DEC(128);
+        else JQ_DEC(256);
+#undef JQ_DEC
+        hipLaunchKernelGGL(jq::attention_merge, dim3((unsigned)(T * a.H)), dim3(128), 2 * n_chunks * sizeof(float), s, m->part, out_f, a.dv,
+                           n_chunks);
+        return 0;
+    }
+    JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attn_rope_store<E>), dim3((unsigned)T), dim3(256), 0, s, a, (typename E::T *)m->q_e));
+    if (type == JQ_TYPE_BF16 && dc <= 256 && !small) {
+        const float sl = a.scale * 1.44269504088896341f;
+        const size_t rows = (size_t)T * gq;
+        // two sets of 16 rows a wave where that still makes a workgroup for every compute unit
+        const bool two = dc <= 128 && (rows + 127) / 128 * a.G >= 256;
+        const dim3 grid((unsigned)((rows + (two ? 127 : 63)) / (two ? 128 : 64)), (unsigned)a.G);
+        const __bf16 *q = (const __bf16 *)m->q_e;
+        __bf16 *o = (__bf16 *)out_e;
+#define JQ_TILES(DC, QF, KT) hipLaunchKernelGGL((jq::attention_tiles_bf16<DC, QF, KT>), grid, dim3(256), 0, s, a, q, o, ldo, sl)
+        if (dc <= 64 && two) JQ_TILES(64, 2, 64);
+        else if (dc <= 64) JQ_TILES(64, 1, 64);
+        else if (dc <= 128 && two) JQ_TILES(128, 2, 64);
+        else if (dc <= 128) JQ_TILES(128, 1, 64);
+        else JQ_TILES(256, 1, 32);
+#undef JQ_TILES
+        return 0;
+    }
+    const size_t lds = ((size_t)a.DP + jq::ANY_CHUNK + 16 + 256) * sizeof(float);
+    if (small)
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attention_any<E, float>), dim3((unsigned)(T * a.H)), dim3(256), lds, s, a,
+                                            (const typename E::T *)m->q_e, out_f, (size_t)a.H * a.dv));
+    else
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attention_any<E, typename E::T>), dim3((unsigned)(T * a.H)), dim3(256), lds, s, a,
+                                            (const typename E::T *)m->q_e, (typename E::T *)out_e, ldo));
+    return 0;
+}
+
+template <class IO>
+int run_scan(const jq::SsmScan &a, const IO *x, IO *out, hipStream_t s) {
+#define JQ_SCAN(LPC, NS)                                                                                                            \
+    hipLaunchKernelGGL((jq::selective_scan<LPC, NS, IO>), dim3((unsigned)((a.C + 256 / LPC - 1) / (256 / LPC))), dim3(256), 0, s, a, x, out)
+    if (a.N <= 4) JQ_SCAN(4, 1);
+    else if (a.N <= 8) JQ_SCAN(4, 2);
+    else if (a.N <= 16) JQ_SCAN(8, 2);
+    else if (a.N <= 32) JQ_SCAN(16, 2);
+    else if (a.N <= 64) JQ_SCAN(16, 4);
+    else if (a.N <= 128) JQ_SCAN(32, 4);
+    else if (a.N <= 256) JQ_SCAN(64, 4);
+    else JQ_SCAN(64, 8);
+#undef JQ_SCAN
+    return 0;
+}
+
+int LayeredModel::run_layers(int T, const uint32_t *want, int n_want, hipStream_t s) {
+    const int w = (int)cfg.width;
+    const size_t sw = dense_stride(w);
+    const bool small = T <= GEMV_MAX_ROWS;             // f32 activations through the GEMV
+    const bool one = T == 1 && w <= FUSED_NORM_MAX_WIDTH;  // and the residual update and norm inside the product's launch
+    const int pos0 = (int)n_past;
+    if (dense_decode(embed, ids, x, T, cfg.embedding_scale, s)) return 1;
+    for (const RotaryTable &r : rots)
+        hipLaunchKernelGGL(jq::rope_angles, dim3(grid_for((size_t)T * (r.c.dims / 2))), dim3(256), 0, s, r.freq, r.c.dims / 2, pos0, T, r.mag, r.cs);
+    if (pos0 == 0) {  // a new sequence: its states start at zero
+        for (Layer &l : layers)
+            if (l.c.mixer == LayerConfig::MAMBA1 &&
+                (zero_floats(l.S, (size_t)l.c.inner * l.c.state, s) || zero_floats(l.tail[l.tail_at], (size_t)(l.c.taps - 1) * l.c.inner, s)))
+                return 1;
+    }
+    float *xc = x, *xo = x2;
+    const float *pending = nullptr;       // the sublayer result not yet in the stream, and the norm it takes first
+    NormWeights post;
+    // the residual update with `pre` as the next norm; out: where the stream goes
+    auto update = [&](const NormWeights &pre, float *out, float *h_out) {
+        jq::ResidualNorm nm{};
+        nm.x = xc, nm.y = pending, nm.post_w = post.w, nm.post_b = post.b, nm.mult = cfg.residual_mult;
+        nm.pre_w = pre.w, nm.pre_b = pre.b, nm.eps = cfg.norm_eps, nm.rms = cfg.rms ? 1 : 0, nm.width = w;
+        nm.x_out = out, nm.h_out = h_out;
+        return nm;
+    };
+    // out [T][wt->n] = wt norm(stream), the stream updated on the way
+    auto norm_product = [&](const NormWeights &pre, const jq_weight *wt, float *out) {
+        if (one) {
+            const jq::ResidualNorm nm = update(pre, xo, nullptr);
+            if (dense_gemv(wt, nullptr, 0, 1, out, wt->n, s, &nm)) return 1;
+            std::swap(xc, xo);
+            return 0;
+        }
+        if (residual_norm(update(pre, xc, small ? h : nullptr), type, small ? nullptr : h_e, sw, T, nullptr, s)) return 1;
+        return small ? dense_gemv(wt, h, w, T, out, wt->n, s) : dense_gemm(wt, h_e, sw, T, out, wt->n, s);
+    };
+    for (Layer &l : layers) {
+        const LayerConfig &c = l.c;
+        if (norm_product(l.norm1, l.in, proj)) return 1;
+        if (c.mixer == LayerConfig::ATTENTION) {
+            jq::AttnLayer a{};
+            a.H = c.heads, a.G = c.kv_heads, a.d = c.dim, a.dv = c.vdim, a.DP = l.DP(), a.DVP = l.DVP(), a.n_ctx = (int)n_ctx;
+            a.rot = c.rot.dims, a.scale = c.scale, a.pos0 = pos0, a.T = T, a.qkv = proj, a.ld = l.in->n, a.cs = l.rot >= 0 ? rots[l.rot].cs : nullptr;
+            a.v_first = c.v_mix && !l.v_first ? first_v : nullptr, a.v_first_out = l.v_first ? first_v : nullptr, a.lambda = l.lambda;
+            a.kc = l.kc, a.vc = l.vc;
+            if (run_attention(this, l, a, small, mid, l.mix_e, s)) return 1;
+        } else {
+            const int C = c.inner, N = c.state, taps = c.taps;
+            const dim3 cgrid(grid_for((size_t)(T + taps - 1) * C));
+            float *t_in = l.tail[l.tail_at], *t_out = l.tail[l.tail_at ^ 1];
+            if (small)
+                hipLaunchKernelGGL((jq::causal_conv_silu<float>), cgrid, dim3(256), 0, s, proj, l.in->n, l.conv, l.conv_b, t_in, t_out,
+                                   conv_f, (size_t)C, T, C, taps);
+            else
+                JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::causal_conv_silu<typename E::T>), cgrid, dim3(256), 0, s, proj, l.in->n, l.conv, l.conv_b,
+                                                    t_in, t_out, (typename E::T *)l.conv_e, dense_stride(C), T, C, taps));
+            l.tail_at ^= 1;
+            const size_t ldp = l.wx->n;
+            if (small ? dense_gemv(l.wx, conv_f, C, T, bc, ldp, s) : dense_gemm(l.wx, l.conv_e, dense_stride(C), T, bc, ldp, s)) return 1;
+            jq::SsmScan a{};
+            a.dt_raw = dt, a.dt_bias = l.dt_b, a.bc = bc + c.dt_rank, a.ld_bc = ldp, a.z = proj + C, a.ld_z = l.in->n;
+            a.A_log2 = l.A_log2, a.D = l.D, a.S = l.S, a.T = T, a.C = C, a.N = N, a.ldx = a.ldo = (size_t)C;
+            if (T == 1) {
+                JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::selective_step<E>), dim3((unsigned)((C + 15) / 16)), dim3(256), 0, s, a, l.wdt->dev,
+                                                    l.wdt->row_bytes, bc, c.dt_rank, conv_f, mid));
+            } else if (small) {
+                if (dense_gemv(l.wdt, bc, ldp, T, dt, C, s) || run_scan<float>(a, conv_f, mid, s)) return 1;
+            } else {
+                const size_t sr = dense_stride(c.dt_rank);
+                if (rows_to_elem(type, bc, ldp, T, c.dt_rank, l.dt_e, sr, s) || dense_gemm(l.wdt, l.dt_e, sr, T, dt, C, s)) return 1;
+                a.ldx = a.ldo = dense_stride(C);
+                JQ_ELEM_OF(type, if (run_scan<typename E::T>(a, (const typename E::T *)l.conv_e, (typename E::T *)l.mix_e, s)) return 1);
+            }
+        }
+        const int mw = l.mix_width();
+        if (small ? dense_gemv(l.o, mid, mw, T, y, w, s) : dense_gemm(l.o, l.mix_e, dense_stride(mw), T, y, w, s)) return 1;
+        pending = y, post = l.norm1b;
+
+        if (c.mlp == LayerConfig::NONE) continue;
+        if (c.mlp == LayerConfig::DENSE) {
+            const jq::GatedUnit unit{c.limit, cfg.act_alpha, cfg.act_shift};
+            if (one) {
+                const jq::ResidualNorm nm = update(l.norm2, xo, nullptr);
+                if (dense_gemv_gated(l.gate, l.up, nullptr, 0, 1, mid, c.ff, unit, s, &nm)) return 1;
+                std::swap(xc, xo);
+            } else {
+                if (residual_norm(update(l.norm2, xc, small ? h : nullptr), type, small ? nullptr : h_e, sw, T, nullptr, s)) return 1;
+                if (small ? dense_gemv_gated(l.gate, l.up, h, w, T, mid, c.ff, unit, s)
+                          : dense_gemm_gated(l.gate, l.up, h_e, sw, T, l.ff_e, dense_stride(c.ff), unit, s))
+                    return 1;
+            }
+            if (small ? dense_gemv(l.down, mid, c.ff, T, y, w, s) : dense_gemm(l.down, l.ff_e, dense_stride(c.ff), T, y, w, s)) return 1;
+        } else {
+            jq_moe *moe = l.moe;
+            int &holder = moe_holder[l.moe_shares];
+            if (layers[holder].moe != moe) moe_swap_scratch(moe, layers[holder].moe);
+            holder = (int)(&l - layers.data());
+            std::lock_guard<std::mutex> lock(moe->mu);
+            if (moe_reserve(moe, cap_tokens)) return 1;
+            if (one && moe_dense_fuses_norm(moe, T)) {
+                const jq::ResidualNorm nm = update(l.norm2, xo, h);
+                if (moe_forward_dense(moe, T, h, nullptr, y, s, &nm)) return 1;
+                std::swap(xc, xo);
+            } else {
+                // the router reads the norm in f32, the experts of a many-token step in their own type
+                if (residual_norm(update(l.norm2, xc, h), type, h_e, sw, T, nullptr, s)) return 1;
+                if (moe_forward_dense(moe, T, h, h_e, y, s)) return 1;
+            }
+        }
+        pending = y, post = l.norm2b;
+    }
+    if (!n_want) return 0;
+    if (one) {
+        const jq::ResidualNorm nm = update(final_norm, xo, nullptr);
+        if (dense_gemv(head, nullptr, 0, 1, logits, vocab, s, &nm)) return 1;
+        for (int i = 1; i < n_want; i++)
+            HIP_TRY(hipMemcpyAsync(logits + (size_t)i * vocab, logits, vocab * sizeof(float), hipMemcpyDeviceToDevice, s));
+        return 0;
+    }
+    const bool few = n_want <= GEMV_MAX_ROWS;
+    if (residual_norm(update(final_norm, nullptr, few ? h : nullptr), type, few ? nullptr : h_e, sw, n_want, want_ids, s)) return 1;
+    return few ? dense_gemv(head, h, w, n_want, logits, vocab, s) : dense_gemm(head, h_e, sw, n_want, logits, vocab, s);
+}
+
+// ---- loading ------------------------------------------------------------------------------------------
+
+struct StackLoader {
+    LayeredModel *m;
+    const jq::SafeTensors &st;
+
+    const jq::SafeTensor *find(const std::string &name, std::initializer_list<uint64_t> shape) {
+        auto it = st.tensors.find(name);
+        if (it == st.tensors.end()) {
+            fail("%s: missing tensor `%s`", m->arch, name.c_str());
+            return nullptr;
+        }
+        if (it->second.shape != std::vector<uint64_t>(shape)) {
+            fail("%s: tensor `%s` does not have the shape the configuration implies", m->arch, name.c_str());
+            return nullptr;
+        }
+        return &it->second;
+    }
+    int host(const std::string &name, std::initializer_list<uint64_t> shape, std::vector<float> *out) {
+        const jq::SafeTensor *t = find(name, shape);
+        if (!t) return 1;
+        out->resize(t->elems);
+        if (!jq::safetensor_to_f32(*t, 0, t->elems, out->data())) return fail("%s: tensor `%s` holds no floats", m->arch, name.c_str());
+        return 0;
+    }
+    int to_device(const std::vector<float> &v, float **out) {
+        if (m->device_alloc(out, v.size())) return 1;
+        HIP_TRY(hipMemcpy(*out, v.data(), v.size() * sizeof(float), hipMemcpyHostToDevice));
+        return 0;
+    }
+    int vec(const std::string &name, std::initializer_list<uint64_t> shape, float **out) {
+        std::vector<float> v;
+        return host(name, shape, &v) || to_device(v, out);
+    }
+    int norm(const std::string &name, NormWeights *out) {
+        const uint64_t w = m->cfg.width;
+        return vec(name, {w}, &out->w) || (!m->cfg.rms && vec(name + ".b", {w}, &out->b));
+    }
+    // One matrix from the named parts' rows, one after the other, in the model's element type.
+    int matrix(const std::vector<std::pair<std::string, uint64_t>> &parts, uint64_t k, jq_weight **out) {
+        uint64_t n = 0;
+        for (const auto &p : parts) n += p.second;
+        std::vector<uint8_t> rows(n * k * m->esz());
+        uint8_t *at = rows.data();
+        std::vector<float> buf;
+        for (const auto &p : parts) {
+            const jq::SafeTensor *t = find(p.first, {p.second, k});
+            if (!t) return 1;
+            if (m->type == JQ_TYPE_BF16 && t->type == jq::SafeTensor::BF16) {
+                memcpy(at, t->data, t->elems * 2);
+            } else if (m->type == JQ_TYPE_F32) {
+                if (!jq::safetensor_to_f32(*t, 0, t->elems, (float *)at)) return fail("%s: tensor `%s` holds no floats", m->arch, p.first.c_str());
+            } else {
+                buf.resize(t->elems);
+                if (!jq::safetensor_to_f32(*t, 0, t->elems, buf.data())) return fail("%s: tensor `%s` holds no floats", m->arch, p.first.c_str());
+                for (uint64_t i = 0; i < t->elems; i++) {  // round to nearest even
+                    uint32_t u;
+                    memcpy(&u, &buf[i], 4);
+                    const uint16_t b = (u & 0x7FFFFFFFu) > 0x7F800000u ? (uint16_t)(u >> 16 | 64) : (uint16_t)((u + 0x7FFFu + (u >> 16 & 1)) >> 16);
+                    memcpy(at + 2 * i, &b, 2);
+                }
+            }
+            at += t->elems * m->esz();
+        }
+        if (jq_upload(m->type, rows.data(), rows.size(), n, k, 0, out)) return 1;
+        m->matrices.push_back(*out);
+        return 0;
+    }
+};
+
+int check_stack(const StackConfig &c) {
+    if (!c.vocab || !c.width) return fail("%s: zero in configuration", c.arch);
+    if (c.width > (uint32_t)NORM_MAX_WIDTH) return fail("%s: width %u exceeds %d", c.arch, c.width, NORM_MAX_WIDTH);
+    int v_mix = -1;
+    for (size_t i = 0; i < c.layers.size(); i++) {
+        const LayerConfig &l = c.layers[i];
+        if (l.mixer == LayerConfig::ATTENTION) {
+            if (l.heads <= 0 || l.kv_heads <= 0 || l.heads % l.kv_heads || l.dim <= 0 || l.vdim <= 0)
+                return fail("%s: layer %zu: %d query heads over %d kv heads of %d and %d", c.arch, i, l.heads, l.kv_heads, l.dim, l.vdim);
+            if (l.vdim > jq::ANY_MAX_DV) return fail("%s: layer %zu: value heads of %d exceed %d", c.arch, i, l.vdim, jq::ANY_MAX_DV);
+            if (l.rot.dims < 0 || l.rot.dims % 2 || l.rot.dims > l.dim) return fail("%s: layer %zu: %d of %d dimensions rotated", c.arch, i, l.rot.dims, l.dim);
+            if (l.v_mix) {
+                if (v_mix >= 0 && c.layers[v_mix].kv_heads * c.layers[v_mix].vdim != l.kv_heads * l.vdim)
+                    return fail("%s: layers %d and %zu mix values of different sizes", c.arch, v_mix, i);
+                if (v_mix < 0) v_mix = (int)i;
+            }
+        } else {
+            if (l.inner <= 0 || l.state <= 0 || l.dt_rank <= 0 || l.taps <= 0) return fail("%s: layer %zu: zero in the mixer", c.arch, i);
+            if (l.state > jq::SCAN_MAX_STATES) return fail("%s: layer %zu: %d states a channel exceed %d", c.arch, i, l.state, jq::SCAN_MAX_STATES);
+        }
+        if (l.mlp != LayerConfig::NONE && l.ff <= 0) return fail("%s: layer %zu: feed-forward of %d", c.arch, i, l.ff);
+        if (l.mlp == LayerConfig::MOE && (l.top <= 0 || l.top > l.experts)) return fail("%s: layer %zu: %d experts used of %d", c.arch, i, l.top, l.experts);
+    }
+    return 0;
+}
+
+// The caches, states and rotary tables of a loaded stack.
+int make_states(LayeredModel *m) {
+    for (Layer &l : m->layers) {
+        const LayerConfig &c = l.c;
+        if (c.mixer == LayerConfig::ATTENTION) {
+            const size_t rows = (size_t)c.kv_heads * m->n_ctx;
+            uint8_t *k = nullptr, *v = nullptr;
+            if (m->device_alloc(&k, rows * l.DP() * m->esz()) || m->device_alloc(&v, rows * l.DVP() * m->esz()))
+                return fail("%s: KV cache allocation failed", m->arch);
+            l.kc = k, l.vc = v;
+            if (c.rot.dims) {
+                for (size_t r = 0; r < m->rots.size(); r++)
+                    if (m->rots[r].c == c.rot) l.rot = (int)r;
+                if (l.rot < 0) {
+                    RotaryTable t;
+                    std::vector<double> freq;
+                    t.c = c.rot, t.mag = (float)rotary_frequencies(c.rot, &freq);
+                    if (m->device_alloc(&t.freq, freq.size())) return 1;
+                    HIP_TRY(hipMemcpy(t.freq, freq.data(), freq.size() * sizeof(double), hipMemcpyHostToDevice));
+                    l.rot = (int)m->rots.size();
+                    m->rots.push_back(t);
+                }
+            }
+        } else if (m->device_alloc(&l.S, (size_t)c.inner * c.state) || m->device_alloc(&l.tail[0], (size_t)(c.taps - 1) * c.inner) ||
+                   m->device_alloc(&l.tail[1], (size_t)(c.taps - 1) * c.inner)) {
+            return 1;
+        }
+    }
+    // layers with experts of the same sizes take turns with one set of scratch buffers
+    m->moe_holder.resize(m->layers.size());
+    for (size_t i = 0; i < m->layers.size(); i++) {
+        Layer &l = m->layers[i];
+        m->moe_holder[i] = (int)i;
+        if (!l.moe) continue;
+        l.moe_shares = (int)i;
+        for (size_t j = 0; j < i && l.moe_shares == (int)i; j++) {
+            const LayerConfig &o = m->layers[j].c;
+            if (m->layers[j].moe && o.experts == l.c.experts && o.top == l.c.top && o.ff == l.c.ff) l.moe_shares = (int)j;
+        }
+    }
+    return 0;
+}
+
+// ---- Bozosun --------------------------------------------------------------------------------------------
+// Layer norms with bias on both sides of every sublayer and a constant on the residual branches; attention with
+// interleaved rotary pairs, YaRN and values mixed with the first such layer's; selective-scan layers; clamped gated
+// units g sigmoid(1.702 g) (u + 1), dense or as experts under a softmax over the chosen logits.
+
+// Typed reads of a configuration object; the first failure is the one reported.
+struct ConfigReader {
+    const char *arch;
+    bool ok = true;
+    std::string where;
+
+    void bad(const char *key, const char *what) {
+        if (ok) fail("%s: config.json: %s%s%s %s", arch, where.c_str(), where.empty() ? "" : ".", key, what);
+        ok = false;
+    }
+    const jq::Json *object(const jq::Json *j, const char *key) {
+        const jq::Json *v = j ? j->find(key) : nullptr;
+        if (!v || v->kind != jq::Json::OBJECT) {
+            bad(key, "is not an object");
+            return nullptr;
+        }
+        return v;
+    }
+    double number(const jq::Json *j, const char *key) {
+        const jq::Json *v = j ? j->find(key) : nullptr;
+        if (!v || v->kind != jq::Json::NUMBER) {
+            bad(key, "is not a number");
+            return 0.0;
+        }
+        return v->num;
+    }
+    int integer(const jq::Json *j, const char *key) {
+        const double v = number(j, key);
+        if (v != std::floor(v) || v < 0 || v > 2147483647.0) {
+            bad(key, "is not a whole number");
+            return 0;
+        }
+        return (int)v;
+    }
+    bool flag(const jq::Json *j, const char *key) {  // absent or null: false
+        const jq::Json *v = j ? j->find(key) : nullptr;
+        if (!v || v->kind == jq::Json::NUL) return false;
+        if (v->kind != jq::Json::BOOL) bad(key, "is not a boolean");
+        return v->b;
+    }
+    const jq::Json *optional(const jq::Json *j, const char *key) {
+        const jq::Json *v = j ? j->find(key) : nullptr;
+        return v && v->kind != jq::Json::NUL ? v : nullptr;
+    }
+};
+
+int bozosun_config(const jq::Json &cfg, StackConfig *out) {
+    ConfigReader r{"Bozosun"};
+    StackConfig &s = *out;
+    s.arch = "Bozosun";
+    s.vocab = (uint32_t)r.integer(&cfg, "vocab"), s.width = (uint32_t)r.integer(&cfg, "width");
+    s.residual_mult = (float)r.number(&cfg, "residual_mult");
+    s.embedding_scale = (float)r.number(r.object(&cfg, "embedding"), "scale");
+    s.norm_eps = (float)r.number(r.object(&cfg, "norm"), "eps");
+    s.act_alpha = 1.702f, s.act_shift = 1.0f;
+    const jq::Json *layers = cfg.find("layers");
+    if (!layers || layers->kind != jq::Json::ARRAY) r.bad("layers", "is not a list");
+    for (size_t i = 0; r.ok && i < layers->items.size(); i++) {
+        const jq::Json *e = &layers->items[i];
+        r.where = "layers[" + std::to_string(i) + "]";
+        LayerConfig l;
+        const jq::Json *type = e->find("type"), *mx = r.object(e, "mixer");
+        if (!type || type->kind != jq::Json::STRING) {
+            r.bad("type", "is not a string");
+        } else if (type->str == "attention") {
+            l.mixer = LayerConfig::ATTENTION;
+            l.heads = r.integer(mx, "heads"), l.kv_heads = r.integer(mx, "kv_heads"), l.dim = r.integer(mx, "dim"), l.vdim = r.integer(mx, "vdim");
+            l.scale = (float)r.number(mx, "scale"), l.v_mix = r.flag(mx, "v_mix");
+            if (const jq::Json *rot = r.optional(mx, "rot")) {
+                l.rot.dims = r.integer(rot, "dims"), l.rot.base = r.number(rot, "base");
+                if (const jq::Json *sc = r.optional(rot, "scaling")) {
+                    l.rot.yarn = true, l.rot.factor = r.number(sc, "factor"), l.rot.original = r.number(sc, "original");
+                    l.rot.fast = r.number(sc, "fast"), l.rot.slow = r.number(sc, "slow");
+                }
+            }
+        } else if (type->str == "mamba1") {
+            l.mixer = LayerConfig::MAMBA1;
+            l.inner = r.integer(mx, "inner"), l.state = r.integer(mx, "state"), l.dt_rank = r.integer(mx, "dt_rank"), l.taps = r.integer(mx, "conv");
+        } else {
+            r.bad("type", "names no mixer of this design");
+        }
+        if (const jq::Json *mlp = r.optional(e, "mlp")) {
+            const jq::Json *kind = mlp->find("kind");
+            if (kind && kind->kind == jq::Json::STRING && kind->str == "dense") {
+                l.mlp = LayerConfig::DENSE;
+                l.ff = r.integer(mlp, "ff"), l.limit = (float)r.number(mlp, "limit");
+            } else if (kind && kind->kind == jq::Json::STRING && kind->str == "moe") {
+                l.mlp = LayerConfig::MOE;
+                const jq::Json *ex = r.object(mlp, "expert"), *ro = r.object(mlp, "router");
+                l.ff = r.integer(ex, "ff"), l.limit = (float)r.number(ex, "limit");
+                l.experts = r.integer(ro, "experts"), l.top = r.integer(ro, "top");
+            } else {
+                r.bad("mlp.kind", "names no feed-forward block of this design");
+            }
+        }
+        s.layers.push_back(l);
+    }
+    return r.ok ? check_stack(s) : 1;
+}
+
+int bozosun_tensors(StackLoader &ld) {
+    LayeredModel *m = ld.m;
+    const StackConfig &c = m->cfg;
+    const uint64_t w = c.width;
+    if (ld.matrix({{"embed", c.vocab}}, w, &m->embed) || ld.matrix({{"head", c.vocab}}, w, &m->head) || ld.norm("final.norm", &m->final_norm))
+        return 1;
+    bool seen_v_mix = false;
+    m->layers.resize(c.layers.size());
+    for (size_t i = 0; i < c.layers.size(); i++) {
+        Layer &l = m->layers[i];
+        l.c = c.layers[i];
+        const LayerConfig &lc = l.c;
+        const std::string p = "l" + std::to_string(i) + ".", mx = p + "mix.", ml = p + "mlp.";
+        if (ld.norm(p + "norm1", &l.norm1) || ld.norm(p + "norm1b", &l.norm1b)) return 1;
+        if (lc.mixer == LayerConfig::ATTENTION) {
+            const uint64_t nq = (uint64_t)lc.heads * lc.dim, nk = (uint64_t)lc.kv_heads * lc.dim, nv = (uint64_t)lc.kv_heads * lc.vdim;
+            if (ld.matrix({{mx + "q", nq}, {mx + "k", nk}, {mx + "v", nv}}, w, &l.in) || ld.matrix({{mx + "o", w}}, (uint64_t)lc.heads * lc.vdim, &l.o))
+                return 1;
+            if (lc.v_mix) {
+                l.v_first = !seen_v_mix, seen_v_mix = true;
+                auto t = ld.st.tensors.find(mx + "vmix");  // a scalar, or a vector of one
+                if (!l.v_first && (t == ld.st.tensors.end() || t->second.elems != 1 || !jq::safetensor_to_f32(t->second, 0, 1, &l.lambda)))
+                    return fail("%s: `%svmix` is missing or no single number", m->arch, mx.c_str());
+            }
+        } else {
+            const uint64_t C = lc.inner, N = lc.state, R = lc.dt_rank;
+            std::vector<float> a_log;
+            if (ld.matrix({{mx + "in", 2 * C}}, w, &l.in) || ld.matrix({{mx + "x", R + 2 * N}}, C, &l.wx) || ld.matrix({{mx + "dt", C}}, R, &l.wdt) ||
+                ld.matrix({{mx + "o", w}}, C, &l.o) || ld.vec(mx + "conv", {C, (uint64_t)lc.taps}, &l.conv) || ld.vec(mx + "conv.b", {C}, &l.conv_b) ||
+                ld.vec(mx + "dt.b", {C}, &l.dt_b) || ld.vec(mx + "D", {C}, &l.D) || ld.host(mx + "A_log", {C, N}, &a_log))
+                return 1;
+            for (float &v : a_log) v = (float)(-std::exp((double)v) * 1.4426950408889634);  // A log2(e)
+            if (ld.to_device(a_log, &l.A_log2)) return 1;
+        }
+        if (lc.mlp == LayerConfig::NONE) continue;
+        if (ld.norm(p + "norm2", &l.norm2) || ld.norm(p + "norm2b", &l.norm2b)) return 1;
+        const uint64_t ff = lc.ff;
+        if (lc.mlp == LayerConfig::DENSE) {
+            if (ld.matrix({{ml + "gate", ff}}, w, &l.gate) || ld.matrix({{ml + "up", ff}}, w, &l.up) || ld.matrix({{ml + "down", w}}, ff, &l.down)) return 1;
+            continue;
+        }
+        std::vector<std::pair<std::string, uint64_t>> g, u, d;
+        for (int e = 0; e < lc.experts; e++) {
+            const std::string ep = ml + "e" + std::to_string(e) + ".";
+            g.emplace_back(ep + "gate", ff), u.emplace_back(ep + "up", ff), d.emplace_back(ep + "down", w);
+        }
+        std::vector<float> router, bias;
+        if (ld.matrix(g, w, &l.gate) || ld.matrix(u, w, &l.up) || ld.matrix(d, ff, &l.down) ||
+            ld.host(ml + "router", {(uint64_t)lc.experts, w}, &router) || ld.host(ml + "router.b", {(uint64_t)lc.experts}, &bias))
+            return 1;
+        jq_moe_config mc{};
+        mc.n_expert = (uint32_t)lc.experts, mc.n_expert_used = (uint32_t)lc.top, mc.hidden = c.width, mc.inter = (uint32_t)ff;
+        mc.gating = 2, mc.norm_topk = 1, mc.swiglu_clamp = lc.limit, mc.act_alpha = c.act_alpha, mc.act_up_shift = c.act_shift;
+        if (jq_moe_create(&mc, router.data(), bias.data(), l.gate, l.up, l.down, nullptr, nullptr, nullptr, &l.moe)) return 1;
+    }
+    return 0;
+}
+
+constexpr uint32_t DEFAULT_CONTEXT = 4096;  // where neither the caller nor the configuration names one
+
+int load_bozosun(const char *path, const ModelLoadOptions &opt, jq_model **out) {
+    std::string err;
+    jq::Json cfg;
+    if (!jq::json_read_file(std::string(path) + "/config.json", &cfg, &err)) return fail("%s", err.c_str());
+    auto m = std::make_unique<LayeredModel>();
+    if (bozosun_config(cfg, &m->cfg)) return 1;
+    m->arch = m->cfg.arch, m->vocab = m->cfg.vocab, m->n_ctx = opt.n_ctx ? opt.n_ctx : DEFAULT_CONTEXT;
+    m->type = opt.compute == JQ_COMPUTE_F32 ? JQ_TYPE_F32 : JQ_TYPE_BF16;
+    auto st = jq::safetensors_open(std::string(path) + "/model.safetensors", &err);
+    if (!st) return fail("%s", err.c_str());
+    if (ensure_init()) return 1;
+    StackLoader ld{m.get(), *st};
+    if (bozosun_tensors(ld) || make_states(m.get()) || m->init_outputs()) return 1;
+    *out = m.release();
+    return 0;
+}
+
+const RegisterModelArch g_register_bozosun({"Bozosun", true, load_bozosun});
+
+}  // namespace
