@@ -98,7 +98,7 @@ def attention(h, w, m, cache, pos0, v_first):
     own = v
     if v_first is not None:
         lam = float(w["vmix"])
-        v = (1.0 - lam) * v + lam * v_first
+        v = (1.0 - lam) * v + lam * v_first.reshape(v.shape)
     cache["k"] = np.concatenate([cache.get("k", np.zeros((0, G, d))), k])
     cache["v"] = np.concatenate([cache.get("v", np.zeros((0, G, dv))), v])
     o = attend(q, cache["k"], cache["v"], pos0, m["scale"])
@@ -153,6 +153,12 @@ def route(h, router, bias, top):
     return ids, e / e.sum(axis=-1, keepdims=True)
 
 
+def route_margin(h, router, bias, top):
+    """Per token, how far the last chosen logit lies above the first one left out (inf where all are chosen)."""
+    z = np.sort(h @ router.T + bias, axis=-1)[:, ::-1]
+    return z[:, top - 1] - z[:, top] if top < z.shape[1] else np.full(len(z), np.inf)
+
+
 def moe_mlp(h, w, mlp):
     ids, wts = route(h, w["router"], w["router.b"], mlp["router"]["top"])
     y = np.zeros_like(h)
@@ -173,6 +179,7 @@ class LayeredOracle:
 
     def reset(self):
         self.n_past = 0
+        self.margin = np.zeros(0)   # per token, the smallest route_margin of its layers
         self.state = [{} for _ in self.cfg["layers"]]
 
     def part(self, prefix):
@@ -186,6 +193,7 @@ class LayeredOracle:
         mult, pos0 = self.cfg["residual_mult"], self.n_past
         x = self.w["embed"][np.asarray(tokens)] * self.cfg["embedding"]["scale"]
         v_first = None
+        margin = np.full(len(tokens), np.inf)
         for i, layer in enumerate(self.cfg["layers"]):
             p, m = f"l{i}.", layer["mixer"]
             h = self.norm(x, p + "norm1")
@@ -203,8 +211,11 @@ class LayeredOracle:
                 h = self.norm(x, p + "norm2")
                 w = self.part(p + "mlp.")
                 y = dense_mlp(h, w, mlp["limit"]) if mlp["kind"] == "dense" else moe_mlp(h, w, mlp)
+                if mlp["kind"] == "moe":
+                    margin = np.minimum(margin, route_margin(h, w["router"], w["router.b"], mlp["router"]["top"]))
                 x = x + mult * self.norm(y, p + "norm2b")
             if layers is not None:
                 layers.append(x.copy())
         self.n_past += len(tokens)
+        self.margin = np.concatenate([self.margin, margin])
         return self.norm(x, "final.norm") @ self.w["head"].T
