@@ -635,6 +635,99 @@ def plugin_moe_leg(prompt_len: int, n_decode: int, share_layers: bool, n_layer: 
     return res
 
 
+def _layered_sizes() -> dict:
+    """Layers of real models' sizes: name -> (Bozosun configuration, the qwen3 / qwen3moe configuration of the same sizes
+    that the library's tuned decoder runs, or None)."""
+    yarn = {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}
+
+    def attn(heads, kv, mlp):
+        return {"type": "attention", "mlp": mlp,
+                "mixer": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "v_mix": True,
+                          "rot": {"dims": 128, "base": 1e6, "scaling": yarn}}}
+
+    def model(width, layers):
+        return {"architecture": "Bozosun", "vocab": 32000, "width": width, "embedding": {"scale": 8.0}, "norm": {"eps": 1e-6},
+                "residual_mult": 0.5, "layers": layers}
+
+    dense = {"kind": "dense", "ff": 12288, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": 768, "limit": 7.0}, "router": {"experts": 128, "top": 8}}
+    scan = {"type": "mamba1", "mixer": {"inner": 8192, "state": 16, "dt_rank": 256, "conv": 4}}
+    base = dict(n_layer=4, vocab=32000, rms_eps=1e-6, rope_theta=1e6, head_dim=128)
+    return {
+        "attention_dense_4096": (model(4096, [attn(32, 8, dense)] * 4), dict(base, hidden=4096, n_head=32, n_kv_head=8, ffn=12288)),
+        "attention_moe_2048": (model(2048, [attn(32, 4, moe)] * 4), dict(base, hidden=2048, n_head=32, n_kv_head=4, ffn=0, n_expert=128,
+                                                                         n_expert_used=8, expert_ffn=768)),
+        "scan_dense_4096": (model(4096, [{**scan, "mlp": dense}] * 4), None),
+    }
+
+
+def _time_model(model, vocab: int, prompts, n_decode: int) -> dict:
+    """Median prefill of each prompt length and greedy decode behind the first, wall clock, logits left on the device."""
+    from joshua_amd import capi
+    from joshua_amd.synth import uniform_u32
+    out = {}
+    for n in prompts:
+        prompt = uniform_u32(31, n, vocab)
+        times = []
+        for _ in range(4):                       # the first one grows the buffers
+            model.reset()
+            capi.stream_synchronize()
+            t0 = time.perf_counter()
+            model.forward_only(prompt, 0)
+            tok = model.greedy()
+            times.append(time.perf_counter() - t0)
+        t = float(np.median(times[1:]))
+        out[f"prefill_{n}_tokens_per_s"], out[f"prefill_{n}_ms"] = round(n / t, 1), round(1e3 * t, 3)
+        if n == prompts[0]:
+            for i in range(8):
+                model.forward_only([tok], n + i)
+                tok = model.greedy()
+            t0 = time.perf_counter()
+            for i in range(n_decode):
+                model.forward_only([tok], n + 8 + i)
+                tok = model.greedy()
+            t = time.perf_counter() - t0
+            out["decode_tokens_per_s"], out["decode_us_per_token"] = round(n_decode / t, 1), round(1e6 * t / n_decode, 1)
+    return out
+
+
+def layered_leg(only: str = "", prompts=(512, 2048), n_decode: int = 96) -> dict:
+    """The layered decoder (plain bf16 weights) at real models' layer sizes, four layers each, beside the qwen3 / qwen3moe
+    decoder (Q4_K_M blocks) of the same sizes; random weights, layers repeating one layer's values."""
+    import tempfile
+
+    from joshua_amd import capi
+    from joshua_amd.synth import layered as sl
+    from joshua_amd.synth.model import qwen3_tensors
+
+    res = {}
+    n_ctx = max(prompts) + n_decode + 8
+    for name, (cfg, like) in _layered_sizes().items():
+        if only and only != name:
+            continue
+        with tempfile.TemporaryDirectory() as tmp:
+            tensors = sl.bozosun_tensors(cfg, 3, share=True)
+            layer_bytes = sum(v.nbytes for k, v in tensors.items() if k.startswith("l"))
+            head_bytes = tensors["head"].nbytes
+            model = capi.Model(sl.write_folder(tmp, cfg, tensors), n_ctx)
+            del tensors
+        r = {"layers": len(cfg["layers"]), "layer_weight_bytes": layer_bytes, "head_bytes": head_bytes,
+             "bozosun_bf16": _time_model(model, cfg["vocab"], prompts, n_decode)}
+        model.close()
+        if like:
+            c = capi.Qwen3Config(like["n_layer"], like["hidden"], like["n_head"], like["n_kv_head"], like["head_dim"], like["ffn"], like["vocab"],
+                                 n_ctx, like["rms_eps"], like["rope_theta"], like.get("n_expert", 0), like.get("n_expert_used", 0),
+                                 like.get("expert_ffn", 0), 1 if like.get("n_expert") else 0)
+            q = capi.Qwen3(c)
+            for tname, qt, d in qwen3_tensors(like, 7, "q4_k_m", share_layers=True):
+                q.set_tensor(tname, qt, d)
+            r["qwen3moe_q4_k_m" if like.get("n_expert") else "qwen3_q4_k_m"] = _time_model(q, like["vocab"], prompts, n_decode)
+            q.close()
+        res[name] = r
+        print(name, json.dumps(r), file=sys.stderr, flush=True)
+    return res
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -662,6 +755,9 @@ def main() -> int:
                          "it through the joshua_npu_* symbols; -1 (default): the whole model, every layer role's bytes drawn "
                          "once, as part of a full run (with the decode leg and all workloads) where 25 GB of temporary "
                          "space are free; 0: never")
+    ap.add_argument("--layered", nargs="?", const="all", default="",
+                    help="only this: the layered decoder with plain weights (Bozosun) at real models' layer sizes beside the qwen3 "
+                         "decoder of equal size; a name picks one of the sizes")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this build has no multi-GPU path (run with --gpus 1)", file=sys.stderr)
@@ -675,6 +771,9 @@ def main() -> int:
         return 2
     dev = torch.device("cuda:0")
     capi.init(0)
+    if args.layered:
+        print(json.dumps({"metric": "layered decoder prefill and decode", "layered": layered_leg("" if args.layered == "all" else args.layered)}))
+        return 0
     m = args.m
 
     blocks = synth.normal_quantized(capi.Q4_K, SEED_W, N * K, 0.02)

@@ -3,6 +3,8 @@
 
 namespace jqh {
 
+constexpr int NORM_GEMV_GRID = 1024;  // workgroups of a product with a fused norm: four a compute unit
+
 #define JQ_ELEM(TYPE, CALL)                                    \
     do {                                                       \
         if ((TYPE) == JQ_TYPE_BF16) {                          \
@@ -22,27 +24,46 @@ namespace jqh {
         else { constexpr int NV = 32; CALL; }                  \
     } while (0)
 
+namespace {
+
+// The one-row product with the norm in front: workgroups enough to fill the chip a few times, groups of rows shared out
+// evenly, one row a group where the matrix is short.
+template <bool GATED>
+int run_norm_gemv(const jq_weight *w, const jq_weight *up, float *Y, const jq::GatedUnit &unit, const jq::ResidualNorm &nm, hipStream_t s) {
+    const int k = (int)w->k, n = (int)w->n;
+    if (nm.width != k || k > FUSED_NORM_MAX_WIDTH || nm.x_out == nm.x) return fail("dense gemv: no fused norm for this row");
+    const uint8_t *wu = up ? up->dev : nullptr;
+    const size_t lds = (size_t)k * sizeof(float);
+    const bool few = n <= 512;
+    const int per = few ? 1 : GATED ? 2 : 4, groups = (n + per - 1) / per, rounds = (groups + NORM_GEMV_GRID - 1) / NORM_GEMV_GRID;
+    const dim3 grid((unsigned)((groups + rounds - 1) / rounds));
+#define JQ_NG(R)                                                                                                        \
+    JQ_ELEM(w->type, JQ_NORM_NV(k, hipLaunchKernelGGL((jq::norm_gemv<E, R, NV, GATED>), grid, dim3(256), lds, s, w->dev, wu, w->row_bytes, \
+                                                      Y, k, n, unit, nm)))
+    if (few && GATED) JQ_NG(2);
+    else if (few) JQ_NG(GATED ? 2 : 1);
+    else JQ_NG(4);
+#undef JQ_NG
+    note_kernel("norm_gemv");
+    HIP_TRY(hipGetLastError());
+    return 0;
+}
+
+}  // namespace
+
 int dense_gemv(const jq_weight *w, const float *X, size_t ldx, int T, float *Y, size_t ldy, hipStream_t s, const jq::ResidualNorm *nm) {
     const int k = (int)w->k, n = (int)w->n;
     const dim3 grid((unsigned)((n + 3) / 4));
-    if (T < 1 || T > GEMV_MAX_ROWS) return fail("dense gemv: %d rows", T);
-    if (nm) {
-        if (T != 1 || nm->width != k || k > FUSED_NORM_MAX_WIDTH || nm->x_out == nm->x) return fail("dense gemv: no fused norm for this row");
-        note_kernel("dense_gemv+norm");
-        JQ_ELEM(w->type, JQ_NORM_NV(k, hipLaunchKernelGGL((jq::dense_gemv<E, 1, NV>), grid, dim3(256), (size_t)k * sizeof(float), s,
-                                                          w->dev, w->row_bytes, nullptr, (size_t)0, Y, ldy, 1, k, n, *nm)));
-    } else {
-        const jq::ResidualNorm none{};
-        note_kernel("dense_gemv");
+    if (T < 1 || T > GEMV_MAX_ROWS || (nm && T != 1)) return fail("dense gemv: %d rows", T);
+    if (nm) return run_norm_gemv<false>(w, nullptr, Y, jq::GatedUnit{}, *nm, s);
+    note_kernel("dense_gemv");
 #define JQ_GEMV(MT)                                                                                                        \
-    JQ_ELEM(w->type, hipLaunchKernelGGL((jq::dense_gemv<E, MT, 0>), grid, dim3(256), 0, s, w->dev, w->row_bytes, X, ldx, Y, \
-                                        ldy, T, k, n, none))
-        if (T == 1) JQ_GEMV(1);
-        else if (T == 2) JQ_GEMV(2);
-        else if (T <= 4) JQ_GEMV(4);
-        else JQ_GEMV(8);
+    JQ_ELEM(w->type, hipLaunchKernelGGL((jq::dense_gemv<E, MT>), grid, dim3(256), 0, s, w->dev, w->row_bytes, X, ldx, Y, ldy, T, k, n))
+    if (T == 1) JQ_GEMV(1);
+    else if (T == 2) JQ_GEMV(2);
+    else if (T <= 4) JQ_GEMV(4);
+    else JQ_GEMV(8);
 #undef JQ_GEMV
-    }
     HIP_TRY(hipGetLastError());
     return 0;
 }
@@ -51,24 +72,17 @@ int dense_gemv_gated(const jq_weight *gate, const jq_weight *up, const float *X,
                      const jq::GatedUnit &unit, hipStream_t s, const jq::ResidualNorm *nm) {
     const int k = (int)gate->k, n = (int)gate->n;
     const dim3 grid((unsigned)((n + 1) / 2));
-    if (T < 1 || T > GEMV_MAX_ROWS) return fail("dense gemv: %d rows", T);
+    if (T < 1 || T > GEMV_MAX_ROWS || (nm && T != 1)) return fail("dense gemv: %d rows", T);
     if (gate->type != up->type || up->n != gate->n || up->k != gate->k) return fail("dense gemv: gate and up differ");
-    if (nm) {
-        if (T != 1 || nm->width != k || k > FUSED_NORM_MAX_WIDTH || nm->x_out == nm->x) return fail("dense gemv: no fused norm for this row");
-        JQ_ELEM(gate->type, JQ_NORM_NV(k, hipLaunchKernelGGL((jq::dense_gemv_gated<E, 1, NV>), grid, dim3(256), (size_t)k * sizeof(float), s,
-                                                             gate->dev, up->dev, gate->row_bytes, nullptr, (size_t)0, Y, ldy, 1, k, n,
-                                                             unit, *nm)));
-    } else {
-        const jq::ResidualNorm none{};
+    if (nm) return run_norm_gemv<true>(gate, up, Y, unit, *nm, s);
 #define JQ_GEMV(MT)                                                                                                              \
-    JQ_ELEM(gate->type, hipLaunchKernelGGL((jq::dense_gemv_gated<E, MT, 0>), grid, dim3(256), 0, s, gate->dev, up->dev, gate->row_bytes, \
-                                           X, ldx, Y, ldy, T, k, n, unit, none))
-        if (T == 1) JQ_GEMV(1);
-        else if (T == 2) JQ_GEMV(2);
-        else if (T <= 4) JQ_GEMV(4);
-        else JQ_GEMV(8);
+    JQ_ELEM(gate->type, hipLaunchKernelGGL((jq::dense_gemv_gated<E, MT>), grid, dim3(256), 0, s, gate->dev, up->dev, gate->row_bytes, X, \
+                                           ldx, Y, ldy, T, k, n, unit))
+    if (T == 1) JQ_GEMV(1);
+    else if (T == 2) JQ_GEMV(2);
+    else if (T <= 4) JQ_GEMV(4);
+    else JQ_GEMV(8);
 #undef JQ_GEMV
-    }
     HIP_TRY(hipGetLastError());
     return 0;
 }

@@ -148,13 +148,13 @@ __global__ __launch_bounds__(256) void attention_any(AttnLayer a, const typename
 }
 
 // Steps of up to 8 tokens, head sizes up to DC (64, 128 or 256): one workgroup per (chunk of ATT_CHUNK keys, KV head, run of
-// up to DEC_HEADS of its query heads, token).  The chunk's keys and values are read once for those heads; the step's own
+// `per` <= DEC_HEADS of its query heads, token): several heads a workgroup where there are workgroups enough.  The chunk's keys and values are read once for those heads; the step's own
 // tokens come from the raw projections, rotated and mixed here, and the workgroups of a token's last chunk store them
 // into the cache.  Partial results (maximum, sum, unnormalised output) go to attention_merge.
 constexpr int DEC_HEADS = 8, DEC_TOKENS = 8;
 
 template <class E, int DC>
-__global__ __launch_bounds__(256) void attention_decode(AttnLayer a, int n_chunks, float *__restrict__ part) {
+__global__ __launch_bounds__(256) void attention_decode(AttnLayer a, int n_chunks, int per, float *__restrict__ part) {
     using T = typename E::T;
     constexpr int CH = E::CH, KSTEPS = DC / (4 * CH), VIM = DC * E::BYTES / 64;
     __shared__ __attribute__((aligned(16))) float qs[DEC_HEADS][DC];
@@ -162,9 +162,12 @@ __global__ __launch_bounds__(256) void attention_decode(AttnLayer a, int n_chunk
     __shared__ __attribute__((aligned(16))) T sk[DEC_TOKENS][DC], sv[DEC_TOKENS][DC];
     __shared__ __attribute__((aligned(16))) float red[2][256 * CH];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int gq = a.H / a.G, runs = (gq + DEC_HEADS - 1) / DEC_HEADS, t = blockIdx.y;
-    const int chunk = (int)blockIdx.x % n_chunks, kvh = (int)blockIdx.x / n_chunks / runs, run = (int)blockIdx.x / n_chunks % runs;
-    const int h0 = kvh * gq + run * DEC_HEADS, nh = min(DEC_HEADS, gq - run * DEC_HEADS);
+    const int gq = a.H / a.G, runs = (gq + per - 1) / per, t = blockIdx.y;
+    // (ids 8 apart run on one XCD: the runs of a chunk's heads share its keys and values in that XCD's L2)
+    const int tri = 8 * ((int)(blockIdx.x >> 3) / runs) + (int)(blockIdx.x & 7), run = (int)(blockIdx.x >> 3) % runs;
+    if (tri >= n_chunks * a.G) return;
+    const int chunk = tri % n_chunks, kvh = tri / n_chunks;
+    const int h0 = kvh * gq + run * per, nh = min(per, gq - run * per);
     const int j0 = chunk * ATT_CHUNK, nj = min(ATT_CHUNK, a.pos0 + t + 1 - j0);
     const size_t pstride = (size_t)a.dv + 2;
     float *po = part + ((size_t)(t * a.H + h0) * n_chunks + chunk) * pstride;
@@ -308,10 +311,15 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
     static_assert(NK * 256 == KT * KCH && NVU * 256 == KT / 2 * KCH, "whole loads a thread");
     __shared__ __attribute__((aligned(16))) uint8_t ks[KT * KROW], vt[DC * VROW];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, n = lane & 15, g = lane >> 4;
-    const int gq = a.H / a.G, rows = a.T * gq, kvh = blockIdx.y;
-    const int tile = (int)gridDim.x - 1 - (int)blockIdx.x;  // the rows that see the most keys first
+    const int gq = a.H / a.G, rows = a.T * gq;
+    // the rows that see the most keys first, every other run of 256 workgroups in reverse: what a compute unit gets
+    // in two runs adds up evenly
+    int id = (int)(blockIdx.y * gridDim.x + blockIdx.x);
+    const int all = (int)(gridDim.x * gridDim.y), lo = id & ~255, hi = min(lo + 256, all);
+    if (id & 256) id = lo + hi - 1 - id;
+    const int kvh = id % a.G, tile = (int)gridDim.x - 1 - id / a.G;
     const int r0 = tile * 64 * QF;
-    const int last_key = a.pos0 + min(r0 + 64 * QF - 1, rows - 1) / gq;
+    const int last_key = a.pos0 + min(r0 + 64 * QF - 1, rows - 1) / gq, first_limit = a.pos0 + r0 / gq;
     const __bf16 *kb = (const __bf16 *)a.kc + (size_t)kvh * a.n_ctx * a.DP, *vb = (const __bf16 *)a.vc + (size_t)kvh * a.n_ctx * a.DVP;
 
     u32x4 qf[QF][DC / 32];
@@ -387,18 +395,23 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
 #pragma unroll
         for (int q = 0; q < QF; q++) {
             float tmax = -INFINITY;
+            if (k0 + KT - 1 > first_limit) {  // the tile reaches past some row's last key (all rows of a workgroup agree)
+#pragma unroll
+                for (int f = 0; f < NF; f++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++)
+                        if (k0 + 16 * f + 4 * g + r > limit[q]) st[q][f][r] = -INFINITY;
+            }
 #pragma unroll
             for (int f = 0; f < NF; f++)
 #pragma unroll
-                for (int r = 0; r < 4; r++) {
-                    const int key = k0 + 16 * f + 4 * g + r;
-                    st[q][f][r] = key <= limit[q] ? st[q][f][r] * scale_log2 : -INFINITY;
-                    tmax = fmaxf(tmax, st[q][f][r]);
-                }
-            tmax = max_xor32(max_xor16(tmax));
+                for (int r = 0; r < 4; r++) tmax = fmaxf(tmax, st[q][f][r]);
+            tmax = max_xor32(max_xor16(tmax)) * scale_log2;  // (scale_log2 > 0)
             const float mnew = fmaxf(mx[q], tmax);
             // (a row that has seen no key of the tiles so far keeps its state: -inf - -inf would be NaN)
-            const float base = mnew == -INFINITY ? 0.0f : mnew, rescale = exp2f(mx[q] - base);
+            const float base = mnew == -INFINITY ? 0.0f : mnew;
+            const bool moved = mnew > mx[q];
+            const float rescale = moved ? __builtin_amdgcn_exp2f(mx[q] - base) : 1.0f;
             mx[q] = mnew;
             float tsum = 0.0f;
 #pragma unroll
@@ -406,7 +419,7 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
                 bf16x4 hi, lo;
 #pragma unroll
                 for (int r = 0; r < 4; r++) {
-                    const float p = exp2f(st[q][f][r] - base);
+                    const float p = __builtin_amdgcn_exp2f(fmaf(st[q][f][r], scale_log2, -base));
                     tsum += p;
                     hi[r] = (__bf16)p;
                     lo[r] = (__bf16)(p - (float)hi[r]);
@@ -416,10 +429,12 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
                 pl[q][f / 2][2 * (f & 1)] = l2.x, pl[q][f / 2][2 * (f & 1) + 1] = l2.y;
             }
             sum[q] = fmaf(sum[q], rescale, tsum);  // this lane's keys; the four lanes of a row are added at the end
+            if (__ballot(moved)) {
 #pragma unroll
-            for (int d = 0; d < DT; d++)
+                for (int d = 0; d < DT; d++)
 #pragma unroll
-                for (int r = 0; r < 4; r++) o[q][d][r] *= rescale;
+                    for (int r = 0; r < 4; r++) o[q][d][r] *= rescale;
+            }
         }
 #pragma unroll
         for (int d = 0; d < DT; d++) {

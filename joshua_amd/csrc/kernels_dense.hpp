@@ -78,31 +78,14 @@ __device__ __forceinline__ void load_acts(const float *__restrict__ x, int c, in
     }
 }
 
-// acc[m][r] += x[m] . rows[r] (m past the rows of x: the last one again) over this thread's chunks (a workgroup of 256 shares the row).  With PRE > 0 the first
-// PRE passes' chunks are already in `pre`.
-template <class E, int MT, int R, int PRE>
-__device__ __forceinline__ void gemv_accumulate(const uint8_t *const (&rows)[R], const u32x4 (&pre)[PRE > 0 ? PRE : 1][R],
-                                                const float *__restrict__ x, size_t ldx, int rows_of_x, int k, float (&acc)[MT][R]) {
+// acc[m][r] += x[m] . rows[r] (m past the rows of x: the last one again) over this thread's chunks (a workgroup of 256
+// shares the row), from pass `p0` on.
+template <class E, int MT, int R>
+__device__ __forceinline__ void gemv_accumulate(const uint8_t *const (&rows)[R], const float *__restrict__ x, size_t ldx, int rows_of_x,
+                                                int k, float (&acc)[MT][R], int p0 = 0) {
     constexpr int STEP = 256 * E::CH;
-    int c = (int)threadIdx.x * E::CH;
-#pragma unroll
-    for (int p = 0; p < PRE; p++, c += STEP) {
-        if (c >= k) break;
-#pragma unroll
-        for (int m = 0; m < MT; m++) {
-            float xv[E::CH];
-            load_acts<E::CH>(x + (MT > 1 ? min(m, rows_of_x - 1) : 0) * ldx, c, k, xv);
-#pragma unroll
-            for (int r = 0; r < R; r++) {
-                float wv[E::CH];
-                E::widen(pre[p][r], wv);
-#pragma unroll
-                for (int i = 0; i < E::CH; i++) acc[m][r] = fmaf(wv[i], xv[i], acc[m][r]);
-            }
-        }
-    }
 #pragma unroll 2
-    for (; c < k; c += STEP) {
+    for (int c = (int)threadIdx.x * E::CH + p0 * STEP; c < k; c += STEP) {
         u32x4 w[R];
 #pragma unroll
         for (int r = 0; r < R; r++) w[r] = chunk_of<E>(rows[r], c);
@@ -135,34 +118,18 @@ __device__ __forceinline__ float gemv_reduce(const float (&acc)[N], float (&red)
     return v < N ? (red[0][v] + red[1][v]) + (red[2][v] + red[3][v]) : 0.0f;
 }
 
-// Y[m, n] = X[m, :] . W[n, :] for m < MT rows, four weight rows a workgroup.  NV > 0: X is the one row that the
-// residual update and norm of `nm` give (every workgroup makes it for itself, workgroup 0 stores it).
-template <class E, int MT, int NV>
+// Y[m, n] = X[m, :] . W[n, :] for m < MT rows, four weight rows a workgroup.
+template <class E, int MT>
 __global__ __launch_bounds__(256) void dense_gemv(const uint8_t *__restrict__ W, size_t pitch, const float *__restrict__ X,
-                                                  size_t ldx, float *__restrict__ Y, size_t ldy, int rows_of_x, int k, int n, ResidualNorm nm) {
-    constexpr int R = 4, PRE = NV > 0 ? 2 : 0;
-    static_assert(NV == 0 || MT == 1, "the fused norm makes one row");
-    extern __shared__ __attribute__((aligned(16))) float hrow[];  // NV > 0: the normed row
+                                                  size_t ldx, float *__restrict__ Y, size_t ldy, int rows_of_x, int k, int n) {
+    constexpr int R = 4;
     __shared__ float red[4][MT * R];
     const int r0 = R * (int)blockIdx.x;
     const uint8_t *rows[R];
 #pragma unroll
     for (int r = 0; r < R; r++) rows[r] = W + (size_t)min(r0 + r, n - 1) * pitch;
-    u32x4 pre[PRE > 0 ? PRE : 1][R];
-    if constexpr (NV > 0) {
-#pragma unroll
-        for (int p = 0; p < PRE; p++) {
-            const int c = ((int)threadIdx.x + 256 * p) * E::CH;
-            if (c < k) {
-#pragma unroll
-                for (int r = 0; r < R; r++) pre[p][r] = chunk_of<E>(rows[r], c);
-            }
-        }
-        residual_norm_row<NV>(nm, 0, hrow, blockIdx.x == 0);
-        __syncthreads();
-    }
     float acc[MT][R] = {};
-    gemv_accumulate<E, MT, R, PRE>(rows, pre, NV > 0 ? hrow : X, ldx, rows_of_x, k, acc);
+    gemv_accumulate<E, MT, R>(rows, X, ldx, rows_of_x, k, acc);
     float flat[MT * R];
 #pragma unroll
     for (int m = 0; m < MT; m++)
@@ -174,34 +141,18 @@ __global__ __launch_bounds__(256) void dense_gemv(const uint8_t *__restrict__ W,
 }
 
 // Y[m, j] = gated(X[m] . Wg[j], X[m] . Wu[j]), two j a workgroup.
-template <class E, int MT, int NV>
+template <class E, int MT>
 __global__ __launch_bounds__(256) void dense_gemv_gated(const uint8_t *__restrict__ Wg, const uint8_t *__restrict__ Wu,
                                                         size_t pitch, const float *__restrict__ X, size_t ldx,
-                                                        float *__restrict__ Y, size_t ldy, int rows_of_x, int k, int n,
-                                                        GatedUnit act, ResidualNorm nm) {
-    constexpr int R = 4, PRE = NV > 0 ? 2 : 0;
-    static_assert(NV == 0 || MT == 1, "the fused norm makes one row");
-    extern __shared__ __attribute__((aligned(16))) float hrow[];
+                                                        float *__restrict__ Y, size_t ldy, int rows_of_x, int k, int n, GatedUnit act) {
+    constexpr int R = 4;
     __shared__ float red[4][MT * R], sums[MT * R];
     const int j0 = 2 * (int)blockIdx.x;
     const uint8_t *rows[R];
 #pragma unroll
     for (int r = 0; r < R; r++) rows[r] = (r & 1 ? Wu : Wg) + (size_t)min(j0 + (r >> 1), n - 1) * pitch;
-    u32x4 pre[PRE > 0 ? PRE : 1][R];
-    if constexpr (NV > 0) {
-#pragma unroll
-        for (int p = 0; p < PRE; p++) {
-            const int c = ((int)threadIdx.x + 256 * p) * E::CH;
-            if (c < k) {
-#pragma unroll
-                for (int r = 0; r < R; r++) pre[p][r] = chunk_of<E>(rows[r], c);
-            }
-        }
-        residual_norm_row<NV>(nm, 0, hrow, blockIdx.x == 0);
-        __syncthreads();
-    }
     float acc[MT][R] = {};
-    gemv_accumulate<E, MT, R, PRE>(rows, pre, NV > 0 ? hrow : X, ldx, rows_of_x, k, acc);
+    gemv_accumulate<E, MT, R>(rows, X, ldx, rows_of_x, k, acc);
     float flat[MT * R];
 #pragma unroll
     for (int m = 0; m < MT; m++)
@@ -212,6 +163,71 @@ __global__ __launch_bounds__(256) void dense_gemv_gated(const uint8_t *__restric
     __syncthreads();
     const int m = (int)threadIdx.x / 2, j = (int)threadIdx.x % 2;
     if (m < min(MT, rows_of_x) && j0 + j < n) Y[m * ldy + j0 + j] = act(sums[m * R + 2 * j], sums[m * R + 2 * j + 1]);
+}
+
+// The one-row products with the residual update and norm of `nm` in front: y = W h, or with GATED
+// y = gated(Wg h, Wu h).  Every workgroup makes the normed row h for itself (workgroup 0 stores it), then walks groups of
+// R weight rows (gated: the gate and up rows of R / 2 columns), the next group's first chunks on their way while the
+// current one's sums come together.
+template <class E, int R, int NV, bool GATED>
+__global__ __launch_bounds__(256) void norm_gemv(const uint8_t *__restrict__ W, const uint8_t *__restrict__ Wu, size_t pitch,
+                                                 float *__restrict__ Y, int k, int n, GatedUnit act, ResidualNorm nm) {
+    constexpr int PRE = 2, PER = GATED ? R / 2 : R, STEP = 256 * E::CH;
+    extern __shared__ __attribute__((aligned(16))) float hrow[];  // [k]
+    __shared__ float red[2][4][R];
+    const int groups = (n + PER - 1) / PER, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const uint8_t *rows[R];
+    u32x4 pre[PRE][R];
+    auto ask = [&](int grp) __attribute__((always_inline)) {
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const int c = grp * PER + (GATED ? r >> 1 : r);
+            rows[r] = (GATED && (r & 1) ? Wu : W) + (size_t)min(c, n - 1) * pitch;
+        }
+#pragma unroll
+        for (int p = 0; p < PRE; p++) {
+            const int c = (int)threadIdx.x * E::CH + p * STEP;
+            if (c < k) {
+#pragma unroll
+                for (int r = 0; r < R; r++) pre[p][r] = chunk_of<E>(rows[r], c);
+            }
+        }
+    };
+    ask(blockIdx.x);
+    residual_norm_row<NV>(nm, 0, hrow, blockIdx.x == 0);
+    __syncthreads();
+    int buf = 0;
+    for (int grp = blockIdx.x; grp < groups; grp += gridDim.x, buf ^= 1) {
+        float acc[1][R] = {};
+#pragma unroll
+        for (int p = 0; p < PRE; p++) {
+            const int c = (int)threadIdx.x * E::CH + p * STEP;
+            if (c < k) {
+                float xv[E::CH];
+                load_acts<E::CH>(hrow, c, k, xv);
+#pragma unroll
+                for (int r = 0; r < R; r++) {
+                    float wv[E::CH];
+                    E::widen(pre[p][r], wv);
+#pragma unroll
+                    for (int i = 0; i < E::CH; i++) acc[0][r] = fmaf(wv[i], xv[i], acc[0][r]);
+                }
+            }
+        }
+        gemv_accumulate<E, 1, R>(rows, hrow, 0, 1, k, acc, PRE);
+        if (grp + (int)gridDim.x < groups) ask(grp + gridDim.x);
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const float s = wave_sum(acc[0][r]);
+            if (lane == 0) red[buf][wave][r] = s;
+        }
+        __syncthreads();  // (the other buffer's readers are past the previous one)
+        if (threadIdx.x < PER && grp * PER + (int)threadIdx.x < n) {
+            auto sum = [&](int r) { return (red[buf][0][r] + red[buf][1][r]) + (red[buf][2][r] + red[buf][3][r]); };
+            const int i = threadIdx.x;
+            Y[grp * PER + i] = GATED ? act(sum(2 * i), sum(2 * i + 1)) : sum(i);
+        }
+    }
 }
 
 // The experts' gated pairs of a decode-sized call: blockIdx.y is the (token, slot) pair, four j a workgroup, every
@@ -246,8 +262,7 @@ __global__ __launch_bounds__(256) void moe_dense_gate_up(const uint8_t *const *_
 #pragma unroll
     for (int r = 0; r < R; r++) rows[r] = (r & 1 ? Wu : Wg)[e] + (size_t)min(j0 + (r >> 1), n - 1) * pitch;
     float acc[1][R] = {};
-    const u32x4 none[1][R] = {};
-    gemv_accumulate<E, 1, R, 0>(rows, none, X + (size_t)t * ldx, 0, 1, k, acc);
+    gemv_accumulate<E, 1, R>(rows, X + (size_t)t * ldx, 0, 1, k, acc);
     const float s = gemv_reduce<R>(acc[0], red);
     if (threadIdx.x < R) sums[threadIdx.x] = s;
     __syncthreads();

@@ -607,6 +607,91 @@ static __global__ __launch_bounds__(GROUP_PAIRS_THREADS) void moe_group_pairs_ra
     }
 }
 
+// The same grouping for longer pair lists, in three launches over runs of GROUP_RUN pairs: a workgroup a run counts its
+// pairs per expert; one workgroup turns the counts into what lies in earlier runs and the totals into start positions;
+// a workgroup a run places its pairs (start + earlier runs + earlier waves of the run + rank within the wave).
+// counts: [runs][E].
+constexpr int GROUP_RUN = 512;
+
+static __global__ __launch_bounds__(GROUP_RUN) void moe_group_count(const uint32_t *__restrict__ ids, int P, int E, int *__restrict__ counts) {
+    extern __shared__ int cnt[];  // [E]
+    for (int e = threadIdx.x; e < E; e += GROUP_RUN) cnt[e] = 0;
+    __syncthreads();
+    const int pidx = (int)blockIdx.x * GROUP_RUN + (int)threadIdx.x;
+    if (pidx < P && ids[pidx] < (uint32_t)E) atomicAdd(&cnt[ids[pidx]], 1);
+    __syncthreads();
+    for (int e = threadIdx.x; e < E; e += GROUP_RUN) counts[(size_t)blockIdx.x * E + e] = cnt[e];
+}
+
+static __global__ __launch_bounds__(GROUP_PAIRS_THREADS) void moe_group_starts(int *__restrict__ counts, int runs, int P, int T, int E,
+                                                                               int *__restrict__ gexp, int *__restrict__ offsets,
+                                                                               int *__restrict__ xrow, int *__restrict__ yrow, int shared_group) {
+    extern __shared__ int start[];  // [E + 1]
+    for (int e = threadIdx.x; e < E; e += GROUP_PAIRS_THREADS) {
+        int sum = 0;
+        for (int r = 0; r < runs; r++) {
+            const int c = counts[(size_t)r * E + e];
+            counts[(size_t)r * E + e] = sum;
+            sum += c;
+        }
+        start[e] = sum;
+    }
+    __syncthreads();
+    if (threadIdx.x < 64) {  // totals -> start positions: each lane a run of experts, a wave scan between the runs
+        const int lane = threadIdx.x, per = (E + 63) / 64, b = lane * per;
+        int local = 0;
+        for (int i = 0; i < per; i++)
+            if (b + i < E) local += start[b + i];
+        int incl = local;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const int v = __shfl_up(incl, off, 64);
+            if (lane >= off) incl += v;
+        }
+        int at = incl - local;
+        for (int i = 0; i < per; i++) {
+            if (b + i < E) {
+                const int c = start[b + i];
+                start[b + i] = at;
+                at += c;
+            }
+        }
+        if (lane == 63) start[E] = incl;
+    }
+    __syncthreads();
+    for (int e = threadIdx.x; e <= E; e += GROUP_PAIRS_THREADS) {
+        offsets[e] = start[e];
+        if (e < E) gexp[e] = e;
+    }
+    if (shared_group) {  // group E: the shared expert over every token, output rows P .. P + T - 1
+        if (threadIdx.x == 0) gexp[E] = E, offsets[E + 1] = P + T;
+        for (int t = threadIdx.x; t < T; t += GROUP_PAIRS_THREADS) xrow[P + t] = t, yrow[P + t] = P + t;
+    }
+}
+
+static __global__ __launch_bounds__(GROUP_RUN) void moe_group_place(const uint32_t *__restrict__ ids, int P, int k_used, int E,
+                                                                    const int *__restrict__ counts, const int *__restrict__ offsets,
+                                                                    int *__restrict__ xrow, int *__restrict__ yrow) {
+    extern __shared__ int hist[];  // [waves][E]
+    constexpr int WAVES = GROUP_RUN / 64;
+    for (int i = threadIdx.x; i < WAVES * E; i += GROUP_RUN) hist[i] = 0;
+    __syncthreads();
+    const int pidx = (int)blockIdx.x * GROUP_RUN + (int)threadIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const uint32_t e = pidx < P ? ids[pidx] : 0xFFFFFFFFu;
+    int before = 0, after = 0;
+    for (int j = 0; j < 64; j++) {
+        const bool same = (uint32_t)__shfl((int)e, j, 64) == e;
+        before += same && j < lane;
+        after += same && j > lane;
+    }
+    if (e < (uint32_t)E && after == 0) hist[wave * E + (int)e] = before + 1;
+    __syncthreads();
+    if (e >= (uint32_t)E) return;
+    int at = offsets[e] + counts[(size_t)blockIdx.x * E + e] + before;
+    for (int w = 0; w < wave; w++) at += hist[w * E + (int)e];
+    xrow[at] = pidx / k_used;
+    yrow[at] = pidx;
+}
 
 // Expert matmuls over the grouped pairs: blockIdx.y = group (its expert is
 // gexp[group]), rows of the expert's weight over blockIdx.x.  The activation row of the pair at sorted

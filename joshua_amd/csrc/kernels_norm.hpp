@@ -18,10 +18,9 @@ struct ResidualNorm {
     float *h_out;                      // or null
 };
 
-// sum over the workgroup of 256, in every thread
+// sum over the workgroup of 256, in every thread; `red` is not used again before another barrier
 __device__ __forceinline__ float sum256(float v, float *red) {
     v = wave_sum(v);
-    __syncthreads();
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
     __syncthreads();
     return (red[0] + red[1]) + (red[2] + red[3]);
@@ -44,13 +43,13 @@ __device__ __forceinline__ void row_stats(const float (&v)[NV], int width, float
         ss = fmaf(d, d, ss);
     }
     *mean = mu;
-    *inv = 1.0f / sqrtf(sum256(ss, red) / (float)width + eps);
+    *inv = 1.0f / sqrtf(sum256(ss, red + 4) / (float)width + eps);
 }
 
 // Row `row` of the update; the normed row goes to `h` (LDS or global), and with `store` x and h to x_out and h_out.
 template <int NV>
 __device__ __forceinline__ void residual_norm_row(const ResidualNorm &a, size_t row, float *h, bool store) {
-    __shared__ float red[4];
+    __shared__ float red[16];  // a row of four for each of the sums
     const float *xr = a.x + row * a.width;
     float x[NV], mean, inv;
     const int c0 = threadIdx.x;
@@ -72,7 +71,7 @@ __device__ __forceinline__ void residual_norm_row(const ResidualNorm &a, size_t 
 #pragma unroll
         for (int i = 0; i < NV; i++) x[i] = fmaf(a.mult, y[i], x[i]);
     }
-    row_stats<NV>(x, a.width, a.eps, a.rms, red, &mean, &inv);
+    row_stats<NV>(x, a.width, a.eps, a.rms, red + 8, &mean, &inv);
 #pragma unroll
     for (int i = 0; i < NV; i++) {
         const int c = c0 + 256 * i;

@@ -8,28 +8,50 @@
 namespace jq {
 
 // out[t, c] = silu(b[c] + sum_j w[c, j] x[t - (taps - 1) + j, c]); inputs in front of the step come from tail_in,
-// the step's last taps - 1 go to tail_out (another buffer: a step may be shorter than the tail).
+// the step's last taps - 1 go to tail_out (another buffer: a step may be shorter than the tail).  A thread takes CONV_RUN
+// tokens of a channel; places T .. T + taps - 2 of the grid are the new tail's.
+constexpr int CONV_RUN = 8;
+
 template <class O>
 __global__ __launch_bounds__(256) void causal_conv_silu(const float *__restrict__ x, size_t ldx, const float *__restrict__ w,
                                                         const float *__restrict__ b, const float *__restrict__ tail_in,
                                                         float *__restrict__ tail_out, O *__restrict__ out, size_t ldo, int T, int C,
                                                         int taps) {
-    const size_t total = (size_t)(T + taps - 1) * C;
-    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
-        const int t = (int)(i / C), c = (int)(i % C);
-        if (t >= T) {
-            const int at = t - (taps - 1);  // place t - T of the new tail
-            tail_out[(size_t)(t - T) * C + c] = at >= 0 ? x[(size_t)at * ldx + c] : tail_in[(size_t)(at + taps - 1) * C + c];
-            continue;
+    const int c = (int)blockIdx.x * 256 + (int)threadIdx.x, t0 = (int)blockIdx.y * CONV_RUN;
+    if (c >= C) return;
+    auto input = [&](int at) { return at >= 0 ? x[(size_t)at * ldx + c] : tail_in[(size_t)(at + taps - 1) * C + c]; };
+    const int nt = min(CONV_RUN, T - t0);
+    if (nt > 0) {
+        float acc[CONV_RUN];
+        const float bias = b[c];
+#pragma unroll
+        for (int u = 0; u < CONV_RUN; u++) acc[u] = bias;
+        if (taps <= 4) {  // the inputs of the run once each
+            float v[CONV_RUN + 3], wt[4];
+#pragma unroll
+            for (int i = 0; i < CONV_RUN + 3; i++) {  // v[i] is the input at t0 - 3 + i
+                const int at = t0 - 3 + i;
+                v[i] = at < T && at >= -(taps - 1) ? input(at) : 0.0f;
+            }
+#pragma unroll
+            for (int j = 0; j < 4; j++) wt[j] = j >= 4 - taps ? w[(size_t)c * taps + j - (4 - taps)] : 0.0f;  // wt[3]: the current token's
+#pragma unroll
+            for (int u = 0; u < CONV_RUN; u++)
+#pragma unroll
+                for (int j = 0; j < 4; j++) acc[u] = fmaf(wt[j], v[u + j], acc[u]);
+        } else {
+            for (int j = 0; j < taps; j++) {
+                const float wj = w[(size_t)c * taps + j];
+#pragma unroll
+                for (int u = 0; u < CONV_RUN; u++)
+                    if (u < nt) acc[u] = fmaf(wj, input(t0 + u - (taps - 1) + j), acc[u]);
+            }
         }
-        float acc = b[c];
-        for (int j = 0; j < taps; j++) {
-            const int at = t - (taps - 1) + j;
-            const float v = at >= 0 ? x[(size_t)at * ldx + c] : tail_in[(size_t)(at + taps - 1) * C + c];
-            acc = fmaf(w[(size_t)c * taps + j], v, acc);
-        }
-        out[(size_t)t * ldo + c] = (O)silu(acc);
+#pragma unroll
+        for (int u = 0; u < CONV_RUN; u++)
+            if (u < nt) out[(size_t)(t0 + u) * ldo + c] = (O)silu(acc[u]);
     }
+    for (int t = max(t0, T); t < min(t0 + CONV_RUN, T + taps - 1); t++) tail_out[(size_t)(t - T) * C + c] = input(t - (taps - 1));
 }
 
 __device__ __forceinline__ float softplus(float v) { return v > 20.0f ? v : log1pf(expf(v)); }
@@ -81,25 +103,48 @@ __global__ __launch_bounds__(256) void selective_scan(SsmScan a, const IO *__res
         A[j] = in ? a.A_log2[(size_t)c * a.N + n] : 0.0f;
         S[j] = in ? a.S[(size_t)c * a.N + n] : 0.0f;
     }
-    for (int t0 = 0; t0 < a.T; t0 += SCAN_RUN) {
-        const int nt = min(SCAN_RUN, a.T - t0), padded = (nt + 3) & ~3;  // (tokens past the end: dt = 0 leaves the states alone)
-        for (int i = tid; i < padded * CPW; i += 256) {
-            const int t = i / CPW, k = i % CPW, cc = c0 + k;
-            float dt = 0.0f, xv = 0.0f, d = 0.0f;
-            if (cc < a.C && t < nt) {
-                dt = softplus(a.dt_raw[(size_t)(t0 + t) * a.C + cc] + a.dt_bias[cc]);
-                xv = (float)x[(size_t)(t0 + t) * a.ldx + cc], d = a.D[cc];
-            }
-            sd[t][k] = float2{dt, dt * xv};
-            sy[t][k] = d * xv;
+    // a run's inputs travel in registers while the run before is worked on (rows past the end: read from the last one)
+    constexpr int NI = (SCAN_RUN * CPW + 255) / 256, NB = (SCAN_RUN * NP + 255) / 256;
+    float rdt[NI], rz[NI], rb[NB], rc[NB], bias[NI], skip[NI], zs[NI];
+    IO rx[NI];
+#pragma unroll
+    for (int i = 0; i < NI; i++) {
+        const int cc = min(c0 + (tid + 256 * i) % CPW, a.C - 1);
+        bias[i] = a.dt_bias[cc], skip[i] = a.D[cc];
+    }
+    auto fetch = [&](int t0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < NI; i++) {
+            const int e = tid + 256 * i, t = min(t0 + e / CPW, a.T - 1), cc = min(c0 + e % CPW, a.C - 1);
+            rdt[i] = a.dt_raw[(size_t)t * a.C + cc], rx[i] = x[(size_t)t * a.ldx + cc], rz[i] = a.z[(size_t)t * a.ld_z + cc];
         }
-        for (int i = tid; i < padded * NP; i += 256) {
-            const int t = i / NP, n = i % NP;
-            const float *p = a.bc + (size_t)(t0 + t) * a.ld_bc;
-            sb[t][n] = n < a.N && t < nt ? p[n] : 0.0f;
-            scc[t][n] = n < a.N && t < nt ? p[a.N + n] : 0.0f;
+#pragma unroll
+        for (int i = 0; i < NB; i++) {
+            const int e = tid + 256 * i, t = min(t0 + e / NP, a.T - 1), n = min(e % NP, a.N - 1);
+            const float *p = a.bc + (size_t)t * a.ld_bc;
+            rb[i] = p[n], rc[i] = p[a.N + n];
+        }
+    };
+    fetch(0);
+    for (int t0 = 0; t0 < a.T; t0 += SCAN_RUN) {
+        const int nt = min(SCAN_RUN, a.T - t0);
+#pragma unroll
+        for (int i = 0; i < NI; i++) {
+            const int e = tid + 256 * i, t = e / CPW, k = e % CPW;
+            if (SCAN_RUN * CPW % 256 == 0 || e < SCAN_RUN * CPW) {
+                const float dt = t < nt ? softplus(rdt[i] + bias[i]) : 0.0f, xv = (float)rx[i];  // (dt = 0 leaves the states alone)
+                sd[t][k] = float2{dt, dt * xv};
+                sy[t][k] = skip[i] * xv;
+                zs[i] = rz[i];
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < NB; i++) {
+            const int e = tid + 256 * i, t = e / NP, n = e % NP;
+            if (SCAN_RUN * NP % 256 == 0 || e < SCAN_RUN * NP) sb[t][n] = n < a.N ? rb[i] : 0.0f, scc[t][n] = n < a.N ? rc[i] : 0.0f;
         }
         __syncthreads();
+        if (t0 + SCAN_RUN < a.T) fetch(t0 + SCAN_RUN);
         for (int t = 0; t < nt; t += 4) {
             float y[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -120,9 +165,10 @@ __global__ __launch_bounds__(256) void selective_scan(SsmScan a, const IO *__res
             }
         }
         __syncthreads();
-        for (int i = tid; i < nt * CPW; i += 256) {
-            const int t = i / CPW, k = i % CPW, cc = c0 + k;
-            if (cc < a.C) out[(size_t)(t0 + t) * a.ldo + cc] = (IO)(sy[t][k] * silu(a.z[(size_t)(t0 + t) * a.ld_z + cc]));
+#pragma unroll
+        for (int i = 0; i < NI; i++) {
+            const int e = tid + 256 * i, t = e / CPW, k = e % CPW;
+            if (t < nt && c0 + k < a.C) out[(size_t)(t0 + t) * a.ldo + c0 + k] = (IO)(sy[t][k] * silu(zs[i]));
         }
         __syncthreads();
     }

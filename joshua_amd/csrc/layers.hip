@@ -214,7 +214,7 @@ int LayeredModel::step(const uint32_t *tokens, uint32_t n, const uint32_t *want,
     if (broken) return fail("%s: an earlier step failed half way; reset the model", arch);
     if (reserve(n, std::max<uint32_t>(n_want, 1))) return 1;
     HIP_TRY(hipMemcpyAsync(ids, tokens, n * sizeof(uint32_t), hipMemcpyHostToDevice, s));
-    if (n_want) HIP_TRY(hipMemcpyAsync(want_ids, want, n_want * sizeof(uint32_t), hipMemcpyHostToDevice, s));
+    if (n_want && n > 1) HIP_TRY(hipMemcpyAsync(want_ids, want, n_want * sizeof(uint32_t), hipMemcpyHostToDevice, s));
     broken = true;
     if (run_layers((int)n, want, (int)n_want, s)) return 1;
     HIP_TRY(hipGetLastError());
@@ -240,9 +240,11 @@ int run_attention(LayeredModel *m, Layer &l, const jq::AttnLayer &a, bool small,
     const int dc = std::max(a.DP, a.DVP), gq = a.H / a.G, T = a.T;
     const size_t ldo = dense_stride((size_t)a.H * a.dv);
     if (small && dc <= 256) {
-        const int n_chunks = (a.pos0 + T + jq::ATT_CHUNK - 1) / jq::ATT_CHUNK, runs = (gq + jq::DEC_HEADS - 1) / jq::DEC_HEADS;
-        const dim3 grid((unsigned)(n_chunks * a.G * runs), (unsigned)T);
-#define JQ_DEC(DC) JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attention_decode<E, DC>), grid, dim3(256), 0, s, a, n_chunks, m->part))
+        const int n_chunks = (a.pos0 + T + jq::ATT_CHUNK - 1) / jq::ATT_CHUNK;
+        // a query head a workgroup until there are four for every compute unit, then more
+        const int per = std::min({gq, jq::DEC_HEADS, std::max(1, n_chunks * a.G * gq * T / 1024)}), runs = (gq + per - 1) / per;
+        const dim3 grid((unsigned)((n_chunks * a.G + 7) / 8 * 8 * runs), (unsigned)T);
+#define JQ_DEC(DC) JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attention_decode<E, DC>), grid, dim3(256), 0, s, a, n_chunks, per, m->part))
         if (dc <= 64) JQ_DEC(64);
         else if (dc <= 128) JQ_DEC(128);
         else JQ_DEC(256);
@@ -252,7 +254,7 @@ int run_attention(LayeredModel *m, Layer &l, const jq::AttnLayer &a, bool small,
         return 0;
     }
     JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attn_rope_store<E>), dim3((unsigned)T), dim3(256), 0, s, a, (typename E::T *)m->q_e));
-    if (type == JQ_TYPE_BF16 && dc <= 256 && !small) {
+    if (type == JQ_TYPE_BF16 && dc <= 256 && !small && a.scale > 0.0f) {
         const float sl = a.scale * 1.44269504088896341f;
         const size_t rows = (size_t)T * gq;
         // two sets of 16 rows a wave where that still makes a workgroup for every compute unit
@@ -344,7 +346,7 @@ int LayeredModel::run_layers(int T, const uint32_t *want, int n_want, hipStream_
             if (run_attention(this, l, a, small, mid, l.mix_e, s)) return 1;
         } else {
             const int C = c.inner, N = c.state, taps = c.taps;
-            const dim3 cgrid(grid_for((size_t)(T + taps - 1) * C));
+            const dim3 cgrid((unsigned)((C + 255) / 256), (unsigned)((T + taps - 1 + jq::CONV_RUN - 1) / jq::CONV_RUN));
             float *t_in = l.tail[l.tail_at], *t_out = l.tail[l.tail_at ^ 1];
             if (small)
                 hipLaunchKernelGGL((jq::causal_conv_silu<float>), cgrid, dim3(256), 0, s, proj, l.in->n, l.conv, l.conv_b, t_in, t_out,

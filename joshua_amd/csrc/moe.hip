@@ -13,10 +13,11 @@ static void moe_free_scratch(jq_moe *m) {
     for (void *p : {(void *)m->logits, (void *)m->wts, (void *)m->G, (void *)m->U, (void *)m->out, (void *)m->sG,
                     (void *)m->sU, (void *)m->sH, (void *)m->sOut, (void *)m->ids, (void *)m->gexp,
                     (void *)m->offsets, (void *)m->xrow, (void *)m->yrow, (void *)m->qacts, (void *)m->qi8.xl,
-                    (void *)m->qi8.xh, (void *)m->qi8.sx, (void *)m->qi8.sxs, (void *)m->gacts, (void *)m->gtab})
+                    (void *)m->qi8.xh, (void *)m->qi8.sx, (void *)m->qi8.sxs, (void *)m->gacts, (void *)m->gtab, (void *)m->group_counts})
         if (p) (void)hipFree(p);
     if (m->backend && m->backend->release) m->backend->release(m);
     m->qacts = nullptr;
+    m->group_counts = nullptr;
     m->gacts = nullptr, m->gtab = nullptr, m->gtab_rows = 0;
     m->qi8 = jq::ActsI8{nullptr, nullptr, nullptr, nullptr};
     m->logits = m->wts = m->G = m->U = m->out = m->sG = m->sU = m->sH = m->sOut = nullptr;
@@ -41,6 +42,7 @@ int moe_reserve(jq_moe *m, size_t T) {
     HIP_TRY(hipMalloc((void **)&m->offsets, (groups + 1) * sizeof(int)));
     HIP_TRY(hipMalloc((void **)&m->xrow, PR * sizeof(int)));
     HIP_TRY(hipMalloc((void **)&m->yrow, PR * sizeof(int)));
+    HIP_TRY(hipMalloc((void **)&m->group_counts, (P + jq::GROUP_RUN - 1) / jq::GROUP_RUN * c.n_expert * sizeof(int)));
     if (m->backend->reserve && m->backend->reserve(m, T)) return 1;
     if (m->sgate) {
         size_t si = m->sgate->n;
@@ -136,6 +138,14 @@ int moe_group_dev(jq_moe *m, size_t T, int extra, hipStream_t s) {
                            m->ids, (int)T, (int)c.n_expert_used, (int)c.n_expert, m->gexp, m->offsets, m->xrow, m->yrow,
                            extra);
     }
+    else if (!no_ranked && (size_t)c.n_expert * (jq::GROUP_RUN / 64) * sizeof(int) <= 65536) {
+        const int runs = (P + jq::GROUP_RUN - 1) / jq::GROUP_RUN, E = (int)c.n_expert;
+        hipLaunchKernelGGL(jq::moe_group_count, dim3((unsigned)runs), dim3(jq::GROUP_RUN), E * sizeof(int), s, m->ids, P, E, m->group_counts);
+        hipLaunchKernelGGL(jq::moe_group_starts, dim3(1), dim3(jq::GROUP_PAIRS_THREADS), (E + 1) * sizeof(int), s, m->group_counts, runs, P,
+                           (int)T, E, m->gexp, m->offsets, m->xrow, m->yrow, extra);
+        hipLaunchKernelGGL(jq::moe_group_place, dim3((unsigned)runs), dim3(jq::GROUP_RUN), E * (jq::GROUP_RUN / 64) * sizeof(int), s, m->ids,
+                           P, (int)c.n_expert_used, E, m->group_counts, m->offsets, m->xrow, m->yrow);
+    }
     else
         hipLaunchKernelGGL(jq::moe_group_pairs, dim3(1), dim3(jq::GROUP_PAIRS_THREADS), (c.n_expert + 1 + (in_lds ? P : 0)) * sizeof(int), s,
                            m->ids, (int)T, (int)c.n_expert_used, (int)c.n_expert, m->gexp, m->offsets, m->xrow, m->yrow,
@@ -165,7 +175,7 @@ void moe_swap_scratch(jq_moe *a, jq_moe *b) {
     std::swap(a->sOut, b->sOut), std::swap(a->ids, b->ids), std::swap(a->gexp, b->gexp);
     std::swap(a->offsets, b->offsets), std::swap(a->xrow, b->xrow), std::swap(a->yrow, b->yrow);
     std::swap(a->qacts, b->qacts), std::swap(a->gacts, b->gacts), std::swap(a->gtab, b->gtab);
-    std::swap(a->dense_x, b->dense_x), std::swap(a->dense_act, b->dense_act);
+    std::swap(a->dense_x, b->dense_x), std::swap(a->dense_act, b->dense_act), std::swap(a->group_counts, b->group_counts);
     std::swap(a->gtab_rows, b->gtab_rows), std::swap(a->gtile_rgs, b->gtile_rgs), std::swap(a->qi8, b->qi8);
 }
 

@@ -49,6 +49,7 @@ struct jq_moe {
     jq::ActsI8 qi8{nullptr, nullptr, nullptr, nullptr};  // activations as int8 planes (decode path, long rows)
     // plain-row experts: activations of the grouped GEMM, [rows][stride] in the experts' type
     uint8_t *dense_x = nullptr, *dense_act = nullptr;
+    int *group_counts = nullptr;  // grouping of long pair lists: pairs per (run, expert)
     const jqh::MoeBackend *backend = nullptr;
     std::mutex mu;
 };

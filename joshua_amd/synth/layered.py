@@ -3,6 +3,7 @@ from __future__ import annotations
 
 import json
 import os
+import re
 import struct
 
 import numpy as np
@@ -80,13 +81,18 @@ def bozosun_tensor(name: str, shape, seed: int) -> np.ndarray:
     return (n / np.sqrt(np.float32(shape[-1]))).astype(np.float32)
 
 
-def bozosun_tensors(cfg: dict, seed: int, override: "dict | None" = None) -> dict:
-    """name -> bf16 bit patterns of a whole model; `override` gives f32 values of some tensors instead."""
-    out = {}
+def bozosun_tensors(cfg: dict, seed: int, override: "dict | None" = None, share: bool = False) -> dict:
+    """name -> bf16 bit patterns of a whole model; `override` gives f32 values of some tensors instead.  `share`: layers
+    and experts repeat the values of the first tensor of their role and shape (for benchmarks: faster to make)."""
+    out, made = {}, {}
     for i, (name, shape) in enumerate(bozosun_shapes(cfg).items()):
+        key = (re.sub(r"^l\d+\.|e\d+\.", "", name), shape)
+        if share and key in made:
+            out[name] = made[key]
+            continue
         x = override[name] if override and name in override else bozosun_tensor(name, shape, seed * 100003 + i)
         assert tuple(np.shape(x)) == tuple(shape), (name, np.shape(x), shape)
-        out[name] = to_bf16(x).reshape(shape)
+        out[name] = made[key] = to_bf16(x).reshape(shape)
     return out
 
 
