@@ -3,8 +3,6 @@
 
 namespace jqh {
 
-constexpr int NORM_GEMV_GRID = 1024;  // workgroups of a product with a fused norm: four a compute unit
-
 #define JQ_ELEM(TYPE, CALL)                                    \
     do {                                                       \
         if ((TYPE) == JQ_TYPE_BF16) {                          \
@@ -16,33 +14,21 @@ constexpr int NORM_GEMV_GRID = 1024;  // workgroups of a product with a fused no
         }                                                      \
     } while (0)
 
-// NV of the row norm for a width: elements a thread.
-#define JQ_NORM_NV(WIDTH, CALL)                                \
-    do {                                                       \
-        if ((WIDTH) <= 1024) { constexpr int NV = 4; CALL; }   \
-        else if ((WIDTH) <= 4096) { constexpr int NV = 16; CALL; } \
-        else { constexpr int NV = 32; CALL; }                  \
-    } while (0)
-
 namespace {
 
-// The one-row product with the norm in front: workgroups enough to fill the chip a few times, groups of rows shared out
-// evenly, one row a group where the matrix is short.
+// The one-row product with the norm in front: a workgroup a compute unit, or a pair of rows a workgroup where there are
+// fewer pairs.
 template <bool GATED>
 int run_norm_gemv(const jq_weight *w, const jq_weight *up, float *Y, const jq::GatedUnit &unit, const jq::ResidualNorm &nm, hipStream_t s) {
     const int k = (int)w->k, n = (int)w->n;
     if (nm.width != k || k > FUSED_NORM_MAX_WIDTH || nm.x_out == nm.x) return fail("dense gemv: no fused norm for this row");
     const uint8_t *wu = up ? up->dev : nullptr;
-    const size_t lds = (size_t)k * sizeof(float);
-    const bool few = n <= 512;
-    const int per = few ? 1 : GATED ? 2 : 4, groups = (n + per - 1) / per, rounds = (groups + NORM_GEMV_GRID - 1) / NORM_GEMV_GRID;
-    const dim3 grid((unsigned)((groups + rounds - 1) / rounds));
-#define JQ_NG(R)                                                                                                        \
-    JQ_ELEM(w->type, JQ_NORM_NV(k, hipLaunchKernelGGL((jq::norm_gemv<E, R, NV, GATED>), grid, dim3(256), lds, s, w->dev, wu, w->row_bytes, \
-                                                      Y, k, n, unit, nm)))
-    if (few && GATED) JQ_NG(2);
-    else if (few) JQ_NG(GATED ? 2 : 1);
-    else JQ_NG(4);
+    const dim3 grid((unsigned)std::min(GATED ? n : (n + 1) / 2, 256)), block(64 * jq::NORM_GEMV_WAVES);
+#define JQ_NG(NV)                                                                                                                   \
+    JQ_ELEM(w->type, hipLaunchKernelGGL((jq::norm_gemv<E, NV, GATED>), grid, block, (size_t)k * sizeof(float), s, w->dev, wu, w->row_bytes, Y, \
+                                        k, n, unit, nm))
+    if (k <= 4096) JQ_NG(4);
+    else JQ_NG(8);
 #undef JQ_NG
     note_kernel("norm_gemv");
     HIP_TRY(hipGetLastError());
@@ -226,13 +212,14 @@ int residual_norm(const jq::ResidualNorm &a, uint32_t type, void *he, size_t str
     if (a.width > NORM_MAX_WIDTH) return fail("residual norm: rows of %d exceed %d", a.width, NORM_MAX_WIDTH);
     if (!rows) return 0;
     const size_t lds = he ? (size_t)a.width * sizeof(float) : 0;
-#define JQ_ROWS(NV)                                                                                                          \
-    JQ_ELEM(type, hipLaunchKernelGGL((jq::residual_norm_rows<E, NV>), dim3((unsigned)rows), dim3(256), lds, s, a, (typename E::T *)he, \
+#define JQ_ROWS(NV, BT)                                                                                                          \
+    JQ_ELEM(type, hipLaunchKernelGGL((jq::residual_norm_rows<E, NV, BT>), dim3((unsigned)rows), dim3(BT), lds, s, a, (typename E::T *)he, \
                                      stride, at))
-    if (a.width <= 1024) JQ_ROWS(4);
-    else if (a.width <= 4096) JQ_ROWS(16);
-    else if (a.width <= 8192) JQ_ROWS(32);
-    else JQ_ROWS(64);
+    if (a.width <= 1024) JQ_ROWS(4, 256);
+    else if (a.width <= 2048) JQ_ROWS(4, 512);
+    else if (a.width <= 4096) JQ_ROWS(4, 1024);
+    else if (a.width <= 8192) JQ_ROWS(8, 1024);
+    else JQ_ROWS(16, 1024);
 #undef JQ_ROWS
     HIP_TRY(hipGetLastError());
     return 0;

@@ -340,13 +340,14 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
 #pragma unroll
         for (int d = 0; d < DT; d++) o[q][d] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
+    // (keys past the last one and columns past the cache's are read from within it: the former are masked, the latter
+    // meet zeros of the query or are never stored)
     u32x4 kpre[NK], vpre[NVU][2];
     auto fetch = [&](int k0) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < NK; i++) {
             const int id = tid + 256 * i, row = id / KCH, c = id % KCH, key = k0 + row;
-            kpre[i] = u32x4{0, 0, 0, 0};
-            if (key <= last_key && 8 * c < a.DP) kpre[i] = *(const u32x4 *)(kb + (size_t)key * a.DP + 8 * c);
+            kpre[i] = *(const u32x4 *)(kb + (size_t)min(key, last_key) * a.DP + (8 * c < a.DP ? 8 * c : 0));
         }
 #pragma unroll
         for (int i = 0; i < NVU; i++) {
@@ -354,8 +355,7 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
 #pragma unroll
             for (int b = 0; b < 2; b++) {
                 const int key = k0 + 2 * pair + b;
-                vpre[i][b] = u32x4{0, 0, 0, 0};
-                if (key <= last_key && 8 * c < a.DVP) vpre[i][b] = *(const u32x4 *)(vb + (size_t)key * a.DVP + 8 * c);
+                vpre[i][b] = *(const u32x4 *)(vb + (size_t)min(key, last_key) * a.DVP + (8 * c < a.DVP ? 8 * c : 0));
             }
         }
     };
@@ -385,7 +385,6 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
             for (int q = 0; q < QF; q++) st[q][f] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int k = 0; k < DC / 32; k++) {
-                if (32 * k >= a.DP) break;
                 const u32x4 kf = *(const u32x4 *)(ks + (16 * f + n) * KROW + 16 * ((4 * k + g) ^ (n & 7)));
 #pragma unroll
                 for (int q = 0; q < QF; q++) st[q][f] = ElemBf16::mma(kf, qf[q][k], st[q][f]);
@@ -416,14 +415,11 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
             float tsum = 0.0f;
 #pragma unroll
             for (int f = 0; f < NF; f++) {
-                bf16x4 hi, lo;
+                f32x4 p;
 #pragma unroll
-                for (int r = 0; r < 4; r++) {
-                    const float p = __builtin_amdgcn_exp2f(fmaf(st[q][f][r], scale_log2, -base));
-                    tsum += p;
-                    hi[r] = (__bf16)p;
-                    lo[r] = (__bf16)(p - (float)hi[r]);
-                }
+                for (int r = 0; r < 4; r++) p[r] = __builtin_amdgcn_exp2f(fmaf(st[q][f][r], scale_log2, -base));
+                tsum += (p[0] + p[1]) + (p[2] + p[3]);
+                const bf16x4 hi = __builtin_convertvector(p, bf16x4), lo = __builtin_convertvector(p - __builtin_convertvector(hi, f32x4), bf16x4);
                 const uint2 h2 = __builtin_bit_cast(uint2, hi), l2 = __builtin_bit_cast(uint2, lo);
                 ph[q][f / 2][2 * (f & 1)] = h2.x, ph[q][f / 2][2 * (f & 1) + 1] = h2.y;
                 pl[q][f / 2][2 * (f & 1)] = l2.x, pl[q][f / 2][2 * (f & 1) + 1] = l2.y;
@@ -438,7 +434,6 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
         }
 #pragma unroll
         for (int d = 0; d < DT; d++) {
-            if (16 * d >= a.DVP) break;
 #pragma unroll
             for (int s = 0; s < NF / 2; s++) {
                 const u32x4 vf = *(const u32x4 *)(vt + (16 * d + n) * VROW + 64 * s + 16 * g);

@@ -166,66 +166,66 @@ __global__ __launch_bounds__(256) void dense_gemv_gated(const uint8_t *__restric
 }
 
 // The one-row products with the residual update and norm of `nm` in front: y = W h, or with GATED
-// y = gated(Wg h, Wu h).  Every workgroup makes the normed row h for itself (workgroup 0 stores it), then walks groups of
-// R weight rows (gated: the gate and up rows of R / 2 columns), the next group's first chunks on their way while the
-// current one's sums come together.
-template <class E, int R, int NV, bool GATED>
-__global__ __launch_bounds__(256) void norm_gemv(const uint8_t *__restrict__ W, const uint8_t *__restrict__ Wu, size_t pitch,
-                                                 float *__restrict__ Y, int k, int n, GatedUnit act, ResidualNorm nm) {
-    constexpr int PRE = 2, PER = GATED ? R / 2 : R, STEP = 256 * E::CH;
+// y = gated(Wg h, Wu h).  A workgroup of 16 waves makes the normed row h for itself (workgroup 0 stores it; few, large
+// workgroups, since each reads the norm's vectors whole); then every wave takes pairs of weight rows (gated: the gate and the
+// up row of a column) on its own, the first chunks of its first pair on their way since before the norm.
+constexpr int NORM_GEMV_WAVES = 16;
+
+template <class E, int NV, bool GATED>
+__global__ __launch_bounds__(64 * NORM_GEMV_WAVES) void norm_gemv(const uint8_t *__restrict__ W, const uint8_t *__restrict__ Wu, size_t pitch,
+                                                                  float *__restrict__ Y, int k, int n, GatedUnit act, ResidualNorm nm) {
+    constexpr int R = 2, PER = GATED ? 1 : 2, STEP = 64 * E::CH, PRE = 4;
     extern __shared__ __attribute__((aligned(16))) float hrow[];  // [k]
-    __shared__ float red[2][4][R];
-    const int groups = (n + PER - 1) / PER, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int groups = (n + PER - 1) / PER, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const uint8_t *rows[R];
     u32x4 pre[PRE][R];
     auto ask = [&](int grp) __attribute__((always_inline)) {
 #pragma unroll
-        for (int r = 0; r < R; r++) {
-            const int c = grp * PER + (GATED ? r >> 1 : r);
-            rows[r] = (GATED && (r & 1) ? Wu : W) + (size_t)min(c, n - 1) * pitch;
-        }
+        for (int r = 0; r < R; r++) rows[r] = (GATED && r ? Wu : W) + (size_t)min(GATED ? grp : 2 * grp + r, n - 1) * pitch;
 #pragma unroll
-        for (int p = 0; p < PRE; p++) {
-            const int c = (int)threadIdx.x * E::CH + p * STEP;
-            if (c < k) {
+        for (int p = 0; p < PRE; p++) {  // (past the row: its last chunk, multiplied by nothing)
+            const int c = min(lane * E::CH + p * STEP, (k - 1) / E::CH * E::CH);
 #pragma unroll
-                for (int r = 0; r < R; r++) pre[p][r] = chunk_of<E>(rows[r], c);
-            }
+            for (int r = 0; r < R; r++) pre[p][r] = chunk_of<E>(rows[r], c);
         }
     };
-    ask(blockIdx.x);
-    residual_norm_row<NV>(nm, 0, hrow, blockIdx.x == 0);
-    __syncthreads();
-    int buf = 0;
-    for (int grp = blockIdx.x; grp < groups; grp += gridDim.x, buf ^= 1) {
-        float acc[1][R] = {};
-#pragma unroll
-        for (int p = 0; p < PRE; p++) {
-            const int c = (int)threadIdx.x * E::CH + p * STEP;
-            if (c < k) {
-                float xv[E::CH];
-                load_acts<E::CH>(hrow, c, k, xv);
-#pragma unroll
-                for (int r = 0; r < R; r++) {
-                    float wv[E::CH];
-                    E::widen(pre[p][r], wv);
-#pragma unroll
-                    for (int i = 0; i < E::CH; i++) acc[0][r] = fmaf(wv[i], xv[i], acc[0][r]);
-                }
-            }
-        }
-        gemv_accumulate<E, 1, R>(rows, hrow, 0, 1, k, acc, PRE);
-        if (grp + (int)gridDim.x < groups) ask(grp + gridDim.x);
+    auto multiply = [&](const u32x4 (&w)[R], int c, float (&acc)[R]) __attribute__((always_inline)) {
+        float xv[E::CH];
+        load_acts<E::CH>(hrow, c, k, xv);
 #pragma unroll
         for (int r = 0; r < R; r++) {
-            const float s = wave_sum(acc[0][r]);
-            if (lane == 0) red[buf][wave][r] = s;
+            float wv[E::CH];
+            E::widen(w[r], wv);
+#pragma unroll
+            for (int i = 0; i < E::CH; i++) acc[r] = fmaf(wv[i], xv[i], acc[r]);
         }
-        __syncthreads();  // (the other buffer's readers are past the previous one)
-        if (threadIdx.x < PER && grp * PER + (int)threadIdx.x < n) {
-            auto sum = [&](int r) { return (red[buf][0][r] + red[buf][1][r]) + (red[buf][2][r] + red[buf][3][r]); };
-            const int i = threadIdx.x;
-            Y[grp * PER + i] = GATED ? act(sum(2 * i), sum(2 * i + 1)) : sum(i);
+    };
+    int grp = (int)blockIdx.x + (int)gridDim.x * wave;
+    ask(min(grp, groups - 1));
+    residual_norm_row<NV, 64 * NORM_GEMV_WAVES>(nm, 0, hrow, blockIdx.x == 0);
+    __syncthreads();
+    for (; grp < groups; grp += (int)gridDim.x * NORM_GEMV_WAVES) {
+        float acc[R] = {};
+#pragma unroll
+        for (int p = 0; p < PRE; p++) {
+            const int c = lane * E::CH + p * STEP;
+            if (c < k) multiply(pre[p], c, acc);
+        }
+#pragma unroll 4
+        for (int c = lane * E::CH + PRE * STEP; c < k; c += STEP) {
+            u32x4 w[R];
+#pragma unroll
+            for (int r = 0; r < R; r++) w[r] = chunk_of<E>(rows[r], c);
+            multiply(w, c, acc);
+        }
+        const int next = grp + (int)gridDim.x * NORM_GEMV_WAVES;
+        if (next < groups) ask(next);
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[r] = wave_sum(acc[r]);
+        if (GATED) {
+            if (lane == 0) Y[grp] = act(acc[0], acc[1]);
+        } else if (lane < R && 2 * grp + lane < n) {
+            Y[2 * grp + lane] = lane ? acc[1] : acc[0];
         }
     }
 }

@@ -1,5 +1,5 @@
 // The residual stream of decoders that normalise in front of and behind a sublayer: x + mult * norm(y), then the norm
-// of the result for the next sublayer, f32 throughout, one workgroup of 256 a row.
+// of the result for the next sublayer, f32 throughout, one workgroup of BT threads a row.
 #pragma once
 #include "kernels_graph.hpp"
 
@@ -18,91 +18,124 @@ struct ResidualNorm {
     float *h_out;                      // or null
 };
 
-// sum over the workgroup of 256, in every thread; `red` is not used again before another barrier
-__device__ __forceinline__ float sum256(float v, float *red) {
+// sum over the workgroup of BT, in every thread; `red` [BT / 64] is not used again before another barrier
+template <int BT>
+__device__ __forceinline__ float sum_block(float v, float *red) {
     v = wave_sum(v);
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
     __syncthreads();
-    return (red[0] + red[1]) + (red[2] + red[3]);
+    float s = 0.0f;
+#pragma unroll
+    for (int i = 0; i < BT / 64; i++) s += red[i];
+    return s;
 }
 
-// One norm over the row held as v[i] at column threadIdx.x + 256 i (0 past the width): mean and 1 / deviation.
-template <int NV>
+// Element i of a thread's share of a row: four columns side by side, every 4 BT.
+template <int BT>
+__device__ __forceinline__ int norm_col(int i) { return 4 * (int)threadIdx.x + 4 * BT * (i / 4) + i % 4; }
+
+// The thread's share of a row; columns past the width are zero.  Every load is issued whatever the width (past it, from
+// the row's end), so that the loads of a row's vectors travel together.
+template <int NV, int BT>
+__device__ __forceinline__ void load_row(const float *__restrict__ p, int width, float (&v)[NV]) {
+    if ((width & 3) == 0) {
+#pragma unroll
+        for (int i = 0; i < NV; i += 4) {
+            const float4 q = *(const float4 *)(p + min(norm_col<BT>(i), width - 4));
+            v[i] = q.x, v[i + 1] = q.y, v[i + 2] = q.z, v[i + 3] = q.w;
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < NV; i++) v[i] = p[min(norm_col<BT>(i), width - 1)];
+    }
+#pragma unroll
+    for (int i = 0; i < NV; i++) v[i] = norm_col<BT>(i) < width ? v[i] : 0.0f;
+}
+
+template <int NV, int BT>
+__device__ __forceinline__ void store_row(float *__restrict__ p, int width, const float (&v)[NV]) {
+    if ((width & 3) == 0) {
+#pragma unroll
+        for (int i = 0; i < NV; i += 4)
+            if (norm_col<BT>(i) < width) *(float4 *)(p + norm_col<BT>(i)) = float4{v[i], v[i + 1], v[i + 2], v[i + 3]};
+    } else {
+#pragma unroll
+        for (int i = 0; i < NV; i++)
+            if (norm_col<BT>(i) < width) p[norm_col<BT>(i)] = v[i];
+    }
+}
+
+// One norm over the row held as v (0 past the width): mean and 1 / deviation.
+template <int NV, int BT>
 __device__ __forceinline__ void row_stats(const float (&v)[NV], int width, float eps, int rms, float *red, float *mean, float *inv) {
     float mu = 0.0f;
     if (!rms) {
         float s = 0.0f;
 #pragma unroll
         for (int i = 0; i < NV; i++) s += v[i];
-        mu = sum256(s, red) / (float)width;
+        mu = sum_block<BT>(s, red) / (float)width;
     }
     float ss = 0.0f;
 #pragma unroll
     for (int i = 0; i < NV; i++) {
-        const float d = (int)threadIdx.x + 256 * i < width ? v[i] - mu : 0.0f;
+        const float d = norm_col<BT>(i) < width ? v[i] - mu : 0.0f;
         ss = fmaf(d, d, ss);
     }
     *mean = mu;
-    *inv = 1.0f / sqrtf(sum256(ss, red + 4) / (float)width + eps);
+    *inv = 1.0f / sqrtf(sum_block<BT>(ss, red + BT / 64) / (float)width + eps);
 }
 
 // Row `row` of the update; the normed row goes to `h` (LDS or global), and with `store` x and h to x_out and h_out.
-template <int NV>
+template <int NV, int BT>
 __device__ __forceinline__ void residual_norm_row(const ResidualNorm &a, size_t row, float *h, bool store) {
-    __shared__ float red[16];  // a row of four for each of the sums
-    const float *xr = a.x + row * a.width;
-    float x[NV], mean, inv;
-    const int c0 = threadIdx.x;
-#pragma unroll
-    for (int i = 0; i < NV; i++) x[i] = c0 + 256 * i < a.width ? xr[c0 + 256 * i] : 0.0f;
+    __shared__ float red[4 * (BT / 64)];  // a part for each of the sums
+    const int w = a.width;
+    float x[NV], g[NV], b[NV], mean, inv;
+    load_row<NV, BT>(a.x + row * w, w, x);
     if (a.y) {
-        const float *yr = a.y + row * a.width;
-        float y[NV];
-#pragma unroll
-        for (int i = 0; i < NV; i++) y[i] = c0 + 256 * i < a.width ? yr[c0 + 256 * i] : 0.0f;
+        float y[NV], pg[NV], pb[NV];
+        load_row<NV, BT>(a.y + row * w, w, y);
+        if (a.post_w) load_row<NV, BT>(a.post_w, w, pg);
+        if (a.post_w && a.post_b) load_row<NV, BT>(a.post_b, w, pb);
+        load_row<NV, BT>(a.pre_w, w, g);
+        if (a.pre_b) load_row<NV, BT>(a.pre_b, w, b);
         if (a.post_w) {
-            row_stats<NV>(y, a.width, a.eps, a.rms, red, &mean, &inv);
+            row_stats<NV, BT>(y, w, a.eps, a.rms, red, &mean, &inv);
 #pragma unroll
-            for (int i = 0; i < NV; i++) {
-                const int c = c0 + 256 * i;
-                if (c < a.width) y[i] = fmaf((y[i] - mean) * inv, a.post_w[c], a.post_b ? a.post_b[c] : 0.0f);
-            }
+            for (int i = 0; i < NV; i++) y[i] = norm_col<BT>(i) < w ? fmaf((y[i] - mean) * inv, pg[i], a.post_b ? pb[i] : 0.0f) : 0.0f;
         }
 #pragma unroll
         for (int i = 0; i < NV; i++) x[i] = fmaf(a.mult, y[i], x[i]);
+    } else {
+        load_row<NV, BT>(a.pre_w, w, g);
+        if (a.pre_b) load_row<NV, BT>(a.pre_b, w, b);
     }
-    row_stats<NV>(x, a.width, a.eps, a.rms, red + 8, &mean, &inv);
+    row_stats<NV, BT>(x, w, a.eps, a.rms, red + 2 * (BT / 64), &mean, &inv);
+    if (store && a.x_out) store_row<NV, BT>(a.x_out + row * w, w, x);
 #pragma unroll
-    for (int i = 0; i < NV; i++) {
-        const int c = c0 + 256 * i;
-        if (c >= a.width) continue;
-        const float v = fmaf((x[i] - mean) * inv, a.pre_w[c], a.pre_b ? a.pre_b[c] : 0.0f);
-        if (h) h[c] = v;
-        if (store) {
-            if (a.x_out) a.x_out[row * a.width + c] = x[i];
-            if (a.h_out) a.h_out[row * a.width + c] = v;
-        }
-    }
+    for (int i = 0; i < NV; i++) x[i] = fmaf((x[i] - mean) * inv, g[i], a.pre_b ? b[i] : 0.0f);
+    if (h) store_row<NV, BT>(h, w, x);
+    if (store && a.h_out) store_row<NV, BT>(a.h_out + row * w, w, x);
 }
 
 // The update of many rows: x in place, h in f32 (h_out) and / or in the products' element type (he, rows `stride`
 // apart, zeros behind the width).  `at`: the rows to take (x_out is then left alone), or null for rows 0, 1, ..
-template <class E, int NV>
-__global__ __launch_bounds__(256) void residual_norm_rows(ResidualNorm a, typename E::T *__restrict__ he, size_t stride,
+template <class E, int NV, int BT>
+__global__ __launch_bounds__(BT) void residual_norm_rows(ResidualNorm a, typename E::T *__restrict__ he, size_t stride,
                                                           const uint32_t *__restrict__ at) {
-    extern __shared__ float hrow[];  // [width] when he is given
+    extern __shared__ __attribute__((aligned(16))) float hrow[];  // [width] when he is given
     const size_t row = at ? at[blockIdx.x] : blockIdx.x;
     if (at) {  // rows of the stream gathered into the first rows of h
         ResidualNorm b = a;
         b.x_out = nullptr, b.h_out = nullptr;
-        residual_norm_row<NV>(b, row, he ? hrow : a.h_out + (size_t)blockIdx.x * a.width, false);
+        residual_norm_row<NV, BT>(b, row, he ? hrow : a.h_out + (size_t)blockIdx.x * a.width, false);
     } else {
-        residual_norm_row<NV>(a, row, he ? hrow : nullptr, true);
+        residual_norm_row<NV, BT>(a, row, he ? hrow : nullptr, true);
     }
     if (!he) return;
     __syncthreads();
     typename E::T *out = he + (size_t)blockIdx.x * stride;
-    for (int c = threadIdx.x; c < (int)stride; c += 256) out[c] = (typename E::T)(c < a.width ? hrow[c] : 0.0f);
+    for (int c = threadIdx.x; c < (int)stride; c += BT) out[c] = (typename E::T)(c < a.width ? hrow[c] : 0.0f);
 }
 
 }  // namespace jq

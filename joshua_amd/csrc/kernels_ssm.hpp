@@ -19,7 +19,8 @@ __global__ __launch_bounds__(256) void causal_conv_silu(const float *__restrict_
                                                         int taps) {
     const int c = (int)blockIdx.x * 256 + (int)threadIdx.x, t0 = (int)blockIdx.y * CONV_RUN;
     if (c >= C) return;
-    auto input = [&](int at) { return at >= 0 ? x[(size_t)at * ldx + c] : tail_in[(size_t)(at + taps - 1) * C + c]; };
+    // (the address is chosen, not the load)
+    auto input = [&](int at) { return *(at >= 0 ? x + (size_t)at * ldx + c : tail_in + (size_t)(at + taps - 1) * C + c); };
     const int nt = min(CONV_RUN, T - t0);
     if (nt > 0) {
         float acc[CONV_RUN];
@@ -31,7 +32,7 @@ __global__ __launch_bounds__(256) void causal_conv_silu(const float *__restrict_
 #pragma unroll
             for (int i = 0; i < CONV_RUN + 3; i++) {  // v[i] is the input at t0 - 3 + i
                 const int at = t0 - 3 + i;
-                v[i] = at < T && at >= -(taps - 1) ? input(at) : 0.0f;
+                v[i] = input(max(min(at, T - 1), -(taps - 1)));  // (beyond either end: meets no weight, or no output)
             }
 #pragma unroll
             for (int j = 0; j < 4; j++) wt[j] = j >= 4 - taps ? w[(size_t)c * taps + j - (4 - taps)] : 0.0f;  // wt[3]: the current token's
@@ -54,7 +55,17 @@ __global__ __launch_bounds__(256) void causal_conv_silu(const float *__restrict_
     for (int t = max(t0, T); t < min(t0 + CONV_RUN, T + taps - 1); t++) tail_out[(size_t)(t - T) * C + c] = input(t - (taps - 1));
 }
 
-__device__ __forceinline__ float softplus(float v) { return v > 20.0f ? v : log1pf(expf(v)); }
+// log(1 + e^v) = max(v, 0) + log1p(e^-|v|), and log1p(e) = 2 atanh(s), s = e / (2 + e) <= 1/3, by its series in s^2: a
+// small result keeps its relative accuracy.
+__device__ __forceinline__ float softplus(float v) {
+    const float e = __builtin_amdgcn_exp2f(-1.44269504088896341f * fabsf(v)), s = e * __builtin_amdgcn_rcpf(2.0f + e), q = s * s;
+    float p = fmaf(q, 1.0f / 15.0f, 1.0f / 13.0f);
+    p = fmaf(q, p, 1.0f / 11.0f), p = fmaf(q, p, 1.0f / 9.0f), p = fmaf(q, p, 1.0f / 7.0f), p = fmaf(q, p, 0.2f), p = fmaf(q, p, 1.0f / 3.0f);
+    return fmaxf(v, 0.0f) + 2.0f * fmaf(q * s, p, s);
+}
+
+// z sigmoid(z)
+__device__ __forceinline__ float gate_silu(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.44269504088896341f * z)); }
 
 template <int LPC>
 __device__ __forceinline__ float sum_lanes(float v) {
@@ -92,7 +103,7 @@ template <int LPC, int NS, class IO>
 __global__ __launch_bounds__(256) void selective_scan(SsmScan a, const IO *__restrict__ x, IO *__restrict__ out) {
     constexpr int CPW = 256 / LPC, NP = LPC * NS, SCAN_RUN = NP <= 128 ? 32 : 4096 / NP;
     __shared__ float2 sd[SCAN_RUN][CPW];                                           // dt, dt x
-    __shared__ float sy[SCAN_RUN][CPW];                                            // D x, then the output
+    __shared__ float sy[SCAN_RUN][CPW];                                            // the states' part of the output
     __shared__ __attribute__((aligned(16))) float sb[SCAN_RUN][NP], scc[SCAN_RUN][NP];
     const int tid = threadIdx.x, ln = tid % LPC, ch = tid / LPC, c0 = (int)blockIdx.x * CPW, c = c0 + ch;
     float S[NS], A[NS];
@@ -105,14 +116,34 @@ __global__ __launch_bounds__(256) void selective_scan(SsmScan a, const IO *__res
     }
     // a run's inputs travel in registers while the run before is worked on (rows past the end: read from the last one)
     constexpr int NI = (SCAN_RUN * CPW + 255) / 256, NB = (SCAN_RUN * NP + 255) / 256;
-    float rdt[NI], rz[NI], rb[NB], rc[NB], bias[NI], skip[NI], zs[NI];
+    float rdt[NI], rz[NI], rb[NB], rc[NB], bias[NI], skip[NI], zs[NI], dx[NI];
     IO rx[NI];
 #pragma unroll
     for (int i = 0; i < NI; i++) {
         const int cc = min(c0 + (tid + 256 * i) % CPW, a.C - 1);
         bias[i] = a.dt_bias[cc], skip[i] = a.D[cc];
     }
+    uint32_t odt[NI], ox[NI], oz[NI], obc[NB];  // this thread's places within a run
+#pragma unroll
+    for (int i = 0; i < NI; i++) {
+        const uint32_t e = tid + 256 * i, t = e / CPW, cc = min(c0 + (int)(e % CPW), a.C - 1);
+        odt[i] = t * (uint32_t)a.C + cc, ox[i] = t * (uint32_t)a.ldx + cc, oz[i] = t * (uint32_t)a.ld_z + cc;
+    }
+#pragma unroll
+    for (int i = 0; i < NB; i++) {
+        const uint32_t e = tid + 256 * i;
+        obc[i] = e / NP * (uint32_t)a.ld_bc + min((int)(e % NP), a.N - 1);
+    }
     auto fetch = [&](int t0) __attribute__((always_inline)) {
+        if (t0 + (256 * NI - 1) / CPW < a.T && t0 + (256 * NB - 1) / NP < a.T) {  // a whole run lies ahead
+            const float *pd = a.dt_raw + (size_t)t0 * a.C, *pz = a.z + (size_t)t0 * a.ld_z, *pb = a.bc + (size_t)t0 * a.ld_bc;
+            const IO *px = x + (size_t)t0 * a.ldx;
+#pragma unroll
+            for (int i = 0; i < NI; i++) rdt[i] = pd[odt[i]], rx[i] = px[ox[i]], rz[i] = pz[oz[i]];
+#pragma unroll
+            for (int i = 0; i < NB; i++) rb[i] = pb[obc[i]], rc[i] = (pb + a.N)[obc[i]];
+            return;
+        }
 #pragma unroll
         for (int i = 0; i < NI; i++) {
             const int e = tid + 256 * i, t = min(t0 + e / CPW, a.T - 1), cc = min(c0 + e % CPW, a.C - 1);
@@ -134,8 +165,7 @@ __global__ __launch_bounds__(256) void selective_scan(SsmScan a, const IO *__res
             if (SCAN_RUN * CPW % 256 == 0 || e < SCAN_RUN * CPW) {
                 const float dt = t < nt ? softplus(rdt[i] + bias[i]) : 0.0f, xv = (float)rx[i];  // (dt = 0 leaves the states alone)
                 sd[t][k] = float2{dt, dt * xv};
-                sy[t][k] = skip[i] * xv;
-                zs[i] = rz[i];
+                dx[i] = skip[i] * xv, zs[i] = rz[i];
             }
         }
 #pragma unroll
@@ -145,30 +175,45 @@ __global__ __launch_bounds__(256) void selective_scan(SsmScan a, const IO *__res
         }
         __syncthreads();
         if (t0 + SCAN_RUN < a.T) fetch(t0 + SCAN_RUN);
-        for (int t = 0; t < nt; t += 4) {
-            float y[4] = {0.f, 0.f, 0.f, 0.f};
+        // four tokens at a time, the next four's operands on their way from LDS meanwhile
+        float2 d[4];
+        float B[4][NS], Cn[4][NS];
+        auto operands = [&](int t) __attribute__((always_inline)) {
 #pragma unroll
             for (int u = 0; u < 4; u++) {
-                const float2 d = sd[t + u][ch];
+                d[u] = sd[t + u][ch];
+#pragma unroll
+                for (int j = 0; j < NS; j++) B[u][j] = sb[t + u][ln * NS + j], Cn[u][j] = scc[t + u][ln * NS + j];
+            }
+        };
+        operands(0);
+        for (int t = 0; t < nt; t += 4) {
+            float decay[4][NS], in[4][NS], cc[4][NS], y[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int u = 0; u < 4; u++)
+#pragma unroll
+                for (int j = 0; j < NS; j++)
+                    decay[u][j] = __builtin_amdgcn_exp2f(d[u].x * A[j]), in[u][j] = d[u].y * B[u][j], cc[u][j] = Cn[u][j];
+            operands(min(t + 4, SCAN_RUN - 4));
+#pragma unroll
+            for (int u = 0; u < 4; u++)
 #pragma unroll
                 for (int j = 0; j < NS; j++) {
-                    const int n = ln * NS + j;
-                    S[j] = fmaf(__builtin_amdgcn_exp2f(d.x * A[j]), S[j], d.y * sb[t + u][n]);
-                    y[u] = fmaf(S[j], scc[t + u][n], y[u]);
+                    S[j] = fmaf(decay[u][j], S[j], in[u][j]);
+                    y[u] = fmaf(S[j], cc[u][j], y[u]);
                 }
-            }
 #pragma unroll
             for (int u = 0; u < 4; u++) y[u] = sum_lanes<LPC>(y[u]);
             if (ln == 0) {
 #pragma unroll
-                for (int u = 0; u < 4; u++) sy[t + u][ch] += y[u];
+                for (int u = 0; u < 4; u++) sy[t + u][ch] = y[u];
             }
         }
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < NI; i++) {
             const int e = tid + 256 * i, t = e / CPW, k = e % CPW;
-            if (t < nt && c0 + k < a.C) out[(size_t)(t0 + t) * a.ldo + c0 + k] = (IO)(sy[t][k] * silu(zs[i]));
+            if (t < nt && c0 + k < a.C) out[(size_t)(t0 + t) * a.ldo + c0 + k] = (IO)((sy[t][k] + dx[i]) * gate_silu(zs[i]));
         }
         __syncthreads();
     }
@@ -203,7 +248,7 @@ __global__ __launch_bounds__(256) void selective_step(SsmScan a, const uint8_t *
         if (c < a.C) a.S[at] = S;
     }
     y = sum_row16(y);
-    if (sub == 0 && c < a.C) out[c] = fmaf(a.D[c], xv, y) * silu(a.z[c]);
+    if (sub == 0 && c < a.C) out[c] = fmaf(a.D[c], xv, y) * gate_silu(a.z[c]);
 }
 
 }  // namespace jq
