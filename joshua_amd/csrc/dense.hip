@@ -23,12 +23,16 @@ int run_norm_gemv(const jq_weight *w, const jq_weight *up, float *Y, const jq::G
     const int k = (int)w->k, n = (int)w->n;
     if (nm.width != k || k > FUSED_NORM_MAX_WIDTH || nm.x_out == nm.x) return fail("dense gemv: no fused norm for this row");
     const uint8_t *wu = up ? up->dev : nullptr;
-    const dim3 grid((unsigned)std::min(GATED ? n : (n + 1) / 2, 256)), block(64 * jq::NORM_GEMV_WAVES);
-#define JQ_NG(NV)                                                                                                                   \
-    JQ_ELEM(w->type, hipLaunchKernelGGL((jq::norm_gemv<E, NV, GATED>), grid, block, (size_t)k * sizeof(float), s, w->dev, wu, w->row_bytes, Y, \
-                                        k, n, unit, nm))
-    if (k <= 4096) JQ_NG(4);
-    else JQ_NG(8);
+    const dim3 grid((unsigned)std::min(GATED ? n : (n + 1) / 2, 256));
+#define JQ_NG(WAVES, NV)                                                                                                             \
+    JQ_ELEM(w->type, hipLaunchKernelGGL((jq::norm_gemv<E, WAVES, NV, GATED>), grid, dim3(64 * WAVES), (size_t)k * sizeof(float), s, w->dev, \
+                                        wu, w->row_bytes, Y, k, n, unit, nm))
+    const bool few = (size_t)n * k <= ((size_t)1 << 20);  // a router, say: the norm is most of it
+    if (few && k <= 1024) JQ_NG(4, 4);
+    else if (few && k <= 4096) JQ_NG(4, 16);
+    else if (k <= 2048) JQ_NG(8, 4);
+    else if (k <= 4096) JQ_NG(16, 4);
+    else JQ_NG(16, 8);
 #undef JQ_NG
     note_kernel("norm_gemv");
     HIP_TRY(hipGetLastError());
@@ -79,7 +83,7 @@ namespace {
 // on.  Runs of at least 4 stages (512 bytes of a row); depends on the shape only, so a shape keeps its order of
 // additions.
 int gemm_splits(size_t tiles, int stages) {
-    if (tiles >= 192) return 1;
+    if (tiles >= 192) return tiles < 384 && stages >= 96 ? 2 : 1;  // long rows: a second workgroup a compute unit pays for the addition
     return (int)std::max<size_t>(1, std::min<size_t>({512 / tiles, (size_t)stages / 4, 16}));
 }
 
@@ -195,7 +199,7 @@ int dense_matmul(uint32_t type, const uint8_t *W, size_t row_bytes, const float 
 
 int dense_decode(const jq_weight *w, const uint32_t *ids, float *out, size_t rows, float scale, hipStream_t s) {
     if (!rows || !w->k) return 0;
-    JQ_ELEM(w->type, hipLaunchKernelGGL((jq::dense_rows_to_f32<E>), dim3(grid_for(rows * w->k)), dim3(256), 0, s, w->dev, w->row_bytes, ids,
+    JQ_ELEM(w->type, hipLaunchKernelGGL((jq::dense_rows_to_f32<E>), dim3((unsigned)std::min<size_t>(rows, 65536), (unsigned)std::min<size_t>((w->k + 1023) / 1024, 64)), dim3(256), 0, s, w->dev, w->row_bytes, ids,
                                         out, rows, (int)w->k, scale));
     HIP_TRY(hipGetLastError());
     return 0;
@@ -211,14 +215,13 @@ int zero_floats(float *p, size_t n, hipStream_t s) {
 int residual_norm(const jq::ResidualNorm &a, uint32_t type, void *he, size_t stride, size_t rows, const uint32_t *at, hipStream_t s) {
     if (a.width > NORM_MAX_WIDTH) return fail("residual norm: rows of %d exceed %d", a.width, NORM_MAX_WIDTH);
     if (!rows) return 0;
-    const size_t lds = he ? (size_t)a.width * sizeof(float) : 0;
 #define JQ_ROWS(NV, BT)                                                                                                          \
-    JQ_ELEM(type, hipLaunchKernelGGL((jq::residual_norm_rows<E, NV, BT>), dim3((unsigned)rows), dim3(BT), lds, s, a, (typename E::T *)he, \
+    JQ_ELEM(type, hipLaunchKernelGGL((jq::residual_norm_rows<E, NV, BT>), dim3((unsigned)rows), dim3(BT), 0, s, a, (typename E::T *)he, \
                                      stride, at))
     if (a.width <= 1024) JQ_ROWS(4, 256);
-    else if (a.width <= 2048) JQ_ROWS(4, 512);
-    else if (a.width <= 4096) JQ_ROWS(4, 1024);
-    else if (a.width <= 8192) JQ_ROWS(8, 1024);
+    else if (a.width <= 2048) JQ_ROWS(8, 256);
+    else if (a.width <= 4096) JQ_ROWS(16, 256);
+    else if (a.width <= 8192) JQ_ROWS(16, 512);
     else JQ_ROWS(16, 1024);
 #undef JQ_ROWS
     HIP_TRY(hipGetLastError());
@@ -269,7 +272,8 @@ int moe_forward_dense(jq_moe *m, size_t T, const float *x, const void *xe, float
         const bool wave = moe_wave_gate(c);
         jq::MoeGateIn gi{m->logits, m->router_bias, moe_gate_params(c), m->ids, m->wts, no_groups, (int)T};
         if (pre) {  // residual update, norm and router logits in one launch; x is what it leaves
-            const jq_weight router{JQ_TYPE_F32, c.n_expert, c.hidden, 0, c.hidden * sizeof(float), (uint8_t *)m->router_w, false};
+            const jq_weight packed{JQ_TYPE_F32, c.n_expert, c.hidden, 0, c.hidden * sizeof(float), (uint8_t *)m->router_w, false};
+            const jq_weight &router = m->router_rows ? *m->router_rows : packed;
             if (pre->h_out != x || T != 1) return fail("moe: the fused norm makes another row");
             if (dense_gemv(&router, nullptr, 0, 1, m->logits, c.n_expert, s, pre)) return 1;
             if (!wave) {  // the gating as a launch of its own

@@ -6,7 +6,7 @@
 namespace jqh {
 
 constexpr int GEMV_MAX_ROWS = 8;   // activation rows up to which a product runs on the GEMV, in f32 activations
-constexpr int NORM_MAX_WIDTH = 16128;
+constexpr int NORM_MAX_WIDTH = 16384;
 constexpr int FUSED_NORM_MAX_WIDTH = 8192;
 
 // Y[t, :] = X[t, :] W^T for T <= GEMV_MAX_ROWS.  With `nm` (one row, width = W's k, at most FUSED_NORM_MAX_WIDTH) X

@@ -166,13 +166,11 @@ __global__ __launch_bounds__(256) void dense_gemv_gated(const uint8_t *__restric
 }
 
 // The one-row products with the residual update and norm of `nm` in front: y = W h, or with GATED
-// y = gated(Wg h, Wu h).  A workgroup of 16 waves makes the normed row h for itself (workgroup 0 stores it; few, large
+// y = gated(Wg h, Wu h).  A workgroup makes the normed row h for itself (workgroup 0 stores it; few, large
 // workgroups, since each reads the norm's vectors whole); then every wave takes pairs of weight rows (gated: the gate and the
 // up row of a column) on its own, the first chunks of its first pair on their way since before the norm.
-constexpr int NORM_GEMV_WAVES = 16;
-
-template <class E, int NV, bool GATED>
-__global__ __launch_bounds__(64 * NORM_GEMV_WAVES) void norm_gemv(const uint8_t *__restrict__ W, const uint8_t *__restrict__ Wu, size_t pitch,
+template <class E, int WAVES, int NV, bool GATED>
+__global__ __launch_bounds__(64 * WAVES) void norm_gemv(const uint8_t *__restrict__ W, const uint8_t *__restrict__ Wu, size_t pitch,
                                                                   float *__restrict__ Y, int k, int n, GatedUnit act, ResidualNorm nm) {
     constexpr int R = 2, PER = GATED ? 1 : 2, STEP = 64 * E::CH, PRE = 4;
     extern __shared__ __attribute__((aligned(16))) float hrow[];  // [k]
@@ -202,9 +200,13 @@ __global__ __launch_bounds__(64 * NORM_GEMV_WAVES) void norm_gemv(const uint8_t 
     };
     int grp = (int)blockIdx.x + (int)gridDim.x * wave;
     ask(min(grp, groups - 1));
-    residual_norm_row<NV, 64 * NORM_GEMV_WAVES>(nm, 0, hrow, blockIdx.x == 0);
+    {
+        float h[NV];
+        residual_norm_row<NV, 64 * WAVES>(nm, h, blockIdx.x == 0);
+        store_row<NV, 64 * WAVES>(hrow, k, h);
+    }
     __syncthreads();
-    for (; grp < groups; grp += (int)gridDim.x * NORM_GEMV_WAVES) {
+    for (; grp < groups; grp += (int)gridDim.x * WAVES) {
         float acc[R] = {};
 #pragma unroll
         for (int p = 0; p < PRE; p++) {
@@ -218,7 +220,7 @@ __global__ __launch_bounds__(64 * NORM_GEMV_WAVES) void norm_gemv(const uint8_t 
             for (int r = 0; r < R; r++) w[r] = chunk_of<E>(rows[r], c);
             multiply(w, c, acc);
         }
-        const int next = grp + (int)gridDim.x * NORM_GEMV_WAVES;
+        const int next = grp + (int)gridDim.x * WAVES;
         if (next < groups) ask(next);
 #pragma unroll
         for (int r = 0; r < R; r++) acc[r] = wave_sum(acc[r]);
@@ -526,10 +528,9 @@ __global__ __launch_bounds__(256) void rows_to_elem(const float *__restrict__ X,
 template <class E>
 __global__ __launch_bounds__(256) void dense_rows_to_f32(const uint8_t *__restrict__ W, size_t pitch, const uint32_t *__restrict__ ids,
                                                          float *__restrict__ out, size_t rows, int k, float scale) {
-    const size_t total = rows * (size_t)k;
-    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
-        const size_t r = i / k, c = i % k;
-        out[i] = (float)((const typename E::T *)(W + (ids ? ids[r] : r) * pitch))[c] * scale;
+    for (size_t r = blockIdx.x; r < rows; r += gridDim.x) {
+        const typename E::T *row = (const typename E::T *)(W + (ids ? ids[r] : r) * pitch);
+        for (int c = (int)blockIdx.y * 256 + (int)threadIdx.x; c < k; c += (int)gridDim.y * 256) out[r * k + c] = (float)row[c] * scale;
     }
 }
 

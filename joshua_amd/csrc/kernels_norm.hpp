@@ -85,16 +85,18 @@ __device__ __forceinline__ void row_stats(const float (&v)[NV], int width, float
     *inv = 1.0f / sqrtf(sum_block<BT>(ss, red + BT / 64) / (float)width + eps);
 }
 
-// Row `row` of the update; the normed row goes to `h` (LDS or global), and with `store` x and h to x_out and h_out.
+// The update of one row by a workgroup; x ends as this thread's share of the normed row.  With `store` the stream goes to
+// x_out and the normed row to h_out.  The norms' vectors are asked for together with the row: a single row's time is its
+// round trips to memory.
 template <int NV, int BT>
-__device__ __forceinline__ void residual_norm_row(const ResidualNorm &a, size_t row, float *h, bool store) {
+__device__ __forceinline__ void residual_norm_row(const ResidualNorm &a, float (&x)[NV], bool store) {
     __shared__ float red[4 * (BT / 64)];  // a part for each of the sums
     const int w = a.width;
-    float x[NV], g[NV], b[NV], mean, inv;
-    load_row<NV, BT>(a.x + row * w, w, x);
+    float g[NV], b[NV], mean, inv;
+    load_row<NV, BT>(a.x, w, x);
     if (a.y) {
         float y[NV], pg[NV], pb[NV];
-        load_row<NV, BT>(a.y + row * w, w, y);
+        load_row<NV, BT>(a.y, w, y);
         if (a.post_w) load_row<NV, BT>(a.post_w, w, pg);
         if (a.post_w && a.post_b) load_row<NV, BT>(a.post_b, w, pb);
         load_row<NV, BT>(a.pre_w, w, g);
@@ -110,32 +112,76 @@ __device__ __forceinline__ void residual_norm_row(const ResidualNorm &a, size_t 
         load_row<NV, BT>(a.pre_w, w, g);
         if (a.pre_b) load_row<NV, BT>(a.pre_b, w, b);
     }
+    if (store && a.x_out) store_row<NV, BT>(a.x_out, w, x);
     row_stats<NV, BT>(x, w, a.eps, a.rms, red + 2 * (BT / 64), &mean, &inv);
-    if (store && a.x_out) store_row<NV, BT>(a.x_out + row * w, w, x);
 #pragma unroll
     for (int i = 0; i < NV; i++) x[i] = fmaf((x[i] - mean) * inv, g[i], a.pre_b ? b[i] : 0.0f);
-    if (h) store_row<NV, BT>(h, w, x);
-    if (store && a.h_out) store_row<NV, BT>(a.h_out + row * w, w, x);
+    if (store && a.h_out) store_row<NV, BT>(a.h_out, w, x);
 }
 
-// The update of many rows: x in place, h in f32 (h_out) and / or in the products' element type (he, rows `stride`
-// apart, zeros behind the width).  `at`: the rows to take (x_out is then left alone), or null for rows 0, 1, ..
+// The update of many rows, a workgroup a row: x in place, h in f32 (h_out) and / or in the products' element type (he, rows
+// `stride` apart, zeros behind the width).  `at`: the rows to take, into the first rows of h (x_out is then left alone), or
+// null for rows 0, 1, ..  A thread has columns BT apart, and the norms' vectors are read as they are needed: what counts here
+// is how many rows are under way at once, that is registers.
 template <class E, int NV, int BT>
 __global__ __launch_bounds__(BT) void residual_norm_rows(ResidualNorm a, typename E::T *__restrict__ he, size_t stride,
-                                                          const uint32_t *__restrict__ at) {
-    extern __shared__ __attribute__((aligned(16))) float hrow[];  // [width] when he is given
+                                                         const uint32_t *__restrict__ at) {
+    using T = typename E::T;
+    constexpr int NW = BT / 64;
+    __shared__ float red[4 * NW];
+    const int w = a.width, c0 = threadIdx.x;
     const size_t row = at ? at[blockIdx.x] : blockIdx.x;
-    if (at) {  // rows of the stream gathered into the first rows of h
-        ResidualNorm b = a;
-        b.x_out = nullptr, b.h_out = nullptr;
-        residual_norm_row<NV, BT>(b, row, he ? hrow : a.h_out + (size_t)blockIdx.x * a.width, false);
-    } else {
-        residual_norm_row<NV, BT>(a, row, he ? hrow : nullptr, true);
+    const float *xr = a.x + row * w;
+    float x[NV];
+    auto stats = [&](const float (&v)[NV], float *r, float *mean, float *inv) __attribute__((always_inline)) {
+        float mu = 0.0f, ss = 0.0f;
+        if (!a.rms) {
+            float s = 0.0f;
+#pragma unroll
+            for (int i = 0; i < NV; i++) s += v[i];
+            mu = sum_block<BT>(s, r) / (float)w;
+        }
+#pragma unroll
+        for (int i = 0; i < NV; i++) {
+            const float d = c0 + BT * i < w ? v[i] - mu : 0.0f;
+            ss = fmaf(d, d, ss);
+        }
+        *mean = mu, *inv = 1.0f / sqrtf(sum_block<BT>(ss, r + NW) / (float)w + a.eps);
+    };
+#pragma unroll
+    for (int i = 0; i < NV; i++) x[i] = c0 + BT * i < w ? xr[c0 + BT * i] : 0.0f;
+    float mean, inv;
+    if (a.y) {
+        const float *yr = a.y + row * w;
+        float y[NV];
+#pragma unroll
+        for (int i = 0; i < NV; i++) y[i] = c0 + BT * i < w ? yr[c0 + BT * i] : 0.0f;
+        if (a.post_w) {
+            stats(y, red, &mean, &inv);
+#pragma unroll
+            for (int i = 0; i < NV; i++) {
+                const int c = c0 + BT * i;
+                if (c < w) y[i] = fmaf((y[i] - mean) * inv, a.post_w[c], a.post_b ? a.post_b[c] : 0.0f);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < NV; i++) x[i] = fmaf(a.mult, y[i], x[i]);
     }
-    if (!he) return;
-    __syncthreads();
-    typename E::T *out = he + (size_t)blockIdx.x * stride;
-    for (int c = threadIdx.x; c < (int)stride; c += BT) out[c] = (typename E::T)(c < a.width ? hrow[c] : 0.0f);
+    stats(x, red + 2 * NW, &mean, &inv);
+    float *xo = at ? nullptr : a.x_out, *ho = a.h_out ? a.h_out + (size_t)blockIdx.x * w : nullptr;
+    T *eo = he ? he + (size_t)blockIdx.x * stride : nullptr;
+#pragma unroll
+    for (int i = 0; i < NV; i++) {
+        const int c = c0 + BT * i;
+        if (c < w) {
+            const float v = fmaf((x[i] - mean) * inv, a.pre_w[c], a.pre_b ? a.pre_b[c] : 0.0f);
+            if (xo) xo[row * w + c] = x[i];
+            if (ho) ho[c] = v;
+            if (eo) eo[c] = (T)v;
+        } else if (eo && c < (int)stride) {
+            eo[c] = (T)0.0f;
+        }
+    }
 }
 
 }  // namespace jq

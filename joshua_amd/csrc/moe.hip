@@ -1,5 +1,5 @@
 // The mixture-of-experts layer object (declared in moe.hpp; C ABI in include/joshua_hip.h).
-#include "moe.hpp"
+#include "dense.hpp"
 
 namespace jqh {
 
@@ -81,7 +81,19 @@ int moe_route_dev(jq_moe *m, size_t T, const float *x, hipStream_t s, jq::MoePai
     const size_t tile_from = (size_t)c.hidden * c.n_expert >= (1u << 20) ? 8 : 32;
     const jq::MoeGateParams gp = moe_gate_params(c);
     const bool wave_gate = moe_wave_gate(c);
-    if (pre)
+    if (m->router_rows) {  // (the kernels below read a row in fours)
+        const size_t E = c.n_expert, h = c.hidden, stride = dense_stride(h);
+        if (pre) return fail("moe: no fused norm for rows of %u", c.hidden);
+        if (T <= (size_t)GEMV_MAX_ROWS) {
+            if (dense_gemv(m->router_rows, x, h, (int)T, m->logits, E, s)) return 1;
+        } else {
+            CallScratch scratch(1);
+            uint8_t *rows = nullptr;
+            if (scratch.get(T * stride * sizeof(float), s, &rows) || rows_to_elem(JQ_TYPE_F32, x, h, T, (int)h, rows, stride, s) ||
+                dense_gemm(m->router_rows, rows, stride, (int)T, m->logits, E, s))
+                return 1;
+        }
+    } else if (pre)
         hipLaunchKernelGGL(jq::moe_router_logits_norm, dim3(c.n_expert), dim3(256), 0, s, m->router_w, *pre, m->logits,
                            (int)c.hidden, (int)c.n_expert);
     else if (T >= tile_from && !no_tile)  // many tokens: a token's activations read once per eight experts (the same bits)
@@ -196,7 +208,7 @@ int jq_moe_create(const jq_moe_config *cfg, const float *router_w, const float *
     if (c.gating > 2) return fail("moe: unknown gating %u", c.gating);
     if (!dense_elem_bytes(gate_exps->type) && ((c.act_alpha != 0.0f && c.act_alpha != 1.0f) || c.act_up_shift != 0.0f))
         return fail("moe: experts in block formats run SwiGLU only");
-    if (c.hidden % 4 != 0) return fail("moe: hidden size %u is not a multiple of 4", c.hidden);
+    if (c.hidden % 4 != 0 && !dense_elem_bytes(gate_exps->type)) return fail("moe: hidden size %u is not a multiple of 4", c.hidden);
     if (c.n_group > 1 && (c.n_expert % c.n_group != 0 || c.topk_group == 0 || c.topk_group > c.n_group))
         return fail("moe: %u experts in %u groups, %u groups kept", c.n_expert, c.n_group, c.topk_group);
     // reference: src/quantized_qwen3_moe.rs:567-571 (expert tensor shaped [n_expert, out, in])
@@ -235,6 +247,7 @@ int jq_moe_create(const jq_moe_config *cfg, const float *router_w, const float *
         fail("moe: router upload failed");
         return cleanup();
     }
+    if (c.hidden % 4 != 0 && jq_upload(JQ_TYPE_F32, router_w, rbytes, c.n_expert, c.hidden, 0, &m->router_rows)) return cleanup();
     if (router_bias) {
         if (hipMalloc((void **)&m->router_bias, c.n_expert * sizeof(float)) != hipSuccess ||
             hipMemcpy(m->router_bias, router_bias, c.n_expert * sizeof(float), hipMemcpyHostToDevice) != hipSuccess) {
@@ -256,6 +269,7 @@ int jq_moe_create(const jq_moe_config *cfg, const float *router_w, const float *
 void jq_moe_free(jq_moe *m) {
     if (!m) return;
     moe_free_scratch(m);
+    jq_free(m->router_rows);
     for (void *p : {(void *)m->router_w, (void *)m->router_bias, (void *)m->pgate, (void *)m->pup, (void *)m->pdown})
         if (p) (void)hipFree(p);
     delete m;

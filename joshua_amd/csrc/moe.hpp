@@ -33,6 +33,7 @@ struct jq_moe {
     jq_moe_config cfg;
     const jq_weight *gate, *up, *down, *sgate, *sup, *sdown;
     float *router_w = nullptr, *router_bias = nullptr;
+    jq_weight *router_rows = nullptr;  // hidden not a multiple of 4 (plain-row experts): the router in padded rows
     const uint8_t **pgate = nullptr, **pup = nullptr, **pdown = nullptr;  // device tables of expert bases
     bool fold_shared = false;  // the shared expert rides along as table entry n_expert of the grouped kernels
     // scratch, grown to the largest token count seen

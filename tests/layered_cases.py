@@ -56,4 +56,11 @@ WIDE = model(72, 90, [
 # many experts: gating past one wave's reach
 CROWD = model(48, 60, [moe(attention(2, 1, 24, 24), 300, 5, 8), moe(mamba(48, 8, 4, 4), 70, 66, 12)], residual_mult=0.9)
 
-ALL = {"mixed": MIXED, "ones": ONES, "wide": WIDE, "crowd": CROWD}
+# sizes that are no multiple of anything
+ODD = model(51, 33, [
+    moe(attention(3, 1, 10, 7, dims=6, v_mix=True), 6, 3, 30),
+    dense(mamba(21, 3, 5, 4), 13),
+    moe(attention(2, 1, 5, 7, dims=2, v_mix=True), 70, 2, 9),
+])
+
+ALL = {"mixed": MIXED, "ones": ONES, "wide": WIDE, "crowd": CROWD, "odd": ODD}
