@@ -229,6 +229,10 @@ int jq_moe_create(const jq_moe_config *cfg, const float *router_w, const float *
                   jq_moe **out);
 void jq_moe_free(jq_moe *moe);
 
+/* A gate of its own on the shared expert of BF16 / F32 experts: its result is multiplied by sigmoid(row . x), one number
+ * a token.  row is [h] f32 on the host. */
+int jq_moe_set_shared_gate(jq_moe *moe, const float *row);
+
 /* Router only: ids[t, s] (descending score) and weights[t, s], s < k
  * (reference: src/quantized_qwen3_moe.rs:424-436 route). */
 int jq_moe_route(jq_moe *moe, size_t n_tokens, const float *x, uint32_t *ids, float *weights,

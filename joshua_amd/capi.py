@@ -30,7 +30,7 @@ TYPE_NAMES = {Q8_0: "Q8_0", Q2_K: "Q2_K", Q4_K: "Q4_K", Q6_K: "Q6_K", IQ2_XXS: "
 EXPORTS = (
     "jq_last_error", "jq_last_kernel", "jq_block_geometry", "jq_init", "jq_upload", "jq_view", "jq_free", "jq_dtype", "jq_rows",
     "jq_cols", "jq_storage_size_in_bytes", "jq_device_ptr", "jq_matmul_t", "jq_matmul_t_f16", "jq_matmul_t_noalloc", "jq_try_matmul_fused", "jq_dequantize", "jq_decode_raw_to_f32", "jq_stream_release",
-    "jq_embedding", "jq_stream_synchronize", "jq_moe_create", "jq_moe_free", "jq_moe_route", "jq_moe_forward",
+    "jq_embedding", "jq_stream_synchronize", "jq_moe_create", "jq_moe_set_shared_gate", "jq_moe_free", "jq_moe_route", "jq_moe_forward",
     "jq_mla_create", "jq_mla_free", "jq_mla_forward", "jq_mla_reset", "jq_mla_cached_tokens",
     "jq_qwen3_create", "jq_qwen3_free", "jq_qwen3_set_tensor", "jq_qwen3_forward", "jq_qwen3_greedy", "jq_qwen3_reset",
     "jq_qwen3_get_config", "jq_qwen3_load_gguf", "jq_type_size_bytes", "jq_gguf_open", "jq_gguf_parse", "jq_gguf_close",
@@ -136,6 +136,7 @@ def lib(path: str = LIB_PATH, beside_torch: bool = True) -> ctypes.CDLL:
         L.jq_embedding.argtypes = [vp, vp, sz, vp, sz, i32, vp]
         L.jq_stream_synchronize.argtypes = [vp]
         L.jq_moe_create.argtypes = [ctypes.POINTER(MoeConfig), vp, vp, vp, vp, vp, vp, vp, vp, ctypes.POINTER(vp)]
+        L.jq_moe_set_shared_gate.argtypes = [vp, vp]
         L.jq_moe_free.argtypes = [vp]
         L.jq_moe_free.restype = None
         L.jq_moe_route.argtypes = [vp, sz, vp, vp, vp, i32, vp]
@@ -364,7 +365,8 @@ class Moe:
     src/quantized_deepseek2.rs:508-672)."""
 
     def __init__(self, cfg: MoeConfig, router_w: np.ndarray, gate_exps: Weight, up_exps: Weight, down_exps: Weight,
-                 router_bias: np.ndarray | None = None, shared: "tuple[Weight, Weight, Weight] | None" = None):
+                 router_bias: np.ndarray | None = None, shared: "tuple[Weight, Weight, Weight] | None" = None,
+                 shared_gate: np.ndarray | None = None):
         self.cfg = cfg
         self._keep = (gate_exps, up_exps, down_exps, shared)
         rw = np.ascontiguousarray(router_w, dtype=np.float32)
@@ -376,6 +378,10 @@ class Moe:
                                    gate_exps.handle, up_exps.handle, down_exps.handle, sh[0], sh[1], sh[2],
                                    ctypes.byref(out)))
         self._h = out
+        if shared_gate is not None:
+            row = np.ascontiguousarray(shared_gate, dtype=np.float32)
+            assert row.size == cfg.hidden
+            _check(lib().jq_moe_set_shared_gate(self._h, row.ctypes.data))
 
     def close(self) -> None:
         if self._h:

@@ -155,7 +155,7 @@ int run_gemm(uint32_t type, jq::DenseGemm a, size_t rows_of_a, size_t k, size_t 
 }  // namespace
 
 int dense_gemm(const jq_weight *w, const void *A, size_t lda, int T, float *C, size_t ldc, hipStream_t s) {
-    if (lda != dense_stride(w->k)) return fail("dense gemm: activation rows of %zu elements for k = %zu", lda, w->k);
+    if (lda < dense_stride(w->k) || lda % DENSE_PAD) return fail("dense gemm: activation rows of %zu elements for k = %zu", lda, w->k);
     jq::DenseGemm a{};
     a.A = (const uint8_t *)A, a.W = w->dev, a.lda = (uint32_t)(lda * dense_elem_bytes(w->type)), a.ldw = (uint32_t)w->row_bytes;
     a.M = T, a.N = (int)w->n, a.C = C, a.ldc = ldc;
@@ -233,24 +233,28 @@ int residual_norm(const jq::ResidualNorm &a, uint32_t type, void *he, size_t str
 namespace {
 
 bool takes_dense(const jq_weight *gate, const jq_weight *up, const jq_weight *down) {
-    return dense_elem_bytes(gate->type) && up->type == gate->type && down->type == gate->type;
+    return dense_elem_bytes(gate->type) && up->type == gate->type && down->type == gate->type;  // (a shared expert's: jq_moe_create)
 }
 
 int reserve_dense(jq_moe *m, size_t T) {
     const jq_moe_config &c = m->cfg;
-    if (m->sgate) return fail("moe: a shared expert beside experts in plain rows is not supported");
     const size_t esz = dense_elem_bytes(m->gate->type), P = T * c.n_expert_used;
     HIP_TRY(hipMalloc((void **)&m->dense_x, T * dense_stride(c.hidden) * esz));
     HIP_TRY(hipMalloc((void **)&m->dense_act, P * dense_stride(c.inter) * esz));
     // (the columns behind inter stay zero: the kernels write the first inter only)
     HIP_TRY(hipMemset(m->dense_act, 0, P * dense_stride(c.inter) * esz));
+    if (m->sgate) {
+        const size_t bytes = T * dense_stride(m->sgate->n) * esz;
+        HIP_TRY(hipMalloc((void **)&m->dense_sact, bytes));
+        HIP_TRY(hipMemset(m->dense_sact, 0, bytes));
+    }
     return 0;
 }
 
 void release_dense(jq_moe *m) {
-    for (uint8_t *p : {m->dense_x, m->dense_act})
+    for (uint8_t *p : {m->dense_x, m->dense_act, m->dense_sact})
         if (p) (void)hipFree(p);
-    m->dense_x = m->dense_act = nullptr;
+    m->dense_x = m->dense_act = m->dense_sact = nullptr;
 }
 
 // One expert is read by every pair that names it on the decode-sized kernels, once a row tile on the grouped GEMM.
@@ -258,36 +262,56 @@ bool decode_sized(const jq_moe_config &c, size_t T) { return T <= (size_t)GEMV_M
 
 }  // namespace
 
+bool moe_dense_decode_sized(const jq_moe *m, size_t T) { return decode_sized(m->cfg, T); }
+
 bool moe_dense_fuses_norm(const jq_moe *m, size_t T) {
     return T == 1 && m->cfg.hidden <= (uint32_t)FUSED_NORM_MAX_WIDTH && decode_sized(m->cfg, T);
 }
 
-int moe_forward_dense(jq_moe *m, size_t T, const float *x, const void *xe, float *y, hipStream_t s, const jq::ResidualNorm *pre) {
+int moe_forward_dense(jq_moe *m, size_t T, const float *x, const void *xe, float *y, hipStream_t s, const MoeDenseExtras &ex) {
     const jq_moe_config &c = m->cfg;
     const uint32_t type = m->gate->type;
     const int P = (int)(T * c.n_expert_used), h = (int)c.hidden, inter = (int)c.inter, ku = (int)c.n_expert_used;
     const jq::GatedUnit unit{c.swiglu_clamp > 0.0f ? c.swiglu_clamp : INFINITY, c.act_alpha == 0.0f ? 1.0f : c.act_alpha, c.act_up_shift};
+    const jq::GatedUnit shared_unit{c.swiglu_clamp_shared > 0.0f ? c.swiglu_clamp_shared : INFINITY, unit.alpha, unit.shift};
     const jq::MoePairGroups no_groups{nullptr, nullptr, nullptr, nullptr, 0};
-    if (decode_sized(c, T)) {
+    const bool decode = decode_sized(c, T);
+    const int sn = m->sgate ? (int)m->sgate->n : 0;
+    if (m->sgate && (m->sgate->type != type || m->sup->type != type || m->sdown->type != type))
+        return fail("moe: a shared expert of another type than the routed ones");
+    // the shared expert's gate
+    const float *sl = ex.logits ? ex.shared_logit : nullptr;
+    size_t ld_sl = ex.ld;
+    if (sn && m->sgate_row && !ex.logits) {
+        if (ex.pre) return fail("moe: no fused norm in front of a gated shared expert");
+        for (size_t t = 0; t < T; t += GEMV_MAX_ROWS)
+            if (dense_gemv(m->sgate_row, x + t * h, h, (int)std::min<size_t>(GEMV_MAX_ROWS, T - t), m->sgate_logit + t, 1, s)) return 1;
+        sl = m->sgate_logit, ld_sl = 1;
+    }
+    // the gating over logits that are there already, as a launch of its own
+    jq::MoeGateParams gp = moe_gate_params(c);
+    gp.ld = ex.logits ? (int)ex.ld : 0;
+    auto gate = [&] { return moe_gate_dev(m, T, ex.logits ? ex.logits : m->logits, gp, no_groups, s); };
+    if (decode) {
         const bool wave = moe_wave_gate(c);
-        jq::MoeGateIn gi{m->logits, m->router_bias, moe_gate_params(c), m->ids, m->wts, no_groups, (int)T};
-        if (pre) {  // residual update, norm and router logits in one launch; x is what it leaves
+        jq::MoeGateIn gi{ex.logits ? ex.logits : m->logits, m->router_bias, gp, m->ids, m->wts, no_groups, (int)T};
+        if (ex.logits) {
+            if (!wave && gate()) return 1;
+        } else if (ex.pre) {  // residual update, norm and router logits in one launch; x is what it leaves
             const jq_weight packed{JQ_TYPE_F32, c.n_expert, c.hidden, 0, c.hidden * sizeof(float), (uint8_t *)m->router_w, false};
             const jq_weight &router = m->router_rows ? *m->router_rows : packed;
-            if (pre->h_out != x || T != 1) return fail("moe: the fused norm makes another row");
-            if (dense_gemv(&router, nullptr, 0, 1, m->logits, c.n_expert, s, pre)) return 1;
-            if (!wave) {  // the gating as a launch of its own
-                size_t sm = (2 * c.n_expert + std::max<uint32_t>(c.n_group, 1) + c.n_expert_used + 4) * sizeof(float);
-                hipLaunchKernelGGL(jq::moe_gate_topk, dim3(1), dim3(256), sm, s, m->logits, m->router_bias, gi.p, m->ids, m->wts, no_groups);
-            }
+            if (ex.pre->h_out != x || T != 1) return fail("moe: the fused norm makes another row");
+            if (dense_gemv(&router, nullptr, 0, 1, m->logits, c.n_expert, s, ex.pre)) return 1;
+            if (!wave && gate()) return 1;
         } else {
             jq::MoeGateIn later{};
             if (moe_route_dev(m, T, x, s, no_groups, jq::ActsI8{nullptr, nullptr, nullptr, nullptr}, nullptr, wave ? &later : nullptr)) return 1;
         }
-        const dim3 grid((unsigned)((inter + 3) / 4), (unsigned)P);
+        const jq::SharedRows sh{sn ? m->sgate->dev : nullptr, sn ? m->sup->dev : nullptr, sn, m->sG, sl, ld_sl, P, shared_unit.limit};
+        const dim3 grid((unsigned)((std::max(inter, sn) + 3) / 4), (unsigned)(P + (sn ? (int)T : 0)));
 #define JQ_GU(NE)                                                                                                             \
     JQ_ELEM(type, hipLaunchKernelGGL((jq::moe_dense_gate_up<E, NE>), grid, dim3(256), 0, s, m->pgate, m->pup, m->gate->row_bytes, x, \
-                                     (size_t)h, m->G, (size_t)inter, h, inter, ku, m->ids, unit, gi))
+                                     (size_t)h, m->G, (size_t)inter, h, inter, ku, m->ids, unit, gi, sh))
         const int ne = (int)(c.n_expert + 63) / 64;
         if (!wave) JQ_GU(0);
         else if (ne == 1) JQ_GU(1);
@@ -295,18 +319,25 @@ int moe_forward_dense(jq_moe *m, size_t T, const float *x, const void *xe, float
         else if (ne == 3) JQ_GU(3);
         else JQ_GU(4);
 #undef JQ_GU
+        jq::SumRun shared_run{}, extra{};
+        if (sn) shared_run = jq::SumRun{m->sdown->dev, m->sdown->row_bytes, m->sG, (size_t)sn, sn};
+        if (ex.W) {
+            if (T != 1 || ex.W->type != type || ex.W->n != c.hidden) return fail("moe: a product that does not join this result");
+            extra = jq::SumRun{ex.W->dev, ex.W->row_bytes, ex.mid, ex.W->k, (int)ex.W->k};
+        }
         JQ_ELEM(type, hipLaunchKernelGGL((jq::moe_dense_down<E>), dim3((unsigned)((h + 3) / 4), (unsigned)T), dim3(256), 0, s, m->pdown,
-                                         m->down->row_bytes, m->G, (size_t)inter, m->ids, m->wts, y, inter, h, ku, (int)c.n_expert));
+                                         m->down->row_bytes, m->G, (size_t)inter, m->ids, m->wts, y, inter, h, ku, (int)c.n_expert, shared_run,
+                                         extra, ex.add));
         HIP_TRY(hipGetLastError());
         return 0;
     }
-    if (pre) return fail("moe: no fused norm for %zu tokens", T);
+    if (ex.pre || ex.W) return fail("moe: no fused norm or product for %zu tokens", T);
     const size_t sx = dense_stride(c.hidden), sa = dense_stride(c.inter);
     if (!xe) {
         if (rows_to_elem(type, x, c.hidden, T, h, m->dense_x, sx, s)) return 1;
         xe = m->dense_x;
     }
-    if (moe_route_dev(m, T, x, s, no_groups) || moe_group_dev(m, T, 0, s)) return 1;
+    if ((ex.logits ? gate() : moe_route_dev(m, T, x, s, no_groups)) || moe_group_dev(m, T, 0, s)) return 1;
     const size_t esz = dense_elem_bytes(type), typical = ((size_t)P + c.n_expert - 1) / c.n_expert;
     jq::DenseGemm a{};
     a.A = (const uint8_t *)xe, a.Wp = m->pgate, a.Wp2 = m->pup, a.lda = (uint32_t)(sx * esz), a.ldw = (uint32_t)m->gate->row_bytes;
@@ -318,8 +349,11 @@ int moe_forward_dense(jq_moe *m, size_t T, const float *x, const void *xe, float
     d.M = P, d.N = h, d.C = m->out, d.ldc = (size_t)h;
     d.offsets = m->offsets, d.yrow = m->yrow, d.groups = (int)c.n_expert;
     if (run_gemm<false, true>(type, d, (size_t)P, c.inter, typical, s)) return 1;
-    hipLaunchKernelGGL(jq::moe_combine, dim3((unsigned)std::min<size_t>((T * h + 255) / 256, 4096)), dim3(256), 0, s, m->out, m->wts, (int)T,
-                       ku, h, (const float *)nullptr, y);
+    if (sn && (dense_gemm_gated(m->sgate, m->sup, xe, sx, (int)T, m->dense_sact, dense_stride(sn), shared_unit, s) ||
+               dense_gemm(m->sdown, m->dense_sact, dense_stride(sn), (int)T, m->sOut, h, s)))
+        return 1;
+    hipLaunchKernelGGL(jq::moe_combine_shared, dim3((unsigned)std::min<size_t>((T * h + 255) / 256, 4096)), dim3(256), 0, s, m->out, m->wts,
+                       (int)T, ku, h, sn ? m->sOut : nullptr, sl, ld_sl, ex.add, y);
     HIP_TRY(hipGetLastError());
     return 0;
 }

@@ -15,8 +15,8 @@ int dense_gemv(const jq_weight *w, const float *X, size_t ldx, int T, float *Y, 
                const jq::ResidualNorm *nm = nullptr);
 int dense_gemv_gated(const jq_weight *gate, const jq_weight *up, const float *X, size_t ldx, int T, float *Y, size_t ldy,
                      const jq::GatedUnit &unit, hipStream_t s, const jq::ResidualNorm *nm = nullptr);
-// The same for any T over activations in the weights' type, rows `lda` elements apart (whole runs of 64, zeros behind
-// the k-th); the gated product leaves its activations in that form too.
+// The same for any T over activations in the weights' type, rows `lda` elements apart (whole runs of 64, numbers behind
+// the k-th up to the next whole run); the gated product leaves its activations in that form too.
 int dense_gemm(const jq_weight *w, const void *A, size_t lda, int T, float *C, size_t ldc, hipStream_t s);
 int dense_gemm_gated(const jq_weight *gate, const jq_weight *up, const void *A, size_t lda, int T, void *act, size_t ld_act,
                      const jq::GatedUnit &unit, hipStream_t s);
@@ -31,8 +31,20 @@ int zero_floats(float *p, size_t n, hipStream_t s);
 int rows_to_elem(uint32_t type, const float *X, size_t ldx, size_t rows, int k, void *out, size_t stride, hipStream_t s);
 
 // The layer with BF16 / F32 experts over x [T, hidden] in f32 and, when the caller has them, the same rows in the
-// experts' type (xe, rows dense_stride(hidden) apart).  With `pre` (one token) the router launch makes x: pre->h_out == x.
-int moe_forward_dense(jq_moe *m, size_t T, const float *x, const void *xe, float *y, hipStream_t s, const jq::ResidualNorm *pre = nullptr);
+// experts' type (xe, rows dense_stride(hidden) apart; x may then be null for calls that are not decode-sized).
+struct MoeDenseExtras {
+    const jq::ResidualNorm *pre = nullptr;  // one token: the router launch makes x (pre->h_out == x)
+    // logits made elsewhere, `ld` floats from a token to the next: the router's, and the shared expert's gate
+    const float *logits = nullptr, *shared_logit = nullptr;
+    size_t ld = 0;
+    const float *add = nullptr;             // rows that join the result (may be y)
+    // one token, decode-sized: another product W mid that joins the result
+    const jq_weight *W = nullptr;
+    const float *mid = nullptr;
+};
+int moe_forward_dense(jq_moe *m, size_t T, const float *x, const void *xe, float *y, hipStream_t s, const MoeDenseExtras &ex = MoeDenseExtras());
+// Whether T tokens run on the decode-sized kernels.
+bool moe_dense_decode_sized(const jq_moe *m, size_t T);
 bool moe_dense_fuses_norm(const jq_moe *m, size_t T);
 
 }  // namespace jqh

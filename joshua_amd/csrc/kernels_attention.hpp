@@ -35,6 +35,13 @@ struct AttnLayer {
     float *v_first_out;      // where this layer's own values go, or null
     float lambda;
     void *kc, *vc;
+    // what the kernels for steps of many tokens know beside this
+    const float *sink;       // [H]: exp(sink) joins the softmax's denominator; or null
+    const float *gate;       // [T][ld_gate]: the outputs are multiplied by its sigmoid; or null
+    size_t ld_gate;
+    __device__ __forceinline__ float gated(float v, int t, int col) const {  // col within [0, H dv)
+        return gate ? v * sigmoid_of(gate[t * ld_gate + col]) : v;
+    }
 };
 
 // Elements 2i and 2i + 1 of a head as rotated.
@@ -133,6 +140,7 @@ __global__ __launch_bounds__(256) void attention_any(AttnLayer a, const typename
         }
         __syncthreads();
     }
+    if (a.sink) l_run += expf(a.sink[h] - m_run);
     O *op = out + (size_t)t * ldo + (size_t)h * a.dv;
 #pragma unroll
     for (int i = 0; i < ANY_MAX_DV / 256; i++) {
@@ -141,7 +149,7 @@ __global__ __launch_bounds__(256) void attention_any(AttnLayer a, const typename
         if (tid < cols && tid + 256 * i < a.dv) {
             float v = 0.0f;
             for (int p = 0; p < parts; p++) v += sums[p * cols + tid];
-            op[tid + 256 * i] = (O)(v / l_run);
+            op[tid + 256 * i] = (O)a.gated(v / l_run, t, h * a.dv + tid + 256 * i);
         }
         __syncthreads();
     }
@@ -449,14 +457,19 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
 #pragma unroll
     for (int q = 0; q < QF; q++) {
         const int r = r0 + (wave * QF + q) * 16 + n;
-        const float inv = 1.0f / sum_xor32(sum_xor16(sum[q]));
+        float total = sum_xor32(sum_xor16(sum[q]));
         if (r >= rows) continue;
-        __bf16 *op = out + (size_t)(r / gq) * ldo + (size_t)(kvh * gq + r % gq) * a.dv;
+        const int t = r / gq, h = kvh * gq + r % gq;
+        if (a.sink) total += __builtin_amdgcn_exp2f(fmaf(a.sink[h], 1.44269504088896341f, -mx[q]));
+        const float inv = 1.0f / total;
+        __bf16 *op = out + (size_t)t * ldo + (size_t)h * a.dv;
 #pragma unroll
         for (int d = 0; d < DT; d++)
 #pragma unroll
-            for (int e = 0; e < 4; e++)
-                if (16 * d + 4 * g + e < a.dv) op[16 * d + 4 * g + e] = (__bf16)(o[q][d][e] * inv);
+            for (int e = 0; e < 4; e++) {
+                const int c = 16 * d + 4 * g + e;
+                if (c < a.dv) op[c] = (__bf16)a.gated(o[q][d][e] * inv, t, h * a.dv + c);
+            }
     }
 }
 

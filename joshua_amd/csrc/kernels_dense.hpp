@@ -232,6 +232,19 @@ __global__ __launch_bounds__(64 * WAVES) void norm_gemv(const uint8_t *__restric
     }
 }
 
+// The shared expert beside a decode-sized call's pairs: rows pairs .. pairs + T - 1 of the gate|up grid.
+struct SharedRows {
+    const uint8_t *gate, *up;  // null: none
+    int n;                     // its activations a token
+    float *act;                // [T][n]
+    const float *logit;        // token t's activations are multiplied by sigmoid(logit[t ld]); null: left alone
+    size_t ld;
+    int pairs;
+    float limit;               // its own clamp
+};
+
+__device__ __forceinline__ float sigmoid_of(float z) { return 1.0f / (1.0f + expf(-z)); }
+
 // The experts' gated pairs of a decode-sized call: blockIdx.y is the (token, slot) pair, four j a workgroup, every
 // weight row read once a pair.  NE > 0: the workgroup's first wave runs the token's gating over the router's logits
 // (moe_gate_topk_wave's arithmetic); the first workgroup of a token's first pair writes ids and weights for the
@@ -240,13 +253,17 @@ template <class E, int NE>
 __global__ __launch_bounds__(256) void moe_dense_gate_up(const uint8_t *const *__restrict__ Wg, const uint8_t *const *__restrict__ Wu,
                                                          size_t pitch, const float *__restrict__ X, size_t ldx,
                                                          float *__restrict__ Y, size_t ldy, int k, int n, int k_used,
-                                                         const uint32_t *__restrict__ ids, GatedUnit act, MoeGateIn gi) {
+                                                         const uint32_t *__restrict__ ids, GatedUnit act, MoeGateIn gi, SharedRows sh) {
     constexpr int R = 8;
     __shared__ float red[4][R], sums[R];
     __shared__ int expert;
-    const int pair = blockIdx.y, t = pair / k_used, slot = pair % k_used;
-    int e;
-    if constexpr (NE > 0) {
+    const bool shared = (int)blockIdx.y >= sh.pairs;  // (the workgroup agrees)
+    const int pair = shared ? (int)blockIdx.y - sh.pairs : (int)blockIdx.y, t = shared ? pair : pair / k_used, slot = pair % k_used;
+    if (shared) Y = sh.act, ldy = (size_t)sh.n, n = sh.n, act.limit = sh.limit;
+    if (R / 2 * (int)blockIdx.x >= n) return;  // (the grid is as wide as the wider of the two)
+    int e = 0;
+    if (shared) {
+    } else if constexpr (NE > 0) {
         if (threadIdx.x < 64) {
             int slot_e;
             moe_gate_topk_wave_body<NE>(t, gi.T, (int)threadIdx.x, gi.logits, gi.bias, gi.p, gi.ids, gi.wts, gi.pg,
@@ -262,38 +279,63 @@ __global__ __launch_bounds__(256) void moe_dense_gate_up(const uint8_t *const *_
     const int j0 = (R / 2) * (int)blockIdx.x;
     const uint8_t *rows[R];
 #pragma unroll
-    for (int r = 0; r < R; r++) rows[r] = (r & 1 ? Wu : Wg)[e] + (size_t)min(j0 + (r >> 1), n - 1) * pitch;
+    for (int r = 0; r < R; r++)
+        rows[r] = (shared ? (r & 1 ? sh.up : sh.gate) : (r & 1 ? Wu : Wg)[e]) + (size_t)min(j0 + (r >> 1), n - 1) * pitch;
     float acc[1][R] = {};
     gemv_accumulate<E, 1, R>(rows, X + (size_t)t * ldx, 0, 1, k, acc);
     const float s = gemv_reduce<R>(acc[0], red);
     if (threadIdx.x < R) sums[threadIdx.x] = s;
     __syncthreads();
     const int j = (int)threadIdx.x;
-    if (j < R / 2 && j0 + j < n) Y[(size_t)pair * ldy + j0 + j] = act(sums[2 * j], sums[2 * j + 1]);
+    if (j < R / 2 && j0 + j < n) {
+        const float v = act(sums[2 * j], sums[2 * j + 1]);
+        Y[(size_t)pair * ldy + j0 + j] = shared && sh.logit ? sigmoid_of(sh.logit[t * sh.ld]) * v : v;
+    }
 }
 
-// y[t, :] = sum over the token's slots of weight * (W_down[expert] act[pair]): down projections and combine of a
+// A product that joins a sum of products: + W[n, :] . x[t, :].
+struct SumRun {
+    const uint8_t *W;   // null: none
+    size_t pitch;
+    const float *x;
+    size_t ldx;
+    int k;
+};
+
+// y[t, :] = sum over the token's slots of weight * (W_down[expert] act[pair]), plus two runs of their own (a shared
+// expert's down projection, the mixer's output projection) and the row `add`: down projections and combine of a
 // decode-sized call.  Four rows a workgroup; its threads share the (slot, chunk) list.
 template <class E>
 __global__ __launch_bounds__(256) void moe_dense_down(const uint8_t *const *__restrict__ Wd, size_t pitch,
                                                       const float *__restrict__ A, size_t lda, const uint32_t *__restrict__ ids,
-                                                      const float *__restrict__ wts, float *__restrict__ y, int k, int n,
-                                                      int k_used, int n_expert) {
+                                                      const float *__restrict__ wts, float *y, int k, int n,
+                                                      int k_used, int n_expert, SumRun run1, SumRun run2, const float *add) {
     constexpr int R = 4;
     __shared__ float red[4][R];
     const int t = blockIdx.y, r0 = R * (int)blockIdx.x;
     const int per = (k + E::CH - 1) / E::CH, total = per * k_used;
+    const int per1 = run1.W ? (run1.k + E::CH - 1) / E::CH : 0, per2 = run2.W ? (run2.k + E::CH - 1) / E::CH : 0;
     float acc[R] = {};
 #pragma unroll 2
-    for (int i = threadIdx.x; i < total; i += 256) {
-        const int slot = i / per, c = (i % per) * E::CH, pair = t * k_used + slot;
-        const uint8_t *base = Wd[min((int)ids[pair], n_expert - 1)];
-        const float wt = wts[pair];
+    for (int i = threadIdx.x; i < total + per1 + per2; i += 256) {
+        const uint8_t *base;
+        const float *x;
+        size_t pt = pitch;
+        int c, kk = k;
+        float wt = 1.0f;
+        if (i < total) {
+            const int slot = i / per, pair = t * k_used + slot;
+            c = (i % per) * E::CH, base = Wd[min((int)ids[pair], n_expert - 1)], x = A + (size_t)pair * lda, wt = wts[pair];
+        } else {
+            const bool first = i < total + per1;
+            c = (i - total - (first ? 0 : per1)) * E::CH, base = first ? run1.W : run2.W, pt = first ? run1.pitch : run2.pitch;
+            x = first ? run1.x + t * run1.ldx : run2.x + t * run2.ldx, kk = first ? run1.k : run2.k;
+        }
         u32x4 w[R];
 #pragma unroll
-        for (int r = 0; r < R; r++) w[r] = chunk_of<E>(base + (size_t)min(r0 + r, n - 1) * pitch, c);
+        for (int r = 0; r < R; r++) w[r] = chunk_of<E>(base + (size_t)min(r0 + r, n - 1) * pt, c);
         float xv[E::CH];
-        load_acts<E::CH>(A + (size_t)pair * lda, c, k, xv);
+        load_acts<E::CH>(x, c, kk, xv);
 #pragma unroll
         for (int r = 0; r < R; r++) {
             float wv[E::CH], d = 0.0f;
@@ -304,7 +346,25 @@ __global__ __launch_bounds__(256) void moe_dense_down(const uint8_t *const *__re
         }
     }
     const float s = gemv_reduce<R>(acc, red);
-    if (threadIdx.x < R && r0 + (int)threadIdx.x < n) y[(size_t)t * n + r0 + threadIdx.x] = s;
+    if (threadIdx.x < R && r0 + (int)threadIdx.x < n) {
+        const size_t at = (size_t)t * n + r0 + threadIdx.x;
+        y[at] = add ? add[at] + s : s;
+    }
+}
+
+// y[t, :] = sum over the slots of weight * out[pair, :], plus the shared expert's rows times sigmoid(logit[t ld]) (logit
+// null: as they are) and the rows `add` (may be y).
+static __global__ __launch_bounds__(256) void moe_combine_shared(const float *__restrict__ out, const float *__restrict__ wts, int T, int k_used,
+                                                                 int h, const float *__restrict__ shared, const float *__restrict__ logit,
+                                                                 size_t ld, const float *add, float *y) {
+    const size_t total = (size_t)T * h;
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
+        const size_t t = i / h, c = i % h;
+        float acc = add ? add[i] : 0.0f;
+        for (int s = 0; s < k_used; s++) acc = fmaf(out[(t * k_used + s) * h + c], wts[t * k_used + s], acc);
+        if (shared) acc = fmaf(shared[i], logit ? sigmoid_of(logit[t * ld]) : 1.0f, acc);
+        y[i] = acc;
+    }
 }
 
 // ---- GEMM -----------------------------------------------------------------------------------------

@@ -208,6 +208,8 @@ struct MoeGateParams {
     int norm_topk;    // divide the k weights by their sum (clamped below at 2^-14)
     float scale;      // multiply the weights (0 or 1: leave alone)
     int n_group, topk_group;
+    int ld;           // floats from a token's logits to the next token's (0: E)
+    __host__ __device__ size_t logits_at(int t) const { return (size_t)t * (ld ? ld : E); }
     // softmax only: the bias is part of the logits (and so of the weights) instead of the selection alone
     __host__ __device__ bool logit_bias() const { return sigmoid == 2; }
     __host__ __device__ bool is_sigmoid() const { return sigmoid == 1; }
@@ -233,7 +235,7 @@ static __global__ __launch_bounds__(256) void moe_gate_topk(const float *__restr
     float *red = selw + p.k_used;
     const int t = blockIdx.x, lane = threadIdx.x, wv = threadIdx.x >> 6;  // `lane` strides the experts by 256
     constexpr int NT = 256;
-    const float *lg = logits + (size_t)t * p.E;
+    const float *lg = logits + p.logits_at(t);
     if (p.is_sigmoid()) {
         for (int e = lane; e < p.E; e += NT) probs[e] = 1.0f / (1.0f + expf(-lg[e]));
     } else {
@@ -343,7 +345,7 @@ __device__ __forceinline__ void moe_gate_topk_wave_body(int t, int T, int lane, 
                                                         const float *__restrict__ bias, const MoeGateParams &p,
                                                         uint32_t *__restrict__ ids, float *__restrict__ wts,
                                                         const MoePairGroups &pg, bool write, int *slot_e) {
-    const float *lg = logits + (size_t)t * p.E;
+    const float *lg = logits + p.logits_at(t);
     float prob[NE], sel[NE];
     {
         float v[NE];

@@ -6,7 +6,7 @@
 namespace jq {
 
 struct ResidualNorm {
-    const float *x;                    // the residual stream, rows `width` apart
+    const float *x;                    // the residual stream
     const float *y;                    // the sublayer's result to add, or null
     const float *post_w, *post_b;      // the norm on y (post_w null: y as it is)
     float mult;
@@ -14,6 +14,7 @@ struct ResidualNorm {
     float eps;
     int rms;                           // both norms: 1 root mean square, 0 mean and variance (with bias)
     int width;
+    size_t ldx;                        // x: from a row to the next (0: width)
     float *x_out;                      // may be x, except where other workgroups read the row
     float *h_out;                      // or null
 };
@@ -131,7 +132,7 @@ __global__ __launch_bounds__(BT) void residual_norm_rows(ResidualNorm a, typenam
     __shared__ float red[4 * NW];
     const int w = a.width, c0 = threadIdx.x;
     const size_t row = at ? at[blockIdx.x] : blockIdx.x;
-    const float *xr = a.x + row * w;
+    const float *xr = a.x + row * (a.ldx ? a.ldx : (size_t)w);
     float x[NV];
     auto stats = [&](const float (&v)[NV], float *r, float *mean, float *inv) __attribute__((always_inline)) {
         float mu = 0.0f, ss = 0.0f;

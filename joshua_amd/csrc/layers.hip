@@ -1,9 +1,11 @@
-// Layered decoders with plain BF16 / F32 weights: a stack whose layers each name a mixer (attention, selective scan)
-// and a feed-forward block (none, dense, mixture of experts), normalised in front and behind.  A design is a reader of
-// its configuration into StackConfig plus its tensor names; the step below runs any of them.
+// Layered decoders with plain BF16 / F32 weights: a stack whose layers each name a mixer (attention, selective scan,
+// latent attention, matrix memory, linear attention with a constant decay) and a feed-forward block (none, dense, mixture
+// of experts).  Mixer and block run one behind the other, each normalised in front and behind, or side by side on one
+// norm; a run of layers may repeat.  A design is a reader of its configuration into StackConfig plus its tensor names;
+// the step below runs any of them.
 #include "dense.hpp"
-#include "kernels_attention.hpp"
-#include "kernels_ssm.hpp"
+#include "kernels_latent.hpp"
+#include "kernels_linear.hpp"
 #include "model.hpp"
 #include "safetensors.hpp"
 
@@ -22,18 +24,27 @@ struct RotaryConfig {
 };
 
 struct LayerConfig {
-    enum Mixer { ATTENTION, MAMBA1 } mixer = ATTENTION;
-    // attention
+    enum Mixer { ATTENTION, MAMBA1, LATENT, MLSTM, LIGHTNING } mixer = ATTENTION;
+    // attention of every kind
     int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
     float scale = 1.0f;
     bool v_mix = false;
     RotaryConfig rot;
+    int q_rank = 0, kv_rank = 0, rot_dim = 0;  // latent attention
+    float gate_cap = 0.0f;                     // matrix memory
+    std::vector<double> decay;                 // constant decay, one a head
     // selective scan
     int inner = 0, state = 0, dt_rank = 0, taps = 0;
     // feed-forward
     enum Mlp { NONE, DENSE, MOE } mlp = NONE;
-    int ff = 0, experts = 0, top = 0;
+    int ff = 0, experts = 0, top = 0, shared_ff = 0;
     float limit = INFINITY;
+
+    bool linear() const { return mixer == MLSTM || mixer == LIGHTNING; }
+    int state_rows() const { return vdim + (mixer == MLSTM ? 1 : 0); }  // of a head of a linear mixer
+    int state_pitch() const { return (dim + 3) / 4 * 4; }
+    int out_pitch() const { return (state_rows() + 3) / 4 * 4; }
+    int latent_pitch() const { return (int)dense_stride(kv_rank + rot_dim); }
 };
 
 struct StackConfig {
@@ -42,6 +53,8 @@ struct StackConfig {
     float embedding_scale = 1.0f, norm_eps = 1e-6f, residual_mult = 1.0f;
     bool rms = false;                         // norms: root mean square instead of mean and variance with bias
     float act_alpha = 1.0f, act_shift = 0.0f;  // the gated unit: g sigmoid(alpha g) (u + shift)
+    bool parallel = false;                    // x + (mixer(h) + block(h)) with h = norm1(x): one norm a layer
+    int loop_start = 0, loop_stop = 0, loop_times = 1;  // layers start .. stop - 1 run that often in a row
     std::vector<LayerConfig> layers;
 };
 
@@ -76,12 +89,17 @@ struct Layer {
     float lambda = 0.0f;
     bool v_first = false;      // the first layer that mixes values: the others mix in its own
     int rot = -1;              // which of the model's rotary tables
-    void *kc = nullptr, *vc = nullptr;
+    // latent attention
+    jq_weight *uq = nullptr, *ukv = nullptr;  // ukv: W_uk's rows, then W_uv's
+    float *dq_norm = nullptr, *dkv_norm = nullptr, *sink = nullptr;
+    // linear mixers
+    float *i_b = nullptr, *f_b = nullptr, *decay = nullptr, *log_decay = nullptr;
+    float *mix_norm = nullptr;
     // selective scan
     jq_weight *wx = nullptr, *wdt = nullptr;
     float *conv = nullptr, *conv_b = nullptr, *dt_b = nullptr, *A_log2 = nullptr, *D = nullptr;
-    float *S = nullptr, *tail[2] = {nullptr, nullptr};
-    int tail_at = 0;
+    // places within a row of `in`'s product: the mixer's output gate, the router with the shared expert's gate behind it
+    int gate_at = 0, router_at = 0;
     // feed-forward
     jq_weight *gate = nullptr, *up = nullptr, *down = nullptr;
     jq_moe *moe = nullptr;
@@ -89,9 +107,20 @@ struct Layer {
     // this layer's activation buffers (shared between layers of equal size)
     void *mix_e = nullptr, *conv_e = nullptr, *dt_e = nullptr, *ff_e = nullptr;
 
-    int DP() const { return (c.dim + 31) / 32 * 32; }
+    int DP() const { return (c.dim + c.rot_dim + 31) / 32 * 32; }
     int DVP() const { return (c.vdim + 31) / 32 * 32; }
-    int mix_width() const { return c.mixer == LayerConfig::ATTENTION ? c.heads * c.vdim : c.inner; }
+    int mix_width() const { return c.mixer == LayerConfig::MAMBA1 ? c.inner : c.heads * c.vdim; }
+};
+
+// One run of a layer within a step, with the cache or state that is its own.
+struct LayerRun {
+    int layer = 0;
+    void *kc = nullptr, *vc = nullptr;  // attention; latent attention: kc holds the rows
+    float *S = nullptr;                 // selective scan, linear mixers
+    size_t S_floats = 0;
+    float *tail[2] = {nullptr, nullptr};  // the scan's convolution, the matrix memory's running maxima: two taking turns
+    size_t tail_floats = 0;
+    int tail_at = 0;
 };
 
 struct RotaryTable {
@@ -105,25 +134,27 @@ struct LayeredModel : jq_model {
     StackConfig cfg;
     uint32_t type = JQ_TYPE_BF16;  // of the matrices, the caches and a many-token step's activations
     std::vector<Layer> layers;
+    std::vector<LayerRun> runs;
     std::vector<RotaryTable> rots;
     jq_weight *embed = nullptr, *head = nullptr;
     NormWeights final_norm;
     std::vector<void *> owned;     // weights and states in device memory
     std::vector<jq_weight *> matrices;
-    // scratch for cap_tokens tokens and cap_want wanted rows
-    size_t cap_tokens = 0, cap_want = 0;
+    // scratch for cap_tokens tokens, cap_want wanted rows and keys and values of cap_keys tokens out of latents
+    size_t cap_tokens = 0, cap_want = 0, cap_keys = 0;
     std::vector<void *> scratch;
     uint32_t *ids = nullptr, *want_ids = nullptr;
     float *x = nullptr, *x2 = nullptr, *h = nullptr, *y = nullptr, *proj = nullptr, *mid = nullptr, *conv_f = nullptr, *bc = nullptr,
-          *dt = nullptr, *first_v = nullptr, *part = nullptr;
-    void *h_e = nullptr, *q_e = nullptr;
+          *dt = nullptr, *first_v = nullptr, *part = nullptr, *lin_o = nullptr, *lin_m = nullptr, *cq = nullptr, *qf = nullptr,
+          *qx = nullptr, *olat = nullptr, *kv = nullptr;
+    void *h_e = nullptr, *q_e = nullptr, *cq_e = nullptr, *k_e = nullptr, *v_e = nullptr;
     std::vector<int> moe_holder;   // per layer index of the first of its size: which layer holds the scratch now
     bool broken = false;           // a step failed half way: the states are those of no sequence
 
     ~LayeredModel() override;
     int step(const uint32_t *tokens, uint32_t n, const uint32_t *want, uint32_t n_want, hipStream_t s) override;
     void forget() override { broken = false; }
-    int reserve(size_t T, size_t W);
+    int reserve(size_t T, size_t W, size_t keys);
     int run_layers(int T, const uint32_t *want, int n_want, hipStream_t s);
     size_t esz() const { return dense_elem_bytes(type); }
 
@@ -149,12 +180,14 @@ LayeredModel::~LayeredModel() {
     free_all(&owned);
 }
 
-int LayeredModel::reserve(size_t T, size_t W) {
-    if (T <= cap_tokens && W <= cap_want) return 0;
+int LayeredModel::reserve(size_t T, size_t W, size_t keys) {
+    if (T <= cap_tokens && W <= cap_want && keys <= cap_keys) return 0;
     T = std::max(T, cap_tokens), W = std::max(W, cap_want);
+    keys = keys <= cap_keys ? cap_keys : std::min<size_t>(n_ctx, std::max(keys, 2 * cap_keys));  // (grows in few steps)
     free_all(&scratch);
-    cap_tokens = cap_want = 0;
-    size_t proj_w = 0, mid_w = 0, inner_w = 0, bc_w = 0, v_w = 0, part_w = 0, q_w = 0;
+    cap_tokens = cap_want = cap_keys = 0;
+    size_t proj_w = 0, mid_w = 0, inner_w = 0, bc_w = 0, v_w = 0, part_w = 0, q_w = 0, lin_w = 0, head_w = 0, cq_w = 0, qf_w = 0, qx_w = 0,
+           olat_w = 0, kv_w = 0, k_w = 0, ve_w = 0;
     for (const Layer &l : layers) {
         const LayerConfig &c = l.c;
         proj_w = std::max(proj_w, l.in->n);
@@ -163,6 +196,14 @@ int LayeredModel::reserve(size_t T, size_t W) {
             q_w = std::max(q_w, (size_t)c.heads * l.DP());
             if (c.v_mix) v_w = std::max(v_w, (size_t)c.kv_heads * c.vdim);
             part_w = std::max(part_w, (size_t)c.heads * ((n_ctx + jq::ATT_CHUNK - 1) / jq::ATT_CHUNK) * (c.vdim + 2));
+        } else if (c.mixer == LayerConfig::LATENT) {
+            const size_t H = c.heads;
+            q_w = std::max(q_w, H * l.DP()), cq_w = std::max(cq_w, (size_t)c.q_rank), qf_w = std::max(qf_w, l.uq->n);
+            qx_w = std::max(qx_w, H * c.latent_pitch()), olat_w = std::max(olat_w, H * c.kv_rank);
+            part_w = std::max(part_w, H * jq::LAT_MAX_SPLIT * (c.kv_rank + 2));
+            kv_w = std::max(kv_w, l.ukv->n), k_w = std::max(k_w, H * l.DP()), ve_w = std::max(ve_w, H * l.DVP());
+        } else if (c.linear()) {
+            lin_w = std::max(lin_w, (size_t)c.heads * c.out_pitch()), head_w = std::max(head_w, (size_t)c.heads);
         } else {
             inner_w = std::max(inner_w, (size_t)c.inner);
             bc_w = std::max(bc_w, l.wx->n);
@@ -181,13 +222,21 @@ int LayeredModel::reserve(size_t T, size_t W) {
     const size_t w = cfg.width, R = std::max(T, W);
     if (get(&ids, T) || get(&want_ids, W) || get(&x, T * w) || get(&x2, w) || get(&h, R * w) || get(&y, T * w) || get(&proj, T * proj_w) ||
         get(&mid, (size_t)GEMV_MAX_ROWS * mid_w) || get(&conv_f, (size_t)GEMV_MAX_ROWS * inner_w) || get(&bc, T * bc_w) ||
-        get(&dt, T * inner_w) || get(&first_v, T * v_w) || get(&part, (size_t)GEMV_MAX_ROWS * part_w))
+        get(&dt, T * inner_w) || get(&first_v, T * v_w) || get(&part, (size_t)GEMV_MAX_ROWS * part_w) || get(&lin_o, T * lin_w) ||
+        get(&lin_m, T * head_w) || get(&cq, (size_t)GEMV_MAX_ROWS * cq_w) || get(&qf, T * qf_w) || get(&qx, (size_t)GEMV_MAX_ROWS * qx_w) ||
+        get(&olat, (size_t)GEMV_MAX_ROWS * olat_w) || get(&kv, keys * kv_w))
         return 1;
     uint8_t *p = nullptr;
     if (get(&p, R * dense_stride(w) * esz())) return 1;
     h_e = p;
     if (get(&p, T * q_w * esz())) return 1;
     q_e = p;
+    if (get(&p, T * dense_stride(cq_w) * esz())) return 1;
+    cq_e = p;
+    if (get(&p, keys * k_w * esz())) return 1;
+    k_e = p;
+    if (get(&p, keys * ve_w * esz())) return 1;
+    v_e = p;
     for (RotaryTable &r : rots)
         if (get(&r.cs, T * (r.c.dims / 2))) return 1;
     std::map<std::pair<int, size_t>, void *> by_size;  // (role, row length)
@@ -206,13 +255,15 @@ int LayeredModel::reserve(size_t T, size_t W) {
         if (l.c.mixer == LayerConfig::MAMBA1 && (rows(1, l.c.inner, &l.conv_e) || rows(2, l.c.dt_rank, &l.dt_e))) return 1;
         if (l.c.mlp == LayerConfig::DENSE && rows(3, l.c.ff, &l.ff_e)) return 1;
     }
-    cap_tokens = T, cap_want = W;
+    cap_tokens = T, cap_want = W, cap_keys = keys;
     return 0;
 }
 
 int LayeredModel::step(const uint32_t *tokens, uint32_t n, const uint32_t *want, uint32_t n_want, hipStream_t s) {
     if (broken) return fail("%s: an earlier step failed half way; reset the model", arch);
-    if (reserve(n, std::max<uint32_t>(n_want, 1))) return 1;
+    bool latent = false;
+    for (const Layer &l : layers) latent |= l.c.mixer == LayerConfig::LATENT;
+    if (reserve(n, std::max<uint32_t>(n_want, 1), latent && n > (uint32_t)GEMV_MAX_ROWS ? n_past + n : 0)) return 1;
     HIP_TRY(hipMemcpyAsync(ids, tokens, n * sizeof(uint32_t), hipMemcpyHostToDevice, s));
     if (n_want && n > 1) HIP_TRY(hipMemcpyAsync(want_ids, want, n_want * sizeof(uint32_t), hipMemcpyHostToDevice, s));
     broken = true;
@@ -233,27 +284,11 @@ int LayeredModel::step(const uint32_t *tokens, uint32_t n, const uint32_t *want,
         }                                                      \
     } while (0)
 
-// The attention of one layer over its projections a.qkv.  Steps of up to 8 tokens leave f32 rows in out_f, longer
-// ones rows of the element type in out_e.
-int run_attention(LayeredModel *m, Layer &l, const jq::AttnLayer &a, bool small, float *out_f, void *out_e, hipStream_t s) {
+// Attention of the queries in q_e over the keys and values in a.kc and a.vc.
+int run_attention_rows(LayeredModel *m, const jq::AttnLayer &a, bool small, float *out_f, void *out_e, hipStream_t s) {
     const uint32_t type = m->type;
     const int dc = std::max(a.DP, a.DVP), gq = a.H / a.G, T = a.T;
     const size_t ldo = dense_stride((size_t)a.H * a.dv);
-    if (small && dc <= 256) {
-        const int n_chunks = (a.pos0 + T + jq::ATT_CHUNK - 1) / jq::ATT_CHUNK;
-        // a query head a workgroup until there are four for every compute unit, then more
-        const int per = std::min({gq, jq::DEC_HEADS, std::max(1, n_chunks * a.G * gq * T / 1024)}), runs = (gq + per - 1) / per;
-        const dim3 grid((unsigned)((n_chunks * a.G + 7) / 8 * 8 * runs), (unsigned)T);
-#define JQ_DEC(DC) JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attention_decode<E, DC>), grid, dim3(256), 0, s, a, n_chunks, per, m->part))
-        if (dc <= 64) JQ_DEC(64);
-        else if (dc <= 128) JQ_DEC(128);
-        else JQ_DEC(256);
-#undef JQ_DEC
-        hipLaunchKernelGGL(jq::attention_merge, dim3((unsigned)(T * a.H)), dim3(128), 2 * n_chunks * sizeof(float), s, m->part, out_f, a.dv,
-                           n_chunks);
-        return 0;
-    }
-    JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attn_rope_store<E>), dim3((unsigned)T), dim3(256), 0, s, a, (typename E::T *)m->q_e));
     if (type == JQ_TYPE_BF16 && dc <= 256 && !small && a.scale > 0.0f) {
         const float sl = a.scale * 1.44269504088896341f;
         const size_t rows = (size_t)T * gq;
@@ -281,6 +316,29 @@ int run_attention(LayeredModel *m, Layer &l, const jq::AttnLayer &a, bool small,
     return 0;
 }
 
+// The attention of one layer over its projections a.qkv.  Steps of up to 8 tokens leave f32 rows in out_f, longer
+// ones rows of the element type in out_e.
+int run_attention(LayeredModel *m, Layer &l, const jq::AttnLayer &a, bool small, float *out_f, void *out_e, hipStream_t s) {
+    const uint32_t type = m->type;
+    const int dc = std::max(a.DP, a.DVP), gq = a.H / a.G, T = a.T;
+    if (small && dc <= 256) {
+        const int n_chunks = (a.pos0 + T + jq::ATT_CHUNK - 1) / jq::ATT_CHUNK;
+        // a query head a workgroup until there are four for every compute unit, then more
+        const int per = std::min({gq, jq::DEC_HEADS, std::max(1, n_chunks * a.G * gq * T / 1024)}), runs = (gq + per - 1) / per;
+        const dim3 grid((unsigned)((n_chunks * a.G + 7) / 8 * 8 * runs), (unsigned)T);
+#define JQ_DEC(DC) JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attention_decode<E, DC>), grid, dim3(256), 0, s, a, n_chunks, per, m->part))
+        if (dc <= 64) JQ_DEC(64);
+        else if (dc <= 128) JQ_DEC(128);
+        else JQ_DEC(256);
+#undef JQ_DEC
+        hipLaunchKernelGGL(jq::attention_merge, dim3((unsigned)(T * a.H)), dim3(128), 2 * n_chunks * sizeof(float), s, m->part, out_f, a.dv,
+                           n_chunks);
+        return 0;
+    }
+    JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::attn_rope_store<E>), dim3((unsigned)T), dim3(256), 0, s, a, (typename E::T *)m->q_e));
+    return run_attention_rows(m, a, small, out_f, out_e, s);
+}
+
 template <class IO>
 int run_scan(const jq::SsmScan &a, const IO *x, IO *out, hipStream_t s) {
 #define JQ_SCAN(LPC, NS)                                                                                                            \
@@ -297,6 +355,123 @@ int run_scan(const jq::SsmScan &a, const IO *x, IO *out, hipStream_t s) {
     return 0;
 }
 
+// The linear mixers: kernels_linear.hpp over the projections, then the norm and gate of the heads' outputs.
+int run_linear(LayeredModel *m, const Layer &l, LayerRun &r, int T, bool small, hipStream_t s) {
+    const LayerConfig &c = l.c;
+    jq::LinearLayer a{};
+    a.H = c.heads, a.d = c.dim, a.dv = c.vdim, a.rows = c.state_rows(), a.DP = c.state_pitch(), a.memory = c.mixer == LayerConfig::MLSTM;
+    a.T = T, a.proj = m->proj, a.ld = l.in->n, a.q_at = 0, a.k_at = c.heads * c.dim, a.v_at = 2 * a.k_at;
+    a.i_at = l.gate_at + c.heads * c.vdim, a.f_at = a.i_at + c.heads;
+    a.q_scale = a.memory ? 1.0f / std::sqrt((float)c.dim) : 1.0f, a.cap = c.gate_cap, a.i_b = l.i_b, a.f_b = l.f_b;
+    a.decay = l.decay, a.log_decay = l.log_decay, a.S = r.S, a.m_in = r.tail[r.tail_at], a.m_out = r.tail[r.tail_at ^ 1];
+    a.o = m->lin_o, a.OP = c.out_pitch(), a.mt = m->lin_m;
+#define JQ_STEPS(LPR, NS)                                                                                                             \
+    hipLaunchKernelGGL((jq::linear_steps<LPR, NS>), dim3((unsigned)((a.rows + 256 / LPR - 1) / (256 / LPR)), (unsigned)a.H), dim3(256), 0, s, a)
+    if (a.d <= 16) JQ_STEPS(4, 1);
+    else if (a.d <= 32) JQ_STEPS(8, 1);
+    else if (a.d <= 64) JQ_STEPS(16, 1);
+    else if (a.d <= 128) JQ_STEPS(16, 2);
+    else if (a.d <= 256) JQ_STEPS(16, 4);
+    else if (a.d <= 512) JQ_STEPS(32, 4);
+    else JQ_STEPS(64, 4);
+#undef JQ_STEPS
+    if (a.memory) r.tail_at ^= 1;
+    jq::LinearNorm n{};
+    n.o = m->lin_o, n.mt = m->lin_m, n.H = a.H, n.dv = a.dv, n.OP = a.OP, n.memory = n.per_head = a.memory, n.w = l.mix_norm;
+    n.gate = m->proj + l.gate_at, n.ld = a.ld, n.eps = m->cfg.norm_eps;
+    const int len = n.per_head ? a.dv : a.H * a.dv;
+    const dim3 grid((unsigned)(n.per_head ? T * a.H : T));
+#define JQ_NORM(BT)                                                                                                                    \
+    do {                                                                                                                               \
+        if (small) hipLaunchKernelGGL((jq::linear_norm_gate<float, BT>), grid, dim3(BT), 0, s, n, m->mid, (size_t)l.mix_width());       \
+        else JQ_ELEM_OF(m->type, hipLaunchKernelGGL((jq::linear_norm_gate<typename E::T, BT>), grid, dim3(BT), 0, s, n,                 \
+                                                    (typename E::T *)l.mix_e, dense_stride(l.mix_width())));                           \
+    } while (0)
+    if (len <= 256) JQ_NORM(64);
+    else if (len <= 2048) JQ_NORM(256);
+    else JQ_NORM(1024);
+#undef JQ_NORM
+    return 0;
+}
+
+int run_latent(LayeredModel *m, const Layer &l, const LayerRun &r, int pos0, int T, bool small, hipStream_t s) {
+    const LayerConfig &c = l.c;
+    const uint32_t type = m->type;
+    const size_t sq = dense_stride(c.q_rank), ld = l.in->n;
+    jq::LatentLayer a{};
+    a.H = c.heads, a.d = c.dim, a.rd = c.rot_dim, a.dv = c.vdim, a.R = c.kv_rank, a.RP = c.latent_pitch(), a.n_ctx = (int)m->n_ctx;
+    a.rot = c.rot.dims, a.pos0 = pos0, a.T = T, a.scale = c.scale, a.eps = m->cfg.norm_eps, a.q = m->qf, a.down = m->proj + c.q_rank, a.ld = ld;
+    a.cs = l.rot >= 0 ? m->rots[l.rot].cs : nullptr, a.norm_w = l.dkv_norm, a.sink = l.sink, a.gate = m->proj + l.gate_at, a.cache = r.kc;
+    // the queries, through their normed latent (the first numbers of a projection row)
+    jq::ResidualNorm nm{};
+    nm.x = m->proj, nm.ldx = ld, nm.pre_w = l.dq_norm, nm.eps = m->cfg.norm_eps, nm.rms = 1, nm.width = c.q_rank;
+    if (T == 1 && c.q_rank <= FUSED_NORM_MAX_WIDTH) {
+        if (dense_gemv(l.uq, nullptr, 0, 1, m->qf, l.uq->n, s, &nm)) return 1;
+    } else if (small) {
+        nm.h_out = m->cq;
+        if (residual_norm(nm, type, nullptr, 0, T, nullptr, s) || dense_gemv(l.uq, m->cq, c.q_rank, T, m->qf, l.uq->n, s)) return 1;
+    } else if (residual_norm(nm, type, m->cq_e, sq, T, nullptr, s) || dense_gemm(l.uq, m->cq_e, sq, T, m->qf, l.uq->n, s)) {
+        return 1;
+    }
+    if (small) {
+        const size_t pitch = l.ukv->row_bytes;
+        const uint8_t *Wuk = l.ukv->dev, *Wuv = Wuk + (size_t)a.H * a.d * pitch;
+        const unsigned H = (unsigned)a.H, Tu = (unsigned)T;
+        const int n_split = std::min(jq::LAT_MAX_SPLIT, (pos0 + T + jq::LAT_RUN - 1) / jq::LAT_RUN);
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_absorb<E>), dim3((unsigned)((a.R + 16 * E::CH - 1) / (16 * E::CH)), H + 1, Tu), dim3(256), 0, s, a,
+                                            Wuk, pitch, m->qx));
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_attention_any<E>), dim3((unsigned)n_split, H, Tu), dim3(256),
+                                            (size_t)(a.RP + jq::LAT_RUN) * sizeof(float), s, a, m->qx, n_split, m->part));
+        hipLaunchKernelGGL(jq::latent_merge, dim3(Tu * H, (unsigned)((a.R + 255) / 256)), dim3(256), 0, s, m->part, a.sink, a.H, a.R, n_split, m->olat);
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_values<E>), dim3((unsigned)((a.dv + 15) / 16), H, Tu), dim3(256), 0, s, a, m->olat, Wuv, pitch,
+                                            m->mid));
+        return 0;
+    }
+    const int n = pos0 + T, DP = l.DP(), DVP = l.DVP();
+    JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_store<E>), dim3((unsigned)T), dim3(256), 0, s, a));
+    if (dense_gemm(l.ukv, r.kc, (size_t)a.RP, n, m->kv, l.ukv->n, s)) return 1;
+    const unsigned gy = (unsigned)std::min((a.H * (DP + DVP) + 255) / 256, 16);
+    JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_expand<E>), dim3((unsigned)n, gy), dim3(256), 0, s, a, m->kv, n, DP, DVP, (typename E::T *)m->k_e,
+                                        (typename E::T *)m->v_e));
+    JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_queries<E>), dim3((unsigned)T), dim3(256), 0, s, a, DP, (typename E::T *)m->q_e));
+    jq::AttnLayer t{};
+    t.H = t.G = a.H, t.d = c.dim + c.rot_dim, t.dv = a.dv, t.DP = DP, t.DVP = DVP, t.n_ctx = n, t.scale = a.scale, t.pos0 = pos0, t.T = T;
+    t.kc = m->k_e, t.vc = m->v_e, t.sink = a.sink, t.gate = a.gate, t.ld_gate = ld;
+    return run_attention_rows(m, t, false, nullptr, l.mix_e, s);
+}
+
+int run_mamba(LayeredModel *m, const Layer &l, LayerRun &r, int T, bool small, hipStream_t s) {
+    const LayerConfig &c = l.c;
+    const uint32_t type = m->type;
+    const int C = c.inner, N = c.state, taps = c.taps;
+    const dim3 cgrid((unsigned)((C + 255) / 256), (unsigned)((T + taps - 1 + jq::CONV_RUN - 1) / jq::CONV_RUN));
+    float *t_in = r.tail[r.tail_at], *t_out = r.tail[r.tail_at ^ 1];
+    if (small)
+        hipLaunchKernelGGL((jq::causal_conv_silu<float>), cgrid, dim3(256), 0, s, m->proj, l.in->n, l.conv, l.conv_b, t_in, t_out, m->conv_f, (size_t)C,
+                           T, C, taps);
+    else
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::causal_conv_silu<typename E::T>), cgrid, dim3(256), 0, s, m->proj, l.in->n, l.conv, l.conv_b, t_in,
+                                            t_out, (typename E::T *)l.conv_e, dense_stride(C), T, C, taps));
+    r.tail_at ^= 1;
+    const size_t ldp = l.wx->n;
+    if (small ? dense_gemv(l.wx, m->conv_f, C, T, m->bc, ldp, s) : dense_gemm(l.wx, l.conv_e, dense_stride(C), T, m->bc, ldp, s)) return 1;
+    jq::SsmScan a{};
+    a.dt_raw = m->dt, a.dt_bias = l.dt_b, a.bc = m->bc + c.dt_rank, a.ld_bc = ldp, a.z = m->proj + C, a.ld_z = l.in->n;
+    a.A_log2 = l.A_log2, a.D = l.D, a.S = r.S, a.T = T, a.C = C, a.N = N, a.ldx = a.ldo = (size_t)C;
+    if (T == 1) {
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::selective_step<E>), dim3((unsigned)((C + 15) / 16)), dim3(256), 0, s, a, l.wdt->dev, l.wdt->row_bytes,
+                                            m->bc, c.dt_rank, m->conv_f, m->mid));
+    } else if (small) {
+        if (dense_gemv(l.wdt, m->bc, ldp, T, m->dt, C, s) || run_scan<float>(a, m->conv_f, m->mid, s)) return 1;
+    } else {
+        const size_t sr = dense_stride(c.dt_rank);
+        if (rows_to_elem(type, m->bc, ldp, T, c.dt_rank, l.dt_e, sr, s) || dense_gemm(l.wdt, l.dt_e, sr, T, m->dt, C, s)) return 1;
+        a.ldx = a.ldo = dense_stride(C);
+        JQ_ELEM_OF(type, if (run_scan<typename E::T>(a, (const typename E::T *)l.conv_e, (typename E::T *)l.mix_e, s)) return 1);
+    }
+    return 0;
+}
+
 int LayeredModel::run_layers(int T, const uint32_t *want, int n_want, hipStream_t s) {
     const int w = (int)cfg.width;
     const size_t sw = dense_stride(w);
@@ -307,10 +482,8 @@ int LayeredModel::run_layers(int T, const uint32_t *want, int n_want, hipStream_
     for (const RotaryTable &r : rots)
         hipLaunchKernelGGL(jq::rope_angles, dim3(grid_for((size_t)T * (r.c.dims / 2))), dim3(256), 0, s, r.freq, r.c.dims / 2, pos0, T, r.mag, r.cs);
     if (pos0 == 0) {  // a new sequence: its states start at zero
-        for (Layer &l : layers)
-            if (l.c.mixer == LayerConfig::MAMBA1 &&
-                (zero_floats(l.S, (size_t)l.c.inner * l.c.state, s) || zero_floats(l.tail[l.tail_at], (size_t)(l.c.taps - 1) * l.c.inner, s)))
-                return 1;
+        for (LayerRun &r : runs)
+            if (zero_floats(r.S, r.S_floats, s) || zero_floats(r.tail[r.tail_at], r.tail_floats, s)) return 1;
     }
     float *xc = x, *xo = x2;
     const float *pending = nullptr;       // the sublayer result not yet in the stream, and the norm it takes first
@@ -323,10 +496,11 @@ int LayeredModel::run_layers(int T, const uint32_t *want, int n_want, hipStream_
         nm.x_out = out, nm.h_out = h_out;
         return nm;
     };
-    // out [T][wt->n] = wt norm(stream), the stream updated on the way
-    auto norm_product = [&](const NormWeights &pre, const jq_weight *wt, float *out) {
+    // out [T][wt->n] = wt norm(stream), the stream updated on the way; `keep`: the normed rows stay, in h up to 8 tokens
+    // and in h_e from there on
+    auto norm_product = [&](const NormWeights &pre, const jq_weight *wt, float *out, bool keep) {
         if (one) {
-            const jq::ResidualNorm nm = update(pre, xo, nullptr);
+            const jq::ResidualNorm nm = update(pre, xo, keep ? h : nullptr);
             if (dense_gemv(wt, nullptr, 0, 1, out, wt->n, s, &nm)) return 1;
             std::swap(xc, xo);
             return 0;
@@ -334,46 +508,51 @@ int LayeredModel::run_layers(int T, const uint32_t *want, int n_want, hipStream_
         if (residual_norm(update(pre, xc, small ? h : nullptr), type, small ? nullptr : h_e, sw, T, nullptr, s)) return 1;
         return small ? dense_gemv(wt, h, w, T, out, wt->n, s) : dense_gemm(wt, h_e, sw, T, out, wt->n, s);
     };
-    for (Layer &l : layers) {
+    // the experts of a layer, their scratch handed over from the layer of their sizes that had it last
+    auto experts = [&](Layer &l, const float *hx, const void *hxe, const MoeDenseExtras &ex) {
+        int &holder = moe_holder[l.moe_shares];
+        if (layers[holder].moe != l.moe) moe_swap_scratch(l.moe, layers[holder].moe);
+        holder = (int)(&l - layers.data());
+        std::lock_guard<std::mutex> lock(l.moe->mu);
+        return moe_reserve(l.moe, cap_tokens) || moe_forward_dense(l.moe, T, hx, hxe, y, s, ex);
+    };
+    for (LayerRun &r : runs) {
+        Layer &l = layers[r.layer];
         const LayerConfig &c = l.c;
-        if (norm_product(l.norm1, l.in, proj)) return 1;
-        if (c.mixer == LayerConfig::ATTENTION) {
+        const bool beside = cfg.parallel && c.mlp != LayerConfig::NONE;
+        if (norm_product(l.norm1, l.in, proj, beside)) return 1;
+        switch (c.mixer) {
+        case LayerConfig::ATTENTION: {
             jq::AttnLayer a{};
             a.H = c.heads, a.G = c.kv_heads, a.d = c.dim, a.dv = c.vdim, a.DP = l.DP(), a.DVP = l.DVP(), a.n_ctx = (int)n_ctx;
             a.rot = c.rot.dims, a.scale = c.scale, a.pos0 = pos0, a.T = T, a.qkv = proj, a.ld = l.in->n, a.cs = l.rot >= 0 ? rots[l.rot].cs : nullptr;
             a.v_first = c.v_mix && !l.v_first ? first_v : nullptr, a.v_first_out = l.v_first ? first_v : nullptr, a.lambda = l.lambda;
-            a.kc = l.kc, a.vc = l.vc;
+            a.kc = r.kc, a.vc = r.vc;
             if (run_attention(this, l, a, small, mid, l.mix_e, s)) return 1;
-        } else {
-            const int C = c.inner, N = c.state, taps = c.taps;
-            const dim3 cgrid((unsigned)((C + 255) / 256), (unsigned)((T + taps - 1 + jq::CONV_RUN - 1) / jq::CONV_RUN));
-            float *t_in = l.tail[l.tail_at], *t_out = l.tail[l.tail_at ^ 1];
-            if (small)
-                hipLaunchKernelGGL((jq::causal_conv_silu<float>), cgrid, dim3(256), 0, s, proj, l.in->n, l.conv, l.conv_b, t_in, t_out,
-                                   conv_f, (size_t)C, T, C, taps);
-            else
-                JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::causal_conv_silu<typename E::T>), cgrid, dim3(256), 0, s, proj, l.in->n, l.conv, l.conv_b,
-                                                    t_in, t_out, (typename E::T *)l.conv_e, dense_stride(C), T, C, taps));
-            l.tail_at ^= 1;
-            const size_t ldp = l.wx->n;
-            if (small ? dense_gemv(l.wx, conv_f, C, T, bc, ldp, s) : dense_gemm(l.wx, l.conv_e, dense_stride(C), T, bc, ldp, s)) return 1;
-            jq::SsmScan a{};
-            a.dt_raw = dt, a.dt_bias = l.dt_b, a.bc = bc + c.dt_rank, a.ld_bc = ldp, a.z = proj + C, a.ld_z = l.in->n;
-            a.A_log2 = l.A_log2, a.D = l.D, a.S = l.S, a.T = T, a.C = C, a.N = N, a.ldx = a.ldo = (size_t)C;
-            if (T == 1) {
-                JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::selective_step<E>), dim3((unsigned)((C + 15) / 16)), dim3(256), 0, s, a, l.wdt->dev,
-                                                    l.wdt->row_bytes, bc, c.dt_rank, conv_f, mid));
-            } else if (small) {
-                if (dense_gemv(l.wdt, bc, ldp, T, dt, C, s) || run_scan<float>(a, conv_f, mid, s)) return 1;
-            } else {
-                const size_t sr = dense_stride(c.dt_rank);
-                if (rows_to_elem(type, bc, ldp, T, c.dt_rank, l.dt_e, sr, s) || dense_gemm(l.wdt, l.dt_e, sr, T, dt, C, s)) return 1;
-                a.ldx = a.ldo = dense_stride(C);
-                JQ_ELEM_OF(type, if (run_scan<typename E::T>(a, (const typename E::T *)l.conv_e, (typename E::T *)l.mix_e, s)) return 1);
-            }
+            break;
+        }
+        case LayerConfig::MAMBA1:
+            if (run_mamba(this, l, r, T, small, s)) return 1;
+            break;
+        case LayerConfig::LATENT:
+            if (run_latent(this, l, r, pos0, T, small, s)) return 1;
+            break;
+        default:
+            if (run_linear(this, l, r, T, small, s)) return 1;
         }
         const int mw = l.mix_width();
-        if (small ? dense_gemv(l.o, mid, mw, T, y, w, s) : dense_gemm(l.o, l.mix_e, dense_stride(mw), T, y, w, s)) return 1;
+        auto output = [&] { return small ? dense_gemv(l.o, mid, mw, T, y, w, s) : dense_gemm(l.o, l.mix_e, dense_stride(mw), T, y, w, s); };
+        if (beside) {  // the block reads the mixer's own input; its router's logits came with the mixer's projections
+            MoeDenseExtras ex;
+            ex.logits = proj + l.router_at, ex.ld = l.in->n, ex.shared_logit = c.shared_ff ? ex.logits + c.experts : nullptr;
+            if (T == 1 && moe_dense_decode_sized(l.moe, 1)) ex.W = l.o, ex.mid = mid;
+            else if (output()) return 1;
+            else ex.add = y;
+            if (experts(l, small ? h : nullptr, small ? nullptr : h_e, ex)) return 1;
+            pending = y, post = NormWeights{};
+            continue;
+        }
+        if (output()) return 1;
         pending = y, post = l.norm1b;
 
         if (c.mlp == LayerConfig::NONE) continue;
@@ -390,22 +569,16 @@ int LayeredModel::run_layers(int T, const uint32_t *want, int n_want, hipStream_
                     return 1;
             }
             if (small ? dense_gemv(l.down, mid, c.ff, T, y, w, s) : dense_gemm(l.down, l.ff_e, dense_stride(c.ff), T, y, w, s)) return 1;
+        } else if (one && moe_dense_fuses_norm(l.moe, T)) {
+            const jq::ResidualNorm nm = update(l.norm2, xo, h);
+            MoeDenseExtras ex;
+            ex.pre = &nm;
+            if (experts(l, h, nullptr, ex)) return 1;
+            std::swap(xc, xo);
         } else {
-            jq_moe *moe = l.moe;
-            int &holder = moe_holder[l.moe_shares];
-            if (layers[holder].moe != moe) moe_swap_scratch(moe, layers[holder].moe);
-            holder = (int)(&l - layers.data());
-            std::lock_guard<std::mutex> lock(moe->mu);
-            if (moe_reserve(moe, cap_tokens)) return 1;
-            if (one && moe_dense_fuses_norm(moe, T)) {
-                const jq::ResidualNorm nm = update(l.norm2, xo, h);
-                if (moe_forward_dense(moe, T, h, nullptr, y, s, &nm)) return 1;
-                std::swap(xc, xo);
-            } else {
-                // the router reads the norm in f32, the experts of a many-token step in their own type
-                if (residual_norm(update(l.norm2, xc, h), type, h_e, sw, T, nullptr, s)) return 1;
-                if (moe_forward_dense(moe, T, h, h_e, y, s)) return 1;
-            }
+            // the router reads the norm in f32, the experts of a many-token step in their own type
+            if (residual_norm(update(l.norm2, xc, h), type, h_e, sw, T, nullptr, s)) return 1;
+            if (experts(l, h, h_e, MoeDenseExtras())) return 1;
         }
         pending = y, post = l.norm2b;
     }
@@ -495,10 +668,29 @@ struct StackLoader {
 int check_stack(const StackConfig &c) {
     if (!c.vocab || !c.width) return fail("%s: zero in configuration", c.arch);
     if (c.width > (uint32_t)NORM_MAX_WIDTH) return fail("%s: width %u exceeds %d", c.arch, c.width, NORM_MAX_WIDTH);
+    const int n_layers = (int)c.layers.size();
+    if (c.loop_start < 0 || c.loop_start > c.loop_stop || c.loop_stop > n_layers || c.loop_times < 1)
+        return fail("%s: layers %d to %d of %d run %d times", c.arch, c.loop_start, c.loop_stop, n_layers, c.loop_times);
     int v_mix = -1;
     for (size_t i = 0; i < c.layers.size(); i++) {
         const LayerConfig &l = c.layers[i];
-        if (l.mixer == LayerConfig::ATTENTION) {
+        if (l.linear()) {
+            if (l.heads <= 0 || l.dim <= 0 || l.vdim <= 0) return fail("%s: layer %zu: zero in the mixer", c.arch, i);
+            if (l.dim > jq::LIN_MAX_DIM) return fail("%s: layer %zu: heads of %d exceed %d", c.arch, i, l.dim, jq::LIN_MAX_DIM);
+            if (l.mixer == LayerConfig::MLSTM && !(l.gate_cap > 0.0f)) return fail("%s: layer %zu: gates capped at %g", c.arch, i, l.gate_cap);
+            if (l.mixer == LayerConfig::LIGHTNING && l.decay.size() != (size_t)l.heads)
+                return fail("%s: layer %zu: %zu decays for %d heads", c.arch, i, l.decay.size(), l.heads);
+            for (double d : l.decay)
+                if (!(d >= 0.0 && d <= 1.0)) return fail("%s: layer %zu: a decay of %g", c.arch, i, d);
+        } else if (l.mixer == LayerConfig::LATENT) {
+            if (l.heads <= 0 || l.dim <= 0 || l.vdim <= 0 || l.q_rank <= 0 || l.kv_rank <= 0 || l.rot_dim < 0)
+                return fail("%s: layer %zu: zero in the mixer", c.arch, i);
+            if (l.kv_rank > jq::LAT_MAX_R) return fail("%s: layer %zu: latents of %d exceed %d", c.arch, i, l.kv_rank, jq::LAT_MAX_R);
+            if (l.q_rank > NORM_MAX_WIDTH) return fail("%s: layer %zu: query latents of %d exceed %d", c.arch, i, l.q_rank, NORM_MAX_WIDTH);
+            if (l.vdim > jq::ANY_MAX_DV) return fail("%s: layer %zu: value heads of %d exceed %d", c.arch, i, l.vdim, jq::ANY_MAX_DV);
+            if (l.rot.dims < 0 || l.rot.dims % 2 || l.rot.dims > l.rot_dim)
+                return fail("%s: layer %zu: %d of %d dimensions rotated", c.arch, i, l.rot.dims, l.rot_dim);
+        } else if (l.mixer == LayerConfig::ATTENTION) {
             if (l.heads <= 0 || l.kv_heads <= 0 || l.heads % l.kv_heads || l.dim <= 0 || l.vdim <= 0)
                 return fail("%s: layer %zu: %d query heads over %d kv heads of %d and %d", c.arch, i, l.heads, l.kv_heads, l.dim, l.vdim);
             if (l.vdim > jq::ANY_MAX_DV) return fail("%s: layer %zu: value heads of %d exceed %d", c.arch, i, l.vdim, jq::ANY_MAX_DV);
@@ -513,39 +705,64 @@ int check_stack(const StackConfig &c) {
             if (l.state > jq::SCAN_MAX_STATES) return fail("%s: layer %zu: %d states a channel exceed %d", c.arch, i, l.state, jq::SCAN_MAX_STATES);
         }
         if (l.mlp != LayerConfig::NONE && l.ff <= 0) return fail("%s: layer %zu: feed-forward of %d", c.arch, i, l.ff);
+        if (c.parallel && l.mlp == LayerConfig::DENSE) return fail("%s: layer %zu: only experts run beside a mixer", c.arch, i);
         if (l.mlp == LayerConfig::MOE && (l.top <= 0 || l.top > l.experts)) return fail("%s: layer %zu: %d experts used of %d", c.arch, i, l.top, l.experts);
     }
     return 0;
 }
 
-// The caches, states and rotary tables of a loaded stack.
+// The cache or state of one run of layer i.
+int make_run(LayeredModel *m, int i) {
+    const Layer &l = m->layers[i];
+    const LayerConfig &c = l.c;
+    LayerRun r;
+    r.layer = i;
+    auto cache = [&](size_t elems, void **out) {  // zeroed: kernels read whole runs of a row
+        uint8_t *p = nullptr;
+        if (m->device_alloc(&p, elems * m->esz())) return fail("%s: cache allocation failed", m->arch);
+        HIP_TRY(hipMemset(p, 0, elems * m->esz()));
+        *out = p;
+        return 0;
+    };
+    if (c.mixer == LayerConfig::ATTENTION) {
+        const size_t rows = (size_t)c.kv_heads * m->n_ctx;
+        if (cache(rows * l.DP(), &r.kc) || cache(rows * l.DVP(), &r.vc)) return 1;
+    } else if (c.mixer == LayerConfig::LATENT) {
+        if (cache((size_t)m->n_ctx * c.latent_pitch(), &r.kc)) return 1;
+    } else {
+        r.S_floats = c.linear() ? (size_t)c.heads * c.state_rows() * c.state_pitch() : (size_t)c.inner * c.state;
+        r.tail_floats = c.linear() ? (size_t)c.heads : (size_t)(c.taps - 1) * c.inner;
+        if (m->device_alloc(&r.S, r.S_floats) || m->device_alloc(&r.tail[0], r.tail_floats) || m->device_alloc(&r.tail[1], r.tail_floats)) return 1;
+    }
+    m->runs.push_back(r);
+    return 0;
+}
+
+// The runs of a loaded stack, each with its cache or state, and the rotary tables.
 int make_states(LayeredModel *m) {
     for (Layer &l : m->layers) {
         const LayerConfig &c = l.c;
-        if (c.mixer == LayerConfig::ATTENTION) {
-            const size_t rows = (size_t)c.kv_heads * m->n_ctx;
-            uint8_t *k = nullptr, *v = nullptr;
-            if (m->device_alloc(&k, rows * l.DP() * m->esz()) || m->device_alloc(&v, rows * l.DVP() * m->esz()))
-                return fail("%s: KV cache allocation failed", m->arch);
-            l.kc = k, l.vc = v;
-            if (c.rot.dims) {
-                for (size_t r = 0; r < m->rots.size(); r++)
-                    if (m->rots[r].c == c.rot) l.rot = (int)r;
-                if (l.rot < 0) {
-                    RotaryTable t;
-                    std::vector<double> freq;
-                    t.c = c.rot, t.mag = (float)rotary_frequencies(c.rot, &freq);
-                    if (m->device_alloc(&t.freq, freq.size())) return 1;
-                    HIP_TRY(hipMemcpy(t.freq, freq.data(), freq.size() * sizeof(double), hipMemcpyHostToDevice));
-                    l.rot = (int)m->rots.size();
-                    m->rots.push_back(t);
-                }
-            }
-        } else if (m->device_alloc(&l.S, (size_t)c.inner * c.state) || m->device_alloc(&l.tail[0], (size_t)(c.taps - 1) * c.inner) ||
-                   m->device_alloc(&l.tail[1], (size_t)(c.taps - 1) * c.inner)) {
-            return 1;
+        if (!c.rot.dims) continue;
+        for (size_t r = 0; r < m->rots.size(); r++)
+            if (m->rots[r].c == c.rot) l.rot = (int)r;
+        if (l.rot < 0) {
+            RotaryTable t;
+            std::vector<double> freq;
+            t.c = c.rot, t.mag = (float)rotary_frequencies(c.rot, &freq);
+            if (m->device_alloc(&t.freq, freq.size())) return 1;
+            HIP_TRY(hipMemcpy(t.freq, freq.data(), freq.size() * sizeof(double), hipMemcpyHostToDevice));
+            l.rot = (int)m->rots.size();
+            m->rots.push_back(t);
         }
     }
+    const StackConfig &sc = m->cfg;
+    for (int i = 0; i < sc.loop_start; i++)
+        if (make_run(m, i)) return 1;
+    for (int pass = 0; pass < sc.loop_times; pass++)
+        for (int i = sc.loop_start; i < sc.loop_stop; i++)
+            if (make_run(m, i)) return 1;
+    for (int i = sc.loop_stop; i < (int)m->layers.size(); i++)
+        if (make_run(m, i)) return 1;
     // layers with experts of the same sizes take turns with one set of scratch buffers
     m->moe_holder.resize(m->layers.size());
     for (size_t i = 0; i < m->layers.size(); i++) {
@@ -555,7 +772,7 @@ int make_states(LayeredModel *m) {
         l.moe_shares = (int)i;
         for (size_t j = 0; j < i && l.moe_shares == (int)i; j++) {
             const LayerConfig &o = m->layers[j].c;
-            if (m->layers[j].moe && o.experts == l.c.experts && o.top == l.c.top && o.ff == l.c.ff) l.moe_shares = (int)j;
+            if (m->layers[j].moe && o.experts == l.c.experts && o.top == l.c.top && o.ff == l.c.ff && o.shared_ff == l.c.shared_ff) l.moe_shares = (int)j;
         }
     }
     return 0;
@@ -605,6 +822,19 @@ struct ConfigReader {
         if (!v || v->kind == jq::Json::NUL) return false;
         if (v->kind != jq::Json::BOOL) bad(key, "is not a boolean");
         return v->b;
+    }
+    std::vector<double> numbers(const jq::Json *j, const char *key) {
+        const jq::Json *v = j ? j->find(key) : nullptr;
+        std::vector<double> out;
+        if (!v || v->kind != jq::Json::ARRAY) {
+            bad(key, "is not a list");
+            return out;
+        }
+        for (const jq::Json &e : v->items) {
+            if (e.kind != jq::Json::NUMBER) bad(key, "is not a list of numbers");
+            out.push_back(e.num);
+        }
+        return out;
     }
     const jq::Json *optional(const jq::Json *j, const char *key) {
         const jq::Json *v = j ? j->find(key) : nullptr;
@@ -724,25 +954,148 @@ int bozosun_tensors(StackLoader &ld) {
     return 0;
 }
 
+// ---- Fasesun --------------------------------------------------------------------------------------------
+// Mixer and experts side by side on one root-mean-square norm; matrix memories, constant-decay linear attention and
+// latent attention with sinks and an output gate; sigmoid-routed experts (a correction for the choice alone) with a gated
+// shared one; a run of layers may repeat with caches of its own a pass; the embedding is the output head.
+
+int fasesun_config(const jq::Json &cfg, StackConfig *out) {
+    ConfigReader r{"Fasesun"};
+    StackConfig &s = *out;
+    s.arch = "Fasesun";
+    s.vocab = (uint32_t)r.integer(&cfg, "vocab"), s.width = (uint32_t)r.integer(&cfg, "width");
+    s.norm_eps = (float)r.number(r.object(&cfg, "norm"), "eps");
+    s.rms = s.parallel = true;
+    if (const jq::Json *loop = r.optional(&cfg, "loop"))
+        s.loop_start = r.integer(loop, "start"), s.loop_stop = r.integer(loop, "stop"), s.loop_times = r.integer(loop, "times");
+    const jq::Json *layers = cfg.find("layers");
+    if (!layers || layers->kind != jq::Json::ARRAY) r.bad("layers", "is not a list");
+    for (size_t i = 0; r.ok && i < layers->items.size(); i++) {
+        const jq::Json *e = &layers->items[i];
+        r.where = "layers[" + std::to_string(i) + "]";
+        LayerConfig l;
+        const jq::Json *type = e->find("type"), *mx = r.object(e, "mixer");
+        l.heads = r.integer(mx, "heads"), l.dim = r.integer(mx, "dim"), l.vdim = r.integer(mx, "vdim");
+        if (!type || type->kind != jq::Json::STRING) {
+            r.bad("type", "is not a string");
+        } else if (type->str == "mlstm") {
+            l.mixer = LayerConfig::MLSTM;
+            l.gate_cap = (float)r.number(mx, "gate_cap");
+        } else if (type->str == "lightning") {
+            l.mixer = LayerConfig::LIGHTNING;
+            l.decay = r.numbers(mx, "decay");
+        } else if (type->str == "latent_attention") {
+            l.mixer = LayerConfig::LATENT;
+            l.q_rank = r.integer(mx, "q_rank"), l.kv_rank = r.integer(mx, "kv_rank"), l.rot_dim = r.integer(mx, "rot_dim");
+            l.scale = (float)r.number(mx, "scale");
+            if (const jq::Json *rot = r.optional(mx, "rot")) l.rot.dims = r.integer(rot, "dims"), l.rot.base = r.number(rot, "base");
+        } else {
+            r.bad("type", "names no mixer of this design");
+        }
+        if (const jq::Json *mlp = r.optional(e, "mlp")) {
+            const jq::Json *kind = mlp->find("kind");
+            if (kind && kind->kind == jq::Json::STRING && kind->str == "moe") {
+                l.mlp = LayerConfig::MOE;
+                const jq::Json *ro = r.object(mlp, "router");
+                l.ff = r.integer(r.object(mlp, "expert"), "ff"), l.experts = r.integer(ro, "experts"), l.top = r.integer(ro, "top");
+                if (const jq::Json *sh = r.optional(mlp, "shared")) l.shared_ff = r.integer(sh, "ff");
+            } else {
+                r.bad("mlp.kind", "names no feed-forward block of this design");
+            }
+        }
+        s.layers.push_back(l);
+    }
+    return r.ok ? check_stack(s) : 1;
+}
+
+int fasesun_tensors(StackLoader &ld) {
+    LayeredModel *m = ld.m;
+    const StackConfig &c = m->cfg;
+    const uint64_t w = c.width;
+    if (ld.matrix({{"embed", c.vocab}}, w, &m->embed) || ld.norm("final.norm", &m->final_norm)) return 1;
+    m->head = m->embed;
+    m->layers.resize(c.layers.size());
+    for (size_t i = 0; i < c.layers.size(); i++) {
+        Layer &l = m->layers[i];
+        l.c = c.layers[i];
+        const LayerConfig &lc = l.c;
+        const std::string p = "l" + std::to_string(i) + ".", mx = p + "mix.", ml = p + "mlp.";
+        const uint64_t H = lc.heads, nv = H * lc.vdim, E = lc.experts;
+        if (ld.norm(p + "norm1", &l.norm1) || ld.matrix({{mx + "o", w}}, nv, &l.o)) return 1;
+        // everything that reads the layer's norm in one product: the mixer's projections, its gates, the router
+        std::vector<std::pair<std::string, uint64_t>> in;
+        if (lc.mixer == LayerConfig::LATENT) {
+            const uint64_t Q = lc.q_rank, R = lc.kv_rank, rd = lc.rot_dim, d = lc.dim;
+            in = {{mx + "dq", Q}, {mx + "dkv", R + rd}, {mx + "g", nv}};
+            l.gate_at = (int)(Q + R + rd);
+            if (ld.vec(mx + "dq.norm", {Q}, &l.dq_norm) || ld.vec(mx + "dkv.norm", {R}, &l.dkv_norm) || ld.vec(mx + "sink", {H}, &l.sink) ||
+                ld.matrix({{mx + "uq", H * (d + rd)}}, Q, &l.uq) || ld.matrix({{mx + "uk", H * d}, {mx + "uv", nv}}, R, &l.ukv))
+                return 1;
+        } else {
+            const uint64_t nk = H * lc.dim;
+            in = {{mx + "q", nk}, {mx + "k", nk}, {mx + "v", nv}, {mx + "g", nv}};
+            l.gate_at = (int)(2 * nk + nv);
+            if (ld.vec(mx + "norm", {nv}, &l.mix_norm)) return 1;
+            if (lc.mixer == LayerConfig::MLSTM) {
+                in.insert(in.end(), {{mx + "i", H}, {mx + "f", H}});
+                if (ld.vec(mx + "i.b", {H}, &l.i_b) || ld.vec(mx + "f.b", {H}, &l.f_b)) return 1;
+            } else {
+                std::vector<float> decay, log_decay;
+                for (double v : lc.decay) decay.push_back((float)v), log_decay.push_back(v > 0.0 ? (float)std::log(v) : -1e4f);
+                if (ld.to_device(decay, &l.decay) || ld.to_device(log_decay, &l.log_decay)) return 1;
+            }
+        }
+        for (const auto &part : in) l.router_at += (int)part.second;
+        if (lc.mlp == LayerConfig::MOE) {
+            in.emplace_back(ml + "router", E);
+            if (lc.shared_ff) in.emplace_back(ml + "shared.sg", 1);
+        }
+        if (ld.matrix(in, w, &l.in)) return 1;
+        if (lc.mlp == LayerConfig::NONE) continue;
+        const uint64_t ff = lc.ff, sf = lc.shared_ff;
+        std::vector<std::pair<std::string, uint64_t>> g, u, d;
+        for (uint64_t e = 0; e < E; e++) {
+            const std::string ep = ml + "e" + std::to_string(e) + ".";
+            g.emplace_back(ep + "gate", ff), u.emplace_back(ep + "up", ff), d.emplace_back(ep + "down", w);
+        }
+        std::vector<float> router, correction;
+        jq_weight *sg = nullptr, *su = nullptr, *sd = nullptr;
+        if (ld.matrix(g, w, &l.gate) || ld.matrix(u, w, &l.up) || ld.matrix(d, ff, &l.down) || ld.host(ml + "router", {E, w}, &router) ||
+            ld.host(ml + "correction", {E}, &correction) ||
+            (sf && (ld.matrix({{ml + "shared.gate", sf}}, w, &sg) || ld.matrix({{ml + "shared.up", sf}}, w, &su) ||
+                    ld.matrix({{ml + "shared.down", w}}, sf, &sd))))
+            return 1;
+        jq_moe_config mc{};
+        mc.n_expert = (uint32_t)E, mc.n_expert_used = (uint32_t)lc.top, mc.hidden = c.width, mc.inter = (uint32_t)ff, mc.gating = 1;
+        if (jq_moe_create(&mc, router.data(), correction.data(), l.gate, l.up, l.down, sg, su, sd, &l.moe)) return 1;
+    }
+    return 0;
+}
+
 constexpr uint32_t DEFAULT_CONTEXT = 4096;  // where neither the caller nor the configuration names one
 
-int load_bozosun(const char *path, const ModelLoadOptions &opt, jq_model **out) {
+int load_layered(const char *path, const ModelLoadOptions &opt, int (*config)(const jq::Json &, StackConfig *), int (*tensors)(StackLoader &),
+                 jq_model **out) {
     std::string err;
     jq::Json cfg;
     if (!jq::json_read_file(std::string(path) + "/config.json", &cfg, &err)) return fail("%s", err.c_str());
     auto m = std::make_unique<LayeredModel>();
-    if (bozosun_config(cfg, &m->cfg)) return 1;
+    if (config(cfg, &m->cfg)) return 1;
     m->arch = m->cfg.arch, m->vocab = m->cfg.vocab, m->n_ctx = opt.n_ctx ? opt.n_ctx : DEFAULT_CONTEXT;
     m->type = opt.compute == JQ_COMPUTE_F32 ? JQ_TYPE_F32 : JQ_TYPE_BF16;
     auto st = jq::safetensors_open(std::string(path) + "/model.safetensors", &err);
     if (!st) return fail("%s", err.c_str());
     if (ensure_init()) return 1;
     StackLoader ld{m.get(), *st};
-    if (bozosun_tensors(ld) || make_states(m.get()) || m->init_outputs()) return 1;
+    if (tensors(ld) || make_states(m.get()) || m->init_outputs()) return 1;
     *out = m.release();
     return 0;
 }
 
+int load_bozosun(const char *path, const ModelLoadOptions &opt, jq_model **out) { return load_layered(path, opt, bozosun_config, bozosun_tensors, out); }
+int load_fasesun(const char *path, const ModelLoadOptions &opt, jq_model **out) { return load_layered(path, opt, fasesun_config, fasesun_tensors, out); }
+
 const RegisterModelArch g_register_bozosun({"Bozosun", true, load_bozosun});
+const RegisterModelArch g_register_fasesun({"Fasesun", true, load_fasesun});
 
 }  // namespace

@@ -13,11 +13,11 @@ static void moe_free_scratch(jq_moe *m) {
     for (void *p : {(void *)m->logits, (void *)m->wts, (void *)m->G, (void *)m->U, (void *)m->out, (void *)m->sG,
                     (void *)m->sU, (void *)m->sH, (void *)m->sOut, (void *)m->ids, (void *)m->gexp,
                     (void *)m->offsets, (void *)m->xrow, (void *)m->yrow, (void *)m->qacts, (void *)m->qi8.xl,
-                    (void *)m->qi8.xh, (void *)m->qi8.sx, (void *)m->qi8.sxs, (void *)m->gacts, (void *)m->gtab, (void *)m->group_counts})
+                    (void *)m->qi8.xh, (void *)m->qi8.sx, (void *)m->qi8.sxs, (void *)m->gacts, (void *)m->gtab, (void *)m->group_counts, (void *)m->sgate_logit})
         if (p) (void)hipFree(p);
     if (m->backend && m->backend->release) m->backend->release(m);
     m->qacts = nullptr;
-    m->group_counts = nullptr;
+    m->group_counts = nullptr, m->sgate_logit = nullptr;
     m->gacts = nullptr, m->gtab = nullptr, m->gtab_rows = 0;
     m->qi8 = jq::ActsI8{nullptr, nullptr, nullptr, nullptr};
     m->logits = m->wts = m->G = m->U = m->out = m->sG = m->sU = m->sH = m->sOut = nullptr;
@@ -50,6 +50,7 @@ int moe_reserve(jq_moe *m, size_t T) {
         HIP_TRY(hipMalloc((void **)&m->sU, T * si * sizeof(float)));
         HIP_TRY(hipMalloc((void **)&m->sH, T * si * sizeof(float)));
         HIP_TRY(hipMalloc((void **)&m->sOut, T * c.hidden * sizeof(float)));
+        HIP_TRY(hipMalloc((void **)&m->sgate_logit, T * sizeof(float)));
     }
     m->cap_tokens = T;
     return 0;
@@ -57,7 +58,7 @@ int moe_reserve(jq_moe *m, size_t T) {
 
 jq::MoeGateParams moe_gate_params(const jq_moe_config &c) {
     return jq::MoeGateParams{(int)c.n_expert, (int)c.n_expert_used, (int)c.gating, (int)c.norm_topk, c.weights_scale,
-                             (int)c.n_group, (int)c.topk_group};
+                             (int)c.n_group, (int)c.topk_group, 0};
 }
 
 bool moe_wave_gate(const jq_moe_config &c) {
@@ -104,7 +105,6 @@ int moe_route_dev(jq_moe *m, size_t T, const float *x, hipStream_t s, jq::MoePai
         hipLaunchKernelGGL(jq::moe_router_logits, dim3(c.n_expert, token_runs), dim3(256), 0, s, m->router_w, x, m->logits,
                            (int)T, (int)c.hidden, (int)c.n_expert, planes);
     if (planes_made) *planes_made = !pre && planes.xl && (c.hidden % 32 == 0 || !(T >= tile_from && !no_tile));
-    size_t sm = (2 * c.n_expert + std::max<uint32_t>(c.n_group, 1) + c.n_expert_used + 4) * sizeof(float);
     if (gate_later) {
         if (wave_gate) {
             *gate_later = jq::MoeGateIn{m->logits, m->router_bias, gp, m->ids, m->wts, pg, (int)T};
@@ -113,20 +113,24 @@ int moe_route_dev(jq_moe *m, size_t T, const float *x, hipStream_t s, jq::MoePai
         }
         gate_later->logits = nullptr;
     }
+    return moe_gate_dev(m, T, m->logits, gp, pg, s);
+}
+
+int moe_gate_dev(jq_moe *m, size_t T, const float *logits, const jq::MoeGateParams &gp, jq::MoePairGroups pg, hipStream_t s) {
+    const jq_moe_config &c = m->cfg;
     // no expert groups and at most 256 experts: one wave a token, reductions in registers
-    if (wave_gate) {
+    if (moe_wave_gate(c)) {
         const int ne = (int)(c.n_expert + 63) / 64;
-#define JQ_GATE(NE) hipLaunchKernelGGL(jq::moe_gate_topk_wave<NE>, dim3((unsigned)T), dim3(64), 0, s, m->logits, m->router_bias, gp, m->ids, m->wts, pg)
+#define JQ_GATE(NE) hipLaunchKernelGGL(jq::moe_gate_topk_wave<NE>, dim3((unsigned)T), dim3(64), 0, s, logits, m->router_bias, gp, m->ids, m->wts, pg)
         if (ne == 1) JQ_GATE(1);
         else if (ne == 2) JQ_GATE(2);
         else if (ne == 3) JQ_GATE(3);
         else JQ_GATE(4);
 #undef JQ_GATE
-        HIP_TRY(hipGetLastError());
-        return 0;
+    } else {
+        const size_t sm = (2 * c.n_expert + std::max<uint32_t>(c.n_group, 1) + c.n_expert_used + 4) * sizeof(float);
+        hipLaunchKernelGGL(jq::moe_gate_topk, dim3((unsigned)T), dim3(256), sm, s, logits, m->router_bias, gp, m->ids, m->wts, pg);
     }
-    hipLaunchKernelGGL(jq::moe_gate_topk, dim3((unsigned)T), dim3(256), sm, s, m->logits, m->router_bias, gp, m->ids,
-                       m->wts, pg);
     HIP_TRY(hipGetLastError());
     return 0;
 }
@@ -188,6 +192,7 @@ void moe_swap_scratch(jq_moe *a, jq_moe *b) {
     std::swap(a->offsets, b->offsets), std::swap(a->xrow, b->xrow), std::swap(a->yrow, b->yrow);
     std::swap(a->qacts, b->qacts), std::swap(a->gacts, b->gacts), std::swap(a->gtab, b->gtab);
     std::swap(a->dense_x, b->dense_x), std::swap(a->dense_act, b->dense_act), std::swap(a->group_counts, b->group_counts);
+    std::swap(a->dense_sact, b->dense_sact), std::swap(a->sgate_logit, b->sgate_logit);
     std::swap(a->gtab_rows, b->gtab_rows), std::swap(a->gtile_rgs, b->gtile_rgs), std::swap(a->qi8, b->qi8);
 }
 
@@ -270,9 +275,20 @@ void jq_moe_free(jq_moe *m) {
     if (!m) return;
     moe_free_scratch(m);
     jq_free(m->router_rows);
+    jq_free(m->sgate_row);
     for (void *p : {(void *)m->router_w, (void *)m->router_bias, (void *)m->pgate, (void *)m->pup, (void *)m->pdown})
         if (p) (void)hipFree(p);
     delete m;
+}
+
+int jq_moe_set_shared_gate(jq_moe *m, const float *row) {
+    if (!m || !row) return fail("jq_moe_set_shared_gate: null argument");
+    if (!m->sgate) return fail("moe: no shared expert to gate");
+    if (!dense_elem_bytes(m->gate->type)) return fail("moe: a gate on the shared expert runs beside BF16 / F32 experts only");
+    std::lock_guard<std::mutex> lock(m->mu);
+    jq_free(m->sgate_row);
+    m->sgate_row = nullptr;
+    return jq_upload(JQ_TYPE_F32, row, m->cfg.hidden * sizeof(float), 1, m->cfg.hidden, 0, &m->sgate_row);
 }
 
 int jq_moe_route(jq_moe *m, size_t n_tokens, const float *x, uint32_t *ids, float *weights, int ptrs_are_device,

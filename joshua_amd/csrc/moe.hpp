@@ -49,7 +49,9 @@ struct jq_moe {
     int gtile_rgs = 8;         // row groups a tile of the current plan: 8 (waves share the rows), 2 (the weight rows), 0 (both: two launches)
     jq::ActsI8 qi8{nullptr, nullptr, nullptr, nullptr};  // activations as int8 planes (decode path, long rows)
     // plain-row experts: activations of the grouped GEMM, [rows][stride] in the experts' type
-    uint8_t *dense_x = nullptr, *dense_act = nullptr;
+    uint8_t *dense_x = nullptr, *dense_act = nullptr, *dense_sact = nullptr;
+    jq_weight *sgate_row = nullptr;    // the shared expert's own gate, one f32 row: its result times sigmoid(row . x)
+    float *sgate_logit = nullptr;      // [tokens]
     int *group_counts = nullptr;  // grouping of long pair lists: pairs per (run, expert)
     const jqh::MoeBackend *backend = nullptr;
     std::mutex mu;
@@ -61,6 +63,8 @@ int moe_reserve(jq_moe *m, size_t T);
 int moe_route_dev(jq_moe *m, size_t T, const float *x, hipStream_t s, jq::MoePairGroups pg,
                   jq::ActsI8 planes = jq::ActsI8{nullptr, nullptr, nullptr, nullptr}, bool *planes_made = nullptr,
                   jq::MoeGateIn *gate_later = nullptr, const jq::MoePreNormArgs *pre = nullptr);
+// The gating alone: ids and weights from logits (rows gp.ld apart).
+int moe_gate_dev(jq_moe *m, size_t T, const float *logits, const jq::MoeGateParams &gp, jq::MoePairGroups pg, hipStream_t s);
 // The routed pairs of T tokens grouped by expert (groups 0 .. n_expert, the last one the folded shared expert's).
 int moe_group_dev(jq_moe *m, size_t T, int extra, hipStream_t s);
 jq::MoeGateParams moe_gate_params(const jq_moe_config &c);

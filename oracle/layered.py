@@ -1,7 +1,8 @@
-"""Plain, slow numpy statement (float64) of the layered decoder: a stack whose layers each name a mixer
-(attention with rotary positions and value mixing, or a selective scan) and a feed-forward block (none, dense or
-mixture of experts), with a norm before and after each.  TEST INFRASTRUCTURE: one function a mechanism, loops
-where a loop says it best, no code shared with the library.
+"""Plain, slow numpy statement (float64) of the layered decoders: a stack whose layers each name a mixer (attention
+with rotary positions and value mixing, a selective scan, latent attention with sinks, a matrix memory, linear
+attention with a constant decay) and a feed-forward block (none, dense or mixture of experts).  `LayeredOracle` (Bozosun)
+puts a norm before and after each, `FasesunOracle` runs mixer and feed-forward block side by side on one norm.
+TEST INFRASTRUCTURE: one function a mechanism, loops where a loop says it best, no code shared with the library.
 
 Tensors are a dict name -> array; the configuration is the parsed config.json.
 """
@@ -18,6 +19,10 @@ def layer_norm(x, w, b, eps):
     mu = x.mean(axis=-1, keepdims=True)
     var = ((x - mu) ** 2).mean(axis=-1, keepdims=True)
     return (x - mu) / np.sqrt(var + eps) * w + b
+
+
+def rms_norm(x, eps):
+    return x / np.sqrt((x ** 2).mean(axis=-1, keepdims=True) + eps)
 
 
 def sigmoid(z):
@@ -138,6 +143,80 @@ def mamba1(h, w, m, state):
     return (y * silu(z)) @ w["o"].T
 
 
+def decayed_memory_step(S, k, v, q, decay):
+    """One head, one token: S <- decay S + k v^T, S^T q.  S [dim, vdim]."""
+    S = decay * S + np.outer(k, v)
+    return S, S.T @ q
+
+
+def lightning(h, w, m, state, eps):
+    """Mixer `lightning`; state {"S"} [heads, dim, vdim] is carried over."""
+    T, H, d, dv = h.shape[0], m["heads"], m["dim"], m["vdim"]
+    q, k = silu(h @ w["q"].T).reshape(T, H, d), silu(h @ w["k"].T).reshape(T, H, d)
+    v = silu(h @ w["v"].T).reshape(T, H, dv)
+    S = state.get("S", np.zeros((H, d, dv))).copy()
+    o = np.zeros((T, H, dv))
+    for t in range(T):
+        for a in range(H):
+            S[a], o[t, a] = decayed_memory_step(S[a], k[t, a], v[t, a], q[t, a], m["decay"][a])
+    state["S"] = S
+    return (rms_norm(o.reshape(T, H * dv), eps) * w["norm"] * sigmoid(h @ w["g"].T)) @ w["o"].T
+
+
+def soft_cap(z, cap):
+    return cap * np.tanh(z / cap)
+
+
+def matrix_memory_step(S, n, mx, q, k, v, log_i, log_f):
+    """One head, one token of a matrix memory with exponential gates, held relative to exp(mx)."""
+    new = max(log_f + mx, log_i)
+    keep, write = np.exp(log_f + mx - new), np.exp(log_i - new)
+    S, n = keep * S + write * np.outer(k, v), keep * n + write * k
+    return S, n, new, S.T @ q / (max(abs(n @ q), np.exp(-new)) + 1e-6)
+
+
+def mlstm(h, w, m, state, eps):
+    """Mixer `mlstm`; state {"S", "n", "m"} is carried over, all of it zero in front of the first token."""
+    T, H, d, dv = h.shape[0], m["heads"], m["dim"], m["vdim"]
+    q, k = (h @ w["q"].T).reshape(T, H, d) * d ** -0.5, (h @ w["k"].T).reshape(T, H, d)
+    v = (h @ w["v"].T).reshape(T, H, dv)
+    log_i = soft_cap(h @ w["i"].T + w["i.b"], m["gate_cap"])
+    log_f = -softplus(-soft_cap(h @ w["f"].T + w["f.b"], m["gate_cap"]))
+    S, n, mx = (state.get(x, z).copy() for x, z in (("S", np.zeros((H, d, dv))), ("n", np.zeros((H, d))), ("m", np.zeros(H))))
+    o = np.zeros((T, H, dv))
+    for t in range(T):
+        for a in range(H):
+            S[a], n[a], mx[a], o[t, a] = matrix_memory_step(S[a], n[a], mx[a], q[t, a], k[t, a], v[t, a], log_i[t, a], log_f[t, a])
+    state.update(S=S, n=n, m=mx)
+    return (rms_norm(o, eps).reshape(T, H * dv) * w["norm"] * sigmoid(h @ w["g"].T)) @ w["o"].T
+
+
+def softmax_with_sink(s, sink):
+    """Weights over the scores s whose denominator also counts exp(sink)."""
+    top = max(s.max(), sink)
+    e = np.exp(s - top)
+    return e / (e.sum() + np.exp(sink - top))
+
+
+def latent_attention(h, w, m, cache, pos0, eps):
+    """Mixer `latent_attention`; cache {"c", "r"}, the latents and the rotated shared keys, is appended to."""
+    T, H, d, rd, dv, R = h.shape[0], m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+    q = ((rms_norm(h @ w["dq"].T, eps) * w["dq.norm"]) @ w["uq"].T).reshape(T, H, d + rd)
+    down = h @ w["dkv"].T
+    qr = rotate_interleaved(q[:, :, d:], pos0, m["rot"])
+    cache["c"] = np.concatenate([cache.get("c", np.zeros((0, R))), rms_norm(down[:, :R], eps) * w["dkv.norm"]])
+    cache["r"] = np.concatenate([cache.get("r", np.zeros((0, rd))), rotate_interleaved(down[:, None, R:], pos0, m["rot"])[:, 0]])
+    k = (cache["c"] @ w["uk"].T).reshape(-1, H, d)
+    v = (cache["c"] @ w["uv"].T).reshape(-1, H, dv)
+    o = np.zeros((T, H, dv))
+    for t in range(T):
+        n = pos0 + t + 1
+        for a in range(H):
+            s = (k[:n, a] @ q[t, a, :d] + cache["r"][:n] @ qr[t, a]) * m["scale"]
+            o[t, a] = softmax_with_sink(s, w["sink"][a]) @ v[:n, a]
+    return (o.reshape(T, H * dv) * sigmoid(h @ w["g"].T)) @ w["o"].T
+
+
 # ---- feed-forward blocks ---------------------------------------------------------------------------
 
 def dense_mlp(h, w, limit):
@@ -166,6 +245,29 @@ def moe_mlp(h, w, mlp):
         for e, p in zip(ids[t], wts[t]):
             ew = {k: w[f"e{e}.{k}"] for k in ("gate", "up", "down")}
             y[t] += p * dense_mlp(h[t:t + 1], ew, mlp["expert"]["limit"])[0]
+    return y
+
+
+def swiglu_mlp(h, w):
+    return (silu(h @ w["gate"].T) * (h @ w["up"].T)) @ w["down"].T
+
+
+def route_sigmoid(h, router, correction, top):
+    """ids [T, top] by descending score + correction, and the chosen experts' scores, as they are."""
+    s = sigmoid(h @ router.T)
+    ids = np.argsort(-(s + correction), axis=-1, kind="stable")[:, :top]
+    return ids, np.take_along_axis(s, ids, axis=-1)
+
+
+def shared_moe_mlp(h, w, mlp):
+    """Sigmoid-routed experts, and a shared one that every token runs behind a gate of its own."""
+    ids, wts = route_sigmoid(h, w["router"], w["correction"], mlp["router"]["top"])
+    y = np.zeros_like(h)
+    for t in range(h.shape[0]):
+        for e, p in zip(ids[t], wts[t]):
+            y[t] += p * swiglu_mlp(h[t:t + 1], {k: w[f"e{e}.{k}"] for k in ("gate", "up", "down")})[0]
+    if mlp.get("shared"):
+        y += sigmoid(h @ w["shared.sg"].T) * swiglu_mlp(h, {k: w[f"shared.{k}"] for k in ("gate", "up", "down")})
     return y
 
 
@@ -219,3 +321,44 @@ class LayeredOracle:
         self.n_past += len(tokens)
         self.margin = np.concatenate([self.margin, margin])
         return self.norm(x, "final.norm") @ self.w["head"].T
+
+
+class FasesunOracle(LayeredOracle):
+    def runs(self):
+        """The layers in the order in which they run."""
+        n, loop = len(self.cfg["layers"]), self.cfg.get("loop")
+        if not loop:
+            return list(range(n))
+        a, b = loop["start"], loop["stop"]
+        return list(range(a)) + list(range(a, b)) * loop["times"] + list(range(b, n))
+
+    def reset(self):
+        super().reset()
+        self.state = [{} for _ in self.runs()]
+
+    def forward(self, tokens, layers=None):
+        eps, pos0 = self.cfg["norm"]["eps"], self.n_past
+        x = self.w["embed"][np.asarray(tokens)]
+        margin = np.full(len(tokens), np.inf)
+        for r, i in enumerate(self.runs()):
+            layer, p = self.cfg["layers"][i], f"l{i}."
+            m, mlp = layer["mixer"], layer.get("mlp")
+            h = rms_norm(x, eps) * self.w[p + "norm1"]
+            w = self.part(p + "mix.")
+            if layer["type"] == "latent_attention":
+                y = latent_attention(h, w, m, self.state[r], pos0, eps)
+            else:
+                y = {"mlstm": mlstm, "lightning": lightning}[layer["type"]](h, w, m, self.state[r], eps)
+            if mlp:
+                w = self.part(p + "mlp.")
+                y = y + shared_moe_mlp(h, w, mlp)
+                z = np.sort(sigmoid(h @ w["router"].T) + w["correction"], axis=-1)[:, ::-1]
+                top = mlp["router"]["top"]
+                if top < z.shape[1]:
+                    margin = np.minimum(margin, z[:, top - 1] - z[:, top])
+            x = x + y
+            if layers is not None:
+                layers.append(x.copy())
+        self.n_past += len(tokens)
+        self.margin = np.concatenate([self.margin, margin])
+        return (rms_norm(x, eps) * self.w["final.norm"]) @ self.w["embed"].T
