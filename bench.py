@@ -636,8 +636,9 @@ def plugin_moe_leg(prompt_len: int, n_decode: int, share_layers: bool, n_layer: 
 
 
 def _layered_sizes() -> dict:
-    """Layers of real models' sizes: name -> (Bozosun configuration, the qwen3 / qwen3moe configuration of the same sizes
-    that the library's tuned decoder runs, or None)."""
+    """Layers of real models' sizes: name -> (configuration of a layered decoder, the closest model of the same sizes to time
+    beside it: a qwen3 / qwen3moe configuration that the library's tuned decoder runs, or another layered decoder's, or
+    None)."""
     yarn = {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}
 
     def attn(heads, kv, mlp):
@@ -653,9 +654,22 @@ def _layered_sizes() -> dict:
     moe = {"kind": "moe", "expert": {"ff": 768, "limit": 7.0}, "router": {"experts": 128, "top": 8}}
     scan = {"type": "mamba1", "mixer": {"inner": 8192, "state": 16, "dt_rank": 256, "conv": 4}}
     base = dict(n_layer=4, vocab=32000, rms_eps=1e-6, rope_theta=1e6, head_dim=128)
+    attn_moe = model(2048, [attn(32, 4, moe)] * 4)
+    scan_moe = model(2048, [{"type": "mamba1", "mixer": {"inner": 4096, "state": 16, "dt_rank": 128, "conv": 4}, "mlp": moe}] * 4)
+
+    def fasesun(kind, **mixer):
+        mlp = {"kind": "moe", "expert": {"ff": 768}, "router": {"experts": 128, "top": 8}, "shared": {"ff": 768}}
+        return {"architecture": "Fasesun", "vocab": 32000, "width": 2048, "norm": {"eps": 1e-6}, "loop": None,
+                "layers": [{"type": kind, "mixer": mixer, "mlp": mlp}] * 4}
+
+    latent = fasesun("latent_attention", heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, scale=192 ** -0.5,
+                     rot={"dims": 64, "base": 1e6})
+    mlstm = fasesun("mlstm", heads=4, dim=256, vdim=512, gate_cap=15.0)
+    lightning = fasesun("lightning", heads=16, dim=128, vdim=128, decay=[1.0 - 2.0 ** (-1 - h / 2) for h in range(16)])
     return {
+        "latent_moe_2048": (latent, attn_moe), "matrix_memory_moe_2048": (mlstm, scan_moe), "constant_decay_moe_2048": (lightning, scan_moe),
         "attention_dense_4096": (model(4096, [attn(32, 8, dense)] * 4), dict(base, hidden=4096, n_head=32, n_kv_head=8, ffn=12288)),
-        "attention_moe_2048": (model(2048, [attn(32, 4, moe)] * 4), dict(base, hidden=2048, n_head=32, n_kv_head=4, ffn=0, n_expert=128,
+        "attention_moe_2048": (attn_moe, dict(base, hidden=2048, n_head=32, n_kv_head=4, ffn=0, n_expert=128,
                                                                          n_expert_used=8, expert_ffn=768)),
         "scan_dense_4096": (model(4096, [{**scan, "mlp": dense}] * 4), None),
     }
@@ -692,8 +706,9 @@ def _time_model(model, vocab: int, prompts, n_decode: int) -> dict:
 
 
 def layered_leg(only: str = "", prompts=(512, 2048), n_decode: int = 96) -> dict:
-    """The layered decoder (plain bf16 weights) at real models' layer sizes, four layers each, beside the qwen3 / qwen3moe
-    decoder (Q4_K_M blocks) of the same sizes; random weights, layers repeating one layer's values."""
+    """The layered decoders (plain bf16 weights) at real models' layer sizes, four layers each, beside the closest model of
+    the same sizes (the qwen3 / qwen3moe decoder over Q4_K_M blocks, or another layered decoder); random weights, layers
+    repeating one layer's values."""
     import tempfile
 
     from joshua_amd import capi
@@ -702,19 +717,26 @@ def layered_leg(only: str = "", prompts=(512, 2048), n_decode: int = 96) -> dict
 
     res = {}
     n_ctx = max(prompts) + n_decode + 8
+
+    def time_layered(cfg):
+        with tempfile.TemporaryDirectory() as tmp:
+            tensors = sl.layered_tensors(cfg, 3, share=True)
+            layer_bytes = sum(v.nbytes for k, v in tensors.items() if k.startswith("l"))
+            head_bytes = tensors["head" if "head" in tensors else "embed"].nbytes
+            model = capi.Model(sl.write_folder(tmp, cfg, tensors), n_ctx)
+            del tensors
+        times = _time_model(model, cfg["vocab"], prompts, n_decode)
+        model.close()
+        return cfg["architecture"].lower() + "_bf16", {"layer_weight_bytes": layer_bytes, "head_bytes": head_bytes, **times}
+
     for name, (cfg, like) in _layered_sizes().items():
         if only and only != name:
             continue
-        with tempfile.TemporaryDirectory() as tmp:
-            tensors = sl.bozosun_tensors(cfg, 3, share=True)
-            layer_bytes = sum(v.nbytes for k, v in tensors.items() if k.startswith("l"))
-            head_bytes = tensors["head"].nbytes
-            model = capi.Model(sl.write_folder(tmp, cfg, tensors), n_ctx)
-            del tensors
-        r = {"layers": len(cfg["layers"]), "layer_weight_bytes": layer_bytes, "head_bytes": head_bytes,
-             "bozosun_bf16": _time_model(model, cfg["vocab"], prompts, n_decode)}
-        model.close()
-        if like:
+        r = {"layers": len(cfg["layers"])}
+        for c in [cfg] + ([like] if like and "architecture" in like else []):
+            key, times = time_layered(c)
+            r[key] = times
+        if like and "architecture" not in like:
             c = capi.Qwen3Config(like["n_layer"], like["hidden"], like["n_head"], like["n_kv_head"], like["head_dim"], like["ffn"], like["vocab"],
                                  n_ctx, like["rms_eps"], like["rope_theta"], like.get("n_expert", 0), like.get("n_expert_used", 0),
                                  like.get("expert_ffn", 0), 1 if like.get("n_expert") else 0)
@@ -756,8 +778,8 @@ def main() -> int:
                          "once, as part of a full run (with the decode leg and all workloads) where 25 GB of temporary "
                          "space are free; 0: never")
     ap.add_argument("--layered", nargs="?", const="all", default="",
-                    help="only this: the layered decoder with plain weights (Bozosun) at real models' layer sizes beside the qwen3 "
-                         "decoder of equal size; a name picks one of the sizes")
+                    help="only this: the layered decoders with plain weights (Bozosun, Fasesun) at real models' layer sizes beside "
+                         "the closest model of equal size; a name picks one of the sizes")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this build has no multi-GPU path (run with --gpus 1)", file=sys.stderr)

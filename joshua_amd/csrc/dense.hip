@@ -117,7 +117,7 @@ int run_gemm(uint32_t type, jq::DenseGemm a, size_t rows_of_a, size_t k, size_t 
     const auto t = tiles(bm, bn);
     if (t.first * t.second > 0x7FFFFFFFull) return fail("dense gemm: too many tiles");
     a.m_tiles = (int)t.first;
-    a.splits = GROUPED ? 1 : gemm_splits(t.first * t.second, a.stages);
+    a.splits = GROUPED || a.heads ? 1 : gemm_splits(t.first * t.second, a.stages);
     CallScratch scratch;
     float *C = a.C;
     if (a.splits > 1) {
@@ -159,6 +159,17 @@ int dense_gemm(const jq_weight *w, const void *A, size_t lda, int T, float *C, s
     jq::DenseGemm a{};
     a.A = (const uint8_t *)A, a.W = w->dev, a.lda = (uint32_t)(lda * dense_elem_bytes(w->type)), a.ldw = (uint32_t)w->row_bytes;
     a.M = T, a.N = (int)w->n, a.C = C, a.ldc = ldc;
+    return run_gemm<false, false>(w->type, a, (size_t)T, w->k, 0, s);
+}
+
+int dense_gemm_heads(const jq_weight *w, size_t w_row, size_t n, const void *A, size_t lda, int T, void *out, int head_w, size_t head_stride,
+                     size_t head_row, hipStream_t s) {
+    if (lda < dense_stride(w->k) || lda % DENSE_PAD) return fail("dense gemm: activation rows of %zu elements for k = %zu", lda, w->k);
+    if (head_w <= 0 || head_w % 4 || n % head_w || head_stride % 4 || head_row % 4 || w_row + n > w->n)
+        return fail("dense gemm: %zu columns by heads of %d", n, head_w);
+    jq::DenseGemm a{};
+    a.A = (const uint8_t *)A, a.W = w->dev + w_row * w->row_bytes, a.lda = (uint32_t)(lda * dense_elem_bytes(w->type)), a.ldw = (uint32_t)w->row_bytes;
+    a.M = T, a.N = (int)n, a.heads = out, a.head_w = head_w, a.head_stride = head_stride, a.head_row = head_row;
     return run_gemm<false, false>(w->type, a, (size_t)T, w->k, 0, s);
 }
 

@@ -18,6 +18,11 @@ int dense_gemv_gated(const jq_weight *gate, const jq_weight *up, const float *X,
 // The same for any T over activations in the weights' type, rows `lda` elements apart (whole runs of 64, numbers behind
 // the k-th up to the next whole run); the gated product leaves its activations in that form too.
 int dense_gemm(const jq_weight *w, const void *A, size_t lda, int T, float *C, size_t ldc, hipStream_t s);
+// The same with the results in the weights' type, by heads of `head_w` columns (a multiple of 4; n is whole heads): column c
+// of row t at out[c / head_w * head_stride + t * head_row + c % head_w], strides in elements, multiples of 4.  w_row: the first
+// of the `n` rows of w to take.
+int dense_gemm_heads(const jq_weight *w, size_t w_row, size_t n, const void *A, size_t lda, int T, void *out, int head_w, size_t head_stride,
+                     size_t head_row, hipStream_t s);
 int dense_gemm_gated(const jq_weight *gate, const jq_weight *up, const void *A, size_t lda, int T, void *act, size_t ld_act,
                      const jq::GatedUnit &unit, hipStream_t s);
 // f32 rows in and out, rows packed: what jq_matmul_t runs for these types.

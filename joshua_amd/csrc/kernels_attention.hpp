@@ -304,7 +304,7 @@ __global__ __launch_bounds__(256) void attention_decode(AttnLayer a, int n_chunk
     if (tid < nh) po[tid * phead] = ml[tid][0], po[tid * phead + 1] = ml[tid][1];
 }
 
-// Steps of many tokens in bf16, head sizes up to DC: a workgroup of four waves takes 64 QF rows, a row being one of
+// Steps of many tokens in bf16, keys of up to DK and values of up to DV elements: a workgroup of four waves takes 64 QF rows, a row being one of
 // the gq query heads of a KV head at one token (row = token gq + head), so the heads share the keys and values staged.
 // Keys go by in tiles of KT.  Per tile and 16 rows:
 //   S^T = K Q^T            (lane: one row's scores of the keys 4 g + r, g = lane / 16)
@@ -312,12 +312,12 @@ __global__ __launch_bounds__(256) void attention_decode(AttnLayer a, int n_chunk
 //   O^T += V^T P^T         (values transposed on their way into LDS, the keys of a run of 32 in the order in which the
 //                           lanes hold their p: place 8 g + r for key 4 g + r, 8 g + 4 + r for key 16 + 4 g + r)
 // The weights p go into the second product as the sum of two bf16 numbers (16 bits of mantissa).
-template <int DC, int QF, int KT>
+template <int DK, int DV, int QF, int KT>
 __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, const __bf16 *__restrict__ qe, __bf16 *__restrict__ out,
                                                                size_t ldo, float scale_log2) {
-    constexpr int KCH = DC / 8, KROW = DC * 2, VROW = KT * 2 + 16, NK = KT * KCH / 256, NVU = KT / 2 * KCH / 256, DT = DC / 16, NF = KT / 16;
-    static_assert(NK * 256 == KT * KCH && NVU * 256 == KT / 2 * KCH, "whole loads a thread");
-    __shared__ __attribute__((aligned(16))) uint8_t ks[KT * KROW], vt[DC * VROW];
+    constexpr int KCH = DK / 8, KROW = DK * 2, VROW = KT * 2 + 16, NK = KT * KCH / 256, NVU = KT / 2 * (DV / 8) / 256, DT = DV / 16, NF = KT / 16;
+    static_assert(NK * 256 == KT * KCH && NVU * 256 == KT / 2 * (DV / 8) && DV % 64 == 0, "whole loads a thread");
+    __shared__ __attribute__((aligned(16))) uint8_t ks[KT * KROW], vt[DV * VROW];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, n = lane & 15, g = lane >> 4;
     const int gq = a.H / a.G, rows = a.T * gq;
     // the rows that see the most keys first, every other run of 256 workgroups in reverse: what a compute unit gets
@@ -330,7 +330,7 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
     const int last_key = a.pos0 + min(r0 + 64 * QF - 1, rows - 1) / gq, first_limit = a.pos0 + r0 / gq;
     const __bf16 *kb = (const __bf16 *)a.kc + (size_t)kvh * a.n_ctx * a.DP, *vb = (const __bf16 *)a.vc + (size_t)kvh * a.n_ctx * a.DVP;
 
-    u32x4 qf[QF][DC / 32];
+    u32x4 qf[QF][DK / 32];
     int limit[QF];
 #pragma unroll
     for (int q = 0; q < QF; q++) {
@@ -338,7 +338,7 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
         limit[q] = a.pos0 + t;
         const uint8_t *qp = (const uint8_t *)(qe + ((size_t)t * a.H + kvh * gq + r % gq) * a.DP);
 #pragma unroll
-        for (int k = 0; k < DC / 32; k++) qf[q][k] = 32 * k < a.DP ? *(const u32x4 *)(qp + 64 * k + 16 * g) : u32x4{0, 0, 0, 0};
+        for (int k = 0; k < DK / 32; k++) qf[q][k] = 32 * k < a.DP ? *(const u32x4 *)(qp + 64 * k + 16 * g) : u32x4{0, 0, 0, 0};
     }
     f32x4 o[QF][DT];
     float mx[QF], sum[QF];
@@ -359,7 +359,7 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
         }
 #pragma unroll
         for (int i = 0; i < NVU; i++) {
-            const int u = tid + 256 * i, c = ((u >> 3) & 7) + 8 * ((u >> 6) % (DC / 64)), pair = (u & 7) + 8 * ((u >> 6) / (DC / 64));
+            const int u = tid + 256 * i, c = ((u >> 3) & 7) + 8 * ((u >> 6) % (DV / 64)), pair = (u & 7) + 8 * ((u >> 6) / (DV / 64));
 #pragma unroll
             for (int b = 0; b < 2; b++) {
                 const int key = k0 + 2 * pair + b;
@@ -376,7 +376,7 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
         }
 #pragma unroll
         for (int i = 0; i < NVU; i++) {
-            const int u = tid + 256 * i, c = ((u >> 3) & 7) + 8 * ((u >> 6) % (DC / 64)), pair = (u & 7) + 8 * ((u >> 6) / (DC / 64));
+            const int u = tid + 256 * i, c = ((u >> 3) & 7) + 8 * ((u >> 6) % (DV / 64)), pair = (u & 7) + 8 * ((u >> 6) / (DV / 64));
             const int run = 2 * pair / 32, k = 2 * pair % 32, at = 64 * run + 2 * (k < 16 ? 8 * (k / 4) + k % 4 : 8 * ((k - 16) / 4) + 4 + k % 4);
 #pragma unroll
             for (int e = 0; e < 8; e++) {
@@ -392,7 +392,7 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_bf16(AttnLayer a, cons
 #pragma unroll
             for (int q = 0; q < QF; q++) st[q][f] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int k = 0; k < DC / 32; k++) {
+            for (int k = 0; k < DK / 32; k++) {
                 const u32x4 kf = *(const u32x4 *)(ks + (16 * f + n) * KROW + 16 * ((4 * k + g) ^ (n & 7)));
 #pragma unroll
                 for (int q = 0; q < QF; q++) st[q][f] = ElemBf16::mma(kf, qf[q][k], st[q][f]);

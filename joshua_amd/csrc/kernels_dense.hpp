@@ -377,6 +377,11 @@ struct DenseGemm {
     int splits;                    // runs of stages, one workgroup each; > 1: C holds the partial sums, [splits][M][width]
     float *C;
     size_t ldc;                    // elements
+    // not gated: the results in the element type instead, columns in runs of head_w (a multiple of 4): column c of row r
+    // at heads[c / head_w * head_stride + r * head_row + c % head_w]
+    void *heads;
+    int head_w;
+    size_t head_stride, head_row;
     void *act;                     // gated, splits 1: the activations, [M][ld_act] in the element type
     size_t ld_act;
     GatedUnit unit;
@@ -515,7 +520,18 @@ __global__ __launch_bounds__(256) void dense_gemm(DenseGemm a) {
         if constexpr (GROUPED) {
             if (a.yrow && !partial) orow = a.yrow[orow];
         }
-        if (!GATED || partial) {
+        if (!GATED && a.heads) {
+#pragma unroll
+            for (int n = 0; n < FN; n++) {
+                const int col = c0 + wn * (BN / 2) + 16 * n + 4 * g;
+                if (col >= a.N) continue;  // (N is whole runs)
+                typename E::T v[4];
+#pragma unroll
+                for (int r = 0; r < 4; r++) v[r] = (typename E::T)acc[n][m][r];
+                typename E::T *hp = (typename E::T *)a.heads + (size_t)(col / a.head_w) * a.head_stride + (size_t)orow * a.head_row + col % a.head_w;
+                __builtin_memcpy(__builtin_assume_aligned(hp, 4 * sizeof(typename E::T)), v, sizeof v);
+            }
+        } else if (!GATED || partial) {
 #pragma unroll
             for (int n = 0; n < FN; n++) {
                 const int col = (GATED ? 2 * c0 : c0) + wn * (BN / 2) + 16 * n + 4 * g;

@@ -95,8 +95,9 @@ __global__ __launch_bounds__(256) void latent_absorb(LatentLayer a, const uint8_
 }
 
 // Any element type and size: a workgroup takes one query head of a token over one of n_split runs of keys, LAT_RUN at a
-// time, with a running maximum; part[t, h, split] = {m, l, o[R]}, unnormalised.
+// time, with a running maximum; part[t, h, split] = {m, l, -, -, o[R]}, unnormalised.
 constexpr int LAT_RUN = 64, LAT_MAX_SPLIT = 64, LAT_MAX_R = 2048;
+__host__ __device__ inline int latent_part_width(int R) { return 4 + (R + 3) / 4 * 4; }
 
 template <class E>
 __global__ __launch_bounds__(256) void latent_attention_any(LatentLayer a, const float *__restrict__ qx, int n_split, float *__restrict__ part) {
@@ -140,58 +141,185 @@ __global__ __launch_bounds__(256) void latent_attention_any(LatentLayer a, const
         }
         __syncthreads();
     }
-    float *po = part + (((size_t)t * a.H + h) * n_split + split) * (a.R + 2);
+    float *po = part + (((size_t)t * a.H + h) * n_split + split) * latent_part_width(a.R);
 #pragma unroll
     for (int i = 0; i < LAT_MAX_R / 256; i++)
-        if (tid + 256 * i < a.R) po[2 + tid + 256 * i] = acc[i];
+        if (tid + 256 * i < a.R) po[4 + tid + 256 * i] = acc[i];
     if (tid == 0) po[0] = m, po[1] = l;
 }
 
-// The runs of a (token, head) merged, with the sink: olat[t, h] = sum_i f_i o_i / (sum_i f_i l_i + exp(sink - m)).  grid
-// (T H, runs of 256 columns).
-static __global__ __launch_bounds__(256) void latent_merge(const float *__restrict__ part, const float *__restrict__ sink, int H, int R,
-                                                           int n_split, float *__restrict__ olat) {
-    __shared__ float f[LAT_MAX_SPLIT], inv;
-    const float *p = part + (size_t)blockIdx.x * n_split * (R + 2);
-    if (threadIdx.x < 64) {
-        const int i = threadIdx.x;
-        const float mi = i < n_split ? p[(size_t)i * (R + 2)] : -INFINITY, li = i < n_split ? p[(size_t)i * (R + 2) + 1] : 0.0f;
-        const float M = wave_max(mi), fi = mi == -INFINITY ? 0.0f : expf(mi - M);  // (a run without keys)
-        float L = wave_sum(fi * li);
-        if (sink) L += expf(sink[blockIdx.x % H] - M);
-        if (i < LAT_MAX_SPLIT) f[i] = fi;
-        if (i == 0) inv = 1.0f / L;
+// The same in bf16 on the matrix cores: a workgroup takes 16 query heads of a token over a run of keys, 64 at a time.
+//   scores  S^T = K Q^T: a wave's 16 keys straight from the cache, the heads' queries in LDS
+//   softmax 16 threads a head, running maximum and sum; p goes on as the sum of two bf16 numbers
+//   sums    O^T += C^T P^T: the cache rows' columns, 64 a wave at a time, transposed through LDS
+// NB: runs of 256 latent columns.
+constexpr int LATM_SROW = 68, LATM_PROW = 144;
+__host__ __device__ inline int latent_query_row(int RP) { return 2 * RP + 16; }  // bytes
+inline size_t latent_mfma_lds(int RP) { return (size_t)16 * latent_query_row(RP) + 16 * LATM_SROW * 4 + 2 * 16 * LATM_PROW + 4 * 64 * LATM_PROW + 64; }
+
+template <int NB>
+__global__ __launch_bounds__(256) void latent_attention_mfma(LatentLayer a, const float *__restrict__ qx, int n_split, float *__restrict__ part) {
+    constexpr int KF = 18;
+    extern __shared__ __attribute__((aligned(16))) uint8_t lmem[];
+    const int qrow = latent_query_row(a.RP);
+    uint8_t *qs = lmem, *ph = qs + 16 * qrow, *pl = ph + 16 * LATM_PROW, *stage = pl + 16 * LATM_PROW;
+    float *sc = (float *)(stage + 4 * 64 * LATM_PROW), *al = sc + 16 * LATM_SROW;
+    const int split = blockIdx.x, h0 = 16 * (int)blockIdx.y, t = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
+    const int n = a.pos0 + t + 1, per = ((n + LAT_RUN - 1) / LAT_RUN + n_split - 1) / n_split * LAT_RUN;
+    const int lo = split * per, hi = min(n, lo + per);
+    const __bf16 *cache = (const __bf16 *)a.cache;
+    for (int e = tid; e < 16 * (a.RP / 4); e += 256) {
+        const int r = e / (a.RP / 4), c = 4 * (e % (a.RP / 4));
+        const f32x4 v = *(const f32x4 *)(qx + ((size_t)t * a.H + min(h0 + r, a.H - 1)) * a.RP + c);
+        *(uint2 *)(qs + r * qrow + 2 * c) = __builtin_bit_cast(uint2, __builtin_convertvector(v, bf16x4));
     }
+    f32x4 o[NB][4];
+#pragma unroll
+    for (int b = 0; b < NB; b++)
+#pragma unroll
+        for (int i = 0; i < 4; i++) o[b][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m = -INFINITY, l = 0.0f;  // of head tid / 16, the same in its 16 threads
+    uint8_t *mine = stage + wave * 64 * LATM_PROW;
     __syncthreads();
-    const int c = (int)blockIdx.y * 256 + (int)threadIdx.x;
-    if (c >= R) return;
-    float v = 0.0f;
-#pragma unroll 8
-    for (int i = 0; i < n_split; i++) v = fmaf(p[(size_t)i * (R + 2) + 2 + c], f[i], v);
-    olat[(size_t)blockIdx.x * R + c] = v * inv;
+    for (int j0 = lo; j0 < hi; j0 += LAT_RUN) {
+        const int nj = min(LAT_RUN, hi - j0);
+        const __bf16 *kr = cache + (size_t)(j0 + min(16 * wave + l16, nj - 1)) * a.RP + 8 * g;
+        f32x4 st{0.f, 0.f, 0.f, 0.f};
+        for (int c0 = 0; c0 < a.RP; c0 += 32 * KF) {  // KF fragments of the row on their way at once
+            u32x4 kf[KF];
+#pragma unroll
+            for (int i = 0; i < KF; i++)
+                if (c0 + 32 * i < a.RP) kf[i] = *(const u32x4 *)(kr + c0 + 32 * i);
+#pragma unroll
+            for (int i = 0; i < KF; i++)
+                if (c0 + 32 * i < a.RP) st = ElemBf16::mma(kf[i], *(const u32x4 *)(qs + l16 * qrow + 2 * (c0 + 32 * i) + 16 * g), st);
+        }
+        *(f32x4 *)(sc + l16 * LATM_SROW + 16 * wave + 4 * g) = st;
+        __syncthreads();
+        {
+            const int hd = tid >> 4, k = 4 * (tid & 15);
+            f32x4 s = *(const f32x4 *)(sc + hd * LATM_SROW + k), p;
+#pragma unroll
+            for (int r = 0; r < 4; r++) s[r] = k + r < nj ? s[r] * a.scale : -INFINITY;
+            const float mn = fmaxf(m, max_row16(fmaxf(fmaxf(s[0], s[1]), fmaxf(s[2], s[3]))));  // (key j0 is there: finite)
+#pragma unroll
+            for (int r = 0; r < 4; r++) p[r] = expf(s[r] - mn);
+            const float keep = expf(m - mn);
+            l = fmaf(l, keep, sum_row16((p[0] + p[1]) + (p[2] + p[3])));
+            m = mn;
+            const bf16x4 hi4 = __builtin_convertvector(p, bf16x4), lo4 = __builtin_convertvector(p - __builtin_convertvector(hi4, f32x4), bf16x4);
+            *(uint2 *)(ph + hd * LATM_PROW + 2 * k) = __builtin_bit_cast(uint2, hi4);
+            *(uint2 *)(pl + hd * LATM_PROW + 2 * k) = __builtin_bit_cast(uint2, lo4);
+            if ((tid & 15) == 0) al[hd] = keep;
+        }
+#pragma unroll
+        for (int b = 0; b < NB; b++) {
+            // unit: tokens 2 pair, 2 pair + 1 and columns 8 c .. 8 c + 7 of this wave's 64
+            u32x4 ra[4], rb[4];
+            const int c0 = 256 * b + 64 * wave + 8 * (lane >> 3 & 7);
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int pair = (lane & 7) + 8 * i;
+                const __bf16 *base = cache + (c0 < a.RP ? c0 : 0);
+                ra[i] = *(const u32x4 *)(base + (size_t)(j0 + min(2 * pair, nj - 1)) * a.RP);
+                rb[i] = *(const u32x4 *)(base + (size_t)(j0 + min(2 * pair + 1, nj - 1)) * a.RP);
+            }
+            __syncthreads();  // p is there; and the fragments of the columns before are read
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int pair = (lane & 7) + 8 * i;
+#pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    const uint32_t x = ra[i][e / 2], y = rb[i][e / 2];
+                    *(uint32_t *)(mine + (8 * (lane >> 3 & 7) + e) * LATM_PROW + 4 * pair) =
+                        e & 1 ? (x >> 16) | (y & 0xFFFF0000u) : (x & 0xFFFFu) | (y << 16);
+                }
+            }
+            __syncthreads();
+            const float keep = al[l16];
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) o[b][i][r] *= keep;
+#pragma unroll
+            for (int ks = 0; ks < 2; ks++) {
+                const u32x4 fh = *(const u32x4 *)(ph + l16 * LATM_PROW + 64 * ks + 16 * g), fl = *(const u32x4 *)(pl + l16 * LATM_PROW + 64 * ks + 16 * g);
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const u32x4 v = *(const u32x4 *)(mine + (16 * i + l16) * LATM_PROW + 64 * ks + 16 * g);
+                    o[b][i] = ElemBf16::mma(v, fh, o[b][i]);
+                    o[b][i] = ElemBf16::mma(v, fl, o[b][i]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+    const int pw = latent_part_width(a.R);
+    if (h0 + l16 < a.H) {
+        float *po = part + (((size_t)t * a.H + h0 + l16) * n_split + split) * pw + 4;
+#pragma unroll
+        for (int b = 0; b < NB; b++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int c = 256 * b + 64 * wave + 16 * i + 4 * g;
+                if (4 + c < pw) *(f32x4 *)(po + c) = o[b][i];
+            }
+    }
+    if ((tid & 15) == 0 && h0 + (tid >> 4) < a.H) {
+        float *po = part + (((size_t)t * a.H + h0 + (tid >> 4)) * n_split + split) * pw;
+        po[0] = m, po[1] = l;
+    }
 }
 
-// out[t, h dv + j] = sigmoid(gate) (W_uv[h dv + j, :] . olat[t, h]): a wave takes four rows; grid (runs of 16 rows, heads, tokens).
+// The runs of a (token, head) merged, with the sink, o = sum_i f_i o_i / (sum_i f_i l_i + exp(sink - m)), then
+// out[t, h dv + j] = sigmoid(gate) (W_uv[h dv + j, :] . o): a wave takes LAT_VROWS rows; grid (runs of 4 LAT_VROWS rows,
+// heads, tokens).
+constexpr int LAT_VROWS = 8;
+
 template <class E>
-__global__ __launch_bounds__(256) void latent_values(LatentLayer a, const float *__restrict__ olat, const uint8_t *__restrict__ Wuv,
+__global__ __launch_bounds__(256) void latent_values(LatentLayer a, const float *__restrict__ part, int n_split, const uint8_t *__restrict__ Wuv,
                                                      size_t pitch, float *__restrict__ out) {
-    const int h = blockIdx.y, t = blockIdx.z, lane = threadIdx.x & 63, j0 = ((int)blockIdx.x * 4 + ((int)threadIdx.x >> 6)) * 4;
+    __shared__ __attribute__((aligned(16))) float ol[LAT_MAX_R];
+    __shared__ float f[LAT_MAX_SPLIT], total;
+    const int h = blockIdx.y, t = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, pw = latent_part_width(a.R);
+    const int j0 = ((int)blockIdx.x * 4 + wave) * LAT_VROWS;
+    const float *p = part + ((size_t)t * a.H + h) * n_split * pw;
+    if (wave == 0) {
+        const float mi = lane < n_split ? p[(size_t)lane * pw] : -INFINITY, li = lane < n_split ? p[(size_t)lane * pw + 1] : 0.0f;
+        const float M = wave_max(mi), fi = mi == -INFINITY ? 0.0f : expf(mi - M);  // (a run without keys)
+        float L = wave_sum(fi * li);
+        if (a.sink) L += expf(a.sink[h] - M);
+        f[lane] = fi;
+        if (lane == 0) total = L;
+    }
+    __syncthreads();
+    const float inv = 1.0f / total;
+    for (int c = threadIdx.x; c < a.R; c += 256) {
+        float v = 0.0f;
+#pragma unroll 16
+        for (int i = 0; i < n_split; i++) v = fmaf(p[(size_t)i * pw + 4 + c], f[i], v);
+        ol[c] = v * inv;
+    }
+    __syncthreads();
     if (j0 >= a.dv) return;
-    const float *x = olat + ((size_t)t * a.H + h) * a.R;
-    float acc[4] = {};
+    float acc[LAT_VROWS] = {};
     for (int c = lane * E::CH; c < a.R; c += 64 * E::CH) {
+        u32x4 w[LAT_VROWS];
+#pragma unroll
+        for (int r = 0; r < LAT_VROWS; r++) w[r] = chunk_of<E>(Wuv + (size_t)(h * a.dv + min(j0 + r, a.dv - 1)) * pitch, c);
         float xv[E::CH];
-        load_acts<E::CH>(x, c, a.R, xv);
+        load_acts<E::CH>(ol, c, a.R, xv);
 #pragma unroll
-        for (int r = 0; r < 4; r++) {
-            float w[E::CH];
-            E::widen(chunk_of<E>(Wuv + (size_t)(h * a.dv + min(j0 + r, a.dv - 1)) * pitch, c), w);
+        for (int r = 0; r < LAT_VROWS; r++) {
+            float wv[E::CH];
+            E::widen(w[r], wv);
 #pragma unroll
-            for (int i = 0; i < E::CH; i++) acc[r] = fmaf(w[i], xv[i], acc[r]);
+            for (int i = 0; i < E::CH; i++) acc[r] = fmaf(wv[i], xv[i], acc[r]);
         }
     }
 #pragma unroll
-    for (int r = 0; r < 4; r++) {
+    for (int r = 0; r < LAT_VROWS; r++) {
         const float v = wave_sum(acc[r]);
         if (lane == r && j0 + r < a.dv) {
             const int col = h * a.dv + j0 + r;
@@ -218,23 +346,37 @@ __global__ __launch_bounds__(256) void latent_expand(LatentLayer a, const float 
     }
 }
 
+// What products written by heads leave of those rows: the keys' rotated part and the zeros behind keys and values.
+template <class E>
+__global__ __launch_bounds__(256) void latent_rest_of_keys(LatentLayer a, int n, int DP, int DVP, typename E::T *__restrict__ kc,
+                                                           typename E::T *__restrict__ vc) {
+    using T = typename E::T;
+    const int j = blockIdx.x, kr = DP - a.d, vr = DVP - a.dv;
+    const T *rot = (const T *)a.cache + (size_t)j * a.RP + a.R;
+    for (int e = threadIdx.x; e < a.H * kr; e += 256) {
+        const int h = e / kr, c = e % kr;
+        kc[((size_t)h * n + j) * DP + a.d + c] = c < a.rd ? rot[c] : (T)0.0f;
+    }
+    for (int e = threadIdx.x; e < a.H * vr; e += 256) vc[((size_t)(e / vr) * n + j) * DVP + a.dv + e % vr] = (T)0.0f;
+}
+
 // The step's queries [T][H][DP], the rotated part turned.
 template <class E>
 __global__ __launch_bounds__(256) void latent_queries(LatentLayer a, int DP, typename E::T *__restrict__ qe) {
-    using T = typename E::T;
+    typedef typename E::T T2 __attribute__((ext_vector_type(2)));
     const int t = blockIdx.x, qd = a.d + a.rd;
     const float *row = a.q + (size_t)t * a.H * qd;
     const float2 *cs = a.cs + (size_t)t * (a.rot / 2);
-    for (int e = threadIdx.x; e < a.H * DP; e += 256) {
-        const int h = e / DP, c = e % DP;
-        float v = 0.0f;
-        if (c < a.d) {
-            v = row[h * qd + c];
-        } else if (c < qd) {
-            const float2 p = rotated_pair(row + h * qd + a.d, (c - a.d) / 2, a.rd, a.rot, cs);
-            v = (c - a.d) & 1 ? p.y : p.x;
-        }
-        qe[((size_t)t * a.H + h) * DP + c] = (T)v;
+    for (int e = threadIdx.x; e < a.H * (DP / 2); e += 256) {
+        const int h = e / (DP / 2), c0 = 2 * (e % (DP / 2));
+        const float *q = row + h * qd;
+        auto element = [&](int c) {
+            if (c < a.d) return q[c];
+            if (c >= qd) return 0.0f;
+            const float2 p = rotated_pair(q + a.d, (c - a.d) / 2, a.rd, a.rot, cs);
+            return (c - a.d) & 1 ? p.y : p.x;
+        };
+        *(T2 *)(qe + ((size_t)t * a.H + h) * DP + c0) = T2{(typename E::T)element(c0), (typename E::T)element(c0 + 1)};
     }
 }
 

@@ -17,7 +17,7 @@
 namespace jq {
 
 struct LinearLayer {
-    int H, d, dv, rows, DP;      // rows: dv, or dv + 1 with the normaliser's; DP: d rounded up to 4, floats from a row of S to the next
+    int H, d, dv, rows, DP;      // rows: dv, or dv + 1 with the normaliser's; DP: d rounded up to 32, floats from a row of S to the next
     int memory;                  // 1: gates, maximum and normaliser; 0: constant decay
     int T;
     const float *proj;           // [T][ld]: the projections of a token, in places q, k, v, zi, zf
@@ -116,6 +116,297 @@ __global__ __launch_bounds__(256) void linear_steps(LinearLayer a) {
         }
     }
     if (a.memory && blockIdx.x == 0 && tid == 0) a.m_out[h] = m;
+}
+
+// ---- many tokens in bf16: runs of LIN_CHUNK tokens ----
+//
+//   linear_prepare      q, k, v of every token in bf16, padded, and its log weights
+//   linear_gates        per head: g, M and m of every token, the maximum in front of every chunk and what a chunk leaves of
+//                       the state before it
+//   linear_chunk_state  per chunk: sum_s exp(g_s - M_end) v_s k_s^T (the normaliser's row has v = 1)
+//   linear_state_pass   per element of the state, chunk after chunk: the state in front of every chunk, in place
+//   linear_chunk_out    per chunk: o_t = sum_{s <= t} exp(g_s - M_t) (q_t . k_s) v_s + exp(m_0 - M_t) S_0 q_t
+//
+// f32 numbers (weights, states) enter a product as the sum of two bf16 numbers; every sum is f32.
+constexpr int LIN_CHUNK = 64, LIN_SEGMENT = 4096;  // tokens a launch set takes at most
+
+struct LinearChunks {
+    int H, DQ, VP, RS, T, nc;    // DQ: d rounded up to 32; VP: elements of a head's v; RS: rows of a chunk's state, rounded up to 16
+    int OP;
+    __bf16 *q, *k, *v;           // [T][H][DQ], [T][H][DQ], [T][H][VP]
+    float *gi, *gf;              // [H][nc LIN_CHUNK]: log write and keep weights; then g and M
+    float *m_at, *carry;         // [H][nc]: m in front of a chunk; the factor on the state across it
+    float *S;                    // [H][nc][RS][DQ]
+    float *o;                    // [T][H][OP]
+};
+
+__device__ __forceinline__ float exp_of(float v) { return __builtin_amdgcn_exp2f(1.44269504088896341f * v); }
+
+static __global__ __launch_bounds__(256) void linear_prepare(LinearLayer a, LinearChunks c) {
+    const int t = blockIdx.x;
+    const float *p = a.proj + (size_t)t * a.ld;
+    const int pairs = a.H * (c.DQ / 2);
+    for (int e = threadIdx.x; e < 2 * pairs; e += 256) {
+        const int key = e >= pairs, i = e - key * pairs, h = i / (c.DQ / 2), d = 2 * (i % (c.DQ / 2));
+        const float *src = p + (key ? a.k_at : a.q_at) + h * a.d;
+        const float f = key ? 1.0f : a.q_scale;
+        __bf16 *dst = (key ? c.k : c.q) + ((size_t)t * a.H + h) * c.DQ + d;
+        dst[0] = (__bf16)(d < a.d ? linear_input(a, src[d]) * f : 0.0f), dst[1] = (__bf16)(d + 1 < a.d ? linear_input(a, src[d + 1]) * f : 0.0f);
+    }
+    for (int e = threadIdx.x; e < a.H * c.VP; e += 256) {
+        const int h = e / c.VP, r = e % c.VP;
+        c.v[(size_t)t * a.H * c.VP + e] = (__bf16)(r < a.dv ? linear_input(a, p[a.v_at + h * a.dv + r]) : r < a.rows ? 1.0f : 0.0f);
+    }
+    for (int h = threadIdx.x; h < a.H; h += 256) {
+        const size_t at = (size_t)h * c.nc * LIN_CHUNK + t;
+        linear_gates_of(a, t, h, &c.gi[at], &c.gf[at]);
+    }
+}
+
+// One workgroup of 16 waves a head, a wave a chunk at a time.
+static __global__ __launch_bounds__(1024) void linear_gates(LinearLayer a, LinearChunks c) {
+    constexpr int MAX = LIN_SEGMENT / LIN_CHUNK;
+    __shared__ float F_end[MAX], g_top[MAX], m_at[MAX];
+    const int h = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    float *gi = c.gi + (size_t)h * c.nc * LIN_CHUNK, *gf = c.gf + (size_t)h * c.nc * LIN_CHUNK;
+    constexpr int PER = MAX / 16;
+    float F[PER], top[PER];
+#pragma unroll
+    for (int u = 0; u < PER; u++) {
+        const int n = wave + 16 * u, t = n * LIN_CHUNK + lane;
+        if (n >= c.nc) continue;
+        const bool live = t < c.T;
+        float f = live ? gf[t] : 0.0f, i = live ? gi[t] : -INFINITY;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const float v = __shfl_up(f, off, 64);
+            if (lane >= off) f += v;
+        }
+        float g = i - f, mx = g;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const float v = __shfl_up(mx, off, 64);
+            if (lane >= off) mx = fmaxf(mx, v);
+        }
+        gi[t] = g, F[u] = f, top[u] = mx;
+        if (lane == 63) F_end[n] = f, g_top[n] = mx;
+    }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+        float m = a.memory ? a.m_in[h] : 0.0f;
+        for (int n = 0; n < c.nc; n++) {
+            m_at[n] = m;
+            c.m_at[h * c.nc + n] = m;
+            const float M = a.memory ? fmaxf(m, g_top[n]) : -F_end[n];
+            c.carry[h * c.nc + n] = expf(m - M);
+            m = F_end[n] + M;
+        }
+        if (a.memory) a.m_out[h] = m;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < PER; u++) {
+        const int n = wave + 16 * u, t = n * LIN_CHUNK + lane;
+        if (n >= c.nc) continue;
+        const float M = a.memory ? fmaxf(m_at[n], top[u]) : -F[u];
+        gf[t] = M;
+        if (a.memory && t < c.T) a.mt[(size_t)t * a.H + h] = F[u] + M;
+    }
+}
+
+// A tile of 64 tokens x 64 columns of bf16, 16 bytes a token and thread pair, on its way into LDS with the tokens side by
+// side: unit u (the thread) holds columns 8 c .. 8 c + 7 of tokens 2 pair and 2 pair + 1.
+struct TileUnit {
+    int c, pair;
+    __device__ __forceinline__ explicit TileUnit(int u) : c((u >> 3) & 7), pair((u & 7) + 8 * (u >> 6)) {}
+};
+constexpr int LIN_TROW = LIN_CHUNK * 2 + 16;  // bytes of a column's tokens
+
+// grid (chunks, runs of 64 state rows, heads)
+static __global__ __launch_bounds__(256) void linear_chunk_state(LinearChunks c) {
+    __shared__ __attribute__((aligned(16))) uint8_t vh[64 * LIN_TROW], vl[64 * LIN_TROW], kt[64 * LIN_TROW];
+    const int n = blockIdx.x, v0 = 64 * (int)blockIdx.y, h = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
+    const TileUnit u(tid);
+    const int t0 = n * LIN_CHUNK + 2 * u.pair, ta = min(t0, c.T - 1), tb = min(t0 + 1, c.T - 1);
+    const float *gi = c.gi + ((size_t)h * c.nc + n) * LIN_CHUNK;
+    const float M = c.gf[((size_t)h * c.nc + n) * LIN_CHUNK + LIN_CHUNK - 1];
+    {
+        const float wa = exp_of(gi[2 * u.pair] - M), wb = exp_of(gi[2 * u.pair + 1] - M);  // (past the last token: 0)
+        u32x4 ra{0, 0, 0, 0}, rb{0, 0, 0, 0};
+        if (v0 + 8 * u.c < c.VP) {
+            ra = *(const u32x4 *)(c.v + ((size_t)ta * c.H + h) * c.VP + v0 + 8 * u.c);
+            rb = *(const u32x4 *)(c.v + ((size_t)tb * c.H + h) * c.VP + v0 + 8 * u.c);
+        }
+        float fa[8], fb[8];
+        ElemBf16::widen(ra, fa), ElemBf16::widen(rb, fb);
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            const float x = wa * fa[e], y = wb * fb[e];
+            const __bf16 xh = (__bf16)x, yh = (__bf16)y, xl = (__bf16)(x - (float)xh), yl = (__bf16)(y - (float)yh);
+            const int at = (8 * u.c + e) * LIN_TROW + 4 * u.pair;
+            *(uint32_t *)(vh + at) = __builtin_bit_cast(uint16_t, xh) | (uint32_t)__builtin_bit_cast(uint16_t, yh) << 16;
+            *(uint32_t *)(vl + at) = __builtin_bit_cast(uint16_t, xl) | (uint32_t)__builtin_bit_cast(uint16_t, yl) << 16;
+        }
+    }
+    const __bf16 *ka = c.k + ((size_t)ta * c.H + h) * c.DQ, *kb = c.k + ((size_t)tb * c.H + h) * c.DQ;
+    const int vrow = v0 + 16 * wave + l16;
+    float *out = c.S + (((size_t)h * c.nc + n) * c.RS + min(vrow, c.RS - 1)) * c.DQ;
+    for (int d0 = 0; d0 < c.DQ; d0 += 64) {
+        const bool in = d0 + 8 * u.c < c.DQ;
+        const u32x4 ra = *(const u32x4 *)(ka + (in ? d0 + 8 * u.c : 0)), rb = *(const u32x4 *)(kb + (in ? d0 + 8 * u.c : 0));
+        if (d0) __syncthreads();
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            const uint32_t lo = ra[e / 2], hi = rb[e / 2];
+            *(uint32_t *)(kt + (8 * u.c + e) * LIN_TROW + 4 * u.pair) = e & 1 ? (lo >> 16) | (hi & 0xFFFF0000u) : (lo & 0xFFFFu) | (hi << 16);
+        }
+        __syncthreads();
+        f32x4 acc[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < 2; ks++) {
+            const int at = 64 * ks + 16 * g, vat = (16 * wave + l16) * LIN_TROW + at;
+            const u32x4 fh = *(const u32x4 *)(vh + vat), fl = *(const u32x4 *)(vl + vat);
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const u32x4 fk = *(const u32x4 *)(kt + (16 * i + l16) * LIN_TROW + at);
+                acc[i] = ElemBf16::mma(fk, fh, acc[i]);
+                acc[i] = ElemBf16::mma(fk, fl, acc[i]);
+            }
+        }
+        if (vrow < c.RS) {
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                if (d0 + 16 * i < c.DQ) *(f32x4 *)(out + d0 + 16 * i + 4 * g) = acc[i];
+        }
+    }
+}
+
+// A thread has four elements of a head's state: S is the sequence's, [H][rows][DP].
+static __global__ __launch_bounds__(256) void linear_state_pass(LinearChunks c, float *__restrict__ S, int rows) {
+    const int per = rows * (c.DQ / 4), e = (int)blockIdx.x * 256 + (int)threadIdx.x, h = blockIdx.y;
+    if (e >= per) return;
+    f32x4 *state = (f32x4 *)(S + (size_t)h * rows * c.DQ) + e;
+    const size_t step = (size_t)c.RS * c.DQ / 4;
+    f32x4 *p = (f32x4 *)(c.S + (size_t)h * c.nc * c.RS * c.DQ) + e;
+    const float *carry = c.carry + h * c.nc;
+    f32x4 s = *state, next[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) next[i] = p[min(i, c.nc - 1) * step];
+    for (int n = 0; n < c.nc; n += 4) {
+        f32x4 now[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) now[i] = next[i];
+#pragma unroll
+        for (int i = 0; i < 4; i++) next[i] = p[min(n + 4 + i, c.nc - 1) * step];  // (the last one again past the end)
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            if (n + i < c.nc) {
+                p[(n + i) * step] = s;
+                const float f = carry[n + i];
+#pragma unroll
+                for (int r = 0; r < 4; r++) s[r] = fmaf(f, s[r], now[i][r]);
+            }
+        }
+    }
+    *state = s;
+}
+
+// x as the sum of two bf16 numbers, for eight elements.
+__device__ __forceinline__ void split_bf16(const f32x4 &a, const f32x4 &b, u32x4 *hi, u32x4 *lo) {
+    const bf16x4 ha = __builtin_convertvector(a, bf16x4), hb = __builtin_convertvector(b, bf16x4);
+    const bf16x4 la = __builtin_convertvector(a - __builtin_convertvector(ha, f32x4), bf16x4);
+    const bf16x4 lb = __builtin_convertvector(b - __builtin_convertvector(hb, f32x4), bf16x4);
+    const uint2 h0 = __builtin_bit_cast(uint2, ha), h1 = __builtin_bit_cast(uint2, hb), l0 = __builtin_bit_cast(uint2, la), l1 = __builtin_bit_cast(uint2, lb);
+    *hi = u32x4{h0.x, h0.y, h1.x, h1.y}, *lo = u32x4{l0.x, l0.y, l1.x, l1.y};
+}
+
+// grid (chunks, runs of 64 state rows, heads); wave w has tokens 16 w .. 16 w + 15 of the chunk, lane l16 one of them.
+static __global__ __launch_bounds__(256) void linear_chunk_out(LinearChunks c) {
+    __shared__ __attribute__((aligned(16))) uint8_t vt[64 * LIN_TROW];
+    __shared__ float gs[LIN_CHUNK];
+    const int n = blockIdx.x, v0 = 64 * (int)blockIdx.y, h = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
+    const size_t at = ((size_t)h * c.nc + n) * LIN_CHUNK;
+    if (tid < LIN_CHUNK) gs[tid] = c.gi[at + tid];
+    {  // values with the tokens of a run of 32 in the order in which the lanes will hold their weights
+        const TileUnit u(tid);
+        const int t0 = n * LIN_CHUNK + 2 * u.pair, ta = min(t0, c.T - 1), tb = min(t0 + 1, c.T - 1);
+        u32x4 ra{0, 0, 0, 0}, rb{0, 0, 0, 0};
+        if (v0 + 8 * u.c < c.VP) {
+            ra = *(const u32x4 *)(c.v + ((size_t)ta * c.H + h) * c.VP + v0 + 8 * u.c);
+            rb = *(const u32x4 *)(c.v + ((size_t)tb * c.H + h) * c.VP + v0 + 8 * u.c);
+        }
+        const int run = 2 * u.pair / 32, k = 2 * u.pair % 32, place = 64 * run + 2 * (k < 16 ? 8 * (k / 4) + k % 4 : 8 * ((k - 16) / 4) + 4 + k % 4);
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            const uint32_t lo = ra[e / 2], hi = rb[e / 2];
+            *(uint32_t *)(vt + (8 * u.c + e) * LIN_TROW + place) = e & 1 ? (lo >> 16) | (hi & 0xFFFF0000u) : (lo & 0xFFFFu) | (hi << 16);
+        }
+    }
+    const int tl = 16 * wave + l16, t = n * LIN_CHUNK + tl;
+    const float M = c.gf[at + tl];
+    const __bf16 *qr = c.q + ((size_t)min(t, c.T - 1) * c.H + h) * c.DQ + 8 * g;
+    const __bf16 *kr[4];
+    const float *sr[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        kr[i] = c.k + ((size_t)min(n * LIN_CHUNK + 16 * i + l16, c.T - 1) * c.H + h) * c.DQ + 8 * g;
+        sr[i] = c.S + (((size_t)h * c.nc + n) * c.RS + min(v0 + 16 * i + l16, c.RS - 1)) * c.DQ + 8 * g;
+    }
+    f32x4 st[4], from[4], acc[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) st[i] = from[i] = acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int d = 0; d < c.DQ; d += 32) {
+        const u32x4 q = *(const u32x4 *)(qr + d);
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (i <= wave) st[i] = ElemBf16::mma(*(const u32x4 *)(kr[i] + d), q, st[i]);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            if (v0 + 16 * i < c.RS) {
+                u32x4 hi, lo;
+                split_bf16(*(const f32x4 *)(sr[i] + d), *(const f32x4 *)(sr[i] + d + 4), &hi, &lo);
+                from[i] = ElemBf16::mma(hi, q, from[i]);
+                from[i] = ElemBf16::mma(lo, q, from[i]);
+            }
+        }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int run = 0; run < 2; run++) {
+        if (2 * run > wave) break;
+        f32x4 p[2];
+#pragma unroll
+        for (int f = 0; f < 2; f++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int s = 32 * run + 16 * f + 4 * g + r;
+                p[f][r] = s <= tl ? st[2 * run + f][r] * exp_of(gs[s] - M) : 0.0f;
+            }
+        u32x4 hi, lo;
+        split_bf16(p[0], p[1], &hi, &lo);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const u32x4 vf = *(const u32x4 *)(vt + (16 * i + l16) * LIN_TROW + 64 * run + 16 * g);
+            acc[i] = ElemBf16::mma(vf, hi, acc[i]);
+            acc[i] = ElemBf16::mma(vf, lo, acc[i]);
+        }
+    }
+    if (t >= c.T) return;
+    const float in = exp_of(c.m_at[h * c.nc + n] - M);
+    float *op = c.o + ((size_t)t * c.H + h) * c.OP + v0 + 4 * g;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        if (v0 + 16 * i + 4 * g < c.OP) {
+            f32x4 o;
+#pragma unroll
+            for (int r = 0; r < 4; r++) o[r] = fmaf(in, from[i][r], acc[i][r]);
+            *(f32x4 *)(op + 16 * i) = o;
+        }
+    }
 }
 
 // The mixer's output rows out of S q: the matrix memory's normaliser, a root mean square norm (over a head, or over all

@@ -42,7 +42,7 @@ struct LayerConfig {
 
     bool linear() const { return mixer == MLSTM || mixer == LIGHTNING; }
     int state_rows() const { return vdim + (mixer == MLSTM ? 1 : 0); }  // of a head of a linear mixer
-    int state_pitch() const { return (dim + 3) / 4 * 4; }
+    int state_pitch() const { return (dim + 31) / 32 * 32; }
     int out_pitch() const { return (state_rows() + 3) / 4 * 4; }
     int latent_pitch() const { return (int)dense_stride(kv_rank + rot_dim); }
 };
@@ -109,6 +109,7 @@ struct Layer {
 
     int DP() const { return (c.dim + c.rot_dim + 31) / 32 * 32; }
     int DVP() const { return (c.vdim + 31) / 32 * 32; }
+    bool latent_by_heads() const { return c.dim % 4 == 0 && c.vdim % 4 == 0; }  // keys and values straight from the product
     int mix_width() const { return c.mixer == LayerConfig::MAMBA1 ? c.inner : c.heads * c.vdim; }
 };
 
@@ -146,8 +147,8 @@ struct LayeredModel : jq_model {
     uint32_t *ids = nullptr, *want_ids = nullptr;
     float *x = nullptr, *x2 = nullptr, *h = nullptr, *y = nullptr, *proj = nullptr, *mid = nullptr, *conv_f = nullptr, *bc = nullptr,
           *dt = nullptr, *first_v = nullptr, *part = nullptr, *lin_o = nullptr, *lin_m = nullptr, *cq = nullptr, *qf = nullptr,
-          *qx = nullptr, *olat = nullptr, *kv = nullptr;
-    void *h_e = nullptr, *q_e = nullptr, *cq_e = nullptr, *k_e = nullptr, *v_e = nullptr;
+          *qx = nullptr, *kv = nullptr, *lin_g = nullptr, *lin_S = nullptr;
+    void *lin_e = nullptr, *h_e = nullptr, *q_e = nullptr, *cq_e = nullptr, *k_e = nullptr, *v_e = nullptr;
     std::vector<int> moe_holder;   // per layer index of the first of its size: which layer holds the scratch now
     bool broken = false;           // a step failed half way: the states are those of no sequence
 
@@ -187,7 +188,8 @@ int LayeredModel::reserve(size_t T, size_t W, size_t keys) {
     free_all(&scratch);
     cap_tokens = cap_want = cap_keys = 0;
     size_t proj_w = 0, mid_w = 0, inner_w = 0, bc_w = 0, v_w = 0, part_w = 0, q_w = 0, lin_w = 0, head_w = 0, cq_w = 0, qf_w = 0, qx_w = 0,
-           olat_w = 0, kv_w = 0, k_w = 0, ve_w = 0;
+           kv_w = 0, k_w = 0, ve_w = 0, lin_e_w = 0, lin_S_w = 0;
+    const size_t seg = std::min<size_t>(T, jq::LIN_SEGMENT), chunks = (seg + jq::LIN_CHUNK - 1) / jq::LIN_CHUNK;
     for (const Layer &l : layers) {
         const LayerConfig &c = l.c;
         proj_w = std::max(proj_w, l.in->n);
@@ -199,11 +201,13 @@ int LayeredModel::reserve(size_t T, size_t W, size_t keys) {
         } else if (c.mixer == LayerConfig::LATENT) {
             const size_t H = c.heads;
             q_w = std::max(q_w, H * l.DP()), cq_w = std::max(cq_w, (size_t)c.q_rank), qf_w = std::max(qf_w, l.uq->n);
-            qx_w = std::max(qx_w, H * c.latent_pitch()), olat_w = std::max(olat_w, H * c.kv_rank);
-            part_w = std::max(part_w, H * jq::LAT_MAX_SPLIT * (c.kv_rank + 2));
-            kv_w = std::max(kv_w, l.ukv->n), k_w = std::max(k_w, H * l.DP()), ve_w = std::max(ve_w, H * l.DVP());
+            qx_w = std::max(qx_w, H * c.latent_pitch());
+            part_w = std::max(part_w, H * jq::LAT_MAX_SPLIT * jq::latent_part_width(c.kv_rank));
+            kv_w = std::max(kv_w, l.latent_by_heads() ? 0 : l.ukv->n), k_w = std::max(k_w, H * l.DP()), ve_w = std::max(ve_w, H * l.DVP());
         } else if (c.linear()) {
             lin_w = std::max(lin_w, (size_t)c.heads * c.out_pitch()), head_w = std::max(head_w, (size_t)c.heads);
+            const size_t H = c.heads, rs = (c.state_rows() + 15) / 16 * 16;
+            lin_e_w = std::max(lin_e_w, H * (2 * c.state_pitch() + rs)), lin_S_w = std::max(lin_S_w, H * rs * c.state_pitch());
         } else {
             inner_w = std::max(inner_w, (size_t)c.inner);
             bc_w = std::max(bc_w, l.wx->n);
@@ -224,8 +228,10 @@ int LayeredModel::reserve(size_t T, size_t W, size_t keys) {
         get(&mid, (size_t)GEMV_MAX_ROWS * mid_w) || get(&conv_f, (size_t)GEMV_MAX_ROWS * inner_w) || get(&bc, T * bc_w) ||
         get(&dt, T * inner_w) || get(&first_v, T * v_w) || get(&part, (size_t)GEMV_MAX_ROWS * part_w) || get(&lin_o, T * lin_w) ||
         get(&lin_m, T * head_w) || get(&cq, (size_t)GEMV_MAX_ROWS * cq_w) || get(&qf, T * qf_w) || get(&qx, (size_t)GEMV_MAX_ROWS * qx_w) ||
-        get(&olat, (size_t)GEMV_MAX_ROWS * olat_w) || get(&kv, keys * kv_w))
+        get(&kv, keys * kv_w))
         return 1;
+    const bool chunked = type == JQ_TYPE_BF16 && T > (size_t)GEMV_MAX_ROWS;
+    if (chunked && lin_S_w && (get(&lin_g, head_w * chunks * (2 * jq::LIN_CHUNK + 2)) || get(&lin_S, chunks * lin_S_w))) return 1;
     uint8_t *p = nullptr;
     if (get(&p, R * dense_stride(w) * esz())) return 1;
     h_e = p;
@@ -233,6 +239,10 @@ int LayeredModel::reserve(size_t T, size_t W, size_t keys) {
     q_e = p;
     if (get(&p, T * dense_stride(cq_w) * esz())) return 1;
     cq_e = p;
+    if (chunked && lin_S_w) {
+        if (get(&p, seg * lin_e_w * esz())) return 1;
+        lin_e = p;
+    }
     if (get(&p, keys * k_w * esz())) return 1;
     k_e = p;
     if (get(&p, keys * ve_w * esz())) return 1;
@@ -287,22 +297,24 @@ int LayeredModel::step(const uint32_t *tokens, uint32_t n, const uint32_t *want,
 // Attention of the queries in q_e over the keys and values in a.kc and a.vc.
 int run_attention_rows(LayeredModel *m, const jq::AttnLayer &a, bool small, float *out_f, void *out_e, hipStream_t s) {
     const uint32_t type = m->type;
-    const int dc = std::max(a.DP, a.DVP), gq = a.H / a.G, T = a.T;
+    const int dk = a.DP, dv = a.DVP, gq = a.H / a.G, T = a.T;
     const size_t ldo = dense_stride((size_t)a.H * a.dv);
-    if (type == JQ_TYPE_BF16 && dc <= 256 && !small && a.scale > 0.0f) {
+    if (type == JQ_TYPE_BF16 && dk <= 256 && dv <= 256 && !small && a.scale > 0.0f) {
         const float sl = a.scale * 1.44269504088896341f;
         const size_t rows = (size_t)T * gq;
         // two sets of 16 rows a wave where that still makes a workgroup for every compute unit
-        const bool two = dc <= 128 && (rows + 127) / 128 * a.G >= 256;
+        const bool two = dk <= 192 && dv <= 128 && (rows + 127) / 128 * a.G >= 256;
         const dim3 grid((unsigned)((rows + (two ? 127 : 63)) / (two ? 128 : 64)), (unsigned)a.G);
         const __bf16 *q = (const __bf16 *)m->q_e;
         __bf16 *o = (__bf16 *)out_e;
-#define JQ_TILES(DC, QF, KT) hipLaunchKernelGGL((jq::attention_tiles_bf16<DC, QF, KT>), grid, dim3(256), 0, s, a, q, o, ldo, sl)
-        if (dc <= 64 && two) JQ_TILES(64, 2, 64);
-        else if (dc <= 64) JQ_TILES(64, 1, 64);
-        else if (dc <= 128 && two) JQ_TILES(128, 2, 64);
-        else if (dc <= 128) JQ_TILES(128, 1, 64);
-        else JQ_TILES(256, 1, 32);
+#define JQ_TILES(DK, DV, QF, KT) hipLaunchKernelGGL((jq::attention_tiles_bf16<DK, DV, QF, KT>), grid, dim3(256), 0, s, a, q, o, ldo, sl)
+        if (dk <= 64 && dv <= 64 && two) JQ_TILES(64, 64, 2, 64);
+        else if (dk <= 64 && dv <= 64) JQ_TILES(64, 64, 1, 64);
+        else if (dk <= 128 && dv <= 128 && two) JQ_TILES(128, 128, 2, 64);
+        else if (dk <= 128 && dv <= 128) JQ_TILES(128, 128, 1, 64);
+        else if (dk <= 192 && dv <= 128 && two) JQ_TILES(192, 128, 2, 64);
+        else if (dk <= 192 && dv <= 128) JQ_TILES(192, 128, 1, 64);
+        else JQ_TILES(256, 256, 1, 32);
 #undef JQ_TILES
         return 0;
     }
@@ -365,17 +377,39 @@ int run_linear(LayeredModel *m, const Layer &l, LayerRun &r, int T, bool small, 
     a.q_scale = a.memory ? 1.0f / std::sqrt((float)c.dim) : 1.0f, a.cap = c.gate_cap, a.i_b = l.i_b, a.f_b = l.f_b;
     a.decay = l.decay, a.log_decay = l.log_decay, a.S = r.S, a.m_in = r.tail[r.tail_at], a.m_out = r.tail[r.tail_at ^ 1];
     a.o = m->lin_o, a.OP = c.out_pitch(), a.mt = m->lin_m;
+    if (m->type == JQ_TYPE_BF16 && !small) {
+        jq::LinearChunks k{};
+        k.H = a.H, k.DQ = a.DP, k.VP = k.RS = (a.rows + 15) / 16 * 16, k.OP = a.OP, k.S = m->lin_S;
+        const unsigned H = (unsigned)a.H, row_runs = (unsigned)((k.RS + 63) / 64);
+        for (int t0 = 0; t0 < T; t0 += jq::LIN_SEGMENT) {
+            jq::LinearLayer b = a;
+            b.T = std::min(jq::LIN_SEGMENT, T - t0), b.proj += (size_t)t0 * b.ld, b.o += (size_t)t0 * b.H * b.OP, b.mt += (size_t)t0 * b.H;
+            b.m_in = r.tail[r.tail_at], b.m_out = r.tail[r.tail_at ^ 1];
+            k.T = b.T, k.nc = (b.T + jq::LIN_CHUNK - 1) / jq::LIN_CHUNK, k.o = b.o;
+            k.q = (__bf16 *)m->lin_e, k.k = k.q + (size_t)k.T * k.H * k.DQ, k.v = k.k + (size_t)k.T * k.H * k.DQ;
+            const size_t places = (size_t)k.H * k.nc * jq::LIN_CHUNK;
+            k.gi = m->lin_g, k.gf = k.gi + places, k.m_at = k.gf + places, k.carry = k.m_at + (size_t)k.H * k.nc;
+            const dim3 grid((unsigned)k.nc, row_runs, H);
+            hipLaunchKernelGGL(jq::linear_prepare, dim3((unsigned)k.T), dim3(256), 0, s, b, k);
+            hipLaunchKernelGGL(jq::linear_gates, dim3(H), dim3(1024), 0, s, b, k);
+            hipLaunchKernelGGL(jq::linear_chunk_state, grid, dim3(256), 0, s, k);
+            hipLaunchKernelGGL(jq::linear_state_pass, dim3((unsigned)((a.rows * (k.DQ / 4) + 255) / 256), H), dim3(256), 0, s, k, r.S, a.rows);
+            hipLaunchKernelGGL(jq::linear_chunk_out, grid, dim3(256), 0, s, k);
+            if (a.memory) r.tail_at ^= 1;
+        }
+    } else {
 #define JQ_STEPS(LPR, NS)                                                                                                             \
     hipLaunchKernelGGL((jq::linear_steps<LPR, NS>), dim3((unsigned)((a.rows + 256 / LPR - 1) / (256 / LPR)), (unsigned)a.H), dim3(256), 0, s, a)
-    if (a.d <= 16) JQ_STEPS(4, 1);
-    else if (a.d <= 32) JQ_STEPS(8, 1);
-    else if (a.d <= 64) JQ_STEPS(16, 1);
-    else if (a.d <= 128) JQ_STEPS(16, 2);
-    else if (a.d <= 256) JQ_STEPS(16, 4);
-    else if (a.d <= 512) JQ_STEPS(32, 4);
-    else JQ_STEPS(64, 4);
+        if (a.d <= 16) JQ_STEPS(4, 1);
+        else if (a.d <= 32) JQ_STEPS(8, 1);
+        else if (a.d <= 64) JQ_STEPS(16, 1);
+        else if (a.d <= 128) JQ_STEPS(16, 2);
+        else if (a.d <= 256) JQ_STEPS(16, 4);
+        else if (a.d <= 512) JQ_STEPS(32, 4);
+        else JQ_STEPS(64, 4);
 #undef JQ_STEPS
-    if (a.memory) r.tail_at ^= 1;
+        if (a.memory) r.tail_at ^= 1;
+    }
     jq::LinearNorm n{};
     n.o = m->lin_o, n.mt = m->lin_m, n.H = a.H, n.dv = a.dv, n.OP = a.OP, n.memory = n.per_head = a.memory, n.w = l.mix_norm;
     n.gate = m->proj + l.gate_at, n.ld = a.ld, n.eps = m->cfg.norm_eps;
@@ -420,19 +454,43 @@ int run_latent(LayeredModel *m, const Layer &l, const LayerRun &r, int pos0, int
         const int n_split = std::min(jq::LAT_MAX_SPLIT, (pos0 + T + jq::LAT_RUN - 1) / jq::LAT_RUN);
         JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_absorb<E>), dim3((unsigned)((a.R + 16 * E::CH - 1) / (16 * E::CH)), H + 1, Tu), dim3(256), 0, s, a,
                                             Wuk, pitch, m->qx));
-        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_attention_any<E>), dim3((unsigned)n_split, H, Tu), dim3(256),
-                                            (size_t)(a.RP + jq::LAT_RUN) * sizeof(float), s, a, m->qx, n_split, m->part));
-        hipLaunchKernelGGL(jq::latent_merge, dim3(Tu * H, (unsigned)((a.R + 255) / 256)), dim3(256), 0, s, m->part, a.sink, a.H, a.R, n_split, m->olat);
-        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_values<E>), dim3((unsigned)((a.dv + 15) / 16), H, Tu), dim3(256), 0, s, a, m->olat, Wuv, pitch,
-                                            m->mid));
+        const size_t lds = jq::latent_mfma_lds(a.RP);
+        if (type == JQ_TYPE_BF16 && a.R <= 1024 && a.RP <= 1152) {
+            const dim3 grid((unsigned)n_split, (H + 15) / 16, Tu);
+#define JQ_LATENT(NB)                                                                                                              \
+    do {                                                                                                                           \
+        static const hipError_t attr = hipFuncSetAttribute((const void *)jq::latent_attention_mfma<NB>,                            \
+                                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)jq::latent_mfma_lds(1152)); \
+        HIP_TRY(attr);                                                                                                             \
+        hipLaunchKernelGGL((jq::latent_attention_mfma<NB>), grid, dim3(256), lds, s, a, m->qx, n_split, m->part);                  \
+    } while (0)
+            if (a.R <= 256) JQ_LATENT(1);
+            else if (a.R <= 512) JQ_LATENT(2);
+            else JQ_LATENT(4);
+#undef JQ_LATENT
+        } else {
+            JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_attention_any<E>), dim3((unsigned)n_split, H, Tu), dim3(256),
+                                                (size_t)(a.RP + jq::LAT_RUN) * sizeof(float), s, a, m->qx, n_split, m->part));
+        }
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_values<E>), dim3((unsigned)((a.dv + 4 * jq::LAT_VROWS - 1) / (4 * jq::LAT_VROWS)), H, Tu), dim3(256),
+                                            0, s, a, m->part, n_split, Wuv, pitch, m->mid));
         return 0;
     }
     const int n = pos0 + T, DP = l.DP(), DVP = l.DVP();
     JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_store<E>), dim3((unsigned)T), dim3(256), 0, s, a));
-    if (dense_gemm(l.ukv, r.kc, (size_t)a.RP, n, m->kv, l.ukv->n, s)) return 1;
-    const unsigned gy = (unsigned)std::min((a.H * (DP + DVP) + 255) / 256, 16);
-    JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_expand<E>), dim3((unsigned)n, gy), dim3(256), 0, s, a, m->kv, n, DP, DVP, (typename E::T *)m->k_e,
-                                        (typename E::T *)m->v_e));
+    if (l.latent_by_heads()) {
+        const size_t nk = (size_t)a.H * a.d, nv = (size_t)a.H * a.dv;
+        if (dense_gemm_heads(l.ukv, 0, nk, r.kc, (size_t)a.RP, n, m->k_e, a.d, (size_t)n * DP, (size_t)DP, s) ||
+            dense_gemm_heads(l.ukv, nk, nv, r.kc, (size_t)a.RP, n, m->v_e, a.dv, (size_t)n * DVP, (size_t)DVP, s))
+            return 1;
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_rest_of_keys<E>), dim3((unsigned)n), dim3(256), 0, s, a, n, DP, DVP, (typename E::T *)m->k_e,
+                                            (typename E::T *)m->v_e));
+    } else {
+        if (dense_gemm(l.ukv, r.kc, (size_t)a.RP, n, m->kv, l.ukv->n, s)) return 1;
+        const unsigned gy = (unsigned)std::min((a.H * (DP + DVP) + 255) / 256, 16);
+        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_expand<E>), dim3((unsigned)n, gy), dim3(256), 0, s, a, m->kv, n, DP, DVP, (typename E::T *)m->k_e,
+                                            (typename E::T *)m->v_e));
+    }
     JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_queries<E>), dim3((unsigned)T), dim3(256), 0, s, a, DP, (typename E::T *)m->q_e));
     jq::AttnLayer t{};
     t.H = t.G = a.H, t.d = c.dim + c.rot_dim, t.dv = a.dv, t.DP = DP, t.DVP = DVP, t.n_ctx = n, t.scale = a.scale, t.pos0 = pos0, t.T = T;

@@ -81,16 +81,72 @@ def bozosun_tensor(name: str, shape, seed: int) -> np.ndarray:
     return (n / np.sqrt(np.float32(shape[-1]))).astype(np.float32)
 
 
-def bozosun_tensors(cfg: dict, seed: int, override: "dict | None" = None, share: bool = False) -> dict:
+def fasesun_shapes(cfg: dict) -> dict:
+    """name -> shape of every tensor of a Fasesun model."""
+    w, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"])}
+
+    def gated(p, ff):
+        out[p + "gate"], out[p + "up"], out[p + "down"] = (ff, w), (ff, w), (w, ff)
+
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, mlp = f"l{i}.", layer["mixer"], layer.get("mlp")
+        H, d, nv = m["heads"], m["dim"], m["heads"] * m["vdim"]
+        out[p + "norm1"] = (w,)
+        x = p + "mix."
+        if layer["type"] == "latent_attention":
+            Q, R, rd = m["q_rank"], m["kv_rank"], m["rot_dim"]
+            out.update({x + "dq": (Q, w), x + "dq.norm": (Q,), x + "uq": (H * (d + rd), Q), x + "dkv": (R + rd, w), x + "dkv.norm": (R,),
+                        x + "uk": (H * d, R), x + "uv": (nv, R), x + "sink": (H,)})
+        else:
+            out.update({x + "q": (H * d, w), x + "k": (H * d, w), x + "v": (nv, w), x + "norm": (nv,)})
+            if layer["type"] == "mlstm":
+                out.update({x + "i": (H, w), x + "i.b": (H,), x + "f": (H, w), x + "f.b": (H,)})
+        out[x + "g"], out[x + "o"] = (nv, w), (w, nv)
+        if not mlp:
+            continue
+        E = mlp["router"]["experts"]
+        for e in range(E):
+            gated(p + f"mlp.e{e}.", mlp["expert"]["ff"])
+        out[p + "mlp.router"], out[p + "mlp.correction"] = (E, w), (E,)
+        if mlp.get("shared"):
+            gated(p + "mlp.shared.", mlp["shared"]["ff"])
+            out[p + "mlp.shared.sg"] = (1, w)
+    out["final.norm"] = (w,)
+    return out
+
+
+def fasesun_tensor(name: str, shape, seed: int) -> np.ndarray:
+    """Seeded f32 values of one tensor: matrices keep their input's scale, norms lie around 1, forget gates mostly open."""
+    role = name.split(".", 1)[-1] if name[0] == "l" and name[1].isdigit() else name
+    n = normal(seed, shape)
+    if name == "embed":
+        return n
+    if "norm" in role:
+        return (1.0 + 0.2 * n).astype(np.float32)
+    if role == "mix.f.b":
+        return (3.0 + 1.5 * n).astype(np.float32)
+    if role in ("mix.i.b", "mix.sink"):
+        return n
+    if role == "mlp.correction":
+        return (0.1 * n).astype(np.float32)
+    return (n / np.sqrt(np.float32(shape[-1]))).astype(np.float32)
+
+
+SHAPES = {"Bozosun": bozosun_shapes, "Fasesun": fasesun_shapes}
+VALUES = {"Bozosun": bozosun_tensor, "Fasesun": fasesun_tensor}
+
+
+def layered_tensors(cfg: dict, seed: int, override: "dict | None" = None, share: bool = False) -> dict:
     """name -> bf16 bit patterns of a whole model; `override` gives f32 values of some tensors instead.  `share`: layers
     and experts repeat the values of the first tensor of their role and shape (for benchmarks: faster to make)."""
     out, made = {}, {}
-    for i, (name, shape) in enumerate(bozosun_shapes(cfg).items()):
-        key = (re.sub(r"^l\d+\.|e\d+\.", "", name), shape)
+    shapes, values = SHAPES[cfg["architecture"]], VALUES[cfg["architecture"]]
+    for i, (name, shape) in enumerate(shapes(cfg).items()):
+        key = (re.sub(r"^l\d+\.|\be\d+\.", "", name), shape)
         if share and key in made:
             out[name] = made[key]
             continue
-        x = override[name] if override and name in override else bozosun_tensor(name, shape, seed * 100003 + i)
+        x = override[name] if override and name in override else values(name, shape, seed * 100003 + i)
         assert tuple(np.shape(x)) == tuple(shape), (name, np.shape(x), shape)
         out[name] = made[key] = to_bf16(x).reshape(shape)
     return out

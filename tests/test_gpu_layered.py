@@ -25,7 +25,7 @@ BOUND = {F32: 5e-5, BF16: 0.06}
 
 
 def build(tmp_path, cfg, seed, compute, n_ctx=320, override=None):
-    tensors = sl.bozosun_tensors(cfg, seed, override)
+    tensors = sl.layered_tensors(cfg, seed, override)
     path = sl.write_folder(str(tmp_path / "model"), cfg, tensors)
     return capi.Model(path, n_ctx, compute), ol.LayeredOracle(cfg, {k: sl.from_bf16(v) for k, v in tensors.items()}), path
 
@@ -328,7 +328,7 @@ def test_steps_that_are_refused(tmp_path):
 
 def test_tensors_that_are_missing_or_misshapen(tmp_path):
     cfg = lc.ONES
-    tensors = sl.bozosun_tensors(cfg, 36)
+    tensors = sl.layered_tensors(cfg, 36)
     for name in ("head", "l0.mix.vmix", "l1.mix.conv.b", "l2.mix.vmix", "l2.mlp.e1.down", "l3.norm1b.b"):
         if name == "l0.mix.vmix":
             continue                                   # the first mixing layer's is not read

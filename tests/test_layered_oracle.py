@@ -14,7 +14,7 @@ from tests import layered_cases as lc
 
 
 def oracle_of(cfg, seed, override=None):
-    return ol.LayeredOracle(cfg, {k: sl.from_bf16(v) for k, v in sl.bozosun_tensors(cfg, seed, override).items()})
+    return ol.LayeredOracle(cfg, {k: sl.from_bf16(v) for k, v in sl.layered_tensors(cfg, seed, override).items()})
 
 
 def test_layer_norm_of_a_known_row():
