@@ -358,6 +358,29 @@ static __global__ __launch_bounds__(256) void moe_combine_shared(const float *__
                                                                  int h, const float *__restrict__ shared, const float *__restrict__ logit,
                                                                  size_t ld, const float *add, float *y) {
     const size_t total = (size_t)T * h;
+    if ((h & 3) == 0) {
+        const int per = h / 4;
+        const f32x4 *o4 = (const f32x4 *)out, *s4 = (const f32x4 *)shared, *a4 = (const f32x4 *)add;
+        for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total / 4; i += (size_t)gridDim.x * 256) {
+            const int t = (int)(i / per), c = (int)(i % per);
+            f32x4 acc = add ? a4[i] : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+            for (int s = 0; s < k_used; s++) {
+                const f32x4 v = o4[((size_t)t * k_used + s) * per + c];
+                const float wt = wts[t * k_used + s];
+#pragma unroll
+                for (int r = 0; r < 4; r++) acc[r] = fmaf(v[r], wt, acc[r]);
+            }
+            if (shared) {
+                const f32x4 v = s4[i];
+                const float wt = logit ? sigmoid_of(logit[t * ld]) : 1.0f;
+#pragma unroll
+                for (int r = 0; r < 4; r++) acc[r] = fmaf(v[r], wt, acc[r]);
+            }
+            ((f32x4 *)y)[i] = acc;
+        }
+        return;
+    }
     for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) {
         const size_t t = i / h, c = i % h;
         float acc = add ? add[i] : 0.0f;

@@ -51,10 +51,10 @@ __global__ __launch_bounds__(256) void latent_store(LatentLayer a) {
 
 // ---- short steps ----
 
-// qx[t, h] = [W_uk[h]^T q | rotated q], RP numbers a row (zeros behind): grid (column runs of 16 chunks, heads + 1, tokens);
+// qx[t, h] = [W_uk[h]^T q | rotated q], RP numbers a row (zeros behind), in f32 or as the matrix cores take them: grid (column runs of 16 chunks, heads + 1, tokens);
 // the workgroups of the row behind the last head store the token's cache row.
-template <class E>
-__global__ __launch_bounds__(256) void latent_absorb(LatentLayer a, const uint8_t *__restrict__ Wuk, size_t pitch, float *__restrict__ qx) {
+template <class E, class O>
+__global__ __launch_bounds__(256) void latent_absorb(LatentLayer a, const uint8_t *__restrict__ Wuk, size_t pitch, O *__restrict__ qx) {
     constexpr int CH = E::CH;
     __shared__ float part[16][16 * CH + 1], red[4];
     const int h = blockIdx.y, t = blockIdx.z, tid = threadIdx.x;
@@ -63,7 +63,7 @@ __global__ __launch_bounds__(256) void latent_absorb(LatentLayer a, const uint8_
         return;
     }
     const float *q = a.q + ((size_t)t * a.H + h) * (a.d + a.rd);
-    float *out = qx + ((size_t)t * a.H + h) * a.RP;
+    O *out = qx + ((size_t)t * a.H + h) * a.RP;
     const int col = tid & 15, grp = tid >> 4, c0 = (int)blockIdx.x * 16 * CH, c = c0 + col * CH;
     float acc[CH] = {};
     if (c < a.R) {
@@ -83,13 +83,13 @@ __global__ __launch_bounds__(256) void latent_absorb(LatentLayer a, const uint8_
         float v = 0.0f;
 #pragma unroll
         for (int g = 0; g < 16; g++) v += part[g][tid];
-        out[c0 + tid] = v;
+        out[c0 + tid] = (O)v;
     }
     if (blockIdx.x == 0) {
         for (int i = tid; i < (a.RP - a.R + 1) / 2; i += 256) {
             const float2 v = rotated_pair(q + a.d, i, a.rd, a.rot, a.cs + (size_t)t * (a.rot / 2));
-            out[a.R + 2 * i] = v.x;
-            if (a.R + 2 * i + 1 < a.RP) out[a.R + 2 * i + 1] = v.y;
+            out[a.R + 2 * i] = (O)v.x;
+            if (a.R + 2 * i + 1 < a.RP) out[a.R + 2 * i + 1] = (O)v.y;
         }
     }
 }
@@ -149,30 +149,51 @@ __global__ __launch_bounds__(256) void latent_attention_any(LatentLayer a, const
 }
 
 // The same in bf16 on the matrix cores: a workgroup takes 16 query heads of a token over a run of keys, 64 at a time.
-//   scores  S^T = K Q^T: a wave's 16 keys straight from the cache, the heads' queries in LDS
+//   scores  S^T = K Q^T: a wave's 16 keys and the heads' queries straight from memory, the first KF fragments of a row kept
 //   softmax 16 threads a head, running maximum and sum; p goes on as the sum of two bf16 numbers
 //   sums    O^T += C^T P^T: the cache rows' columns, 64 a wave at a time, transposed through LDS
 // NB: runs of 256 latent columns.
 constexpr int LATM_SROW = 68, LATM_PROW = 144;
-__host__ __device__ inline int latent_query_row(int RP) { return 2 * RP + 16; }  // bytes
-inline size_t latent_mfma_lds(int RP) { return (size_t)16 * latent_query_row(RP) + 16 * LATM_SROW * 4 + 2 * 16 * LATM_PROW + 4 * 64 * LATM_PROW + 64; }
 
 template <int NB>
-__global__ __launch_bounds__(256) void latent_attention_mfma(LatentLayer a, const float *__restrict__ qx, int n_split, float *__restrict__ part) {
+__global__ __launch_bounds__(256, 1) void latent_attention_mfma(LatentLayer a, const __bf16 *__restrict__ qx, int n_split, float *__restrict__ part) {
     constexpr int KF = 18;
-    extern __shared__ __attribute__((aligned(16))) uint8_t lmem[];
-    const int qrow = latent_query_row(a.RP);
-    uint8_t *qs = lmem, *ph = qs + 16 * qrow, *pl = ph + 16 * LATM_PROW, *stage = pl + 16 * LATM_PROW;
-    float *sc = (float *)(stage + 4 * 64 * LATM_PROW), *al = sc + 16 * LATM_SROW;
+    __shared__ __attribute__((aligned(16))) uint8_t ph[16 * LATM_PROW], pl[16 * LATM_PROW], stage[4 * 64 * LATM_PROW];
+    __shared__ __attribute__((aligned(16))) float sc[16 * LATM_SROW];
+    __shared__ float al[16];
     const int split = blockIdx.x, h0 = 16 * (int)blockIdx.y, t = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
     const int n = a.pos0 + t + 1, per = ((n + LAT_RUN - 1) / LAT_RUN + n_split - 1) / n_split * LAT_RUN;
     const int lo = split * per, hi = min(n, lo + per);
     const __bf16 *cache = (const __bf16 *)a.cache;
-    for (int e = tid; e < 16 * (a.RP / 4); e += 256) {
-        const int r = e / (a.RP / 4), c = 4 * (e % (a.RP / 4));
-        const f32x4 v = *(const f32x4 *)(qx + ((size_t)t * a.H + min(h0 + r, a.H - 1)) * a.RP + c);
-        *(uint2 *)(qs + r * qrow + 2 * c) = __builtin_bit_cast(uint2, __builtin_convertvector(v, bf16x4));
+    // this wave's 16 keys of a tile, the first KF fragments of a row: on their way since before they are needed
+    u32x4 kf[KF], qf[KF];
+    auto fetch_keys = [&](int j0) __attribute__((always_inline)) {
+        const __bf16 *kr = cache + (size_t)min(j0 + 16 * wave + l16, hi - 1) * a.RP + 8 * g;
+#pragma unroll
+        for (int i = 0; i < KF; i++)
+            if (32 * i < a.RP) kf[i] = *(const u32x4 *)(kr + 32 * i);
+    };
+    // rows of a tile for the sums: tokens 2 pair, 2 pair + 1 and columns 8 c .. 8 c + 7 of this wave's 64
+    const int uc = lane >> 3 & 7;
+    u32x4 ra[4], rb[4];
+    auto fetch_columns = [&](int j0, int b) __attribute__((always_inline)) {
+        const int c0 = 256 * b + 64 * wave + 8 * uc;
+        const __bf16 *base = cache + (c0 < a.RP ? c0 : 0);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int j = j0 + 2 * ((lane & 7) + 8 * i);
+            ra[i] = *(const u32x4 *)(base + (size_t)min(j, hi - 1) * a.RP);
+            rb[i] = *(const u32x4 *)(base + (size_t)min(j + 1, hi - 1) * a.RP);
+        }
+    };
+    const __bf16 *qr = qx + ((size_t)t * a.H + min(h0 + l16, a.H - 1)) * a.RP + 8 * g;
+    if (lo < hi) {
+        fetch_keys(lo);
+#pragma unroll
+        for (int i = 0; i < KF; i++)
+            if (32 * i < a.RP) qf[i] = *(const u32x4 *)(qr + 32 * i);
+        fetch_columns(lo, 0);
     }
     f32x4 o[NB][4];
 #pragma unroll
@@ -181,20 +202,16 @@ __global__ __launch_bounds__(256) void latent_attention_mfma(LatentLayer a, cons
         for (int i = 0; i < 4; i++) o[b][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = -INFINITY, l = 0.0f;  // of head tid / 16, the same in its 16 threads
     uint8_t *mine = stage + wave * 64 * LATM_PROW;
-    __syncthreads();
     for (int j0 = lo; j0 < hi; j0 += LAT_RUN) {
         const int nj = min(LAT_RUN, hi - j0);
-        const __bf16 *kr = cache + (size_t)(j0 + min(16 * wave + l16, nj - 1)) * a.RP + 8 * g;
         f32x4 st{0.f, 0.f, 0.f, 0.f};
-        for (int c0 = 0; c0 < a.RP; c0 += 32 * KF) {  // KF fragments of the row on their way at once
-            u32x4 kf[KF];
 #pragma unroll
-            for (int i = 0; i < KF; i++)
-                if (c0 + 32 * i < a.RP) kf[i] = *(const u32x4 *)(kr + c0 + 32 * i);
-#pragma unroll
-            for (int i = 0; i < KF; i++)
-                if (c0 + 32 * i < a.RP) st = ElemBf16::mma(kf[i], *(const u32x4 *)(qs + l16 * qrow + 2 * (c0 + 32 * i) + 16 * g), st);
-        }
+        for (int i = 0; i < KF; i++)
+            if (32 * i < a.RP) st = ElemBf16::mma(kf[i], qf[i], st);
+        const __bf16 *kr = cache + (size_t)min(j0 + 16 * wave + l16, hi - 1) * a.RP + 8 * g;
+        for (int c = 32 * KF; c < a.RP; c += 32)
+            st = ElemBf16::mma(*(const u32x4 *)(kr + c), *(const u32x4 *)(qr + c), st);
+        if (j0 + LAT_RUN < hi) fetch_keys(j0 + LAT_RUN);
         *(f32x4 *)(sc + l16 * LATM_SROW + 16 * wave + 4 * g) = st;
         __syncthreads();
         {
@@ -215,16 +232,6 @@ __global__ __launch_bounds__(256) void latent_attention_mfma(LatentLayer a, cons
         }
 #pragma unroll
         for (int b = 0; b < NB; b++) {
-            // unit: tokens 2 pair, 2 pair + 1 and columns 8 c .. 8 c + 7 of this wave's 64
-            u32x4 ra[4], rb[4];
-            const int c0 = 256 * b + 64 * wave + 8 * (lane >> 3 & 7);
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int pair = (lane & 7) + 8 * i;
-                const __bf16 *base = cache + (c0 < a.RP ? c0 : 0);
-                ra[i] = *(const u32x4 *)(base + (size_t)(j0 + min(2 * pair, nj - 1)) * a.RP);
-                rb[i] = *(const u32x4 *)(base + (size_t)(j0 + min(2 * pair + 1, nj - 1)) * a.RP);
-            }
             __syncthreads();  // p is there; and the fragments of the columns before are read
 #pragma unroll
             for (int i = 0; i < 4; i++) {
@@ -232,10 +239,11 @@ __global__ __launch_bounds__(256) void latent_attention_mfma(LatentLayer a, cons
 #pragma unroll
                 for (int e = 0; e < 8; e++) {
                     const uint32_t x = ra[i][e / 2], y = rb[i][e / 2];
-                    *(uint32_t *)(mine + (8 * (lane >> 3 & 7) + e) * LATM_PROW + 4 * pair) =
-                        e & 1 ? (x >> 16) | (y & 0xFFFF0000u) : (x & 0xFFFFu) | (y << 16);
+                    *(uint32_t *)(mine + (8 * uc + e) * LATM_PROW + 4 * pair) = e & 1 ? (x >> 16) | (y & 0xFFFF0000u) : (x & 0xFFFFu) | (y << 16);
                 }
             }
+            if (b + 1 < NB) fetch_columns(j0, b + 1);
+            else if (j0 + LAT_RUN < hi) fetch_columns(j0 + LAT_RUN, 0);
             __syncthreads();
             const float keep = al[l16];
 #pragma unroll
@@ -285,6 +293,22 @@ __global__ __launch_bounds__(256) void latent_values(LatentLayer a, const float 
     const int h = blockIdx.y, t = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, pw = latent_part_width(a.R);
     const int j0 = ((int)blockIdx.x * 4 + wave) * LAT_VROWS;
     const float *p = part + ((size_t)t * a.H + h) * n_split * pw;
+    const bool works = j0 < a.dv;  // (the wave agrees)
+    // the rows' first pieces are on their way while the runs are merged
+    u32x4 w0[LAT_VROWS];
+    const uint8_t *rows[LAT_VROWS];
+#pragma unroll
+    for (int r = 0; r < LAT_VROWS; r++) {
+        rows[r] = Wuv + (size_t)(h * a.dv + min(j0 + r, a.dv - 1)) * pitch;
+        w0[r] = chunk_of<E>(rows[r], min(lane * E::CH, (a.R - 1) / E::CH * E::CH));
+    }
+    float first[2][16];  // the first columns' sums of the first runs
+#pragma unroll
+    for (int j = 0; j < 2; j++)
+#pragma unroll
+        for (int i = 0; i < 16; i++) first[j][i] = p[(size_t)min(i, n_split - 1) * pw + 4 + min((int)threadIdx.x + 256 * j, a.R - 1)];
+    const int my_col = h * a.dv + min(j0 + (lane & (LAT_VROWS - 1)), a.dv - 1);
+    const float z = a.gate[(size_t)t * a.ld + my_col];
     if (wave == 0) {
         const float mi = lane < n_split ? p[(size_t)lane * pw] : -INFINITY, li = lane < n_split ? p[(size_t)lane * pw + 1] : 0.0f;
         const float M = wave_max(mi), fi = mi == -INFINITY ? 0.0f : expf(mi - M);  // (a run without keys)
@@ -295,19 +319,32 @@ __global__ __launch_bounds__(256) void latent_values(LatentLayer a, const float 
     }
     __syncthreads();
     const float inv = 1.0f / total;
-    for (int c = threadIdx.x; c < a.R; c += 256) {
+#pragma unroll
+    for (int j = 0; j < 2; j++) {
+        const int c = (int)threadIdx.x + 256 * j;
+        float v = 0.0f;
+#pragma unroll
+        for (int i = 0; i < 16; i++)
+            if (i < n_split) v = fmaf(first[j][i], f[i], v);
+        if (c < a.R) {
+#pragma unroll 16
+            for (int i = 16; i < n_split; i++) v = fmaf(p[(size_t)i * pw + 4 + c], f[i], v);
+            ol[c] = v * inv;
+        }
+    }
+    for (int c = (int)threadIdx.x + 512; c < a.R; c += 256) {
         float v = 0.0f;
 #pragma unroll 16
         for (int i = 0; i < n_split; i++) v = fmaf(p[(size_t)i * pw + 4 + c], f[i], v);
         ol[c] = v * inv;
     }
     __syncthreads();
-    if (j0 >= a.dv) return;
+    if (!works) return;
     float acc[LAT_VROWS] = {};
     for (int c = lane * E::CH; c < a.R; c += 64 * E::CH) {
         u32x4 w[LAT_VROWS];
 #pragma unroll
-        for (int r = 0; r < LAT_VROWS; r++) w[r] = chunk_of<E>(Wuv + (size_t)(h * a.dv + min(j0 + r, a.dv - 1)) * pitch, c);
+        for (int r = 0; r < LAT_VROWS; r++) w[r] = c < 64 * E::CH ? w0[r] : chunk_of<E>(rows[r], c);
         float xv[E::CH];
         load_acts<E::CH>(ol, c, a.R, xv);
 #pragma unroll
@@ -321,10 +358,7 @@ __global__ __launch_bounds__(256) void latent_values(LatentLayer a, const float 
 #pragma unroll
     for (int r = 0; r < LAT_VROWS; r++) {
         const float v = wave_sum(acc[r]);
-        if (lane == r && j0 + r < a.dv) {
-            const int col = h * a.dv + j0 + r;
-            out[(size_t)t * a.H * a.dv + col] = v * sigmoid_of(a.gate[(size_t)t * a.ld + col]);
-        }
+        if (lane == r && j0 + r < a.dv) out[(size_t)t * a.H * a.dv + my_col] = v * sigmoid_of(z);
     }
 }
 

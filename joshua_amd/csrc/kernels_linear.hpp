@@ -146,16 +146,19 @@ static __global__ __launch_bounds__(256) void linear_prepare(LinearLayer a, Line
     const int t = blockIdx.x;
     const float *p = a.proj + (size_t)t * a.ld;
     const int pairs = a.H * (c.DQ / 2);
+    auto input = [&](float v) { return a.memory ? v : gate_silu(v); };
     for (int e = threadIdx.x; e < 2 * pairs; e += 256) {
         const int key = e >= pairs, i = e - key * pairs, h = i / (c.DQ / 2), d = 2 * (i % (c.DQ / 2));
         const float *src = p + (key ? a.k_at : a.q_at) + h * a.d;
         const float f = key ? 1.0f : a.q_scale;
         __bf16 *dst = (key ? c.k : c.q) + ((size_t)t * a.H + h) * c.DQ + d;
-        dst[0] = (__bf16)(d < a.d ? linear_input(a, src[d]) * f : 0.0f), dst[1] = (__bf16)(d + 1 < a.d ? linear_input(a, src[d + 1]) * f : 0.0f);
+        const float x = src[min(d, a.d - 1)], y = src[min(d + 1, a.d - 1)];
+        const __bf16 lo = (__bf16)(d < a.d ? input(x) * f : 0.0f), hi = (__bf16)(d + 1 < a.d ? input(y) * f : 0.0f);
+        *(uint32_t *)dst = __builtin_bit_cast(uint16_t, lo) | (uint32_t)__builtin_bit_cast(uint16_t, hi) << 16;
     }
     for (int e = threadIdx.x; e < a.H * c.VP; e += 256) {
         const int h = e / c.VP, r = e % c.VP;
-        c.v[(size_t)t * a.H * c.VP + e] = (__bf16)(r < a.dv ? linear_input(a, p[a.v_at + h * a.dv + r]) : r < a.rows ? 1.0f : 0.0f);
+        c.v[(size_t)t * a.H * c.VP + e] = (__bf16)(r < a.dv ? input(p[a.v_at + h * a.dv + r]) : r < a.rows ? 1.0f : 0.0f);
     }
     for (int h = threadIdx.x; h < a.H; h += 256) {
         const size_t at = (size_t)h * c.nc * LIN_CHUNK + t;
@@ -323,15 +326,16 @@ __device__ __forceinline__ void split_bf16(const f32x4 &a, const f32x4 &b, u32x4
     *hi = u32x4{h0.x, h0.y, h1.x, h1.y}, *lo = u32x4{l0.x, l0.y, l1.x, l1.y};
 }
 
-// grid (chunks, runs of 64 state rows, heads); wave w has tokens 16 w .. 16 w + 15 of the chunk, lane l16 one of them.
+// grid (chunks, runs of 64 state rows, heads).  First wave w has the weights of tokens 16 w .. 16 w + 15, then state rows
+// 16 w .. 16 w + 15 of the run and all tokens: a state is read and split once a workgroup.
 static __global__ __launch_bounds__(256) void linear_chunk_out(LinearChunks c) {
-    __shared__ __attribute__((aligned(16))) uint8_t vt[64 * LIN_TROW];
-    __shared__ float gs[LIN_CHUNK];
+    __shared__ __attribute__((aligned(16))) uint8_t vt[64 * LIN_TROW], ph[64 * LIN_TROW], pl[64 * LIN_TROW];
+    __shared__ float gs[LIN_CHUNK], Ms[LIN_CHUNK];
     const int n = blockIdx.x, v0 = 64 * (int)blockIdx.y, h = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
     const size_t at = ((size_t)h * c.nc + n) * LIN_CHUNK;
-    if (tid < LIN_CHUNK) gs[tid] = c.gi[at + tid];
-    {  // values with the tokens of a run of 32 in the order in which the lanes will hold their weights
+    if (tid < LIN_CHUNK) gs[tid] = c.gi[at + tid], Ms[tid] = c.gf[at + tid];
+    {
         const TileUnit u(tid);
         const int t0 = n * LIN_CHUNK + 2 * u.pair, ta = min(t0, c.T - 1), tb = min(t0 + 1, c.T - 1);
         u32x4 ra{0, 0, 0, 0}, rb{0, 0, 0, 0};
@@ -339,72 +343,95 @@ static __global__ __launch_bounds__(256) void linear_chunk_out(LinearChunks c) {
             ra = *(const u32x4 *)(c.v + ((size_t)ta * c.H + h) * c.VP + v0 + 8 * u.c);
             rb = *(const u32x4 *)(c.v + ((size_t)tb * c.H + h) * c.VP + v0 + 8 * u.c);
         }
-        const int run = 2 * u.pair / 32, k = 2 * u.pair % 32, place = 64 * run + 2 * (k < 16 ? 8 * (k / 4) + k % 4 : 8 * ((k - 16) / 4) + 4 + k % 4);
 #pragma unroll
         for (int e = 0; e < 8; e++) {
             const uint32_t lo = ra[e / 2], hi = rb[e / 2];
-            *(uint32_t *)(vt + (8 * u.c + e) * LIN_TROW + place) = e & 1 ? (lo >> 16) | (hi & 0xFFFF0000u) : (lo & 0xFFFFu) | (hi << 16);
+            *(uint32_t *)(vt + (8 * u.c + e) * LIN_TROW + 4 * u.pair) = e & 1 ? (lo >> 16) | (hi & 0xFFFF0000u) : (lo & 0xFFFFu) | (hi << 16);
         }
     }
-    const int tl = 16 * wave + l16, t = n * LIN_CHUNK + tl;
-    const float M = c.gf[at + tl];
-    const __bf16 *qr = c.q + ((size_t)min(t, c.T - 1) * c.H + h) * c.DQ + 8 * g;
-    const __bf16 *kr[4];
-    const float *sr[4];
+    const __bf16 *qr[4], *kr[4];
 #pragma unroll
     for (int i = 0; i < 4; i++) {
-        kr[i] = c.k + ((size_t)min(n * LIN_CHUNK + 16 * i + l16, c.T - 1) * c.H + h) * c.DQ + 8 * g;
-        sr[i] = c.S + (((size_t)h * c.nc + n) * c.RS + min(v0 + 16 * i + l16, c.RS - 1)) * c.DQ + 8 * g;
+        const size_t row = ((size_t)min(n * LIN_CHUNK + 16 * i + l16, c.T - 1) * c.H + h) * c.DQ + 8 * g;
+        qr[i] = c.q + row, kr[i] = c.k + row;
     }
-    f32x4 st[4], from[4], acc[4];
+    const bool rows_here = v0 + 16 * wave < c.RS;  // (the wave agrees)
+    const float *sr = c.S + (((size_t)h * c.nc + n) * c.RS + min(v0 + 16 * wave + l16, c.RS - 1)) * c.DQ + 8 * g;
+    f32x4 st[4], from[4];
 #pragma unroll
-    for (int i = 0; i < 4; i++) st[i] = from[i] = acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int d = 0; d < c.DQ; d += 32) {
-        const u32x4 q = *(const u32x4 *)(qr + d);
+    for (int i = 0; i < 4; i++) st[i] = from[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    struct Step {  // 32 columns' operands
+        u32x4 q[4], k[4];
+        f32x4 s0, s1;
+    };
+    auto fetch = [&](int d, Step &x) __attribute__((always_inline)) {
+        x.s0 = *(const f32x4 *)(sr + d), x.s1 = *(const f32x4 *)(sr + d + 4);
+#pragma unroll
+        for (int i = 0; i < 4; i++) x.q[i] = *(const u32x4 *)(qr[i] + d), x.k[i] = *(const u32x4 *)(kr[i] + d);
+    };
+    auto multiply = [&](const Step &x) __attribute__((always_inline)) {
+        const u32x4 own = wave == 0 ? x.q[0] : wave == 1 ? x.q[1] : wave == 2 ? x.q[2] : x.q[3];
 #pragma unroll
         for (int i = 0; i < 4; i++)
-            if (i <= wave) st[i] = ElemBf16::mma(*(const u32x4 *)(kr[i] + d), q, st[i]);
+            if (i <= wave) st[i] = ElemBf16::mma(x.k[i], own, st[i]);
+        u32x4 hi, lo;
+        split_bf16(x.s0, x.s1, &hi, &lo);
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            if (v0 + 16 * i < c.RS) {
-                u32x4 hi, lo;
-                split_bf16(*(const f32x4 *)(sr[i] + d), *(const f32x4 *)(sr[i] + d + 4), &hi, &lo);
-                from[i] = ElemBf16::mma(hi, q, from[i]);
-                from[i] = ElemBf16::mma(lo, q, from[i]);
+            from[i] = ElemBf16::mma(hi, x.q[i], from[i]);
+            from[i] = ElemBf16::mma(lo, x.q[i], from[i]);
+        }
+    };
+    Step even, odd;  // the next columns' operands travel while these are multiplied
+    fetch(0, even);
+    for (int d = 0; d < c.DQ; d += 64) {
+        if (d + 32 < c.DQ) fetch(d + 32, odd);
+        multiply(even);
+        if (d + 64 < c.DQ) fetch(d + 64, even);
+        if (d + 32 < c.DQ) multiply(odd);
+    }
+    __syncthreads();
+    {
+        const int tl = 16 * wave + l16;
+        const float M = Ms[tl];
+#pragma unroll
+        for (int i = 0; i < 4; i++) {  // keys 16 i + 4 g + r of token tl
+            f32x4 p;
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int s = 16 * i + 4 * g + r;
+                p[r] = s <= tl ? st[i][r] * exp_of(gs[s] - M) : 0.0f;
             }
+            const bf16x4 hi = __builtin_convertvector(p, bf16x4), lo = __builtin_convertvector(p - __builtin_convertvector(hi, f32x4), bf16x4);
+            *(uint2 *)(ph + tl * LIN_TROW + 32 * i + 8 * g) = __builtin_bit_cast(uint2, hi);
+            *(uint2 *)(pl + tl * LIN_TROW + 32 * i + 8 * g) = __builtin_bit_cast(uint2, lo);
         }
     }
     __syncthreads();
+    if (!rows_here) return;
+    f32x4 acc[4];
 #pragma unroll
-    for (int run = 0; run < 2; run++) {
-        if (2 * run > wave) break;
-        f32x4 p[2];
+    for (int i = 0; i < 4; i++) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int f = 0; f < 2; f++)
+    for (int ks = 0; ks < 2; ks++) {
+        const u32x4 vf = *(const u32x4 *)(vt + (16 * wave + l16) * LIN_TROW + 64 * ks + 16 * g);
 #pragma unroll
-            for (int r = 0; r < 4; r++) {
-                const int s = 32 * run + 16 * f + 4 * g + r;
-                p[f][r] = s <= tl ? st[2 * run + f][r] * exp_of(gs[s] - M) : 0.0f;
-            }
-        u32x4 hi, lo;
-        split_bf16(p[0], p[1], &hi, &lo);
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const u32x4 vf = *(const u32x4 *)(vt + (16 * i + l16) * LIN_TROW + 64 * run + 16 * g);
-            acc[i] = ElemBf16::mma(vf, hi, acc[i]);
-            acc[i] = ElemBf16::mma(vf, lo, acc[i]);
+        for (int i = 2 * ks; i < 4; i++) {  // (tokens in front of the run of keys have no weight there)
+            acc[i] = ElemBf16::mma(vf, *(const u32x4 *)(ph + (16 * i + l16) * LIN_TROW + 64 * ks + 16 * g), acc[i]);
+            acc[i] = ElemBf16::mma(vf, *(const u32x4 *)(pl + (16 * i + l16) * LIN_TROW + 64 * ks + 16 * g), acc[i]);
         }
     }
-    if (t >= c.T) return;
-    const float in = exp_of(c.m_at[h * c.nc + n] - M);
-    float *op = c.o + ((size_t)t * c.H + h) * c.OP + v0 + 4 * g;
+    const float m0 = c.m_at[h * c.nc + n];
+    const int col = v0 + 16 * wave + 4 * g;
 #pragma unroll
     for (int i = 0; i < 4; i++) {
-        if (v0 + 16 * i + 4 * g < c.OP) {
+        const int t = n * LIN_CHUNK + 16 * i + l16;
+        if (t < c.T && col < c.OP) {
+            const float in = exp_of(m0 - Ms[16 * i + l16]);
             f32x4 o;
 #pragma unroll
             for (int r = 0; r < 4; r++) o[r] = fmaf(in, from[i][r], acc[i][r]);
-            *(f32x4 *)(op + 16 * i) = o;
+            *(f32x4 *)(c.o + ((size_t)t * c.H + h) * c.OP + col) = o;
         }
     }
 }
@@ -430,15 +457,30 @@ __global__ __launch_bounds__(BT) void linear_norm_gate(LinearNorm a, O *__restri
     float inv_den = 1.0f;
     if (a.memory) inv_den = 1.0f / (fmaxf(fabsf(src[a.dv]), expf(-a.mt[(size_t)t * a.H + h0])) + 1e-6f);  // (per head then)
     auto value = [&](int c) { return (a.per_head ? src[c] : src[(size_t)(c / a.dv) * a.OP + c % a.dv]) * inv_den; };
-    float ss = 0.0f;
-    for (int c = threadIdx.x; c < n; c += BT) {
-        const float v = value(c);
-        ss = fmaf(v, v, ss);
+    const float *g = a.gate + (size_t)t * a.ld + (size_t)h0 * a.dv, *w = a.w + (size_t)h0 * a.dv;
+    // a thread's first columns stay in registers, everything of theirs asked for at once
+    constexpr int KEEP = 4;
+    float v[KEEP], gv[KEEP], wv[KEEP], ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < KEEP; i++) {
+        const int c = min((int)threadIdx.x + BT * i, n - 1);
+        v[i] = value(c), gv[i] = g[c], wv[i] = w[c];
+    }
+#pragma unroll
+    for (int i = 0; i < KEEP; i++)
+        if ((int)threadIdx.x + BT * i < n) ss = fmaf(v[i], v[i], ss);
+    for (int c = (int)threadIdx.x + KEEP * BT; c < n; c += BT) {
+        const float x = value(c);
+        ss = fmaf(x, x, ss);
     }
     const float inv = 1.0f / sqrtf(sum_block<BT>(ss, red) / (float)n + a.eps);
-    const float *g = a.gate + (size_t)t * a.ld + (size_t)h0 * a.dv, *w = a.w + (size_t)h0 * a.dv;
     O *dst = out + (size_t)t * ldo + (size_t)h0 * a.dv;
-    for (int c = threadIdx.x; c < n; c += BT) dst[c] = (O)(value(c) * inv * w[c] * sigmoid_of(g[c]));
+#pragma unroll
+    for (int i = 0; i < KEEP; i++) {
+        const int c = (int)threadIdx.x + BT * i;
+        if (c < n) dst[c] = (O)(v[i] * inv * wv[i] * sigmoid_of(gv[i]));
+    }
+    for (int c = (int)threadIdx.x + KEEP * BT; c < n; c += BT) dst[c] = (O)(value(c) * inv * w[c] * sigmoid_of(g[c]));
 }
 
 }  // namespace jq

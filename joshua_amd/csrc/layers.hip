@@ -422,7 +422,7 @@ int run_linear(LayeredModel *m, const Layer &l, LayerRun &r, int T, bool small, 
                                                     (typename E::T *)l.mix_e, dense_stride(l.mix_width())));                           \
     } while (0)
     if (len <= 256) JQ_NORM(64);
-    else if (len <= 2048) JQ_NORM(256);
+    else if (len <= 1024) JQ_NORM(256);
     else JQ_NORM(1024);
 #undef JQ_NORM
     return 0;
@@ -452,23 +452,17 @@ int run_latent(LayeredModel *m, const Layer &l, const LayerRun &r, int pos0, int
         const uint8_t *Wuk = l.ukv->dev, *Wuv = Wuk + (size_t)a.H * a.d * pitch;
         const unsigned H = (unsigned)a.H, Tu = (unsigned)T;
         const int n_split = std::min(jq::LAT_MAX_SPLIT, (pos0 + T + jq::LAT_RUN - 1) / jq::LAT_RUN);
-        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_absorb<E>), dim3((unsigned)((a.R + 16 * E::CH - 1) / (16 * E::CH)), H + 1, Tu), dim3(256), 0, s, a,
-                                            Wuk, pitch, m->qx));
-        const size_t lds = jq::latent_mfma_lds(a.RP);
-        if (type == JQ_TYPE_BF16 && a.R <= 1024 && a.RP <= 1152) {
+        const dim3 absorb((unsigned)((a.R + 16 * (type == JQ_TYPE_BF16 ? jq::ElemBf16::CH : jq::ElemF32::CH) - 1) /
+                                     (16 * (type == JQ_TYPE_BF16 ? jq::ElemBf16::CH : jq::ElemF32::CH))), H + 1, Tu);
+        if (type == JQ_TYPE_BF16 && a.R <= 1024) {
             const dim3 grid((unsigned)n_split, (H + 15) / 16, Tu);
-#define JQ_LATENT(NB)                                                                                                              \
-    do {                                                                                                                           \
-        static const hipError_t attr = hipFuncSetAttribute((const void *)jq::latent_attention_mfma<NB>,                            \
-                                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)jq::latent_mfma_lds(1152)); \
-        HIP_TRY(attr);                                                                                                             \
-        hipLaunchKernelGGL((jq::latent_attention_mfma<NB>), grid, dim3(256), lds, s, a, m->qx, n_split, m->part);                  \
-    } while (0)
-            if (a.R <= 256) JQ_LATENT(1);
-            else if (a.R <= 512) JQ_LATENT(2);
-            else JQ_LATENT(4);
-#undef JQ_LATENT
+            __bf16 *qb = (__bf16 *)m->qx;
+            hipLaunchKernelGGL((jq::latent_absorb<jq::ElemBf16, __bf16>), absorb, dim3(256), 0, s, a, Wuk, pitch, qb);
+            if (a.R <= 256) hipLaunchKernelGGL((jq::latent_attention_mfma<1>), grid, dim3(256), 0, s, a, qb, n_split, m->part);
+            else if (a.R <= 512) hipLaunchKernelGGL((jq::latent_attention_mfma<2>), grid, dim3(256), 0, s, a, qb, n_split, m->part);
+            else hipLaunchKernelGGL((jq::latent_attention_mfma<4>), grid, dim3(256), 0, s, a, qb, n_split, m->part);
         } else {
+            JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_absorb<E, float>), absorb, dim3(256), 0, s, a, Wuk, pitch, m->qx));
             JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_attention_any<E>), dim3((unsigned)n_split, H, Tu), dim3(256),
                                                 (size_t)(a.RP + jq::LAT_RUN) * sizeof(float), s, a, m->qx, n_split, m->part));
         }

@@ -14,53 +14,12 @@ from joshua_amd.synth import layered as sl
 from joshua_amd.synth import normal
 from oracle import layered as ol
 from tests import layered_cases as lc
+from tests.layered_cases import build, check, error, feed, tokens
 
 pytestmark = pytest.mark.gpu
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-F32, BF16 = capi.COMPUTE_F32, capi.COMPUTE_DEFAULT
-# root mean square of a position's difference over that of its logits: f32 against f64; bf16 activations through the
-# small stacks here
-BOUND = {F32: 5e-5, BF16: 0.06}
-
-
-def build(tmp_path, cfg, seed, compute, n_ctx=320, override=None):
-    tensors = sl.layered_tensors(cfg, seed, override)
-    path = sl.write_folder(str(tmp_path / "model"), cfg, tensors)
-    return capi.Model(path, n_ctx, compute), ol.LayeredOracle(cfg, {k: sl.from_bf16(v) for k, v in tensors.items()}), path
-
-
-def error(got, want):
-    """Per position: rms of the difference (mean taken off) over the rms of the logits."""
-    d = got - want
-    d = d - d.mean(axis=-1, keepdims=True)
-    w = want - want.mean(axis=-1, keepdims=True)
-    return np.sqrt((d ** 2).mean(axis=-1) / (w ** 2).mean())
-
-
-# how far apart a router's logits may lie for 16-bit activations to choose another expert
-CLOSE_CALL = 0.05
-
-
-def check(got, want, compute, what="", margin=None):
-    """`margin`: the statement's route_margin per token; in bf16 a token with a close call may run another expert."""
-    e = error(got, want)
-    bound = np.full(e.shape, BOUND[compute])
-    if margin is not None and compute == BF16:
-        bound[margin < CLOSE_CALL] = 1.0
-        assert (margin < CLOSE_CALL).mean() < 0.9
-    assert np.all(e <= bound), (what, float((e / bound).max()), int((e / bound).argmax()))
-
-
-def feed(m, toks, cuts):
-    """The logits of every token, the tokens cut into steps at `cuts`."""
-    m.reset()
-    edges = [0] + [c for c in cuts if 0 < c < len(toks)] + [len(toks)]
-    return np.concatenate([m.logits_at(toks[a:b], a, range(b - a)) for a, b in zip(edges, edges[1:])])
-
-
-def tokens(cfg, seed, n):
-    return np.random.default_rng(seed).integers(0, cfg["vocab"], n)
+F32, BF16, BOUND = lc.F32, lc.BF16, lc.BOUND
 
 
 # ---- products and experts alone --------------------------------------------------------------------------
@@ -144,8 +103,8 @@ def test_prompts_and_steps_match(tmp_path, name, compute):
     m, o, _ = build(tmp_path, cfg, 11, compute)
     toks = tokens(cfg, 12, 83)
     want = o.forward(toks)
-    check(feed(m, toks, []), want, compute, "whole", o.margin)
-    check(feed(m, toks, [1, 2, 3, 5, 13, 22, 24, 55, 56, 57, 65, 67]), want, compute, "cut", o.margin)
+    check(feed(m, toks, []), want, compute, "whole", o)
+    check(feed(m, toks, [1, 2, 3, 5, 13, 22, 24, 55, 56, 57, 65, 67]), want, compute, "cut", o)
 
 
 LAYERS = {
@@ -164,8 +123,8 @@ def test_one_layer_of_a_kind(tmp_path, kind, compute):
     m, o, _ = build(tmp_path, cfg, 13, compute)
     toks = tokens(cfg, 14, 70)
     want = o.forward(toks)
-    check(feed(m, toks, []), want, compute, "whole", o.margin)
-    check(feed(m, toks, [40, 41, 42, 50]), want, compute, "cut", o.margin)
+    check(feed(m, toks, []), want, compute, "whole", o)
+    check(feed(m, toks, [40, 41, 42, 50]), want, compute, "cut", o)
 
 
 @pytest.mark.parametrize("size", [1, 2, 3, 7, 8, 9, 16, 31, 33, 64, 65])
@@ -265,7 +224,7 @@ def test_long_decoding(tmp_path, compute):
     m, o, _ = build(tmp_path, cfg, 29, compute)
     toks = tokens(cfg, 30, 300)
     want = o.forward(toks)
-    check(feed(m, toks, range(20, 300)), want, compute, margin=o.margin)
+    check(feed(m, toks, range(20, 300)), want, compute, oracle=o)
 
 
 def test_wanted_places_in_any_order(tmp_path):

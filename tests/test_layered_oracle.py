@@ -11,10 +11,7 @@ from joshua_amd import capi
 from joshua_amd.synth import layered as sl
 from oracle import layered as ol
 from tests import layered_cases as lc
-
-
-def oracle_of(cfg, seed, override=None):
-    return ol.LayeredOracle(cfg, {k: sl.from_bf16(v) for k, v in sl.layered_tensors(cfg, seed, override).items()})
+from tests.layered_cases import oracle_of
 
 
 def test_layer_norm_of_a_known_row():
@@ -114,7 +111,7 @@ def test_configurations_are_checked_before_any_device_call(tmp_path):
         capi.Model(str(tmp_path), 16)
     attempt(tmp_path, "{\"architecture\": ", "JSON")
     attempt(tmp_path, {"vocab": 3}, "no \"architecture\"")
-    attempt(tmp_path, {"architecture": "Other"}, "no model of architecture `Other`: expected `Bozosun`")
+    attempt(tmp_path, {"architecture": "Other"}, "no model of architecture `Other`: expected `Bozosun`, `Fasesun`")
 
     def broken(change):
         cfg = copy.deepcopy(lc.MIXED)
