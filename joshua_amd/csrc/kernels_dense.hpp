@@ -633,6 +633,24 @@ __global__ __launch_bounds__(256) void dense_rows_to_f32(const uint8_t *__restri
     }
 }
 
+// ---- tiles transposed through LDS -----------------------------------------------------------------
+//
+// 64 rows (tokens) x 64 columns of bf16, a column's tokens side by side: what a product over the tokens reads.  A lane
+// brings columns 8 c .. 8 c + 7 of tokens 2 pair and 2 pair + 1 and writes them as eight words.  Column rows are 144 bytes
+// apart; runs of 16 bytes are exchanged by the column so that the lanes of a write (8 c's, 8 pairs) meet 64 banks.
+constexpr int TILE_COL = 144;  // bytes
+__device__ __forceinline__ int tile_word(int c, int e, int pair) { return (8 * c + e) * TILE_COL + 4 * (pair ^ 4 * (c & 6)); }
+// tokens 8 j .. 8 j + 7 of a column
+__device__ __forceinline__ int tile_chunk(int col, int j) { return col * TILE_COL + 16 * (j ^ (col >> 3 & 6)); }
+
+__device__ __forceinline__ void tile_put(uint8_t *tile, int c, int pair, const u32x4 &a, const u32x4 &b) {
+#pragma unroll
+    for (int e = 0; e < 8; e++) {
+        const uint32_t lo = a[e / 2], hi = b[e / 2];
+        *(uint32_t *)(tile + tile_word(c, e, pair)) = e & 1 ? (lo >> 16) | (hi & 0xFFFF0000u) : (lo & 0xFFFFu) | (hi << 16);
+    }
+}
+
 static __global__ __launch_bounds__(256) void fill_zero(float *__restrict__ p, size_t n) {
     for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) p[i] = 0.0f;
 }

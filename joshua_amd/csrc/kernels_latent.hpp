@@ -153,12 +153,12 @@ __global__ __launch_bounds__(256) void latent_attention_any(LatentLayer a, const
 //   softmax 16 threads a head, running maximum and sum; p goes on as the sum of two bf16 numbers
 //   sums    O^T += C^T P^T: the cache rows' columns, 64 a wave at a time, transposed through LDS
 // NB: runs of 256 latent columns.
-constexpr int LATM_SROW = 68, LATM_PROW = 144;
+constexpr int LATM_SROW = 68, LATM_PROW = 144;  // floats, bytes
 
 template <int NB>
 __global__ __launch_bounds__(256, 1) void latent_attention_mfma(LatentLayer a, const __bf16 *__restrict__ qx, int n_split, float *__restrict__ part) {
     constexpr int KF = 18;
-    __shared__ __attribute__((aligned(16))) uint8_t ph[16 * LATM_PROW], pl[16 * LATM_PROW], stage[4 * 64 * LATM_PROW];
+    __shared__ __attribute__((aligned(16))) uint8_t ph[16 * LATM_PROW], pl[16 * LATM_PROW], stage[4 * 64 * TILE_COL];
     __shared__ __attribute__((aligned(16))) float sc[16 * LATM_SROW];
     __shared__ float al[16];
     const int split = blockIdx.x, h0 = 16 * (int)blockIdx.y, t = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
@@ -176,15 +176,18 @@ __global__ __launch_bounds__(256, 1) void latent_attention_mfma(LatentLayer a, c
     };
     // rows of a tile for the sums: tokens 2 pair, 2 pair + 1 and columns 8 c .. 8 c + 7 of this wave's 64
     const int uc = lane >> 3 & 7;
-    u32x4 ra[4], rb[4];
-    auto fetch_columns = [&](int j0, int b) __attribute__((always_inline)) {
-        const int c0 = 256 * b + 64 * wave + 8 * uc;
-        const __bf16 *base = cache + (c0 < a.RP ? c0 : 0);
+    u32x4 ra[NB][4], rb[NB][4];
+    auto fetch_columns = [&](int j0) __attribute__((always_inline)) {
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int j = j0 + 2 * ((lane & 7) + 8 * i);
-            ra[i] = *(const u32x4 *)(base + (size_t)min(j, hi - 1) * a.RP);
-            rb[i] = *(const u32x4 *)(base + (size_t)min(j + 1, hi - 1) * a.RP);
+        for (int b = 0; b < NB; b++) {
+            const int c0 = 256 * b + 64 * wave + 8 * uc;
+            const __bf16 *base = cache + (c0 < a.RP ? c0 : 0);
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int j = j0 + 2 * ((lane & 7) + 8 * i);
+                ra[b][i] = *(const u32x4 *)(base + (size_t)min(j, hi - 1) * a.RP);
+                rb[b][i] = *(const u32x4 *)(base + (size_t)min(j + 1, hi - 1) * a.RP);
+            }
         }
     };
     const __bf16 *qr = qx + ((size_t)t * a.H + min(h0 + l16, a.H - 1)) * a.RP + 8 * g;
@@ -193,7 +196,7 @@ __global__ __launch_bounds__(256, 1) void latent_attention_mfma(LatentLayer a, c
 #pragma unroll
         for (int i = 0; i < KF; i++)
             if (32 * i < a.RP) qf[i] = *(const u32x4 *)(qr + 32 * i);
-        fetch_columns(lo, 0);
+        fetch_columns(lo);
     }
     f32x4 o[NB][4];
 #pragma unroll
@@ -201,7 +204,7 @@ __global__ __launch_bounds__(256, 1) void latent_attention_mfma(LatentLayer a, c
 #pragma unroll
         for (int i = 0; i < 4; i++) o[b][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = -INFINITY, l = 0.0f;  // of head tid / 16, the same in its 16 threads
-    uint8_t *mine = stage + wave * 64 * LATM_PROW;
+    uint8_t *mine = stage + wave * 64 * TILE_COL;
     for (int j0 = lo; j0 < hi; j0 += LAT_RUN) {
         const int nj = min(LAT_RUN, hi - j0);
         f32x4 st{0.f, 0.f, 0.f, 0.f};
@@ -234,16 +237,8 @@ __global__ __launch_bounds__(256, 1) void latent_attention_mfma(LatentLayer a, c
         for (int b = 0; b < NB; b++) {
             __syncthreads();  // p is there; and the fragments of the columns before are read
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int pair = (lane & 7) + 8 * i;
-#pragma unroll
-                for (int e = 0; e < 8; e++) {
-                    const uint32_t x = ra[i][e / 2], y = rb[i][e / 2];
-                    *(uint32_t *)(mine + (8 * uc + e) * LATM_PROW + 4 * pair) = e & 1 ? (x >> 16) | (y & 0xFFFF0000u) : (x & 0xFFFFu) | (y << 16);
-                }
-            }
-            if (b + 1 < NB) fetch_columns(j0, b + 1);
-            else if (j0 + LAT_RUN < hi) fetch_columns(j0 + LAT_RUN, 0);
+            for (int i = 0; i < 4; i++) tile_put(mine, uc, (lane & 7) + 8 * i, ra[b][i], rb[b][i]);
+            if (b + 1 == NB && j0 + LAT_RUN < hi) fetch_columns(j0 + LAT_RUN);
             __syncthreads();
             const float keep = al[l16];
 #pragma unroll
@@ -255,7 +250,7 @@ __global__ __launch_bounds__(256, 1) void latent_attention_mfma(LatentLayer a, c
                 const u32x4 fh = *(const u32x4 *)(ph + l16 * LATM_PROW + 64 * ks + 16 * g), fl = *(const u32x4 *)(pl + l16 * LATM_PROW + 64 * ks + 16 * g);
 #pragma unroll
                 for (int i = 0; i < 4; i++) {
-                    const u32x4 v = *(const u32x4 *)(mine + (16 * i + l16) * LATM_PROW + 64 * ks + 16 * g);
+                    const u32x4 v = *(const u32x4 *)(mine + tile_chunk(16 * i + l16, 4 * ks + g));
                     o[b][i] = ElemBf16::mma(v, fh, o[b][i]);
                     o[b][i] = ElemBf16::mma(v, fl, o[b][i]);
                 }
@@ -285,7 +280,8 @@ __global__ __launch_bounds__(256, 1) void latent_attention_mfma(LatentLayer a, c
 // heads, tokens).
 constexpr int LAT_VROWS = 8;
 
-template <class E>
+// NS: runs whose numbers are asked for ahead (n_split of them at most matter).
+template <class E, int NS>
 __global__ __launch_bounds__(256) void latent_values(LatentLayer a, const float *__restrict__ part, int n_split, const uint8_t *__restrict__ Wuv,
                                                      size_t pitch, float *__restrict__ out) {
     __shared__ __attribute__((aligned(16))) float ol[LAT_MAX_R];
@@ -302,11 +298,11 @@ __global__ __launch_bounds__(256) void latent_values(LatentLayer a, const float 
         rows[r] = Wuv + (size_t)(h * a.dv + min(j0 + r, a.dv - 1)) * pitch;
         w0[r] = chunk_of<E>(rows[r], min(lane * E::CH, (a.R - 1) / E::CH * E::CH));
     }
-    float first[2][16];  // the first columns' sums of the first runs
+    float first[2][NS];  // the first columns' sums of the first runs
 #pragma unroll
     for (int j = 0; j < 2; j++)
 #pragma unroll
-        for (int i = 0; i < 16; i++) first[j][i] = p[(size_t)min(i, n_split - 1) * pw + 4 + min((int)threadIdx.x + 256 * j, a.R - 1)];
+        for (int i = 0; i < NS; i++) first[j][i] = p[(size_t)min(i, n_split - 1) * pw + 4 + min((int)threadIdx.x + 256 * j, a.R - 1)];
     const int my_col = h * a.dv + min(j0 + (lane & (LAT_VROWS - 1)), a.dv - 1);
     const float z = a.gate[(size_t)t * a.ld + my_col];
     if (wave == 0) {
@@ -324,13 +320,9 @@ __global__ __launch_bounds__(256) void latent_values(LatentLayer a, const float 
         const int c = (int)threadIdx.x + 256 * j;
         float v = 0.0f;
 #pragma unroll
-        for (int i = 0; i < 16; i++)
+        for (int i = 0; i < NS; i++)
             if (i < n_split) v = fmaf(first[j][i], f[i], v);
-        if (c < a.R) {
-#pragma unroll 16
-            for (int i = 16; i < n_split; i++) v = fmaf(p[(size_t)i * pw + 4 + c], f[i], v);
-            ol[c] = v * inv;
-        }
+        if (c < a.R) ol[c] = v * inv;
     }
     for (int c = (int)threadIdx.x + 512; c < a.R; c += 256) {
         float v = 0.0f;
@@ -397,10 +389,25 @@ __global__ __launch_bounds__(256) void latent_rest_of_keys(LatentLayer a, int n,
 // The step's queries [T][H][DP], the rotated part turned.
 template <class E>
 __global__ __launch_bounds__(256) void latent_queries(LatentLayer a, int DP, typename E::T *__restrict__ qe) {
-    typedef typename E::T T2 __attribute__((ext_vector_type(2)));
+    using T = typename E::T;
+    typedef T T2 __attribute__((ext_vector_type(2)));
+    typedef T T4 __attribute__((ext_vector_type(4)));
     const int t = blockIdx.x, qd = a.d + a.rd;
     const float *row = a.q + (size_t)t * a.H * qd;
     const float2 *cs = a.cs + (size_t)t * (a.rot / 2);
+    if (((a.d | a.rd | a.rot) & 3) == 0) {
+        for (int e = threadIdx.x; e < a.H * (DP / 4); e += 256) {
+            const int h = e / (DP / 4), c = 4 * (e % (DP / 4)), i = c - a.d;
+            f32x4 v = *(const f32x4 *)(row + h * qd + min(c, qd - 4));
+            if (i >= 0 && i < a.rot) {
+                const f32x4 r = *(const f32x4 *)(cs + i / 2);
+                v = f32x4{v[0] * r[0] - v[1] * r[1], v[1] * r[0] + v[0] * r[1], v[2] * r[2] - v[3] * r[3], v[3] * r[2] + v[2] * r[3]};
+            }
+            if (c >= qd) v = f32x4{0.f, 0.f, 0.f, 0.f};
+            *(T4 *)(qe + ((size_t)t * a.H + h) * DP + c) = T4{(T)v[0], (T)v[1], (T)v[2], (T)v[3]};
+        }
+        return;
+    }
     for (int e = threadIdx.x; e < a.H * (DP / 2); e += 256) {
         const int h = e / (DP / 2), c0 = 2 * (e % (DP / 2));
         const float *q = row + h * qd;
@@ -410,7 +417,7 @@ __global__ __launch_bounds__(256) void latent_queries(LatentLayer a, int DP, typ
             const float2 p = rotated_pair(q + a.d, (c - a.d) / 2, a.rd, a.rot, cs);
             return (c - a.d) & 1 ? p.y : p.x;
         };
-        *(T2 *)(qe + ((size_t)t * a.H + h) * DP + c0) = T2{(typename E::T)element(c0), (typename E::T)element(c0 + 1)};
+        *(T2 *)(qe + ((size_t)t * a.H + h) * DP + c0) = T2{(T)element(c0), (T)element(c0 + 1)};
     }
 }
 

@@ -217,17 +217,16 @@ static __global__ __launch_bounds__(1024) void linear_gates(LinearLayer a, Linea
     }
 }
 
-// A tile of 64 tokens x 64 columns of bf16, 16 bytes a token and thread pair, on its way into LDS with the tokens side by
-// side: unit u (the thread) holds columns 8 c .. 8 c + 7 of tokens 2 pair and 2 pair + 1.
+// A thread's part of a transposed tile of 64 tokens x 64 columns.
 struct TileUnit {
     int c, pair;
     __device__ __forceinline__ explicit TileUnit(int u) : c((u >> 3) & 7), pair((u & 7) + 8 * (u >> 6)) {}
 };
-constexpr int LIN_TROW = LIN_CHUNK * 2 + 16;  // bytes of a column's tokens
+constexpr int LIN_PROW = LIN_CHUNK * 2 + 16;  // bytes of a token's weights
 
 // grid (chunks, runs of 64 state rows, heads)
 static __global__ __launch_bounds__(256) void linear_chunk_state(LinearChunks c) {
-    __shared__ __attribute__((aligned(16))) uint8_t vh[64 * LIN_TROW], vl[64 * LIN_TROW], kt[64 * LIN_TROW];
+    __shared__ __attribute__((aligned(16))) uint8_t vh[64 * TILE_COL], vl[64 * TILE_COL], kt[64 * TILE_COL];
     const int n = blockIdx.x, v0 = 64 * (int)blockIdx.y, h = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
     const TileUnit u(tid);
@@ -247,7 +246,7 @@ static __global__ __launch_bounds__(256) void linear_chunk_state(LinearChunks c)
         for (int e = 0; e < 8; e++) {
             const float x = wa * fa[e], y = wb * fb[e];
             const __bf16 xh = (__bf16)x, yh = (__bf16)y, xl = (__bf16)(x - (float)xh), yl = (__bf16)(y - (float)yh);
-            const int at = (8 * u.c + e) * LIN_TROW + 4 * u.pair;
+            const int at = tile_word(u.c, e, u.pair);
             *(uint32_t *)(vh + at) = __builtin_bit_cast(uint16_t, xh) | (uint32_t)__builtin_bit_cast(uint16_t, yh) << 16;
             *(uint32_t *)(vl + at) = __builtin_bit_cast(uint16_t, xl) | (uint32_t)__builtin_bit_cast(uint16_t, yl) << 16;
         }
@@ -259,22 +258,18 @@ static __global__ __launch_bounds__(256) void linear_chunk_state(LinearChunks c)
         const bool in = d0 + 8 * u.c < c.DQ;
         const u32x4 ra = *(const u32x4 *)(ka + (in ? d0 + 8 * u.c : 0)), rb = *(const u32x4 *)(kb + (in ? d0 + 8 * u.c : 0));
         if (d0) __syncthreads();
-#pragma unroll
-        for (int e = 0; e < 8; e++) {
-            const uint32_t lo = ra[e / 2], hi = rb[e / 2];
-            *(uint32_t *)(kt + (8 * u.c + e) * LIN_TROW + 4 * u.pair) = e & 1 ? (lo >> 16) | (hi & 0xFFFF0000u) : (lo & 0xFFFFu) | (hi << 16);
-        }
+        tile_put(kt, u.c, u.pair, ra, rb);
         __syncthreads();
         f32x4 acc[4];
 #pragma unroll
         for (int i = 0; i < 4; i++) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int ks = 0; ks < 2; ks++) {
-            const int at = 64 * ks + 16 * g, vat = (16 * wave + l16) * LIN_TROW + at;
+            const int vat = tile_chunk(16 * wave + l16, 4 * ks + g);
             const u32x4 fh = *(const u32x4 *)(vh + vat), fl = *(const u32x4 *)(vl + vat);
 #pragma unroll
             for (int i = 0; i < 4; i++) {
-                const u32x4 fk = *(const u32x4 *)(kt + (16 * i + l16) * LIN_TROW + at);
+                const u32x4 fk = *(const u32x4 *)(kt + tile_chunk(16 * i + l16, 4 * ks + g));
                 acc[i] = ElemBf16::mma(fk, fh, acc[i]);
                 acc[i] = ElemBf16::mma(fk, fl, acc[i]);
             }
@@ -326,69 +321,91 @@ __device__ __forceinline__ void split_bf16(const f32x4 &a, const f32x4 &b, u32x4
     *hi = u32x4{h0.x, h0.y, h1.x, h1.y}, *lo = u32x4{l0.x, l0.y, l1.x, l1.y};
 }
 
-// grid (chunks, runs of 64 state rows, heads).  First wave w has the weights of tokens 16 w .. 16 w + 15, then state rows
-// 16 w .. 16 w + 15 of the run and all tokens: a state is read and split once a workgroup.
-static __global__ __launch_bounds__(256) void linear_chunk_out(LinearChunks c) {
-    __shared__ __attribute__((aligned(16))) uint8_t vt[64 * LIN_TROW], ph[64 * LIN_TROW], pl[64 * LIN_TROW];
+// grid (chunks, runs of 64 VT state rows, heads).  q and k pass through LDS in blocks of 64 columns.  Wave w has the weights
+// of tokens 16 w .. 16 w + 15, and 16 VT of the run's state rows for all tokens: a state is read and split once a workgroup.
+template <int VT>
+__global__ __launch_bounds__(256) void linear_chunk_out(LinearChunks c) {
+    __shared__ __attribute__((aligned(16))) uint8_t vt[64 * VT * TILE_COL], mem[2 * 64 * LIN_PROW];
     __shared__ float gs[LIN_CHUNK], Ms[LIN_CHUNK];
-    const int n = blockIdx.x, v0 = 64 * (int)blockIdx.y, h = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
+    uint8_t *qs = mem, *ks = mem + 64 * 128, *ph = mem, *pl = mem + 64 * LIN_PROW;  // (the weights come when q and k are through)
+    const int n = blockIdx.x, v0 = 64 * VT * (int)blockIdx.y, h = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
     const size_t at = ((size_t)h * c.nc + n) * LIN_CHUNK;
     if (tid < LIN_CHUNK) gs[tid] = c.gi[at + tid], Ms[tid] = c.gf[at + tid];
+    // row r of a block: eight chunks of 16 bytes, chunk j at place j ^ (r & 7)
+    const int r0 = tid >> 3, ch = tid & 7;
+    const size_t row0 = ((size_t)min(n * LIN_CHUNK + r0, c.T - 1) * c.H + h) * c.DQ, row1 = ((size_t)min(n * LIN_CHUNK + r0 + 32, c.T - 1) * c.H + h) * c.DQ;
+    const int place = 16 * (ch ^ (r0 & 7));
+    u32x4 pre[4];
+    auto fetch = [&](int d) __attribute__((always_inline)) {
+        const int col = d + 8 * ch < c.DQ ? d + 8 * ch : 0;
+        pre[0] = *(const u32x4 *)(c.q + row0 + col), pre[1] = *(const u32x4 *)(c.q + row1 + col);
+        pre[2] = *(const u32x4 *)(c.k + row0 + col), pre[3] = *(const u32x4 *)(c.k + row1 + col);
+    };
+    fetch(0);
+    const float *sr[VT];
+#pragma unroll
+    for (int j = 0; j < VT; j++) sr[j] = c.S + (((size_t)h * c.nc + n) * c.RS + min(v0 + 16 * (VT * wave + j) + l16, c.RS - 1)) * c.DQ + 8 * g;
+    f32x4 state[VT][4];  // 64 columns of this wave's rows
+    auto fetch_state = [&](int d) __attribute__((always_inline)) {
+#pragma unroll
+        for (int j = 0; j < VT; j++) {
+            state[j][0] = *(const f32x4 *)(sr[j] + d), state[j][1] = *(const f32x4 *)(sr[j] + d + 4);
+            if (d + 32 < c.DQ) state[j][2] = *(const f32x4 *)(sr[j] + d + 32), state[j][3] = *(const f32x4 *)(sr[j] + d + 36);
+        }
+    };
+    fetch_state(0);
     {
         const TileUnit u(tid);
         const int t0 = n * LIN_CHUNK + 2 * u.pair, ta = min(t0, c.T - 1), tb = min(t0 + 1, c.T - 1);
-        u32x4 ra{0, 0, 0, 0}, rb{0, 0, 0, 0};
-        if (v0 + 8 * u.c < c.VP) {
-            ra = *(const u32x4 *)(c.v + ((size_t)ta * c.H + h) * c.VP + v0 + 8 * u.c);
-            rb = *(const u32x4 *)(c.v + ((size_t)tb * c.H + h) * c.VP + v0 + 8 * u.c);
-        }
 #pragma unroll
-        for (int e = 0; e < 8; e++) {
-            const uint32_t lo = ra[e / 2], hi = rb[e / 2];
-            *(uint32_t *)(vt + (8 * u.c + e) * LIN_TROW + 4 * u.pair) = e & 1 ? (lo >> 16) | (hi & 0xFFFF0000u) : (lo & 0xFFFFu) | (hi << 16);
+        for (int j = 0; j < VT; j++) {
+            const int col = v0 + 64 * j + 8 * u.c;
+            u32x4 ra{0, 0, 0, 0}, rb{0, 0, 0, 0};
+            if (col < c.VP) {
+                ra = *(const u32x4 *)(c.v + ((size_t)ta * c.H + h) * c.VP + col);
+                rb = *(const u32x4 *)(c.v + ((size_t)tb * c.H + h) * c.VP + col);
+            }
+            tile_put(vt + 64 * j * TILE_COL, u.c, u.pair, ra, rb);
         }
     }
-    const __bf16 *qr[4], *kr[4];
+    f32x4 st[4], from[VT][4];
 #pragma unroll
     for (int i = 0; i < 4; i++) {
-        const size_t row = ((size_t)min(n * LIN_CHUNK + 16 * i + l16, c.T - 1) * c.H + h) * c.DQ + 8 * g;
-        qr[i] = c.q + row, kr[i] = c.k + row;
+        st[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < VT; j++) from[j][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    const bool rows_here = v0 + 16 * wave < c.RS;  // (the wave agrees)
-    const float *sr = c.S + (((size_t)h * c.nc + n) * c.RS + min(v0 + 16 * wave + l16, c.RS - 1)) * c.DQ + 8 * g;
-    f32x4 st[4], from[4];
-#pragma unroll
-    for (int i = 0; i < 4; i++) st[i] = from[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    struct Step {  // 32 columns' operands
-        u32x4 q[4], k[4];
-        f32x4 s0, s1;
-    };
-    auto fetch = [&](int d, Step &x) __attribute__((always_inline)) {
-        x.s0 = *(const f32x4 *)(sr + d), x.s1 = *(const f32x4 *)(sr + d + 4);
-#pragma unroll
-        for (int i = 0; i < 4; i++) x.q[i] = *(const u32x4 *)(qr[i] + d), x.k[i] = *(const u32x4 *)(kr[i] + d);
-    };
-    auto multiply = [&](const Step &x) __attribute__((always_inline)) {
-        const u32x4 own = wave == 0 ? x.q[0] : wave == 1 ? x.q[1] : wave == 2 ? x.q[2] : x.q[3];
-#pragma unroll
-        for (int i = 0; i < 4; i++)
-            if (i <= wave) st[i] = ElemBf16::mma(x.k[i], own, st[i]);
-        u32x4 hi, lo;
-        split_bf16(x.s0, x.s1, &hi, &lo);
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            from[i] = ElemBf16::mma(hi, x.q[i], from[i]);
-            from[i] = ElemBf16::mma(lo, x.q[i], from[i]);
-        }
-    };
-    Step even, odd;  // the next columns' operands travel while these are multiplied
-    fetch(0, even);
     for (int d = 0; d < c.DQ; d += 64) {
-        if (d + 32 < c.DQ) fetch(d + 32, odd);
-        multiply(even);
-        if (d + 64 < c.DQ) fetch(d + 64, even);
-        if (d + 32 < c.DQ) multiply(odd);
+        if (d) __syncthreads();
+        *(u32x4 *)(qs + r0 * 128 + place) = pre[0], *(u32x4 *)(qs + (r0 + 32) * 128 + place) = pre[1];
+        *(u32x4 *)(ks + r0 * 128 + place) = pre[2], *(u32x4 *)(ks + (r0 + 32) * 128 + place) = pre[3];
+        __syncthreads();
+        u32x4 hi[VT][2], lo[VT][2];
+#pragma unroll
+        for (int j = 0; j < VT; j++)
+#pragma unroll
+            for (int kk = 0; kk < 2; kk++) split_bf16(state[j][2 * kk], state[j][2 * kk + 1], &hi[j][kk], &lo[j][kk]);
+        if (d + 64 < c.DQ) fetch(d + 64), fetch_state(d + 64);
+#pragma unroll
+        for (int kk = 0; kk < 2; kk++) {
+            if (d + 32 * kk >= c.DQ) break;
+            const int piece = 16 * ((4 * kk + g) ^ (l16 & 7));
+            u32x4 q[4];
+#pragma unroll
+            for (int i = 0; i < 4; i++) q[i] = *(const u32x4 *)(qs + (16 * i + l16) * 128 + piece);
+            const u32x4 own = *(const u32x4 *)(qs + (16 * wave + l16) * 128 + piece);
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                if (i <= wave) st[i] = ElemBf16::mma(*(const u32x4 *)(ks + (16 * i + l16) * 128 + piece), own, st[i]);
+#pragma unroll
+            for (int j = 0; j < VT; j++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    from[j][i] = ElemBf16::mma(hi[j][kk], q[i], from[j][i]);
+                    from[j][i] = ElemBf16::mma(lo[j][kk], q[i], from[j][i]);
+                }
+        }
     }
     __syncthreads();
     {
@@ -403,35 +420,38 @@ static __global__ __launch_bounds__(256) void linear_chunk_out(LinearChunks c) {
                 p[r] = s <= tl ? st[i][r] * exp_of(gs[s] - M) : 0.0f;
             }
             const bf16x4 hi = __builtin_convertvector(p, bf16x4), lo = __builtin_convertvector(p - __builtin_convertvector(hi, f32x4), bf16x4);
-            *(uint2 *)(ph + tl * LIN_TROW + 32 * i + 8 * g) = __builtin_bit_cast(uint2, hi);
-            *(uint2 *)(pl + tl * LIN_TROW + 32 * i + 8 * g) = __builtin_bit_cast(uint2, lo);
+            *(uint2 *)(ph + tl * LIN_PROW + 32 * i + 8 * g) = __builtin_bit_cast(uint2, hi);
+            *(uint2 *)(pl + tl * LIN_PROW + 32 * i + 8 * g) = __builtin_bit_cast(uint2, lo);
         }
     }
     __syncthreads();
-    if (!rows_here) return;
-    f32x4 acc[4];
-#pragma unroll
-    for (int i = 0; i < 4; i++) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int ks = 0; ks < 2; ks++) {
-        const u32x4 vf = *(const u32x4 *)(vt + (16 * wave + l16) * LIN_TROW + 64 * ks + 16 * g);
-#pragma unroll
-        for (int i = 2 * ks; i < 4; i++) {  // (tokens in front of the run of keys have no weight there)
-            acc[i] = ElemBf16::mma(vf, *(const u32x4 *)(ph + (16 * i + l16) * LIN_TROW + 64 * ks + 16 * g), acc[i]);
-            acc[i] = ElemBf16::mma(vf, *(const u32x4 *)(pl + (16 * i + l16) * LIN_TROW + 64 * ks + 16 * g), acc[i]);
-        }
-    }
     const float m0 = c.m_at[h * c.nc + n];
-    const int col = v0 + 16 * wave + 4 * g;
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-        const int t = n * LIN_CHUNK + 16 * i + l16;
-        if (t < c.T && col < c.OP) {
-            const float in = exp_of(m0 - Ms[16 * i + l16]);
-            f32x4 o;
+    for (int j = 0; j < VT; j++) {
+        const int row = 16 * (VT * wave + j), col = v0 + row + 4 * g;
+        if (v0 + row >= c.RS) break;  // (the wave agrees)
+        f32x4 acc[4];
 #pragma unroll
-            for (int r = 0; r < 4; r++) o[r] = fmaf(in, from[i][r], acc[i][r]);
-            *(f32x4 *)(c.o + ((size_t)t * c.H + h) * c.OP + col) = o;
+        for (int i = 0; i < 4; i++) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k = 0; k < 2; k++) {
+            const u32x4 vf = *(const u32x4 *)(vt + 64 * (row / 64) * TILE_COL + tile_chunk(row % 64 + l16, 4 * k + g));
+#pragma unroll
+            for (int i = 2 * k; i < 4; i++) {  // (tokens in front of the run of keys have no weight there)
+                acc[i] = ElemBf16::mma(vf, *(const u32x4 *)(ph + (16 * i + l16) * LIN_PROW + 64 * k + 16 * g), acc[i]);
+                acc[i] = ElemBf16::mma(vf, *(const u32x4 *)(pl + (16 * i + l16) * LIN_PROW + 64 * k + 16 * g), acc[i]);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int t = n * LIN_CHUNK + 16 * i + l16;
+            if (t < c.T && col < c.OP) {
+                const float in = exp_of(m0 - Ms[16 * i + l16]);
+                f32x4 o;
+#pragma unroll
+                for (int r = 0; r < 4; r++) o[r] = fmaf(in, from[j][i][r], acc[i][r]);
+                *(f32x4 *)(c.o + ((size_t)t * c.H + h) * c.OP + col) = o;
+            }
         }
     }
 }

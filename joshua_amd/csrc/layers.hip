@@ -394,7 +394,8 @@ int run_linear(LayeredModel *m, const Layer &l, LayerRun &r, int T, bool small, 
             hipLaunchKernelGGL(jq::linear_gates, dim3(H), dim3(1024), 0, s, b, k);
             hipLaunchKernelGGL(jq::linear_chunk_state, grid, dim3(256), 0, s, k);
             hipLaunchKernelGGL(jq::linear_state_pass, dim3((unsigned)((a.rows * (k.DQ / 4) + 255) / 256), H), dim3(256), 0, s, k, r.S, a.rows);
-            hipLaunchKernelGGL(jq::linear_chunk_out, grid, dim3(256), 0, s, k);
+            if (k.RS <= 64) hipLaunchKernelGGL((jq::linear_chunk_out<1>), grid, dim3(256), 0, s, k);
+            else hipLaunchKernelGGL((jq::linear_chunk_out<2>), dim3((unsigned)k.nc, (unsigned)((k.RS + 127) / 128), H), dim3(256), 0, s, k);
             if (a.memory) r.tail_at ^= 1;
         }
     } else {
@@ -466,8 +467,11 @@ int run_latent(LayeredModel *m, const Layer &l, const LayerRun &r, int pos0, int
             JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_attention_any<E>), dim3((unsigned)n_split, H, Tu), dim3(256),
                                                 (size_t)(a.RP + jq::LAT_RUN) * sizeof(float), s, a, m->qx, n_split, m->part));
         }
-        JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_values<E>), dim3((unsigned)((a.dv + 4 * jq::LAT_VROWS - 1) / (4 * jq::LAT_VROWS)), H, Tu), dim3(256),
-                                            0, s, a, m->part, n_split, Wuv, pitch, m->mid));
+        const dim3 values((unsigned)((a.dv + 4 * jq::LAT_VROWS - 1) / (4 * jq::LAT_VROWS)), H, Tu);
+#define JQ_VALUES(NS) JQ_ELEM_OF(type, hipLaunchKernelGGL((jq::latent_values<E, NS>), values, dim3(256), 0, s, a, m->part, n_split, Wuv, pitch, m->mid))
+        if (n_split <= 16) JQ_VALUES(16);
+        else JQ_VALUES(jq::LAT_MAX_SPLIT);
+#undef JQ_VALUES
         return 0;
     }
     const int n = pos0 + T, DP = l.DP(), DVP = l.DVP();
