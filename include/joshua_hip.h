@@ -411,7 +411,7 @@ int jq_qwen3_load_gguf(const char *path, uint32_t n_ctx, jq_model **out);
 
 /* ---- Models of any architecture ------------------------------------------------------
  * jq_model_load picks the loader by what the path holds: a GGUF file by its general.architecture (qwen3, qwen3moe),
- * a folder with config.json and model.safetensors by the configuration's "architecture" (Bozosun).  The jq_qwen3_*
+ * a folder with config.json and model.safetensors by the configuration's "architecture" (Bozosun, Fasesun).  The jq_qwen3_*
  * calls above and these work on the same objects.  No counterpart in the reference, whose model object is one Rust
  * type per architecture. */
 #define JQ_COMPUTE_DEFAULT 0u  /* the precision the architecture is served with */
